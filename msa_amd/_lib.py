@@ -1,4 +1,4 @@
-"""ctypes binding of the C ABI declared in ``include/msa_amd.h``.
+"""ctypes binding of the C ABIs declared in ``include/msa_amd.h`` and ``include/msa_seq.h``.
 
 There is no fallback: if the HIP library is missing or a call fails, an exception is raised.
 """
@@ -10,6 +10,8 @@ from typing import Optional
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.environ.get("MSA_AMD_LIB", os.path.join(HERE, "libmsa_amd.so"))   # override: an alternative build
+
+SEQ_LIB_PATH = os.path.join(HERE, "libmsa_seq.so")
 
 MSA_BF16, MSA_F32 = 0, 1
 MODE_COSINE, MODE_SCALED_DOT = 0, 1
@@ -75,34 +77,96 @@ SIGNATURES = {
 }
 
 
+class SeqBatch(C.Structure):
+    """``msa_seq_batch``."""
+    _fields_ = [("cu", _vp), ("row_seq", _vp), ("slot", _vp), ("pos", _vp), ("n_seq", _i32), ("rows", _i32),
+                ("max_rows", _i32), ("reserved", _i32)]
+
+
+class DynTanh(C.Structure):
+    """``msa_dyn_tanh``."""
+    _fields_ = [("w", _vp), ("b", _vp), ("alpha", _f32), ("reserved", _i32)]
+
+
+class RowsArgs(C.Structure):
+    """``msa_rows_args``."""
+    _fields_ = [("x", _vp), ("x_b", _vp), ("w", _vp), ("out", _vp), ("x_stride", _i64), ("x_b_stride", _i64),
+                ("out_stride", _i64), ("M", _i32), ("N", _i32), ("K", _i32), ("groups", _i32), ("n_b", _i32), ("gelu_n", _i32),
+                ("cap", _f32), ("reserved", _i32), ("add", _vp),
+                ("x_in", _vp), ("x_out", _vp), ("gate", _vp), ("gate_stride", _i64), ("gate_bias", _vp), ("norm", DynTanh),
+                ("h", _vp), ("shift", _vp), ("prev", _vp), ("h_shift", _vp),
+                ("taps", _vp), ("conv_bias", _vp), ("conv_state", _vp), ("conv_lo", _i32), ("conv_n", _i32), ("conv_k", _i32),
+                ("reserved2", _i32),
+                ("z_bias", _vp), ("u_bias", _vp), ("gru_state", _vp), ("out2", _vp), ("gru_n", _i32), ("reserved3", _i32),
+                ("slot", _vp)]
+
+
+ROWS_PLAIN, ROWS_F32, ROWS_RESIDUAL, ROWS_MAMBA, ROWS_GRU = range(5)
+_batch = C.POINTER(SeqBatch)
+
+# include/msa_seq.h
+SEQ_SIGNATURES = {
+    "msa_seq_residual_norm": (C.c_int, [_vp, _vp, _i64, _vp, _i64, _vp, _vp, _i32, _i32, C.POINTER(DynTanh), _vp, _vp, _vp, _vp,
+                                        _batch, _vp]),
+    "msa_seq_gelu": (C.c_int, [_vp, _i64, _i32, _i32, _i32, _vp]),
+    "msa_seq_softcap": (C.c_int, [_vp, _i32, _i64, _f32, _vp, _vp]),
+    "msa_seq_join": (C.c_int, [_vp, _vp, _i32, _i32, _i32, _vp, _vp]),
+    "msa_seq_conv_silu": (C.c_int, [_vp, _i64, _vp, _vp, _i32, _i32, _i32, _vp, _vp, _i64, _batch, _vp]),
+    "msa_seq_ssd_scan": (C.c_int, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _batch,
+                                   _vp]),
+    "msa_seq_ssd_chunked_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32, _i32]),
+    "msa_seq_ssd_chunked": (C.c_int, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _vp, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _batch,
+                                      _vp, _sz, _vp]),
+    "msa_seq_group_rmsnorm": (C.c_int, [_vp, _i32, _i32, _i32, _i32, _vp, _f32, _vp, _vp]),
+    "msa_seq_min_gru_workspace_bytes": (_sz, [_i32, _i32, _i32, _i32]),
+    "msa_seq_min_gru": (C.c_int, [_vp, _i64, _vp, _vp, _i32, _i32, _vp, _vp, _batch, _vp, _sz, _vp]),
+    "msa_seq_latent_append": (C.c_int, [_vp, _i64, _vp, _f32, _i32, _i32, _vp, _i64, _batch, _vp]),
+    "msa_seq_latent_attn": (C.c_int, [_vp, _vp, _i64, _vp, _f32, _i32, _i32, _i32, _vp, _batch, _vp]),
+    "msa_seq_latent_decode_workspace_bytes": (_sz, [_i32, _i32, _i32, _i64]),
+    "msa_seq_latent_decode": (C.c_int, [_vp, _vp, _i64, _vp, _f32, _i32, _i32, _i32, _i64, _vp, _batch, _vp, _sz, _vp]),
+    "msa_seq_flash": (C.c_int, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _f32, _i32, _i32, _i32, _i32, _vp, _batch, _vp]),
+    "msa_rows_linear": (C.c_int, [C.POINTER(RowsArgs), _i32, _vp]),
+}
+# entry points of include/msa_amd.h that libmsa_seq.so holds too (the error text is per library)
+SEQ_SHARED = ("msa_last_error", "msa_abi_version", "msa_greedy_sample")
+
+
 class MsaError(RuntimeError):
     def __init__(self, code: int, where: str, message: str):
         super().__init__(f"{where} failed with code {code}: {message}")
         self.code = code
 
 
-_lib: Optional[C.CDLL] = None
+_libs = {}
+
+
+def _open(path: str, table) -> C.CDLL:
+    if path in _libs:
+        return _libs[path]
+    if not os.path.exists(path):
+        raise ImportError(f"{path} is missing: build it with `python -m msa_amd.build` "
+                          "(there is no CPU or PyTorch fallback for this path)")
+    lib = C.CDLL(path)
+    for name, (res, args) in table.items():
+        fn = getattr(lib, name)          # AttributeError if the library lacks a declared symbol
+        fn.restype, fn.argtypes = res, args
+    _libs[path] = lib
+    return lib
 
 
 def load() -> C.CDLL:
     """Loads the library and declares every entry point; raises if it is missing."""
-    global _lib
-    if _lib is not None:
-        return _lib
-    if not os.path.exists(LIB_PATH):
-        raise ImportError(f"{LIB_PATH} is missing: build it with `python -m msa_amd.build` "
-                          "(there is no CPU or PyTorch fallback for this path)")
-    lib = C.CDLL(LIB_PATH)
-    for name, (res, args) in SIGNATURES.items():
-        fn = getattr(lib, name)          # AttributeError if the library lacks a declared symbol
-        fn.restype, fn.argtypes = res, args
-    _lib = lib
-    return lib
+    return _open(LIB_PATH, SIGNATURES)
 
 
-def check(code: int, where: str) -> None:
+def load_seq() -> C.CDLL:
+    """The same for the library of the recurrent / latent-attention layers."""
+    return _open(SEQ_LIB_PATH, {**SEQ_SIGNATURES, **{n: SIGNATURES[n] for n in SEQ_SHARED}})
+
+
+def check(code: int, where: str, lib: Optional[C.CDLL] = None) -> None:
     if code != 0:
-        raise MsaError(code, where, load().msa_last_error().decode("utf-8", "replace"))
+        raise MsaError(code, where, (lib or load()).msa_last_error().decode("utf-8", "replace"))
 
 
 def ptr(t) -> Optional[int]:

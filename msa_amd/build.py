@@ -1,9 +1,11 @@
-"""Builds ``libmsa_amd.so`` (the C-ABI library) from ``csrc/*.hip`` for gfx950 with hipcc.
+"""Builds the C-ABI libraries from ``csrc/*.hip`` for gfx950 with hipcc: ``libmsa_amd.so`` (routing / sparse attention)
+and ``libmsa_seq.so`` (recurrent and latent-attention layers).
 
-``python -m msa_amd.build`` compiles in-tree; the library then travels with the source tree.
+``python -m msa_amd.build`` compiles both in-tree; the libraries then travel with the source tree.
 """
 from __future__ import annotations
 
+import fcntl
 import os
 import re
 import subprocess
@@ -13,6 +15,8 @@ from concurrent.futures import ThreadPoolExecutor
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libmsa_amd.so")
+SEQ_LIB = os.path.join(HERE, "libmsa_seq.so")
+SHARED = ("status.hip", "glue.hip")          # linked into both libraries
 ARCH = "gfx950"
 # packed fp32 VALU ops are switched off for all device code of this library
 FLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-Xclang", "-target-feature", "-Xclang",
@@ -21,6 +25,15 @@ FLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-Xclang", "-ta
 
 def sources():
     return sorted(os.path.join(CSRC, f) for f in os.listdir(CSRC) if f.endswith(".hip"))
+
+
+def seq_sources():
+    """What ``libmsa_seq.so`` is made of: the ``seq_*`` sources and the shared ones."""
+    return [s for s in sources() if os.path.basename(s).startswith("seq_") or os.path.basename(s) in SHARED]
+
+
+def main_sources():
+    return [s for s in sources() if not os.path.basename(s).startswith("seq_")]
 
 
 def _compile(src: str) -> str:
@@ -122,25 +135,46 @@ def _check_contracts(src: str) -> None:
         raise RuntimeError("inline-asm contract broken in %s:\n  %s" % (src, "\n  ".join(problems[:20])))
 
 
+def _link(objs, lib: str) -> str:
+    tmp = lib + ".tmp"
+    r = subprocess.run(["hipcc", "-shared", "-fPIC", f"--offload-arch={ARCH}", *objs, "-o", tmp],
+                       capture_output=True, text=True)
+    if r.returncode != 0:
+        raise RuntimeError(f"link failed:\n{r.stderr}")
+    os.replace(tmp, lib)
+    return lib
+
+
+def build_seq(jobs: int = 8) -> str:
+    """Compiles and links ``libmsa_seq.so`` alone."""
+    with ThreadPoolExecutor(max_workers=jobs) as ex:
+        return _link(list(ex.map(_compile, seq_sources())), SEQ_LIB)
+
+
+def ensure_seq() -> str:
+    """``libmsa_seq.so``, compiled if it is missing (a fresh checkout); concurrent callers wait for the first."""
+    if not os.path.exists(SEQ_LIB):
+        with open(SEQ_LIB + ".lock", "w") as lock:
+            fcntl.flock(lock, fcntl.LOCK_EX)
+            if not os.path.exists(SEQ_LIB):
+                build_seq()
+    return SEQ_LIB
+
+
 def build(jobs: int = 8) -> str:
-    """Compiles every source (always, even if the library exists), checks the inline-asm contracts on the device
-    assembly and links the shared library."""
+    """Compiles every source (always, even if the libraries exist), checks the inline-asm contracts on the device
+    assembly and links both shared libraries."""
     srcs = sources()
     for gen, inc in (("gen_scan_asm.py", "scan_asm.inc"), ("gen_flash_asm.py", "flash_asm.inc")):
         if subprocess.run([sys.executable, os.path.join(CSRC, gen), "--check"]).returncode != 0:
             raise RuntimeError(f"csrc/{inc} is not what csrc/{gen} generates: run the generator")
     with ThreadPoolExecutor(max_workers=min(jobs, len(srcs) + len(CONTRACTS))) as ex:
         checks = [ex.submit(_check_contracts, s) for s in srcs if os.path.basename(s) in CONTRACTS]
-        objs = list(ex.map(_compile, srcs))
+        objs = dict(zip(srcs, ex.map(_compile, srcs)))
         for c in checks:
             c.result()
-    tmp = LIB + ".tmp"
-    r = subprocess.run(["hipcc", "-shared", "-fPIC", f"--offload-arch={ARCH}", *objs, "-o", tmp],
-                       capture_output=True, text=True)
-    if r.returncode != 0:
-        raise RuntimeError(f"link failed:\n{r.stderr}")
-    os.replace(tmp, LIB)
-    return LIB
+    _link([objs[s] for s in seq_sources()], SEQ_LIB)
+    return _link([objs[s] for s in main_sources()], LIB)
 
 
 if __name__ == "__main__":

@@ -4,7 +4,8 @@ as the reference's ``CustomDynamicCache`` (src/utils/cache.py:14-172) without th
 class; pooled tensors are kept in the reference's ``[1, Hkv, C, D]`` view convention."""
 from __future__ import annotations
 
-from typing import Dict, List, Optional, Tuple
+from dataclasses import dataclass
+from typing import Dict, Hashable, List, Optional, Sequence, Tuple
 
 import torch
 
@@ -108,3 +109,71 @@ def compact_cache_reference_layout(key_cache: torch.Tensor, value_cache: torch.T
         rows = rows * mask.view(B, max_len, 1, 1).to(rows.dtype)
         out.append(rows.permute(0, 2, 1, 3).contiguous())
     return out[0], out[1], mask
+
+
+@dataclass(frozen=True)
+class StateSpec:
+    """One tensor a layer keeps per sequence: a fixed-size state (zeros for a new sequence), or with ``per_token`` one row
+    of ``shape`` per token."""
+    shape: Tuple[int, ...]
+    dtype: torch.dtype
+    per_token: bool = False
+
+
+class SequenceStateCache:
+    """What sequences leave behind between steps, for models whose layers keep recurrent states, convolution inputs and
+    per-token rows side by side.  Sequences own a slot; ``tensors[run][name]`` is ``[slots, *shape]``, or
+    ``[slots, capacity, *shape]`` for per-token rows.  A closed sequence's slot is given to the next one, its fixed states
+    cleared at that moment (rows need no clearing: nothing reads past a sequence's length)."""
+
+    def __init__(self, specs: Sequence[Dict[str, StateSpec]], device, slots: int = 1, capacity: int = 256):
+        self.specs, self.device = list(specs), device
+        self.slots, self.capacity = 0, max(1, capacity)
+        self.tensors: List[Dict[str, torch.Tensor]] = [{} for _ in self.specs]
+        self.slot_of: Dict[Hashable, int] = {}
+        self.length: Dict[Hashable, int] = {}
+        self._free: List[int] = []
+        self._resize(max(1, slots), self.capacity)
+
+    def _resize(self, slots: int, capacity: int) -> None:
+        for spec, held in zip(self.specs, self.tensors):
+            for name, s in spec.items():
+                shape = (slots, capacity) + s.shape if s.per_token else (slots,) + s.shape
+                old = held.get(name)
+                if old is not None and old.shape == shape:
+                    continue
+                new = torch.zeros(shape, dtype=s.dtype, device=self.device)
+                if old is not None and s.per_token:
+                    new[:old.shape[0], :old.shape[1]].copy_(old)
+                elif old is not None:
+                    new[:old.shape[0]].copy_(old)
+                held[name] = new
+        self._free += range(self.slots, slots)
+        self.slots, self.capacity = slots, capacity
+
+    def open(self, key: Hashable) -> int:
+        """Gives ``key`` a cleared slot."""
+        if key in self.slot_of:
+            raise KeyError(f"sequence {key!r} is already open")
+        if not self._free:
+            self._resize(2 * self.slots, self.capacity)
+        slot = self._free.pop(0)
+        for spec, held in zip(self.specs, self.tensors):
+            for name, s in spec.items():
+                if not s.per_token:
+                    held[name][slot].zero_()
+        self.slot_of[key], self.length[key] = slot, 0
+        return slot
+
+    def close(self, key: Hashable) -> None:
+        """Gives the sequence's slot back."""
+        self._free.append(self.slot_of.pop(key))
+        del self.length[key]
+
+    def reserve(self, tokens: int) -> None:
+        """Room for sequences of ``tokens`` tokens (grows by at least half; contents are kept)."""
+        if tokens > self.capacity:
+            self._resize(self.slots, max(tokens, self.capacity + self.capacity // 2))
+
+    def advance(self, key: Hashable, tokens: int) -> None:
+        self.length[key] += tokens

@@ -96,3 +96,119 @@ class MSAConfig:
     def __post_init__(self):
         if isinstance(self.msa_config, dict) and not isinstance(self.msa_config, DotDict):
             self.msa_config = DotDict(self.msa_config)
+
+
+# ------------------------------------------------------------------------------ recurrent / latent-attention decoders
+def _fields(cls, d: dict, where: str):
+    """Builds dataclass ``cls`` from ``d``; unknown or missing keys are an error that names the place."""
+    names = [f for f in cls.__dataclass_fields__]
+    unknown = sorted(set(d) - set(names))
+    if unknown:
+        raise ValueError(f"{where}: unknown keys {unknown}")
+    try:
+        return cls(**d)
+    except TypeError as e:
+        raise ValueError(f"{where}: {e}") from None
+
+
+@dataclass
+class Mamba2Config:
+    """State-space mixer: ``heads`` of ``vdim`` value and ``state`` state dimensions, ``groups`` of heads sharing B / C,
+    ``conv`` taps, output norm in ``norm_groups`` parts."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv: int
+    norm_groups: int
+
+    def __post_init__(self):
+        if self.heads % self.groups or self.inner % self.norm_groups:
+            raise ValueError(f"mamba2: {self.heads} heads in {self.groups} groups, {self.inner} columns in {self.norm_groups} parts")
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def conv_channels(self) -> int:
+        return self.inner + 2 * self.groups * self.state
+
+
+@dataclass
+class MinGRUConfig:
+    width: int
+
+
+@dataclass
+class LatentAttentionConfig:
+    heads: int
+    dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+
+
+@dataclass
+class DenseMLPConfig:
+    ff: int
+    kind: str = "dense"
+
+    def __post_init__(self):
+        if self.kind != "dense":
+            raise NotImplementedError(f"unsupported feed-forward {self.kind!r}")
+
+
+MIXER_CONFIGS = {"mamba2": Mamba2Config, "mingru": MinGRUConfig, "latent_attention": LatentAttentionConfig}
+
+
+@dataclass
+class HybridLayerConfig:
+    type: str
+    mixer: Union[Mamba2Config, MinGRUConfig, LatentAttentionConfig]
+    mlp: Union[DenseMLPConfig, None]
+
+
+@dataclass
+class LoopConfig:
+    """Layers ``start .. stop - 1`` run ``times`` times in a row with the same weights."""
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass
+class HybridConfig:
+    """A decoder whose layers each name their mixer and feed-forward, with an optional looped range of layers, dynamic-tanh
+    norms, token shift and gated residuals (the Gevonex architecture)."""
+    vocab: int
+    width: int
+    layers: List[HybridLayerConfig]
+    norm_eps: float
+    loop: Union[LoopConfig, None] = None
+    logit_softcap: Union[float, None] = None
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "HybridConfig":
+        layers = []
+        for i, e in enumerate(d["layers"]):
+            where = f"layers[{i}]"
+            if e["type"] not in MIXER_CONFIGS:
+                raise NotImplementedError(f"{where}: unsupported mixer {e['type']!r}")
+            mlp = e.get("mlp")
+            layers.append(HybridLayerConfig(e["type"], _fields(MIXER_CONFIGS[e["type"]], e["mixer"], where + ".mixer"),
+                                            None if mlp is None else _fields(DenseMLPConfig, mlp, where + ".mlp")))
+        loop = d.get("loop")
+        loop = None if loop is None else _fields(LoopConfig, loop, "loop")
+        if loop is not None and not (0 <= loop.start < loop.stop <= len(layers) and loop.times >= 1):
+            raise ValueError(f"loop: {loop} over {len(layers)} layers")
+        return cls(d["vocab"], d["width"], layers, d["norm"]["eps"], loop, d.get("logit_softcap"))
+
+    @property
+    def runs(self) -> List[tuple]:
+        """``(layer, pass)`` in the order they run; the pass is None outside the loop.  Each run has its own state."""
+        n, lp = len(self.layers), self.loop
+        if lp is None:
+            return [(i, None) for i in range(n)]
+        return ([(i, None) for i in range(lp.start)] + [(i, t) for t in range(lp.times) for i in range(lp.start, lp.stop)]
+                + [(i, None) for i in range(lp.stop, n)])

@@ -1,21 +1,8 @@
-// Error plumbing and the memory-bank handle (host code only).
-#include <stdarg.h>
+// The memory-bank handle (host code only).
 #include <stdlib.h>
 #include <string.h>
 
 #include "common.h"
-
-static thread_local char g_err[512] = "";
-
-void msa_set_error(const char* fmt, ...) {
-  va_list ap;
-  va_start(ap, fmt);
-  vsnprintf(g_err, sizeof(g_err), fmt, ap);
-  va_end(ap);
-}
-
-extern "C" const char* msa_last_error(void) { return g_err; }
-extern "C" int msa_abi_version(void) { return 1; }
 
 extern "C" int msa_bank_create(msa_bank** out, int32_t n_layers, int64_t C, int32_t Hkv, int32_t D,
                                int32_t dtype, const int32_t* doc_chunk_off_host,

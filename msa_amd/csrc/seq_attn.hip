@@ -1,0 +1,549 @@
+// Attention over latents with a learned sink in the softmax denominator.
+//
+// Decoding works on the latents themselves: a head's query is multiplied by its key matrix beforehand, so all heads of a
+// token share one pass over the cached rows (scores and values come from the same bytes).  Prefill works on keys and
+// values expanded per head, which costs a fraction of the multiplications per (query, key) pair.
+//   latent_attn_kernel    any rank and type: a workgroup per (row, head), fp32 arithmetic throughout
+//   latent_decode_kernel  bf16: a workgroup per (row, range of keys, up to 32 heads), 16x16x32 MFMA, then a combine step
+//   flash_sink_kernel     bf16 prefill: 32 query columns per wavefront, transposed score tile, 32x32x16 MFMA
+#include <algorithm>
+
+#include "seq_common.h"
+
+namespace {
+
+typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8_t;
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4_t;
+typedef __attribute__((__vector_size__(16 * sizeof(float)))) float floatx16_t;
+typedef short shortx4_t __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) shortx4_t lds_shortx4_t;
+
+constexpr float kLog2e = 1.4426950408889634f;
+
+// Transposing LDS read of 16-bit elements: within each group of 16 lanes, lanes 4 r .. 4 r + 3 name the four 8-byte
+// pieces of row r (r = 0..3, 16 elements) and lane j receives element j of rows 0..3.
+__device__ __forceinline__ shortx4_t lds_read_tr16(const bf16_t* p) {
+  return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_shortx4_t*)(p));
+}
+__device__ __forceinline__ bf16x8_t join8(shortx4_t lo, shortx4_t hi) {
+  return __builtin_bit_cast(bf16x8_t, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+}
+__device__ __forceinline__ float half_wave_max(float x) {
+  const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+  return fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
+}
+__device__ __forceinline__ float half_wave_sum(float x) {
+  const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+  return __uint_as_float(r[0]) + __uint_as_float(r[1]);
+}
+
+// ------------------------------------------------------------------------------------------------ any rank and type
+constexpr int kMaxCols = 8;            // rank <= 256 * kMaxCols
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_attn_kernel(const T* __restrict__ q, const T* __restrict__ cache, int64_t Lcap,
+                                                          const float* __restrict__ sink, float scale, int32_t H, int32_t rank,
+                                                          T* __restrict__ ctx, msa_seq_batch b) {
+  extern __shared__ float qs[];        // [rank], then 64 scores
+  float* sc = qs + rank;
+  const int row = blockIdx.x, head = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int s = b.row_seq[row];
+  const int n_keys = (int)(b.pos[s] + (row - b.cu[s]) + 1);
+  const T* c = cache + (int64_t)b.slot[s] * Lcap * rank;
+  const int64_t qat = ((int64_t)row * H + head) * rank;
+  for (int i = tid; i < rank; i += 256) qs[i] = to_f32<T>(q[qat + i]);
+  float m = sink[head], l = 1.f;       // the sink is the softmax's first member
+  float acc[kMaxCols] = {};
+  __syncthreads();
+  for (int k0 = 0; k0 < n_keys; k0 += 64) {
+    const int nk = min(64, n_keys - k0);
+    for (int j = wave; j < nk; j += 4) {
+      float d = 0.f;
+      for (int i = lane; i < rank; i += 64) d += qs[i] * to_f32<T>(c[(int64_t)(k0 + j) * rank + i]);
+#pragma unroll
+      for (int o = 32; o > 0; o >>= 1) d += __shfl_xor(d, o);
+      if (lane == 0) sc[j] = d * scale;
+    }
+    __syncthreads();
+    const float mine = lane < nk ? sc[lane] : -INFINITY;
+    float mx = mine;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o));
+    const float m_new = fmaxf(m, mx), alpha = expf(m - m_new);
+    const float p = expf(mine - m_new);
+    float sum = p;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) sum += __shfl_xor(sum, o);
+    l = l * alpha + sum;
+    m = m_new;
+    __syncthreads();
+    if (wave == 0) sc[lane] = p;
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < kMaxCols; ++u) {
+      const int i = tid + 256 * u;
+      if (i >= rank) break;
+      float a = acc[u] * alpha;
+      for (int j = 0; j < nk; ++j) a += sc[j] * to_f32<T>(c[(int64_t)(k0 + j) * rank + i]);
+      acc[u] = a;
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int u = 0; u < kMaxCols; ++u) {
+    const int i = tid + 256 * u;
+    if (i < rank) ctx[qat + i] = from_f32<T>(acc[u] / l);
+  }
+}
+
+// ------------------------------------------------------------------------------------------------ decode
+constexpr int kDecKeys = 64;           // keys per tile
+constexpr int kDecMaxRank = 512;
+
+struct DecArgs {
+  const bf16_t* q;
+  const bf16_t* cache;
+  float* part_acc;     // [rows, n_split, H, rank]
+  float* part_ml;      // [rows, n_split, H, 2]
+  int64_t Lcap;
+  float scale_log2e;
+  int32_t H, rank, n_split;
+};
+
+// HT tiles of 16 heads.  Wavefront w scores keys 16 w .. + 16 of a tile and owns the latent columns of tiles w, w + 4, ...
+// of the product with the probabilities.
+template <int HT>
+__global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_batch b) {
+  constexpr int kHeads = 16 * HT, kPStride = kDecKeys + 8, kPer = 256 / kHeads;   // threads per head in the softmax
+  constexpr int kSStride = kDecKeys + 4;
+  constexpr int kCT = kDecMaxRank / 16 / 4;
+  extern __shared__ __align__(16) char lds[];
+  const int rankp = (a.rank + 31) / 32 * 32, stride = rankp + 8;
+  bf16_t* cs = reinterpret_cast<bf16_t*>(lds);                   // [64][stride]
+  bf16_t* qs = cs + kDecKeys * stride;                           // [kHeads][stride]
+  bf16_t* ps = qs + kHeads * stride;                             // [kHeads][kPStride]
+  float* ss = reinterpret_cast<float*>(ps + kHeads * kPStride);  // [kHeads][kSStride]
+  float* al = ss + kHeads * kSStride;                            // [kHeads]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
+  const int split = blockIdx.x, h0 = blockIdx.y * kHeads, row = blockIdx.z;
+  const int s = b.row_seq[row];
+  const int n_keys = (int)(b.pos[s] + (row - b.cu[s]) + 1);
+  const int tiles = (n_keys + kDecKeys - 1) / kDecKeys, per = (tiles + a.n_split - 1) / a.n_split;
+  const int first = split * per * kDecKeys, last = min(n_keys, first + per * kDecKeys);
+  const bf16_t* c = a.cache + (int64_t)b.slot[s] * a.Lcap * a.rank;
+  const int units = rankp / 8;                                   // 16-byte pieces of a row, zero behind the rank
+
+  for (int i = tid; i < kHeads * units; i += 256) {
+    const int h = i / units, u = i % units;
+    uint4 w = make_uint4(0, 0, 0, 0);
+    if (h0 + h < a.H && u * 8 < a.rank) w = *reinterpret_cast<const uint4*>(a.q + ((int64_t)row * a.H + h0 + h) * a.rank + u * 8);
+    *reinterpret_cast<uint4*>(qs + h * stride + u * 8) = w;
+  }
+  constexpr int kPieces = kDecKeys * (kDecMaxRank / 8) / 256;    // pieces of a tile per thread (16)
+  uint4 next[kPieces];
+  const int total = kDecKeys * units;
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int i = 0; i < kPieces; ++i) {
+      const int idx = tid + 256 * i, key = idx / units, u = idx % units;
+      next[i] = make_uint4(0, 0, 0, 0);
+      if (idx < total && k0 + key < last && u * 8 < a.rank)
+        next[i] = *reinterpret_cast<const uint4*>(c + (int64_t)(k0 + key) * a.rank + u * 8);
+    }
+  };
+  auto stash = [&]() {
+#pragma unroll
+    for (int i = 0; i < kPieces; ++i) {
+      const int idx = tid + 256 * i;
+      if (idx < total) *reinterpret_cast<uint4*>(cs + (idx / units) * stride + (idx % units) * 8) = next[i];
+    }
+  };
+  floatx4_t o[HT][kCT];
+#pragma unroll
+  for (int h = 0; h < HT; ++h)
+#pragma unroll
+    for (int t = 0; t < kCT; ++t) o[h][t] = floatx4_t{0.f, 0.f, 0.f, 0.f};
+  const int col_tiles = rankp / 16;
+  float m = -INFINITY, l = 0.f;        // of head tid / kPer, the same in its kPer threads
+  if (first < last) fetch(first);
+  for (int k0 = first; k0 < last; k0 += kDecKeys) {
+    __syncthreads();
+    stash();
+    __syncthreads();
+    if (k0 + kDecKeys < last) fetch(k0 + kDecKeys);
+    floatx4_t sc[HT];
+#pragma unroll
+    for (int h = 0; h < HT; ++h) sc[h] = floatx4_t{0.f, 0.f, 0.f, 0.f};
+    for (int kk = 0; kk < rankp; kk += 32) {
+      const bf16x8_t kb = *reinterpret_cast<const bf16x8_t*>(cs + (wave * 16 + l16) * stride + kk + 8 * g);
+#pragma unroll
+      for (int h = 0; h < HT; ++h) {
+        const bf16x8_t qa = *reinterpret_cast<const bf16x8_t*>(qs + (h * 16 + l16) * stride + kk + 8 * g);
+        sc[h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qa, kb, sc[h], 0, 0, 0);
+      }
+    }
+#pragma unroll
+    for (int h = 0; h < HT; ++h)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss[(h * 16 + 4 * g + e) * kSStride + wave * 16 + l16] = sc[h][e] * a.scale_log2e;
+    __syncthreads();
+    {
+      constexpr int kEach = kDecKeys / kPer;                     // keys per thread
+      const int h = tid / kPer, j0 = (tid % kPer) * kEach;
+      float v[kEach], mx = m;
+#pragma unroll
+      for (int j = 0; j < kEach; ++j) {
+        v[j] = k0 + j0 + j < last ? ss[h * kSStride + j0 + j] : -INFINITY;
+        mx = fmaxf(mx, v[j]);
+      }
+#pragma unroll
+      for (int d = 1; d < kPer; d <<= 1) mx = fmaxf(mx, __shfl_xor(mx, d));
+      const float alpha = exp2f(m - mx);                         // a tile has at least one key: mx is finite
+      float sum = 0.f;
+#pragma unroll
+      for (int j = 0; j < kEach; j += 2) {
+        const float p0 = exp2f(v[j] - mx), p1 = exp2f(v[j + 1] - mx);
+        sum += p0 + p1;
+        *reinterpret_cast<uint32_t*>(ps + h * kPStride + j0 + j) = pack_bf16x2(p0, p1);
+      }
+#pragma unroll
+      for (int d = 1; d < kPer; d <<= 1) sum += __shfl_xor(sum, d);
+      l = l * alpha + sum;
+      m = mx;
+      if (tid % kPer == 0) al[h] = alpha;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int h = 0; h < HT; ++h) {
+      float f[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) f[e] = al[h * 16 + 4 * g + e];
+#pragma unroll
+      for (int t = 0; t < kCT; ++t)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[h][t][e] *= f[e];
+    }
+#pragma unroll
+    for (int kk = 0; kk < kDecKeys; kk += 32) {
+      bf16x8_t pa[HT];
+#pragma unroll
+      for (int h = 0; h < HT; ++h) pa[h] = *reinterpret_cast<const bf16x8_t*>(ps + (h * 16 + l16) * kPStride + kk + 8 * g);
+#pragma unroll
+      for (int t = 0; t < kCT; ++t) {
+        const int ct = wave + 4 * t;
+        if (ct >= col_tiles) break;
+        const bf16_t* at = cs + (kk + 8 * g + (l16 >> 2)) * stride + ct * 16 + (l16 & 3) * 4;
+        const bf16x8_t vb = join8(lds_read_tr16(at), lds_read_tr16(at + 4 * stride));
+#pragma unroll
+        for (int h = 0; h < HT; ++h) o[h][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[h], vb, o[h][t], 0, 0, 0);
+      }
+    }
+  }
+  // o[h][t][e] belongs to head 16 h + 4 g + e, latent column 16 (wave + 4 t) + l16
+  const int64_t at = ((int64_t)row * a.n_split + split) * a.H;
+#pragma unroll
+  for (int h = 0; h < HT; ++h)
+#pragma unroll
+    for (int t = 0; t < kCT; ++t) {
+      const int col = (wave + 4 * t) * 16 + l16;
+      if (col >= a.rank) continue;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int head = h0 + h * 16 + 4 * g + e;
+        if (head < a.H) a.part_acc[(at + head) * a.rank + col] = o[h][t][e];
+      }
+    }
+  if (tid % kPer == 0 && h0 + tid / kPer < a.H) {
+    a.part_ml[(at + h0 + tid / kPer) * 2] = m;
+    a.part_ml[(at + h0 + tid / kPer) * 2 + 1] = l;
+  }
+}
+
+// A workgroup per (row, head): folds the key ranges and the sink.
+__global__ __launch_bounds__(128) void latent_combine_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
+                                                             const float* __restrict__ sink, int32_t H, int32_t rank, int32_t n_split,
+                                                             bf16_t* __restrict__ ctx) {
+  const int row = blockIdx.x, head = blockIdx.y;
+  const float sk = sink[head] * kLog2e;
+  float m = sk;
+  for (int i = 0; i < n_split; ++i) m = fmaxf(m, part_ml[(((int64_t)row * n_split + i) * H + head) * 2]);
+  float l = exp2f(sk - m);
+  for (int i = 0; i < n_split; ++i) {
+    const float* ml = part_ml + (((int64_t)row * n_split + i) * H + head) * 2;
+    if (ml[0] > -INFINITY) l += exp2f(ml[0] - m) * ml[1];
+  }
+  const float inv = 1.0f / l;
+  for (int c = threadIdx.x; c < rank; c += 128) {
+    float v = 0.f;
+    for (int i = 0; i < n_split; ++i) {
+      const int64_t at = ((int64_t)row * n_split + i) * H + head;
+      const float mi = part_ml[at * 2];
+      if (mi > -INFINITY) v += exp2f(mi - m) * part_acc[at * rank + c];
+    }
+    ctx[((int64_t)row * H + head) * rank + c] = f32_to_bf16(v * inv);
+  }
+}
+
+int latent_splits(int32_t rows, int32_t H, int64_t max_keys) {
+  const int64_t tiles = std::max<int64_t>(1, (max_keys + kDecKeys - 1) / kDecKeys);
+  const int64_t blocks = (int64_t)rows * ((H + 31) / 32);
+  return (int)std::min<int64_t>(std::min<int64_t>(tiles, 128), std::max<int64_t>(1, (2 * device_compute_units() + blocks - 1) / blocks));
+}
+
+// ------------------------------------------------------------------------------------------------ prefill
+struct FlashArgs {
+  const bf16_t* q;
+  const bf16_t* k;
+  const bf16_t* v;
+  const int64_t* kv_off;
+  const float* sink;
+  bf16_t* out;
+  int64_t q_stride, k_stride, v_stride;
+  float scale_log2e;
+  int32_t H, D, E;
+};
+constexpr int kFlashKeys = 64, kFlashRows = 128;
+
+// DP / EP: D and E padded to a multiple of 32 (zeros in LDS).  Two stages of K and V tiles in LDS; the next tile is
+// fetched into registers while this one is multiplied.
+template <int DP, int EP>
+__global__ __launch_bounds__(256, (DP + EP <= 256) ? 2 : 1) void flash_sink_kernel(FlashArgs a, msa_seq_batch b) {
+  constexpr int kKS = DP + 8, kVS = EP + 8;
+  constexpr int kKP = kFlashKeys * DP / 8 / 256, kVP = kFlashKeys * EP / 8 / 256;   // 16-byte pieces per thread
+  extern __shared__ __align__(16) bf16_t fl[];
+  bf16_t* kt = fl;                                   // [2][64][kKS]
+  bf16_t* vt = fl + 2 * kFlashKeys * kKS;            // [2][64][kVS]
+  const int head = blockIdx.x, s = blockIdx.z;
+  const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo;
+  const int blk = (n_tok + kFlashRows - 1) / kFlashRows - 1 - (int)blockIdx.y;   // long ones first
+  if (blk < 0) return;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 31, half = lane >> 5;
+  const int tok = blk * kFlashRows + wave * 32 + col;
+  const bool ok = tok < n_tok;
+  const int base = (int)b.pos[s];
+  const int limit = ok ? base + tok + 1 : 0;
+  const int kmax = base + min(n_tok, (blk + 1) * kFlashRows);
+  const int wave_min = base + blk * kFlashRows + wave * 32 + 1;      // the wavefront's first column sees this many keys
+  const bf16_t* kg = a.k + a.kv_off[s] * a.k_stride + (int64_t)head * a.D;
+  const bf16_t* vg = a.v + a.kv_off[s] * a.v_stride + (int64_t)head * a.E;
+
+  bf16x8_t qf[DP / 16];
+  {
+    const bf16_t* qr = a.q + (int64_t)(lo + (ok ? tok : 0)) * a.q_stride + (int64_t)head * a.D;
+#pragma unroll
+    for (int i = 0; i < DP / 16; ++i) {
+      const int d = 16 * i + 8 * half;
+      const uint4 w = ok && d < a.D ? *reinterpret_cast<const uint4*>(qr + d) : make_uint4(0, 0, 0, 0);
+      qf[i] = __builtin_bit_cast(bf16x8_t, w);
+    }
+  }
+  uint4 kn[kKP], vn[kVP];
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int i = 0; i < kKP; ++i) {
+      const int idx = tid + 256 * i, key = idx / (DP / 8), d = idx % (DP / 8) * 8;
+      kn[i] = k0 + key < kmax && d < a.D ? *reinterpret_cast<const uint4*>(kg + (int64_t)(k0 + key) * a.k_stride + d) : make_uint4(0, 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < kVP; ++i) {
+      const int idx = tid + 256 * i, key = idx / (EP / 8), d = idx % (EP / 8) * 8;
+      vn[i] = k0 + key < kmax && d < a.E ? *reinterpret_cast<const uint4*>(vg + (int64_t)(k0 + key) * a.v_stride + d) : make_uint4(0, 0, 0, 0);
+    }
+  };
+  auto stash = [&](int stage) {
+#pragma unroll
+    for (int i = 0; i < kKP; ++i) {
+      const int idx = tid + 256 * i;
+      *reinterpret_cast<uint4*>(kt + (stage * kFlashKeys + idx / (DP / 8)) * kKS + idx % (DP / 8) * 8) = kn[i];
+    }
+#pragma unroll
+    for (int i = 0; i < kVP; ++i) {
+      const int idx = tid + 256 * i;
+      *reinterpret_cast<uint4*>(vt + (stage * kFlashKeys + idx / (EP / 8)) * kVS + idx % (EP / 8) * 8) = vn[i];
+    }
+  };
+  floatx16_t o[EP / 32];
+#pragma unroll
+  for (int d = 0; d < EP / 32; ++d)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) o[d][e] = 0.f;
+  float m = a.sink[head] * kLog2e, l = half == 0 ? 1.f : 0.f;       // the sink: first member of every column's softmax
+  fetch(0);
+  stash(0);
+  __syncthreads();
+  int stage = 0;
+  for (int k0 = 0; k0 < kmax; k0 += kFlashKeys, stage ^= 1) {
+    const bool more = k0 + kFlashKeys < kmax;
+    if (more) fetch(k0 + kFlashKeys);
+    const bf16_t* kb = kt + stage * kFlashKeys * kKS;
+    const bf16_t* vb = vt + stage * kFlashKeys * kVS;
+    floatx16_t sc[2];
+#pragma unroll
+    for (int rb = 0; rb < 2; ++rb)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) sc[rb][e] = 0.f;
+#pragma unroll
+    for (int i = 0; i < DP / 16; ++i)
+#pragma unroll
+      for (int rb = 0; rb < 2; ++rb) {
+        const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(kb + (rb * 32 + col) * kKS + 16 * i + 8 * half);
+        sc[rb] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[i], sc[rb], 0, 0, 0);
+      }
+    float mx = -INFINITY;
+    if (k0 + kFlashKeys > wave_min) {
+#pragma unroll
+      for (int rb = 0; rb < 2; ++rb)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) {
+          const int key = k0 + 32 * rb + 8 * (e >> 2) + 4 * half + (e & 3);
+          sc[rb][e] = key < limit ? sc[rb][e] : -INFINITY;
+        }
+    }
+#pragma unroll
+    for (int rb = 0; rb < 2; ++rb)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) mx = fmaxf(mx, sc[rb][e]);
+    mx = half_wave_max(mx * a.scale_log2e);
+    // the reference value only follows the maximum when it is well behind it: the probabilities stay below 2^6
+    if (__any(mx > m + 6.0f)) {
+      const float m_new = fmaxf(m, mx), alpha = __builtin_amdgcn_exp2f(m - m_new);
+      l *= alpha;
+#pragma unroll
+      for (int d = 0; d < EP / 32; ++d)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) o[d][e] *= alpha;
+      m = m_new;
+    }
+#pragma unroll
+    for (int rb = 0; rb < 2; ++rb)
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        uint32_t pw[4];
+#pragma unroll
+        for (int x = 0; x < 4; ++x) {
+          const float p0 = __builtin_amdgcn_exp2f(fmaf(sc[rb][8 * j + 2 * x], a.scale_log2e, -m));
+          const float p1 = __builtin_amdgcn_exp2f(fmaf(sc[rb][8 * j + 2 * x + 1], a.scale_log2e, -m));
+          l += p0 + p1;
+          pw[x] = pack_bf16x2(p0, p1);
+        }
+        const bf16x8_t pb = __builtin_bit_cast(bf16x8_t, make_uint4(pw[0], pw[1], pw[2], pw[3]));
+        // keys 32 rb + 16 j + {4 half .. + 3, 8 + 4 half .. + 3}, in the order the score tile's rows hold them
+        const bf16_t* vrow = vb + (rb * 32 + j * 16 + 4 * half + ((lane & 15) >> 2)) * kVS + (lane & 16) + (lane & 3) * 4;
+#pragma unroll
+        for (int d = 0; d < EP / 32; ++d) {
+          const bf16x8_t vf = join8(lds_read_tr16(vrow + d * 32), lds_read_tr16(vrow + 8 * kVS + d * 32));
+          o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, pb, o[d], 0, 0, 0);
+        }
+      }
+    if (more) stash(stage ^ 1);
+    __syncthreads();
+  }
+  l = half_wave_sum(l);
+  if (!ok) return;
+  const float inv = 1.0f / l;
+  bf16_t* dst = a.out + ((int64_t)(lo + tok) * a.H + head) * a.E;
+#pragma unroll
+  for (int d = 0; d < EP / 32; ++d)
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      const int at = d * 32 + 8 * x + 4 * half;
+      if (at < a.E)
+        *reinterpret_cast<uint2*>(dst + at) = make_uint2(pack_bf16x2(o[d][4 * x] * inv, o[d][4 * x + 1] * inv),
+                                                         pack_bf16x2(o[d][4 * x + 2] * inv, o[d][4 * x + 3] * inv));
+    }
+}
+
+template <int DP, int EP>
+int launch_flash(const FlashArgs& a, const msa_seq_batch& b, hipStream_t st) {
+  constexpr int lds = 2 * kFlashKeys * (DP + 8 + EP + 8) * 2;
+  static std::atomic<int> raised{0};
+  MSA_HIP(raise_dynamic_lds_limit(raised, reinterpret_cast<const void*>(flash_sink_kernel<DP, EP>), lds));
+  flash_sink_kernel<DP, EP><<<dim3(a.H, (b.max_rows + kFlashRows - 1) / kFlashRows, b.n_seq), 256, lds, st>>>(a, b);
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+
+template <int HT>
+int launch_decode(const DecArgs& a, const msa_seq_batch& b, hipStream_t st) {
+  const int stride = (a.rank + 31) / 32 * 32 + 8, heads = 16 * HT;
+  const int lds = (kDecKeys + heads) * stride * 2 + heads * (kDecKeys + 8) * 2 + heads * (kDecKeys + 4) * 4 + heads * 4;
+  static std::atomic<int> raised{0};
+  MSA_HIP(raise_dynamic_lds_limit(raised, reinterpret_cast<const void*>(latent_decode_kernel<HT>), 160 * 1024));
+  MSA_REQUIRE(lds <= 160 * 1024, "msa_seq_latent_decode: %d bytes of LDS", lds);
+  latent_decode_kernel<HT><<<dim3(a.n_split, (a.H + heads - 1) / heads, b.rows), 256, lds, st>>>(a, b);
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+
+}  // namespace
+
+extern "C" int msa_seq_latent_attn(const void* q, const void* cache, int64_t Lcap, const float* sink, float scale, int32_t dtype,
+                                   int32_t H, int32_t rank, void* ctx, const msa_seq_batch* batch, void* stream) {
+  MSA_CHECK_BATCH(batch, "msa_seq_latent_attn");
+  MSA_CHECK_DTYPE(dtype, "msa_seq_latent_attn");
+  MSA_REQUIRE(q && cache && sink && ctx && Lcap > 0 && H > 0 && H <= 65535 && rank > 0 && rank <= 256 * kMaxCols,
+              "msa_seq_latent_attn: H=%d rank=%d (up to %d)", H, rank, 256 * kMaxCols);
+  const dim3 grid(batch->rows, H);
+  const size_t lds = (rank + 64) * sizeof(float);
+  if (dtype == MSA_BF16)
+    latent_attn_kernel<bf16_t><<<grid, 256, lds, as_stream(stream)>>>((const bf16_t*)q, (const bf16_t*)cache, Lcap, sink, scale, H, rank,
+                                                                      (bf16_t*)ctx, *batch);
+  else
+    latent_attn_kernel<float><<<grid, 256, lds, as_stream(stream)>>>((const float*)q, (const float*)cache, Lcap, sink, scale, H, rank,
+                                                                     (float*)ctx, *batch);
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+
+extern "C" size_t msa_seq_latent_decode_workspace_bytes(int32_t rows, int32_t H, int32_t rank, int64_t max_keys) {
+  if (rows <= 0 || H <= 0 || rank <= 0 || max_keys <= 0) return 0;
+  return (size_t)rows * latent_splits(rows, H, max_keys) * H * (rank + 2) * sizeof(float);
+}
+
+extern "C" int msa_seq_latent_decode(const void* q, const void* cache, int64_t Lcap, const float* sink, float scale, int32_t dtype,
+                                     int32_t H, int32_t rank, int64_t max_keys, void* ctx, const msa_seq_batch* batch, void* workspace,
+                                     size_t workspace_bytes, void* stream) {
+  MSA_CHECK_BATCH(batch, "msa_seq_latent_decode");
+  MSA_REQUIRE(dtype == MSA_BF16, "msa_seq_latent_decode: bf16 only");
+  MSA_REQUIRE(q && cache && sink && ctx && workspace, "msa_seq_latent_decode: null pointer");
+  MSA_REQUIRE(H > 0 && H <= 4096 && rank > 0 && rank % 8 == 0 && rank <= kDecMaxRank, "msa_seq_latent_decode: H=%d rank=%d (a multiple of 8 up to %d)",
+              H, rank, kDecMaxRank);
+  MSA_REQUIRE(batch->rows <= 65535 && max_keys > 0 && max_keys <= Lcap && Lcap < ((int64_t)1 << 31), "msa_seq_latent_decode: %d rows, %lld keys",
+              batch->rows, (long long)max_keys);
+  MSA_REQUIRE((((uintptr_t)q | (uintptr_t)cache) & 15) == 0, "msa_seq_latent_decode: q and cache must be 16-byte aligned");
+  const int splits = latent_splits(batch->rows, H, max_keys);
+  if (workspace_bytes < msa_seq_latent_decode_workspace_bytes(batch->rows, H, rank, max_keys)) {
+    msa_set_error("msa_seq_latent_decode: workspace of %zu bytes is too small", workspace_bytes);
+    return MSA_ESIZE;
+  }
+  float* acc = static_cast<float*>(workspace);
+  float* ml = acc + (int64_t)batch->rows * splits * H * rank;
+  const DecArgs a{(const bf16_t*)q, (const bf16_t*)cache, acc, ml, Lcap, scale * kLog2e, H, rank, splits};
+  hipStream_t st = as_stream(stream);
+  const int rc = H <= 16 ? launch_decode<1>(a, *batch, st) : launch_decode<2>(a, *batch, st);
+  if (rc != MSA_OK) return rc;
+  latent_combine_kernel<<<dim3(batch->rows, H), 128, 0, st>>>(acc, ml, sink, H, rank, splits, (bf16_t*)ctx);
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+
+extern "C" int msa_seq_flash(const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v, int64_t v_stride,
+                             const int64_t* kv_off, const float* sink, float scale, int32_t dtype, int32_t H, int32_t D, int32_t E,
+                             void* out, const msa_seq_batch* batch, void* stream) {
+  MSA_CHECK_BATCH(batch, "msa_seq_flash");
+  MSA_REQUIRE(dtype == MSA_BF16, "msa_seq_flash: bf16 only");
+  MSA_REQUIRE(q && k && v && kv_off && sink && out && scale > 0.f, "msa_seq_flash: null pointer or scale <= 0");
+  MSA_REQUIRE(H > 0 && D > 0 && E > 0 && D % 8 == 0 && E % 8 == 0 && D <= 256 && E <= 256, "msa_seq_flash: D=%d E=%d (multiples of 8 up to 256)", D, E);
+  MSA_REQUIRE(q_stride >= (int64_t)H * D && k_stride >= (int64_t)H * D && v_stride >= (int64_t)H * E && q_stride % 8 == 0 &&
+                  k_stride % 8 == 0 && v_stride % 8 == 0 && (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)out) & 15) == 0,
+              "msa_seq_flash: strides or alignment");
+  MSA_REQUIRE(batch->n_seq <= 65535 && (batch->max_rows + kFlashRows - 1) / kFlashRows <= 65535, "msa_seq_flash: step too large");
+  const FlashArgs a{(const bf16_t*)q, (const bf16_t*)k, (const bf16_t*)v, kv_off, sink, (bf16_t*)out, q_stride, k_stride, v_stride,
+                    scale * kLog2e, H, D, E};
+  hipStream_t st = as_stream(stream);
+  if (D <= 64 && E <= 64) return launch_flash<64, 64>(a, *batch, st);
+  if (D <= 128 && E <= 64) return launch_flash<128, 64>(a, *batch, st);
+  if (D <= 128 && E <= 128) return launch_flash<128, 128>(a, *batch, st);
+  if (D <= 192 && E <= 128) return launch_flash<192, 128>(a, *batch, st);
+  return launch_flash<256, 256>(a, *batch, st);
+}

@@ -1,0 +1,66 @@
+// Helpers shared by the recurrent / latent-attention layer kernels (msa_seq.h).
+#pragma once
+
+#include "../../include/msa_seq.h"
+#include "common.h"
+
+template <typename T>
+__device__ __forceinline__ float to_f32(T v);
+template <>
+__device__ __forceinline__ float to_f32<bf16_t>(bf16_t v) { return bf16_to_f32(v); }
+template <>
+__device__ __forceinline__ float to_f32<float>(float v) { return v; }
+template <typename T>
+__device__ __forceinline__ T from_f32(float v);
+template <>
+__device__ __forceinline__ bf16_t from_f32<bf16_t>(float v) { return f32_to_bf16(v); }
+template <>
+__device__ __forceinline__ float from_f32<float>(float v) { return v; }
+
+__device__ __forceinline__ float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
+__device__ __forceinline__ float silu_f(float x) { return x / (1.0f + expf(-x)); }
+__device__ __forceinline__ float softplus_f(float x) { return x > 30.f ? x : log1pf(expf(x)); }
+__device__ __forceinline__ float gelu_tanh_f(float z) {
+  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+
+// VEC consecutive elements of a row (VEC = 4 needs 8- / 16-byte alignment), as fp32.
+template <typename T, int VEC>
+__device__ __forceinline__ void load_vec(const T* p, float (&v)[VEC]) {
+  if constexpr (VEC == 4 && sizeof(T) == 2) {
+    const uint2 w = *reinterpret_cast<const uint2*>(p);
+    v[0] = bf16lo(w.x); v[1] = bf16hi(w.x); v[2] = bf16lo(w.y); v[3] = bf16hi(w.y);
+  } else if constexpr (VEC == 4) {
+    const float4 w = *reinterpret_cast<const float4*>(p);
+    v[0] = w.x; v[1] = w.y; v[2] = w.z; v[3] = w.w;
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) v[i] = to_f32<T>(p[i]);
+  }
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void store_vec(T* p, const float (&v)[VEC]) {
+  if constexpr (VEC == 4 && sizeof(T) == 2) {
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
+  } else if constexpr (VEC == 4) {
+    *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) p[i] = from_f32<T>(v[i]);
+  }
+}
+
+// Host side: 16-byte vectors are usable when every given address is aligned and every stride a multiple of 4 elements.
+static inline bool vec4_ok(std::initializer_list<const void*> ps, std::initializer_list<int64_t> strides) {
+  for (const void* p : ps)
+    if (((uintptr_t)p & 15) != 0) return false;
+  for (int64_t s : strides)
+    if (s % 4 != 0) return false;
+  return true;
+}
+
+#define MSA_CHECK_BATCH(b, who)                                                                                     \
+  MSA_REQUIRE((b) && (b)->cu && (b)->row_seq && (b)->slot && (b)->pos && (b)->n_seq > 0 && (b)->rows >= (b)->n_seq && \
+                  (b)->max_rows > 0 && (b)->max_rows <= (b)->rows && (b)->rows < (1 << 24),                         \
+              "%s: bad batch", who)
+#define MSA_CHECK_DTYPE(d, who) MSA_REQUIRE((d) == MSA_BF16 || (d) == MSA_F32, "%s: bad dtype %d", who, d)

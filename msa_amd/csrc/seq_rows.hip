@@ -1,0 +1,228 @@
+// Weight-streaming linear for the rows of a decode step (M <= 16, bf16), with the recurrent decoder's element-wise work in
+// the epilogue: gelu, softcap, the gated residual with the next norm and token shift, the causal convolution, the minimal
+// gated recurrence.  Like the skinny linear of the attention model a workgroup owns a few 16-row groups of the weights and
+// splits K over its wavefronts (16x16x32 MFMA: the 16 activation rows are exactly one operand); partial sums meet in LDS
+// and are added in wavefront order.  Everything behind the sums is element-wise in this model (dynamic tanh has no row
+// statistics), so a layer's chain of launches is one per weight matrix plus the state-space / attention step.
+#include <algorithm>
+
+#include "seq_common.h"
+
+namespace {
+
+typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8_t;
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4_t;
+typedef unsigned int u32x4_t __attribute__((ext_vector_type(4)));
+
+constexpr int kMaxWaves = 16;
+constexpr int kGruGroup = 16;
+
+// Units of 32 J elements of K (J 16-byte vectors per lane): shorter when three row groups share the registers.
+template <int R>
+constexpr int kVectors = R == 3 ? 2 : 4;
+
+template <int EPI, int R>
+__global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_args a, int32_t rows_per_wg) {
+  constexpr int J = kVectors<R>, kUnit = 32 * J;
+  extern __shared__ __align__(16) float part[];   // [waves][R][64][4]
+  const int tid = threadIdx.x, lane = tid & 63, waves = blockDim.x >> 6;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int n_l = lane & 15, g = lane >> 4;
+  const int n_base = blockIdx.x * rows_per_wg, grp = blockIdx.y;
+  const int row_bytes = a.K * 2;
+  const int rows_w = min(rows_per_wg, a.N - n_base);
+  const bool second = n_base >= a.n_b;
+  const int64_t xs = second ? a.x_b_stride : a.x_stride;
+  const char* xbase = static_cast<const char*>(second ? a.x_b : a.x) + (int64_t)grp * row_bytes;
+  const __amdgpu_buffer_rsrc_t rs_w = __builtin_amdgcn_make_buffer_rsrc(
+      const_cast<char*>(static_cast<const char*>(a.w)) + ((int64_t)grp * a.N + n_base) * row_bytes, 0, rows_w * row_bytes, 0x00020000);
+  const __amdgpu_buffer_rsrc_t rs_x = __builtin_amdgcn_make_buffer_rsrc(
+      const_cast<char*>(xbase), 0, (int)((a.M - 1) * xs * 2 + row_bytes), 0x00020000);
+  const int voff_w = n_l * row_bytes + g * 16, voff_x = n_l * (int)(xs * 2) + g * 16;
+  constexpr int kFar = 0x7ff00000;          // past every extent, whatever is added: reads zeros
+  const int units = (a.K + kUnit - 1) / kUnit;
+  const int u0 = units * wave / waves, u1 = units * (wave + 1) / waves;
+
+  floatx4_t acc[R];
+#pragma unroll
+  for (int r = 0; r < R; ++r) acc[r] = floatx4_t{0.f, 0.f, 0.f, 0.f};
+  u32x4_t fw[2][R][J], fx[2][J];
+  auto load_unit = [&](int slot, int u) {
+    const int k_off = u * kUnit * 2;
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+      const bool in = k_off + j * 64 + g * 16 < row_bytes;        // pieces behind K read as zero
+      fx[slot][j] = __builtin_amdgcn_raw_buffer_load_b128(rs_x, in ? voff_x : kFar, k_off + j * 64, 0);
+#pragma unroll
+      for (int r = 0; r < R; ++r)
+        fw[slot][r][j] = __builtin_amdgcn_raw_buffer_load_b128(rs_w, in ? voff_w + r * 16 * row_bytes : kFar, k_off + j * 64, 0);
+    }
+  };
+  auto mul_unit = [&](int slot) {
+#pragma unroll
+    for (int j = 0; j < J; ++j)
+#pragma unroll
+      for (int r = 0; r < R; ++r)
+        acc[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, fx[slot][j]),
+                                                         __builtin_bit_cast(bf16x8_t, fw[slot][r][j]), acc[r], 0, 0, 0);
+  };
+  if (u0 < u1) load_unit(0, u0);
+  int u = u0;
+  for (; u + 2 <= u1; u += 2) {
+    load_unit(1, u + 1);
+    mul_unit(0);
+    if (u + 2 < u1) load_unit(0, u + 2);
+    mul_unit(1);
+  }
+  if (u < u1) mul_unit(0);
+
+#pragma unroll
+  for (int r = 0; r < R; ++r) *reinterpret_cast<floatx4_t*>(&part[((wave * R + r) * 64 + lane) * 4]) = acc[r];
+  __syncthreads();
+
+  // output i of a row group: lane i / 4, element i % 4 of its accumulator
+  auto total = [&](int r, int i) {
+    float v = 0.f;
+    for (int w = 0; w < waves; ++w) v += part[(w * R + r) * 256 + i];
+    return v;
+  };
+  auto row_of = [](int i) { return 4 * (i >> 6) + (i & 3); };
+  auto col_of = [](int i) { return (i >> 2) & 15; };
+  bf16_t* out16 = static_cast<bf16_t*>(a.out);
+
+  if constexpr (EPI == MSA_ROWS_GRU) {
+    if (!second) {
+      for (int i = tid; i < 256; i += blockDim.x) {
+        const int m = row_of(i), c = n_base / (3 * kGruGroup) * kGruGroup + col_of(i);
+        if (m >= a.M || c >= a.gru_n) continue;
+        const float z = sigmoid_f(total(0, i) + a.z_bias[c]), uu = total(1, i) + a.u_bias[c], gt = total(2, i);
+        float* st = a.gru_state + (int64_t)a.slot[m] * a.gru_n + c;
+        const float S = (1.0f - z) * *st + z * (uu >= 0.f ? uu + 0.5f : sigmoid_f(uu));
+        *st = S;
+        static_cast<bf16_t*>(a.out2)[(int64_t)m * a.gru_n + c] = f32_to_bf16(S * silu_f(gt));
+      }
+      return;
+    }
+  }
+  for (int o = tid; o < R * 256; o += blockDim.x) {
+    const int r = o >> 8, i = o & 255;
+    const int m = row_of(i), nr = 16 * r + col_of(i), n = n_base + nr;
+    if (m >= a.M || nr >= rows_w) continue;
+    float v = total(r, i);
+    const int64_t col = (int64_t)grp * a.N + n;
+    if constexpr (EPI == MSA_ROWS_PLAIN || EPI == MSA_ROWS_GRU) {
+      if (EPI == MSA_ROWS_PLAIN && n < a.gelu_n) v = gelu_tanh_f(v);
+      out16[m * a.out_stride + col] = f32_to_bf16(v);
+    } else if constexpr (EPI == MSA_ROWS_F32) {
+      if (a.cap > 0.f) v = a.cap * tanhf(v / a.cap);
+      if (a.add) v += a.add[col];
+      static_cast<float*>(a.out)[m * a.out_stride + col] = v;
+    } else if constexpr (EPI == MSA_ROWS_MAMBA) {
+      const int c = n - a.conv_lo;
+      if (c >= 0 && c < a.conv_n) {
+        float* keep = a.conv_state + (int64_t)a.slot[m] * (a.conv_k - 1) * a.conv_n + c;
+        const float* tp = a.taps + (int64_t)c * a.conv_k;
+        float y = a.conv_bias[c];
+        for (int j = 0; j + 1 < a.conv_k; ++j) {
+          const float old = keep[(int64_t)j * a.conv_n];
+          y += tp[j] * old;
+          if (j > 0) keep[(int64_t)(j - 1) * a.conv_n] = old;
+        }
+        y += tp[a.conv_k - 1] * v;
+        if (a.conv_k > 1) keep[(int64_t)(a.conv_k - 2) * a.conv_n] = v;
+        v = silu_f(y);
+      }
+      out16[m * a.out_stride + col] = f32_to_bf16(v);
+    } else {
+      const int64_t at = (int64_t)m * a.N + n;
+      const float gate = bf16_to_f32(static_cast<const bf16_t*>(a.gate)[m * a.gate_stride + n]) + a.gate_bias[n];
+      const float x = a.x_in[at] + sigmoid_f(gate) * v;
+      a.x_out[at] = x;
+      if (a.norm.w) {
+        const float h = tanhf(a.norm.alpha * x) * a.norm.w[n] + a.norm.b[n];
+        if (a.h) static_cast<bf16_t*>(a.h)[at] = f32_to_bf16(h);
+        if (a.shift) {
+          float* prev = a.prev + (int64_t)a.slot[m] * a.N + n;
+          const float before = *prev;
+          *prev = h;
+          static_cast<bf16_t*>(a.h_shift)[at] = f32_to_bf16(h + (before - h) * a.shift[n]);
+        }
+      }
+    }
+  }
+}
+
+template <int EPI, int R>
+int launch_rows(const msa_rows_args& a, int waves, int rows_per_wg, hipStream_t st) {
+  const size_t lds = (size_t)waves * R * 256 * sizeof(float);       // at most 48 KB
+  rows_linear_kernel<EPI, R><<<dim3((a.N + rows_per_wg - 1) / rows_per_wg, a.groups), waves * 64, lds, st>>>(a, rows_per_wg);
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+
+}  // namespace
+
+extern "C" int msa_rows_linear(const msa_rows_args* args, int32_t epilogue, void* stream) {
+  MSA_REQUIRE(args != nullptr, "msa_rows_linear: null arguments");
+  msa_rows_args a = *args;
+  MSA_REQUIRE(a.x && a.w && a.M > 0 && a.M <= 16 && a.N > 0 && a.K > 0 && a.K % 8 == 0 && a.groups > 0 && a.groups <= 65535,
+              "msa_rows_linear: M=%d (1..16) N=%d K=%d (a multiple of 8) groups=%d", a.M, a.N, a.K, a.groups);
+  MSA_REQUIRE(a.x_stride >= (int64_t)a.K * a.groups && a.x_stride % 8 == 0 && a.x_stride * 32 < ((int64_t)1 << 30) &&
+                  (int64_t)64 * a.K * 2 < ((int64_t)1 << 30), "msa_rows_linear: x_stride=%lld K=%d", (long long)a.x_stride, a.K);
+  const bool two = a.n_b < a.N;
+  MSA_REQUIRE(a.n_b > 0 && (!two || (a.x_b && a.groups == 1 && a.x_b_stride >= a.K && a.x_b_stride % 8 == 0 &&
+                                     a.x_b_stride * 32 < ((int64_t)1 << 30))), "msa_rows_linear: second operand");
+  MSA_REQUIRE((((uintptr_t)a.x | (uintptr_t)a.x_b | (uintptr_t)a.w) & 15) == 0, "msa_rows_linear: x / x_b / w must be 16-byte aligned");
+  switch (epilogue) {
+    case MSA_ROWS_PLAIN:
+    case MSA_ROWS_F32:
+      MSA_REQUIRE(a.out && a.out_stride >= (int64_t)a.N * a.groups, "msa_rows_linear: output");
+      break;
+    case MSA_ROWS_RESIDUAL:
+      MSA_REQUIRE(a.x_in && a.x_out && a.gate && a.gate_bias && a.gate_stride >= a.N && a.groups == 1 && !two, "msa_rows_linear: residual arguments");
+      MSA_REQUIRE(!a.norm.w || (a.norm.b && (a.h || a.shift)), "msa_rows_linear: norm arguments");
+      MSA_REQUIRE(!a.shift || (a.norm.w && a.prev && a.h_shift && a.slot), "msa_rows_linear: shift arguments");
+      break;
+    case MSA_ROWS_MAMBA:
+      MSA_REQUIRE(a.out && a.out_stride >= a.N && a.groups == 1 && a.taps && a.conv_bias && a.slot && a.conv_k >= 1 && a.conv_lo >= 0 &&
+                      a.conv_n > 0 && a.conv_lo + a.conv_n <= a.n_b && (a.conv_k == 1 || a.conv_state), "msa_rows_linear: convolution arguments");
+      break;
+    case MSA_ROWS_GRU:
+      MSA_REQUIRE(a.out2 && a.z_bias && a.u_bias && a.gru_state && a.slot && a.groups == 1 && a.gru_n > 0 &&
+                      a.n_b == (a.gru_n + kGruGroup - 1) / kGruGroup * 3 * kGruGroup && (!two || (a.out && a.out_stride >= a.N)),
+                  "msa_rows_linear: recurrence arguments");
+      break;
+    default:
+      msa_set_error("msa_rows_linear: epilogue %d", epilogue);
+      return MSA_EINVAL;
+  }
+  // Row groups per workgroup: two when N alone fills the chip (the activations are then read half as often); fewer than 16
+  // rows when that leaves compute units without a workgroup.  Wavefronts: a few thousand in the launch, and a share of K each.
+  const bool gru = epilogue == MSA_ROWS_GRU;
+  int R = gru ? 3 : ((int64_t)a.N * a.groups >= 6144 && (!two || a.n_b % 32 == 0) && a.N >= 32) ? 2 : 1;
+  int rows_per_wg = 16 * R;
+  MSA_REQUIRE(!two || a.n_b % rows_per_wg == 0, "msa_rows_linear: n_b=%d must be a multiple of %d", a.n_b, rows_per_wg);
+  if (R == 1 && !two && a.groups == 1 && (a.N + 15) / 16 < device_compute_units())
+    rows_per_wg = std::min(16, std::max(8, (a.N + device_compute_units() - 1) / device_compute_units()));
+  const int64_t wgs = (int64_t)((a.N + rows_per_wg - 1) / rows_per_wg) * a.groups;
+  const int kUnit = 32 * (R == 3 ? kVectors<3> : kVectors<1>);
+  const int units = (a.K + kUnit - 1) / kUnit;
+  int waves = (int)std::min<int64_t>(kMaxWaves, std::max<int64_t>(1, (4096 + wgs - 1) / wgs));
+  waves = std::max(1, std::min(waves, units));
+  for (int cand = waves; cand >= std::max(1, waves / 2); --cand)
+    if (units % cand == 0) { waves = cand; break; }
+  hipStream_t st = as_stream(stream);
+  switch (epilogue * 4 + R) {
+    case MSA_ROWS_PLAIN * 4 + 1: return launch_rows<MSA_ROWS_PLAIN, 1>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_PLAIN * 4 + 2: return launch_rows<MSA_ROWS_PLAIN, 2>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_F32 * 4 + 1: return launch_rows<MSA_ROWS_F32, 1>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_F32 * 4 + 2: return launch_rows<MSA_ROWS_F32, 2>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_RESIDUAL * 4 + 1: return launch_rows<MSA_ROWS_RESIDUAL, 1>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_RESIDUAL * 4 + 2: return launch_rows<MSA_ROWS_RESIDUAL, 2>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_MAMBA * 4 + 1: return launch_rows<MSA_ROWS_MAMBA, 1>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_MAMBA * 4 + 2: return launch_rows<MSA_ROWS_MAMBA, 2>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_GRU * 4 + 3: return launch_rows<MSA_ROWS_GRU, 3>(a, waves, rows_per_wg, st);
+  }
+  msa_set_error("msa_rows_linear: no kernel for epilogue %d with %d row groups", epilogue, R);
+  return MSA_EINVAL;
+}

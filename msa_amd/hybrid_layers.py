@@ -1,0 +1,226 @@
+"""Layers of the hybrid decoder: token mixers (state space, minimal gated recurrence, latent attention), the dense
+feed-forward and the gated-residual layer around them.
+
+A mixer projects its input with one matrix (``w_in``, rows padded so that a second matrix can follow in one launch), keeps
+its own per-sequence state (``state_specs``) and has two forms of the work between its projections: ``mix`` for any rows of a
+step, and ``decode`` for up to 16 sequences' single rows with the projection folded in.  The residual gates read the norm
+output before the token shift, so a layer's first matrix is ``[w_in ; gate]`` over two operands.
+"""
+from __future__ import annotations
+
+from typing import Callable, Dict, Tuple
+
+import torch
+import torch.nn.functional as F
+
+from . import seq_ops
+from .cache import StateSpec
+from .config import HybridLayerConfig, LatentAttentionConfig, Mamba2Config, MinGRUConfig
+
+Get = Callable[[str], torch.Tensor]
+F32 = torch.float32
+ROW_PAD = 32                  # rows of a matrix that another one follows are padded to this
+
+
+def _pad_rows(w: torch.Tensor, multiple: int = ROW_PAD) -> torch.Tensor:
+    pad = -w.shape[0] % multiple
+    return torch.cat([w, w.new_zeros(pad, w.shape[1])]) if pad else w
+
+
+def head_linear(x: torch.Tensor, w: torch.Tensor, heads: int) -> torch.Tensor:
+    """Per-head products: ``x [T, heads K]``, ``w [heads N, K]`` -> ``[T, heads N]``."""
+    T, K = x.shape[0], w.shape[1]
+    if x.dtype == torch.bfloat16 and K % 8 == 0 and x.stride(0) % 8 == 0:
+        if T <= seq_ops.MAX_ROWS:
+            return seq_ops.rows_linear(x, w, groups=heads)
+        return torch.cat([seq_ops.rows_linear(x[i:i + seq_ops.MAX_ROWS], w, groups=heads) for i in range(0, T, seq_ops.MAX_ROWS)])
+    y = torch.bmm(x.reshape(T, heads, K).transpose(0, 1).contiguous(), w.view(heads, -1, K).transpose(1, 2).contiguous())
+    return y.transpose(0, 1).reshape(T, -1)
+
+
+class Mamba2Mixer:
+    """State-space layer: ``[z | x | B | C | dt]`` from one projection, causal convolution + silu of x, B, C, scalar-decay
+    recurrence per head, output gate, grouped RMS norm."""
+
+    def __init__(self, c: Mamba2Config, width: int, eps: float):
+        self.c, self.eps = c, eps
+
+    def shapes(self, width: int) -> Dict[str, Tuple[int, ...]]:
+        c = self.c
+        ch = c.conv_channels
+        return {"in": (c.inner + ch + c.heads, width), "conv": (ch, c.conv), "conv.b": (ch,), "dt_bias": (c.heads,),
+                "A_log": (c.heads,), "D": (c.heads,), "norm": (c.inner,), "o": (width, c.inner)}
+
+    def load(self, get: Get) -> None:
+        self.w_in, self.w_o = _pad_rows(get("in")), get("o")
+        self.taps, self.conv_b, self.dt_bias, self.A_log, self.D, self.norm = (
+            get(n).to(F32).contiguous() for n in ("conv", "conv.b", "dt_bias", "A_log", "D", "norm"))
+
+    def state_specs(self, dtype) -> Dict[str, StateSpec]:
+        c = self.c
+        return {"conv": StateSpec((c.conv - 1, c.conv_channels), F32), "ssm": StateSpec((c.heads, c.state, c.vdim), F32)}
+
+    def decode_ok(self) -> bool:
+        return self.c.inner % 8 == 0
+
+    def _columns(self, proj):
+        c = self.c
+        a, b = c.inner, c.inner + c.conv_channels
+        return proj[:, :a], proj[:, a:b], proj[:, b:b + c.heads]
+
+    def _scan(self, xbc, z, dt, state, batch):
+        c = self.c
+        chunked = (xbc.dtype == torch.bfloat16 and batch.max_rows >= (1 << 30) and c.state % 16 == 0 and c.state <= 256
+                   and c.vdim % 8 == 0)
+        v = seq_ops.ssd(xbc, z, dt, self.dt_bias, self.A_log, self.D, c.heads, c.vdim, c.state, c.groups, state["ssm"], batch,
+                        chunked=chunked)
+        return seq_ops.group_rmsnorm(v, self.norm, c.norm_groups, self.eps)
+
+    def mix(self, proj, state, batch):
+        z, xbc, dt = self._columns(proj)
+        return self._scan(seq_ops.conv_silu(xbc, self.taps, self.conv_b, state["conv"], batch), z, dt, state, batch)
+
+    def decode(self, w, hs, h, state, batch):
+        n_b = self.w_in.shape[0]
+        out = seq_ops.rows_conv(hs, w, h, n_b, self.c.inner, self.taps, self.conv_b, state["conv"], batch.slot)
+        z, xbc, dt = self._columns(out)
+        return self._scan(xbc, z, dt, state, batch), out[:, n_b:]
+
+
+class MinGRUMixer:
+    """Gated recurrence whose gates read only the current token; z, candidate and output gate come from one projection with
+    their rows interleaved (16 channels at a time)."""
+
+    def __init__(self, c: MinGRUConfig, width: int, eps: float):
+        self.c = c
+
+    def shapes(self, width: int):
+        n = self.c.width
+        return {"z": (n, width), "z.b": (n,), "x": (n, width), "x.b": (n,), "g": (n, width), "o": (width, n)}
+
+    def load(self, get: Get) -> None:
+        self.w_in, self.w_o = seq_ops.interleave_gru(get("z"), get("x"), get("g")), get("o")
+        self.z_b, self.u_b = get("z.b").to(F32).contiguous(), get("x.b").to(F32).contiguous()
+
+    def state_specs(self, dtype):
+        return {"gru": StateSpec((self.c.width,), F32)}
+
+    def decode_ok(self) -> bool:
+        return self.c.width % 8 == 0
+
+    def mix(self, proj, state, batch):
+        return seq_ops.min_gru(proj, self.z_b, self.u_b, self.c.width, state["gru"], batch)
+
+    def decode(self, w, hs, h, state, batch):
+        act, out = seq_ops.rows_gru(hs, w, h, self.c.width, self.z_b, self.u_b, state["gru"], batch.slot)
+        return act, out[:, self.w_in.shape[0]:]
+
+
+class LatentAttention:
+    """Attention without positions over a shared low-rank latent per token (the only thing cached), with a learned sink per
+    head.  Long portions expand the latents to keys and values; short ones multiply the queries by the key matrices and
+    attend to the latents themselves."""
+
+    ABSORB_ROWS = seq_ops.MAX_ROWS        # portions up to this many tokens
+
+    def __init__(self, c: LatentAttentionConfig, width: int, eps: float):
+        self.c, self.eps = c, eps
+
+    def shapes(self, width: int):
+        c = self.c
+        return {"q": (c.heads * c.dim, width), "dkv": (c.kv_rank, width), "dkv.norm": (c.kv_rank,),
+                "uk": (c.heads * c.dim, c.kv_rank), "uv": (c.heads * c.vdim, c.kv_rank), "sink": (c.heads,),
+                "o": (width, c.heads * c.vdim)}
+
+    def load(self, get: Get) -> None:
+        c = self.c
+        q, dkv = get("q"), get("dkv")
+        if q.shape[0] % 8:                 # keep the latent columns 16-byte aligned
+            q = _pad_rows(q, 8)
+        self.c_at = q.shape[0]
+        self.w_in, self.w_o = _pad_rows(torch.cat([q, dkv])), get("o")
+        self.uk, self.uv = get("uk").contiguous(), get("uv").contiguous()
+        self.uk_t = self.uk.view(c.heads, c.dim, c.kv_rank).transpose(1, 2).reshape(c.heads * c.kv_rank, c.dim).contiguous()
+        self.c_norm, self.sink = get("dkv.norm").to(F32).contiguous(), get("sink").to(F32).contiguous()
+
+    def state_specs(self, dtype):
+        return {"latent": StateSpec((self.c.kv_rank,), dtype, per_token=True)}
+
+    def decode_ok(self) -> bool:
+        c = self.c
+        return c.dim % 8 == 0 and c.kv_rank % 8 == 0 and (c.heads * c.vdim) % 8 == 0
+
+    def _absorbed(self, q, cache, batch):
+        c = self.c
+        qa = head_linear(q, self.uk_t, c.heads)
+        ctx = seq_ops.latent_attn(qa.view(batch.rows, c.heads, c.kv_rank), cache, self.sink, c.scale, batch, batch.max_keys)
+        return head_linear(ctx.view(batch.rows, -1), self.uv, c.heads)
+
+    def mix(self, proj, state, batch):
+        c, cache = self.c, state["latent"]
+        q = proj[:, :c.heads * c.dim]
+        seq_ops.latent_append(proj[:, self.c_at:self.c_at + c.kv_rank], self.c_norm, self.eps, cache, batch)
+        if batch.max_rows <= self.ABSORB_ROWS or not seq_ops.flash_ok(q.dtype, c.dim, c.vdim, c.scale) or proj.stride(0) % 8:
+            return self._absorbed(q, cache, batch)
+        ends = [p + n for p, n in zip(batch.positions, batch.counts)]
+        if batch.n_seq == 1:
+            lat, off = cache[batch.slots[0], :ends[0]], [0]
+        else:
+            lat = torch.cat([cache[s, :e] for s, e in zip(batch.slots, ends)])
+            off = [sum(ends[:i]) for i in range(batch.n_seq)]
+        return seq_ops.flash(q, F.linear(lat, self.uk), F.linear(lat, self.uv),
+                             torch.tensor(off, dtype=torch.int64).to(q.device), self.sink, c.scale, c.heads, batch)
+
+    def decode(self, w, hs, h, state, batch):
+        c, n_b = self.c, self.w_in.shape[0]
+        out = seq_ops.rows_linear(hs, w, x_b=h, n_b=n_b)
+        seq_ops.latent_append(out[:, self.c_at:self.c_at + c.kv_rank], self.c_norm, self.eps, state["latent"], batch)
+        return self._absorbed(out[:, :c.heads * c.dim], state["latent"], batch), out[:, n_b:]
+
+
+MIXERS = {"mamba2": Mamba2Mixer, "mingru": MinGRUMixer, "latent_attention": LatentAttention}
+
+
+def norm_shapes(name: str, width: int):
+    return {name: (width,), name + ".alpha": (), name + ".b": (width,)}
+
+
+def load_norm(get: Get, name: str) -> seq_ops.DynTanhNorm:
+    return seq_ops.DynTanhNorm(get(name).to(F32).contiguous(), get(name + ".b").to(F32).contiguous(), float(get(name + ".alpha")))
+
+
+class HybridLayer:
+    """Token shift and gated residuals around a mixer and an optional dense feed-forward."""
+
+    def __init__(self, c: HybridLayerConfig, width: int, eps: float):
+        self.width, self.mlp = width, c.mlp
+        self.mixer = MIXERS[c.type](c.mixer, width, eps)
+
+    def shapes(self) -> Dict[str, Tuple[int, ...]]:
+        W = self.width
+        out = {**norm_shapes("norm1", W), "shift": (W,), "rg1": (W, W), "rg1.b": (W,)}
+        out.update({"mix." + n: s for n, s in self.mixer.shapes(W).items()})
+        if self.mlp is not None:
+            out.update({**norm_shapes("norm2", W), "rg2": (W, W), "rg2.b": (W,), "mlp.up": (self.mlp.ff, W), "mlp.down": (W, self.mlp.ff)})
+        return out
+
+    def load(self, get: Get) -> None:
+        self.norm1, self.shift = load_norm(get, "norm1"), get("shift").to(F32).contiguous()
+        self.mixer.load(lambda n: get("mix." + n))
+        # the mixer's matrix and the gate's lie behind one another: one launch when decoding
+        self.w_in = torch.cat([self.mixer.w_in, get("rg1")]).contiguous()
+        self.n_mix = self.mixer.w_in.shape[0]
+        self.mixer.w_in = self.w_in[:self.n_mix]
+        self.w_gate, self.gate_b, self.w_o = self.w_in[self.n_mix:], get("rg1.b").to(F32).contiguous(), self.mixer.w_o.contiguous()
+        if self.mlp is not None:
+            self.norm2 = load_norm(get, "norm2")
+            up = _pad_rows(get("mlp.up"))
+            self.n_up = up.shape[0]
+            self.w_up, self.w_down = torch.cat([up, get("rg2")]).contiguous(), get("mlp.down").contiguous()
+            self.gate2_b = get("rg2.b").to(F32).contiguous()
+
+    def state_specs(self, dtype) -> Dict[str, StateSpec]:
+        return {"shift": StateSpec((self.width,), F32), **self.mixer.state_specs(dtype)}
+
+    def decode_ok(self) -> bool:
+        return self.width % 8 == 0 and (self.mlp is None or self.mlp.ff % 8 == 0) and self.mixer.decode_ok()

@@ -13,6 +13,7 @@ import torch.nn.functional as F
 from . import ops
 from .cache import CustomDynamicCache, create_cache
 from .config import MSAConfig
+from .generation import greedy_decode
 from .memory_sparse_attention import MemorySparseAttention, RMSNorm, rotary_embedding
 from .prefill import query_position_ids, source_block_position_ids
 
@@ -183,51 +184,18 @@ class MSAForCausalLM(nn.Module):
         tok_buf = tok.clone()
         ones = torch.ones((B, 1), dtype=attention_mask.dtype, device=dev)
         gen_ids = torch.full((B, 1), -1, dtype=doc_ids.dtype, device=dev)
-        out_buf = torch.zeros((B, max_new_tokens), dtype=tok.dtype, device=dev)
-        out_buf[:, :1] = tok
-        col = torch.ones((B, 1), dtype=torch.long, device=dev)
 
         fold_head = (dev.type == "cuda" and self.lm_head.weight.dtype == torch.bfloat16 and B <= ops.SKINNY_MAX_ROWS
                      and cfg.hidden_size % 128 == 0 and self.lm_head.bias is None)
 
-        native_sample = (dev.type == "cuda" and tok_buf.is_contiguous() and pos_buf.is_contiguous()
-                         and pos_buf.dtype == torch.int64 and pos_buf.numel() == B)
-        sample_scratch = torch.empty(B * 32, dtype=torch.int64, device=dev) if native_sample else None
-
-        def step():
-            # everything is in-place on fixed buffers so the same launches can be replayed as a graph
+        def step_logits():
             if fold_head:                          # final norm folded into the weight-streaming LM head
                 h = self.model(tok_buf, ones, pos_buf, cache, gen_ids, final_norm=False)
-                logits = ops.skinny_linear(h.view(B, -1), self.lm_head.weight, norm_weight=self.model.norm.weight,
-                                           eps=self.model.norm.variance_epsilon).view(B, 1, -1)
-            else:
-                logits = self.lm_head(self.model(tok_buf, ones, pos_buf, cache, gen_ids))
-            if native_sample:                      # argmax + token bookkeeping in two small launches
-                ops.greedy_sample(logits.view(B, -1), tok_buf, pos_buf, out_buf, col, sample_scratch)
-                return
-            new_tok = logits.argmax(-1)
-            tok_buf.copy_(new_tok)
-            pos_buf.add_(1)
-            out_buf.scatter_(1, col, new_tok)
-            col.add_(1)
+                return ops.skinny_linear(h.view(B, -1), self.lm_head.weight, norm_weight=self.model.norm.weight,
+                                         eps=self.model.norm.variance_epsilon)
+            return self.lm_head(self.model(tok_buf, ones, pos_buf, cache, gen_ids))
 
-        done = 0
-        if use_graph and n_steps > 3:
-            for _ in range(2):                     # warm-up: workspaces and library handles exist before capture
-                step()
-                done += 1
-            torch.cuda.synchronize()
-            graph = torch.cuda.CUDAGraph()
-            with torch.cuda.graph(graph):
-                step()
-            done += 0                              # capture records the launches without running them
-            while done < n_steps:
-                graph.replay()
-                done += 1
-        else:
-            while done < n_steps:
-                step()
-                done += 1
+        out_buf = greedy_decode(step_logits, tok_buf, pos_buf, max_new_tokens, use_graph)
         if timings is not None:
             torch.cuda.synchronize()
             timings["decode_s"] = time.perf_counter() - t0

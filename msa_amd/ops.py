@@ -498,7 +498,7 @@ def decode_attn_fused(qkv: torch.Tensor, Hq: int, Hkv: int, D: int, positions: t
 
 def greedy_sample(logits: torch.Tensor, tok: torch.Tensor, pos: Optional[torch.Tensor] = None,
                   out: Optional[torch.Tensor] = None, col: Optional[torch.Tensor] = None,
-                  scratch: Optional[torch.Tensor] = None) -> torch.Tensor:
+                  scratch: Optional[torch.Tensor] = None, lib=None) -> torch.Tensor:
     """Row-wise argmax of ``logits [B, V]`` written to ``tok`` (int64, ``B`` elements) with the bookkeeping of a
     greedy decode step done in place: ``pos += 1``; ``out[b, col[b]] = tok[b]``; ``col += 1``.  Returns ``tok``."""
     _need_cuda(logits, tok, pos, out, col)
@@ -512,9 +512,10 @@ def greedy_sample(logits: torch.Tensor, tok: torch.Tensor, pos: Optional[torch.T
         raise ValueError("out [B, max_new] int64 and col go together")
     if scratch is None:
         scratch = torch.empty(B * 32, dtype=torch.int64, device=logits.device)
-    check(_lib.load().msa_greedy_sample(ptr(logits), dtype_code(logits.dtype), B, V, ptr(scratch), ptr(tok), ptr(pos),
+    lib = lib or _lib.load()              # either library holds it
+    check(lib.msa_greedy_sample(ptr(logits), dtype_code(logits.dtype), B, V, ptr(scratch), ptr(tok), ptr(pos),
                                         ptr(out), out.stride(0) if out is not None else 0, ptr(col),
-                                        out.shape[1] if out is not None else 0, _stream()), "msa_greedy_sample")
+                                        out.shape[1] if out is not None else 0, _stream()), "msa_greedy_sample", lib)
     return tok
 
 

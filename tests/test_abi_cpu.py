@@ -11,8 +11,8 @@ from msa_amd import _lib
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
-def _declared():
-    text = open(os.path.join(ROOT, "include", "msa_amd.h")).read()
+def _declared(header="msa_amd.h"):
+    text = open(os.path.join(ROOT, "include", header)).read()
     text = re.sub(r"/\*.*?\*/", "", text, flags=re.S)
     return sorted(set(re.findall(r"\b(msa_[a-z0-9_]+)\s*\(", text)))
 
@@ -27,15 +27,63 @@ def test_header_symbols_exported_and_bound():
     assert lib.msa_abi_version() == 1
 
 
-def test_header_arity_matches_ctypes_table():
-    text = open(os.path.join(ROOT, "include", "msa_amd.h")).read()
+def test_seq_header_symbols_exported_and_bound():
+    lib = _lib.load_seq()
+    names = _declared("msa_seq.h")
+    assert len(names) >= 12
+    for n in names + list(_lib.SEQ_SHARED):
+        assert hasattr(lib, n), f"{n} not exported"
+    assert sorted(_lib.SEQ_SIGNATURES) == names
+    assert lib.msa_abi_version() == 1
+
+
+@pytest.mark.parametrize("header,table", [("msa_amd.h", _lib.SIGNATURES), ("msa_seq.h", _lib.SEQ_SIGNATURES)])
+def test_header_arity_matches_ctypes_table(header, table):
+    text = open(os.path.join(ROOT, "include", header)).read()
     text = re.sub(r"/\*.*?\*/", "", text, flags=re.S)
-    for name, (_, args) in _lib.SIGNATURES.items():
+    for name, (_, args) in table.items():
         m = re.search(r"\b%s\s*\(([^;]*?)\)\s*;" % name, text, flags=re.S)
         assert m, name
         params = m.group(1).strip()
         n = 0 if params in ("", "void") else len(params.split(","))
         assert n == len(args), f"{name}: header has {n} parameters, ctypes table {len(args)}"
+
+
+def test_seq_structures_match_the_header(tmp_path):
+    """Sizes and field offsets of the structures handed over by pointer, against the host compiler's."""
+    import subprocess
+    structs = {"msa_seq_batch": _lib.SeqBatch, "msa_dyn_tanh": _lib.DynTanh, "msa_rows_args": _lib.RowsArgs}
+    src = ['#include <stdio.h>', '#include "msa_seq.h"', "int main() {"]
+    for c_name, py in structs.items():
+        src.append(f'printf("{c_name} %zu\\n", sizeof({c_name}));')
+        src += [f'printf("{c_name}.{f[0]} %zu\\n", offsetof({c_name}, {f[0]}));' for f in py._fields_]
+    src.append("return 0; }")
+    (tmp_path / "s.c").write_text("\n".join(src))
+    subprocess.run(["gcc", "-I", os.path.join(ROOT, "include"), str(tmp_path / "s.c"), "-o", str(tmp_path / "s")], check=True)
+    got = dict(l.split() for l in subprocess.run([str(tmp_path / "s")], check=True, capture_output=True, text=True).stdout.splitlines())
+    for c_name, py in structs.items():
+        assert int(got[c_name]) == C.sizeof(py), c_name
+        for f in py._fields_:
+            assert int(got[f"{c_name}.{f[0]}"]) == getattr(py, f[0]).offset, f"{c_name}.{f[0]}"
+
+
+def test_seq_validation_errors_without_gpu():
+    lib = _lib.load_seq()
+    a = _lib.RowsArgs()
+    assert lib.msa_rows_linear(C.byref(a), 0, None) == -1
+    a.x = a.w = a.out = 4096
+    a.M, a.N, a.K, a.groups, a.n_b, a.x_stride, a.out_stride = 17, 16, 64, 1, 16, 64, 16
+    assert lib.msa_rows_linear(C.byref(a), 0, None) == -1 and b"M=17" in lib.msa_last_error()
+    a.M, a.K, a.x_stride = 16, 60, 64
+    assert lib.msa_rows_linear(C.byref(a), 0, None) == -1 and b"multiple of 8" in lib.msa_last_error()
+    a.K, a.n_b = 64, 8
+    assert lib.msa_rows_linear(C.byref(a), 0, None) == -1 and b"second operand" in lib.msa_last_error()
+    assert lib.msa_seq_softcap(None, 0, 1, 0.0, None, None) == -1
+    b = _lib.SeqBatch(4096, 4096, 4096, 4096, 1, 4, 4, 0)
+    assert lib.msa_seq_flash(4096, 96, 4096, 96, 4096, 96, 4096, 4096, 1.0, 0, 1, 300, 96, 4096, C.byref(b), None) == -1
+    assert b"D=300" in lib.msa_last_error()
+    assert lib.msa_seq_min_gru(4096, 96, 4096, 4096, 0, 32, 4096, 4096, C.byref(_lib.SeqBatch(4096, 4096, 4096, 4096, 1, 999, 999, 0)),
+                               None, 0, None) == -3 and b"workspace" in lib.msa_last_error()
 
 
 def test_validation_errors_without_gpu():
