@@ -68,10 +68,9 @@ int msa_seq_conv_silu(const void* in, int64_t in_stride, const float* taps, cons
 int msa_seq_ssd_scan(const void* xbc, int64_t xbc_stride, const void* z, int64_t z_stride, const void* dt_raw, int64_t dt_stride,
                      const float* dt_bias, const float* A_log, const float* D, int32_t dtype, int32_t H, int32_t P, int32_t N,
                      int32_t G, float* state, void* v, const msa_seq_batch* batch, void* stream);
-/* The same recurrence for long bf16 portions of one sequence or several, in chunks of MSA_SSD_CHUNK tokens on the
- * matrix cores: chunk states, their recurrence, chunk outputs.  N a multiple of 16 up to 256, P a multiple of 8. */
-#define MSA_SSD_CHUNK 64
-size_t msa_seq_ssd_chunked_workspace_bytes(int32_t rows, int32_t n_seq, int32_t H, int32_t P, int32_t N);
+/* The same recurrence for long bf16 portions, in chunks of 64 or 128 tokens on the matrix cores: chunk states, their
+ * recurrence, chunk outputs.  N a multiple of 8 up to 256, P a multiple of 8. */
+size_t msa_seq_ssd_chunked_workspace_bytes(int32_t max_rows, int32_t n_seq, int32_t H, int32_t P, int32_t N);
 int msa_seq_ssd_chunked(const void* xbc, int64_t xbc_stride, const void* z, int64_t z_stride, const void* dt_raw, int64_t dt_stride,
                         const float* dt_bias, const float* A_log, const float* D, int32_t dtype, int32_t H, int32_t P,
                         int32_t N, int32_t G, float* state, void* v, const msa_seq_batch* batch, void* workspace,

@@ -70,8 +70,8 @@ class Mamba2Mixer:
 
     def _scan(self, xbc, z, dt, state, batch):
         c = self.c
-        chunked = (xbc.dtype == torch.bfloat16 and batch.max_rows >= (1 << 30) and c.state % 16 == 0 and c.state <= 256
-                   and c.vdim % 8 == 0)
+        chunked = (xbc.dtype == torch.bfloat16 and batch.max_rows >= seq_ops.SSD_CHUNKED_ROWS and c.state % 8 == 0
+                   and c.state <= 256 and c.vdim % 8 == 0)
         v = seq_ops.ssd(xbc, z, dt, self.dt_bias, self.A_log, self.D, c.heads, c.vdim, c.state, c.groups, state["ssm"], batch,
                         chunked=chunked)
         return seq_ops.group_rmsnorm(v, self.norm, c.norm_groups, self.eps)

@@ -12,7 +12,7 @@ from . import _lib
 from ._lib import dtype_code, ptr
 
 MAX_ROWS = 16           # rows of a step that the weight-streaming kernels take
-SSD_CHUNK = 64
+SSD_CHUNKED_ROWS = 64   # portions from this many tokens on are cut into chunks
 
 
 def _check(code: int, where: str) -> None:
@@ -179,7 +179,7 @@ def ssd(xbc, z, dt_raw, dt_bias, A_log, D, H: int, P: int, N: int, G: int, state
     args = [ptr(xbc), _rows(xbc), ptr(z), _rows(z), ptr(dt_raw), _rows(dt_raw), ptr(dt_bias), ptr(A_log), ptr(D),
             dtype_code(xbc.dtype), H, P, N, G, ptr(state), ptr(v), batch.ref]
     if chunked:
-        ws = _workspace(xbc.device, lib.msa_seq_ssd_chunked_workspace_bytes(T, batch.n_seq, H, P, N))
+        ws = _workspace(xbc.device, lib.msa_seq_ssd_chunked_workspace_bytes(batch.max_rows, batch.n_seq, H, P, N))
         _check(lib.msa_seq_ssd_chunked(*args, ptr(ws), ws.numel(), _stream()), "msa_seq_ssd_chunked")
     else:
         _check(lib.msa_seq_ssd_scan(*args, _stream()), "msa_seq_ssd_scan")
