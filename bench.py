@@ -422,7 +422,14 @@ def main():
                     help="also run one plain 1 GiB device copy (reference point for rocprof FETCH_SIZE / WRITE_SIZE)")
     ap.add_argument("--ceiling-only", action="store_true",
                     help="run only the register-only MFMA loop (other_kernels.mfma_ceiling) and print its figures")
+    ap.add_argument("--hybrid", action="store_true",
+                    help="run the hybrid decoder's benchmark (bench_hybrid.py) instead: prefill and decode throughput and every "
+                         "kernel beside the attention model's")
     args = ap.parse_args()
+    if args.hybrid:
+        import bench_hybrid
+        bench_hybrid.main([])
+        return
     if args.gpus != 1:
         sys.exit("bench.py: this build runs on exactly one GPU (no sharding, no collectives); use --gpus 1")
     if not torch.cuda.is_available():

@@ -102,10 +102,11 @@ class HybridForCausalLM:
     def step(self, cache: SequenceStateCache, entries: Sequence[Entry]) -> Optional[torch.Tensor]:
         """Feeds every entry's tokens behind what its sequence has been fed before (a key not seen before starts a
         sequence).  Returns fp32 logits ``[wanted, vocab]`` in the order of the entries and their wanted places, or None."""
+        entries = [(k, torch.as_tensor(t, dtype=torch.int64).cpu(), w) for k, t, w in entries]
         for key, tokens, want in entries:
             if not len(tokens) or any(not 0 <= w < len(tokens) for w in want):
                 raise ValueError(f"sequence {key!r}: no tokens, or a wanted place outside them")
-            if any(not 0 <= t < self.config.vocab for t in tokens):
+            if not 0 <= int(tokens.min()) <= int(tokens.max()) < self.config.vocab:
                 raise ValueError(f"sequence {key!r}: token outside the vocabulary")
         cache.reserve(max(cache.length.get(k, 0) + len(t) for k, t, _ in entries))
         for key, _, _ in entries:
@@ -114,7 +115,7 @@ class HybridForCausalLM:
         counts = [len(t) for _, t, _ in entries]
         batch = seq_ops.StepBatch(counts, [cache.slot_of[k] for k, _, _ in entries], [cache.length[k] for k, _, _ in entries],
                                   self.device)
-        tokens = torch.tensor([t for _, ts, _ in entries for t in ts], dtype=torch.int64).to(self.device)
+        tokens = torch.cat([t for _, t, _ in entries]).to(self.device)
         rows, at = [], 0
         for (_, ts, want) in entries:
             rows += [at + w for w in want]
@@ -213,7 +214,7 @@ class HybridForCausalLM:
         ``max_new_tokens`` greedily.  Returns ``(tokens [B, max_new_tokens], cache)``; the sequences ``0 .. B - 1`` stay open
         in the cache, with every token but the last fed."""
         import time
-        prompts = [[t for t, m in zip(ids, mask) if m] for ids, mask in zip(input_ids.tolist(), attention_mask.tolist())]
+        prompts = [ids[mask != 0] for ids, mask in zip(input_ids.cpu(), attention_mask.cpu())]
         B = len(prompts)
         cache = cache if cache is not None else self.create_cache(B)
         longest = max(len(p) for p in prompts)
