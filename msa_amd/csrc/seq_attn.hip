@@ -110,15 +110,14 @@ struct DecArgs {
   int32_t H, rank, n_split;
 };
 
-// HT tiles of 16 heads.  Wavefront w scores keys 16 w .. + 16 of a tile and owns the latent columns of tiles w, w + 4, ...
-// of the product with the probabilities.
-template <int HT>
+// HT tiles of 16 heads, RP: the rank padded to 64, 128, 256 or 512 (zeros in LDS).  Wavefront w scores keys 16 w .. + 16 of a
+// tile and owns the latent columns of tiles w, w + 4, ... of the product with the probabilities.
+template <int HT, int RP>
 __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_batch b) {
   constexpr int kHeads = 16 * HT, kPStride = kDecKeys + 8, kPer = 256 / kHeads;   // threads per head in the softmax
-  constexpr int kSStride = kDecKeys + 4;
-  constexpr int kCT = kDecMaxRank / 16 / 4;
+  constexpr int kSStride = kDecKeys + 4, stride = RP + 8;
+  constexpr int kCT = RP / 16 / 4, units = RP / 8;               // 16-byte pieces of a row, zero behind the rank
   extern __shared__ __align__(16) char lds[];
-  const int rankp = (a.rank + 31) / 32 * 32, stride = rankp + 8;
   bf16_t* cs = reinterpret_cast<bf16_t*>(lds);                   // [64][stride]
   bf16_t* qs = cs + kDecKeys * stride;                           // [kHeads][stride]
   bf16_t* ps = qs + kHeads * stride;                             // [kHeads][kPStride]
@@ -131,41 +130,42 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_b
   const int tiles = (n_keys + kDecKeys - 1) / kDecKeys, per = (tiles + a.n_split - 1) / a.n_split;
   const int first = split * per * kDecKeys, last = min(n_keys, first + per * kDecKeys);
   const bf16_t* c = a.cache + (int64_t)b.slot[s] * a.Lcap * a.rank;
-  const int units = rankp / 8;                                   // 16-byte pieces of a row, zero behind the rank
 
-  for (int i = tid; i < kHeads * units; i += 256) {
-    const int h = i / units, u = i % units;
-    uint4 w = make_uint4(0, 0, 0, 0);
-    if (h0 + h < a.H && u * 8 < a.rank) w = *reinterpret_cast<const uint4*>(a.q + ((int64_t)row * a.H + h0 + h) * a.rank + u * 8);
-    *reinterpret_cast<uint4*>(qs + h * stride + u * 8) = w;
-  }
-  constexpr int kPieces = kDecKeys * (kDecMaxRank / 8) / 256;    // pieces of a tile per thread (16)
+  // a thread's pieces: column u of rows r0, r0 + 256 / units, ...
+  const int u = tid % units * 8, r0 = tid / units;
+  constexpr int kStep = 256 / units, kPieces = kDecKeys / kStep, kQPieces = (kHeads + kStep - 1) / kStep;
   uint4 next[kPieces];
-  const int total = kDecKeys * units;
   auto fetch = [&](int k0) {
+    const bf16_t* at = c + (int64_t)(k0 + r0) * a.rank + u;
 #pragma unroll
     for (int i = 0; i < kPieces; ++i) {
-      const int idx = tid + 256 * i, key = idx / units, u = idx % units;
       next[i] = make_uint4(0, 0, 0, 0);
-      if (idx < total && k0 + key < last && u * 8 < a.rank)
-        next[i] = *reinterpret_cast<const uint4*>(c + (int64_t)(k0 + key) * a.rank + u * 8);
+      if (k0 + r0 + kStep * i < last && u < a.rank) next[i] = *reinterpret_cast<const uint4*>(at + (int64_t)(kStep * i) * a.rank);
     }
   };
   auto stash = [&]() {
 #pragma unroll
-    for (int i = 0; i < kPieces; ++i) {
-      const int idx = tid + 256 * i;
-      if (idx < total) *reinterpret_cast<uint4*>(cs + (idx / units) * stride + (idx % units) * 8) = next[i];
-    }
+    for (int i = 0; i < kPieces; ++i) *reinterpret_cast<uint4*>(cs + (r0 + kStep * i) * stride + u) = next[i];
   };
+  if (first < last) fetch(first);
+  {
+    uint4 qw[kQPieces];
+#pragma unroll
+    for (int i = 0; i < kQPieces; ++i) {
+      const int h = h0 + r0 + kStep * i;
+      qw[i] = make_uint4(0, 0, 0, 0);
+      if (h < a.H && u < a.rank) qw[i] = *reinterpret_cast<const uint4*>(a.q + ((int64_t)row * a.H + h) * a.rank + u);
+    }
+#pragma unroll
+    for (int i = 0; i < kQPieces; ++i)
+      if (kHeads >= kStep || r0 < kHeads) *reinterpret_cast<uint4*>(qs + (r0 + kStep * i) * stride + u) = qw[i];
+  }
   floatx4_t o[HT][kCT];
 #pragma unroll
   for (int h = 0; h < HT; ++h)
 #pragma unroll
     for (int t = 0; t < kCT; ++t) o[h][t] = floatx4_t{0.f, 0.f, 0.f, 0.f};
-  const int col_tiles = rankp / 16;
   float m = -INFINITY, l = 0.f;        // of head tid / kPer, the same in its kPer threads
-  if (first < last) fetch(first);
   for (int k0 = first; k0 < last; k0 += kDecKeys) {
     __syncthreads();
     stash();
@@ -174,7 +174,8 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_b
     floatx4_t sc[HT];
 #pragma unroll
     for (int h = 0; h < HT; ++h) sc[h] = floatx4_t{0.f, 0.f, 0.f, 0.f};
-    for (int kk = 0; kk < rankp; kk += 32) {
+#pragma unroll
+    for (int kk = 0; kk < RP; kk += 32) {
       const bf16x8_t kb = *reinterpret_cast<const bf16x8_t*>(cs + (wave * 16 + l16) * stride + kk + 8 * g);
 #pragma unroll
       for (int h = 0; h < HT; ++h) {
@@ -198,11 +199,11 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_b
       }
 #pragma unroll
       for (int d = 1; d < kPer; d <<= 1) mx = fmaxf(mx, __shfl_xor(mx, d));
-      const float alpha = exp2f(m - mx);                         // a tile has at least one key: mx is finite
+      const float alpha = __builtin_amdgcn_exp2f(m - mx);        // a tile has at least one key: mx is finite
       float sum = 0.f;
 #pragma unroll
       for (int j = 0; j < kEach; j += 2) {
-        const float p0 = exp2f(v[j] - mx), p1 = exp2f(v[j + 1] - mx);
+        const float p0 = __builtin_amdgcn_exp2f(v[j] - mx), p1 = __builtin_amdgcn_exp2f(v[j + 1] - mx);
         sum += p0 + p1;
         *reinterpret_cast<uint32_t*>(ps + h * kPStride + j0 + j) = pack_bf16x2(p0, p1);
       }
@@ -215,13 +216,14 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_b
     __syncthreads();
 #pragma unroll
     for (int h = 0; h < HT; ++h) {
-      float f[4];
+      const float4 f = *reinterpret_cast<const float4*>(al + h * 16 + 4 * g);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) f[e] = al[h * 16 + 4 * g + e];
-#pragma unroll
-      for (int t = 0; t < kCT; ++t)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) o[h][t][e] *= f[e];
+      for (int t = 0; t < kCT; ++t) {
+        o[h][t][0] *= f.x;
+        o[h][t][1] *= f.y;
+        o[h][t][2] *= f.z;
+        o[h][t][3] *= f.w;
+      }
     }
 #pragma unroll
     for (int kk = 0; kk < kDecKeys; kk += 32) {
@@ -230,9 +232,7 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_b
       for (int h = 0; h < HT; ++h) pa[h] = *reinterpret_cast<const bf16x8_t*>(ps + (h * 16 + l16) * kPStride + kk + 8 * g);
 #pragma unroll
       for (int t = 0; t < kCT; ++t) {
-        const int ct = wave + 4 * t;
-        if (ct >= col_tiles) break;
-        const bf16_t* at = cs + (kk + 8 * g + (l16 >> 2)) * stride + ct * 16 + (l16 & 3) * 4;
+        const bf16_t* at = cs + (kk + 8 * g + (l16 >> 2)) * stride + (wave + 4 * t) * 16 + (l16 & 3) * 4;
         const bf16x8_t vb = join8(lds_read_tr16(at), lds_read_tr16(at + 4 * stride));
 #pragma unroll
         for (int h = 0; h < HT; ++h) o[h][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[h], vb, o[h][t], 0, 0, 0);
@@ -259,35 +259,53 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_b
   }
 }
 
-// A workgroup per (row, head): folds the key ranges and the sink.
+// A workgroup per (row, head): folds the key ranges and the sink.  The ranges' weights first, then one pass over their sums.
+constexpr int kMaxSplits = 128;
 __global__ __launch_bounds__(128) void latent_combine_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
                                                              const float* __restrict__ sink, int32_t H, int32_t rank, int32_t n_split,
                                                              bf16_t* __restrict__ ctx) {
-  const int row = blockIdx.x, head = blockIdx.y;
+  __shared__ float ws[kMaxSplits], red[4];
+  const int row = blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
+  const int64_t first = (int64_t)row * n_split * H + head;
   const float sk = sink[head] * kLog2e;
-  float m = sk;
-  for (int i = 0; i < n_split; ++i) m = fmaxf(m, part_ml[(((int64_t)row * n_split + i) * H + head) * 2]);
-  float l = exp2f(sk - m);
-  for (int i = 0; i < n_split; ++i) {
-    const float* ml = part_ml + (((int64_t)row * n_split + i) * H + head) * 2;
-    if (ml[0] > -INFINITY) l += exp2f(ml[0] - m) * ml[1];
+  float mi = -INFINITY, li = 0.f;
+  if (tid < n_split) {
+    const float2 ml = *reinterpret_cast<const float2*>(part_ml + (first + (int64_t)tid * H) * 2);
+    mi = ml.x;
+    li = ml.y;
   }
-  const float inv = 1.0f / l;
-  for (int c = threadIdx.x; c < rank; c += 128) {
-    float v = 0.f;
+  float m = fmaxf(mi, sk);
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) m = fmaxf(m, __shfl_xor(m, o));
+  if ((tid & 63) == 0) red[tid >> 6] = m;
+  __syncthreads();
+  m = fmaxf(red[0], red[1]);
+  const float w = __builtin_amdgcn_exp2f(mi - m);                // 0 for a range without keys
+  float l = w * li;
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) l += __shfl_xor(l, o);
+  if ((tid & 63) == 0) red[2 + (tid >> 6)] = l;
+  ws[tid] = w;
+  __syncthreads();
+  const float inv = 1.0f / (red[2] + red[3] + __builtin_amdgcn_exp2f(sk - m));
+  for (int c = tid * 4; c < rank; c += 512) {
+    float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+    const float* src = part_acc + first * rank + c;
+#pragma unroll 8
     for (int i = 0; i < n_split; ++i) {
-      const int64_t at = ((int64_t)row * n_split + i) * H + head;
-      const float mi = part_ml[at * 2];
-      if (mi > -INFINITY) v += exp2f(mi - m) * part_acc[at * rank + c];
+      const float4 p = *reinterpret_cast<const float4*>(src + (int64_t)i * H * rank);
+      const float f = ws[i];
+      v.x += f * p.x; v.y += f * p.y; v.z += f * p.z; v.w += f * p.w;
     }
-    ctx[((int64_t)row * H + head) * rank + c] = f32_to_bf16(v * inv);
+    *reinterpret_cast<uint2*>(ctx + ((int64_t)row * H + head) * rank + c) =
+        make_uint2(pack_bf16x2(v.x * inv, v.y * inv), pack_bf16x2(v.z * inv, v.w * inv));
   }
 }
 
 int latent_splits(int32_t rows, int32_t H, int64_t max_keys) {
   const int64_t tiles = std::max<int64_t>(1, (max_keys + kDecKeys - 1) / kDecKeys);
   const int64_t blocks = (int64_t)rows * ((H + 31) / 32);
-  return (int)std::min<int64_t>(std::min<int64_t>(tiles, 128), std::max<int64_t>(1, (2 * device_compute_units() + blocks - 1) / blocks));
+  return (int)std::min<int64_t>(std::min<int64_t>(tiles, kMaxSplits), std::max<int64_t>(1, (device_compute_units() + blocks - 1) / blocks));
 }
 
 // ------------------------------------------------------------------------------------------------ prefill
@@ -463,16 +481,23 @@ int launch_flash(const FlashArgs& a, const msa_seq_batch& b, hipStream_t st) {
   return MSA_OK;
 }
 
-template <int HT>
+template <int HT, int RP>
 int launch_decode(const DecArgs& a, const msa_seq_batch& b, hipStream_t st) {
-  const int stride = (a.rank + 31) / 32 * 32 + 8, heads = 16 * HT;
-  const int lds = (kDecKeys + heads) * stride * 2 + heads * (kDecKeys + 8) * 2 + heads * (kDecKeys + 4) * 4 + heads * 4;
+  constexpr int stride = RP + 8, heads = 16 * HT;
+  constexpr int lds = (kDecKeys + heads) * stride * 2 + heads * (kDecKeys + 8) * 2 + heads * (kDecKeys + 4) * 4 + heads * 4;
+  static_assert(lds <= 160 * 1024, "tiles must fit LDS");
   static std::atomic<int> raised{0};
-  MSA_HIP(raise_dynamic_lds_limit(raised, reinterpret_cast<const void*>(latent_decode_kernel<HT>), 160 * 1024));
-  MSA_REQUIRE(lds <= 160 * 1024, "msa_seq_latent_decode: %d bytes of LDS", lds);
-  latent_decode_kernel<HT><<<dim3(a.n_split, (a.H + heads - 1) / heads, b.rows), 256, lds, st>>>(a, b);
+  MSA_HIP(raise_dynamic_lds_limit(raised, reinterpret_cast<const void*>(latent_decode_kernel<HT, RP>), lds));
+  latent_decode_kernel<HT, RP><<<dim3(a.n_split, (a.H + heads - 1) / heads, b.rows), 256, lds, st>>>(a, b);
   MSA_LAUNCH_CHECK();
   return MSA_OK;
+}
+template <int HT>
+int launch_decode(const DecArgs& a, const msa_seq_batch& b, hipStream_t st) {
+  if (a.rank <= 64) return launch_decode<HT, 64>(a, b, st);
+  if (a.rank <= 128) return launch_decode<HT, 128>(a, b, st);
+  if (a.rank <= 256) return launch_decode<HT, 256>(a, b, st);
+  return launch_decode<HT, 512>(a, b, st);
 }
 
 }  // namespace

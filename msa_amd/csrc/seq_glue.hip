@@ -38,23 +38,33 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResNorm a, msa_seq_b
     load_vec<float, VEC>(a.norm.b + col, nb);
   }
   if (a.shift) load_vec<float, VEC>(a.shift + col, sh);
-  auto value = [&](int t, float (&v)[VEC]) {
-    load_vec<float, VEC>(a.x_in + (int64_t)t * a.W + col, v);
+  struct Raw { float x[VEC], y[VEC], g[VEC]; };
+  auto fetch = [&](int t, Raw& r) {
+    load_vec<float, VEC>(a.x_in + (int64_t)t * a.W + col, r.x);
     if (!a.y) return;
-    float y[VEC], g[VEC];
-    load_vec<T, VEC>(static_cast<const T*>(a.y) + t * a.y_stride + col, y);
-    load_vec<T, VEC>(static_cast<const T*>(a.gate) + t * a.gate_stride + col, g);
+    load_vec<T, VEC>(static_cast<const T*>(a.y) + t * a.y_stride + col, r.y);
+    load_vec<T, VEC>(static_cast<const T*>(a.gate) + t * a.gate_stride + col, r.g);
+  };
+  auto combine = [&](const Raw& r, float (&v)[VEC]) {
 #pragma unroll
-    for (int i = 0; i < VEC; ++i) v[i] += sigmoid_f(g[i] + gb[i]) * y[i];
+    for (int i = 0; i < VEC; ++i) v[i] = a.y ? r.x[i] + sigmoid_f(r.g[i] + gb[i]) * r.y[i] : r.x[i];
+  };
+  auto value = [&](int t, float (&v)[VEC]) {
+    Raw r;
+    fetch(t, r);
+    combine(r, v);
   };
   auto normed = [&](const float (&v)[VEC], float (&h)[VEC]) {
 #pragma unroll
-    for (int i = 0; i < VEC; ++i) h[i] = tanhf(a.norm.alpha * v[i]) * nw[i] + nb[i];
+    for (int i = 0; i < VEC; ++i) h[i] = tanh_f(a.norm.alpha * v[i]) * nw[i] + nb[i];
   };
   float before[VEC] = {};
+  Raw next;                             // the row ahead is on its way while this one is finished
+  fetch(t0, next);
   for (int t = t0; t < t1; ++t) {
     float v[VEC], h[VEC];
-    value(t, v);
+    combine(next, v);
+    if (t + 1 < t1) fetch(t + 1, next);
     if (a.x_out) store_vec<float, VEC>(a.x_out + (int64_t)t * a.W + col, v);
     if (!norm) continue;
     normed(v, h);
@@ -109,7 +119,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void softcap_kernel(const T* __restrict__ in, int64_t n, float cap, float* __restrict__ out) {
   for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
     const float v = to_f32<T>(in[i]);
-    out[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
+    out[i] = cap > 0.f ? cap * tanh_f(v / cap) : v;
   }
 }
 
@@ -128,29 +138,57 @@ __global__ __launch_bounds__(256) void join_kernel(const float* __restrict__ x, 
   }
 }
 
-// One workgroup per (row, part).
-template <typename T>
-__global__ __launch_bounds__(256) void group_rmsnorm_kernel(const T* __restrict__ v, int32_t n, int32_t parts,
+// A wavefront per (row, part): the part stays in registers between the sum of squares and the output when it fits
+// (VEC = 8: 16-byte accesses).
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void group_rmsnorm_kernel(const T* __restrict__ v, int64_t items, int32_t n, int32_t parts,
                                                             const float* __restrict__ w, float eps, T* __restrict__ out) {
-  __shared__ float part_sum[4];
-  const int len = n / parts;
-  const int64_t at = (int64_t)blockIdx.x * n + (int64_t)blockIdx.y * len;
-  const float* wg = w + blockIdx.y * len;
-  float ssq = 0.f;
-  for (int i = threadIdx.x; i < len; i += 256) {
-    const float x = to_f32<T>(v[at + i]);
-    ssq += x * x;
+  constexpr int kKeep = 4;
+  const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= items) return;
+  const int lane = threadIdx.x & 63, len = n / parts;
+  const int64_t at = item * len;
+  const float* wg = w + item % parts * len;
+  float keep[kKeep][VEC], ssq = 0.f;
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k) {
+    const int i = (k * 64 + lane) * VEC;
+    if (i < len) {
+      load_vec<T, VEC>(v + at + i, keep[k]);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ssq += keep[k][e] * keep[k][e];
+    }
+  }
+  for (int i = (kKeep * 64 + lane) * VEC; i < len; i += 64 * VEC) {
+    float x[VEC];
+    load_vec<T, VEC>(v + at + i, x);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ssq += x[e] * x[e];
   }
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) ssq += __shfl_xor(ssq, o);
-  if ((threadIdx.x & 63) == 0) part_sum[threadIdx.x >> 6] = ssq;
-  __syncthreads();
-  const float inv = 1.0f / sqrtf((part_sum[0] + part_sum[1] + part_sum[2] + part_sum[3]) / (float)len + eps);
-  for (int i = threadIdx.x; i < len; i += 256) out[at + i] = from_f32<T>(to_f32<T>(v[at + i]) * inv * wg[i]);
+  const float inv = 1.0f / sqrtf(ssq / (float)len + eps);
+  auto finish = [&](int i, float (&x)[VEC]) {
+    float g[VEC];
+    load_vec<float, VEC>(wg + i, g);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) x[e] *= inv * g[e];
+    store_vec<T, VEC>(out + at + i, x);
+  };
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k) {
+    const int i = (k * 64 + lane) * VEC;
+    if (i < len) finish(i, keep[k]);
+  }
+  for (int i = (kKeep * 64 + lane) * VEC; i < len; i += 64 * VEC) {
+    float x[VEC];
+    load_vec<T, VEC>(v + at + i, x);
+    finish(i, x);
+  }
 }
 
 // One wavefront per row.
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void latent_append_kernel(const T* __restrict__ in, int64_t stride, const float* __restrict__ w,
                                                             float eps, int32_t rank, T* __restrict__ cache, int64_t Lcap,
                                                             msa_seq_batch b) {
@@ -159,17 +197,26 @@ __global__ __launch_bounds__(256) void latent_append_kernel(const T* __restrict_
   const int s = b.row_seq[row];
   const int64_t p = b.pos[s] + (row - b.cu[s]);
   const T* src = in + row * stride;
+  T* dst = cache + ((int64_t)b.slot[s] * Lcap + p) * rank;
   float ssq = 0.f;
-  for (int i = lane; i < rank; i += 64) {
-    const float x = to_f32<T>(src[i]);
-    ssq += x * x;
+  for (int i = lane * VEC; i < rank; i += 64 * VEC) {
+    float x[VEC];
+    load_vec<T, VEC>(src + i, x);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ssq += x[e] * x[e];
   }
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) ssq += __shfl_xor(ssq, o);
   if (p >= Lcap) return;
   const float inv = 1.0f / sqrtf(ssq / (float)rank + eps);
-  T* dst = cache + ((int64_t)b.slot[s] * Lcap + p) * rank;
-  for (int i = lane; i < rank; i += 64) dst[i] = from_f32<T>(to_f32<T>(src[i]) * inv * w[i]);
+  for (int i = lane * VEC; i < rank; i += 64 * VEC) {
+    float x[VEC], g[VEC];
+    load_vec<T, VEC>(src + i, x);
+    load_vec<float, VEC>(w + i, g);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) x[e] *= inv * g[e];
+    store_vec<T, VEC>(dst + i, x);
+  }
 }
 
 int grid_for(int64_t items) { return (int)std::min<int64_t>(std::max<int64_t>(1, (items + 255) / 256), 8192); }
@@ -192,7 +239,7 @@ extern "C" int msa_seq_residual_norm(const float* x_in, const void* y, int64_t y
   ResNorm a{x_in, y, gate, gate_bias, y ? x_out : nullptr, with_norm ? *norm : msa_dyn_tanh{}, with_norm ? h : nullptr,
             shift, prev, h_shift, y_stride, gate_stride, W, 1};
   a.rows_per_wg = batch->rows <= 256 ? 1 : 8;
-  const bool vec = vec4_ok({x_in, y, gate, gate_bias, x_out, a.norm.w, a.norm.b, h, shift, prev, h_shift}, {W, y_stride, gate_stride});
+  const bool vec = vec_ok(4, {x_in, y, gate, gate_bias, x_out, a.norm.w, a.norm.b, h, shift, prev, h_shift}, {W, y_stride, gate_stride});
   const int V = vec ? 4 : 1;
   const dim3 grid((batch->rows + a.rows_per_wg - 1) / a.rows_per_wg, (W + 256 * V - 1) / (256 * V));
   hipStream_t st = as_stream(stream);
@@ -210,7 +257,7 @@ extern "C" int msa_seq_residual_norm(const float* x_in, const void* y, int64_t y
 extern "C" int msa_seq_gelu(void* y, int64_t y_stride, int32_t dtype, int32_t rows, int32_t n, void* stream) {
   MSA_REQUIRE(y && rows > 0 && n > 0 && y_stride >= n, "msa_seq_gelu: bad arguments");
   MSA_CHECK_DTYPE(dtype, "msa_seq_gelu");
-  const bool vec = vec4_ok({y}, {y_stride, n});
+  const bool vec = vec_ok(4, {y}, {y_stride, n});
   const int grid = grid_for((int64_t)rows * n / (vec ? 4 : 1));
   hipStream_t st = as_stream(stream);
   if (dtype == MSA_BF16) {
@@ -248,11 +295,17 @@ extern "C" int msa_seq_group_rmsnorm(const void* v, int32_t dtype, int32_t rows,
   MSA_REQUIRE(v && w && out && rows > 0 && n > 0 && parts > 0 && n % parts == 0 && parts <= 65535,
               "msa_seq_group_rmsnorm: n=%d in %d parts", n, parts);
   MSA_CHECK_DTYPE(dtype, "msa_seq_group_rmsnorm");
-  const dim3 grid(rows, parts);
-  if (dtype == MSA_BF16)
-    group_rmsnorm_kernel<bf16_t><<<grid, 256, 0, as_stream(stream)>>>((const bf16_t*)v, n, parts, w, eps, (bf16_t*)out);
-  else
-    group_rmsnorm_kernel<float><<<grid, 256, 0, as_stream(stream)>>>((const float*)v, n, parts, w, eps, (float*)out);
+  const int64_t items = (int64_t)rows * parts;
+  const unsigned grid = (unsigned)((items + 3) / 4);
+  const bool vec = vec_ok(8, {v, w, out}, {n / parts});
+  hipStream_t st = as_stream(stream);
+  if (dtype == MSA_BF16) {
+    if (vec) group_rmsnorm_kernel<bf16_t, 8><<<grid, 256, 0, st>>>((const bf16_t*)v, items, n, parts, w, eps, (bf16_t*)out);
+    else group_rmsnorm_kernel<bf16_t, 1><<<grid, 256, 0, st>>>((const bf16_t*)v, items, n, parts, w, eps, (bf16_t*)out);
+  } else {
+    if (vec) group_rmsnorm_kernel<float, 8><<<grid, 256, 0, st>>>((const float*)v, items, n, parts, w, eps, (float*)out);
+    else group_rmsnorm_kernel<float, 1><<<grid, 256, 0, st>>>((const float*)v, items, n, parts, w, eps, (float*)out);
+  }
   MSA_LAUNCH_CHECK();
   return MSA_OK;
 }
@@ -263,10 +316,15 @@ extern "C" int msa_seq_latent_append(const void* in, int64_t in_stride, const fl
   MSA_CHECK_DTYPE(dtype, "msa_seq_latent_append");
   MSA_REQUIRE(in && w && cache && rank > 0 && in_stride >= rank && Lcap > 0, "msa_seq_latent_append: bad arguments");
   const int grid = (batch->rows + 3) / 4;
-  if (dtype == MSA_BF16)
-    latent_append_kernel<bf16_t><<<grid, 256, 0, as_stream(stream)>>>((const bf16_t*)in, in_stride, w, eps, rank, (bf16_t*)cache, Lcap, *batch);
-  else
-    latent_append_kernel<float><<<grid, 256, 0, as_stream(stream)>>>((const float*)in, in_stride, w, eps, rank, (float*)cache, Lcap, *batch);
+  const bool vec = vec_ok(8, {in, w, cache}, {in_stride, rank});
+  hipStream_t st = as_stream(stream);
+  if (dtype == MSA_BF16) {
+    if (vec) latent_append_kernel<bf16_t, 8><<<grid, 256, 0, st>>>((const bf16_t*)in, in_stride, w, eps, rank, (bf16_t*)cache, Lcap, *batch);
+    else latent_append_kernel<bf16_t, 1><<<grid, 256, 0, st>>>((const bf16_t*)in, in_stride, w, eps, rank, (bf16_t*)cache, Lcap, *batch);
+  } else {
+    if (vec) latent_append_kernel<float, 8><<<grid, 256, 0, st>>>((const float*)in, in_stride, w, eps, rank, (float*)cache, Lcap, *batch);
+    else latent_append_kernel<float, 1><<<grid, 256, 0, st>>>((const float*)in, in_stride, w, eps, rank, (float*)cache, Lcap, *batch);
+  }
   MSA_LAUNCH_CHECK();
   return MSA_OK;
 }

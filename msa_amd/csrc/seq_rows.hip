@@ -114,7 +114,7 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_ar
       if (EPI == MSA_ROWS_PLAIN && n < a.gelu_n) v = gelu_tanh_f(v);
       out16[m * a.out_stride + col] = f32_to_bf16(v);
     } else if constexpr (EPI == MSA_ROWS_F32) {
-      if (a.cap > 0.f) v = a.cap * tanhf(v / a.cap);
+      if (a.cap > 0.f) v = a.cap * tanh_f(v / a.cap);
       if (a.add) v += a.add[col];
       static_cast<float*>(a.out)[m * a.out_stride + col] = v;
     } else if constexpr (EPI == MSA_ROWS_MAMBA) {
@@ -139,7 +139,7 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_ar
       const float x = a.x_in[at] + sigmoid_f(gate) * v;
       a.x_out[at] = x;
       if (a.norm.w) {
-        const float h = tanhf(a.norm.alpha * x) * a.norm.w[n] + a.norm.b[n];
+        const float h = tanh_f(a.norm.alpha * x) * a.norm.w[n] + a.norm.b[n];
         if (a.h) static_cast<bf16_t*>(a.h)[at] = f32_to_bf16(h);
         if (a.shift) {
           float* prev = a.prev + (int64_t)a.slot[m] * a.N + n;

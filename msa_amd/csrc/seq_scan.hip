@@ -44,11 +44,77 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(const T* __restrict__ in
     }
 }
 
+// The same for 2 <= K <= 5 and aligned rows: a thread owns eight channels and slides its window of K - 1 inputs along.
+template <typename T, int K>
+__global__ __launch_bounds__(256) void conv_silu_vec_kernel(const T* __restrict__ in, int64_t in_stride, const float* __restrict__ taps,
+                                                            const float* __restrict__ bias, int32_t C, float* __restrict__ state,
+                                                            T* __restrict__ out, int64_t out_stride, msa_seq_batch b) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
+  const int s = blockIdx.z;
+  const int lo = b.cu[s], n = b.cu[s + 1] - lo;
+  const int t0 = blockIdx.y * kConvRows;
+  if (c >= C || t0 >= n) return;
+  const int t1 = min(n, t0 + kConvRows);
+  float* keep = state + (int64_t)b.slot[s] * (K - 1) * C + c;
+  const T* src = in + (int64_t)lo * in_stride + c;
+  float tp[K][8], bs[8], win[K - 1][8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e)
+#pragma unroll
+    for (int j = 0; j < K; ++j) tp[j][e] = taps[(int64_t)(c + e) * K + j];
+  load_vec<float, 8>(bias + c, bs);
+  auto input = [&](int u, float (&x)[8]) {                   // input u of the sequence's new tokens, or a kept one (u < 0)
+    if (u >= 0) load_vec<T, 8>(src + u * in_stride, x);
+    else load_vec<float, 8>(keep + (int64_t)(K - 1 + u) * C, x);
+  };
+#pragma unroll
+  for (int j = 0; j < K - 1; ++j) input(t0 - (K - 1) + j, win[j]);
+#pragma unroll 4
+  for (int t = t0; t < t1; ++t) {
+    float x[8], y[8];
+    load_vec<T, 8>(src + t * in_stride, x);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float acc = bs[e] + tp[K - 1][e] * x[e];
+#pragma unroll
+      for (int j = 0; j < K - 1; ++j) acc += tp[j][e] * win[j][e];
+      y[e] = silu_f(acc);
+#pragma unroll
+      for (int j = 0; j + 1 < K - 1; ++j) win[j][e] = win[j + 1][e];
+      win[K - 2][e] = x[e];
+    }
+    store_vec<T, 8>(out + (int64_t)(lo + t) * out_stride + c, y);
+  }
+  if (blockIdx.y == 0) {
+    float last[K - 1][8];
+#pragma unroll
+    for (int i = 0; i < K - 1; ++i) input(n - (K - 1) + i, last[i]);
+#pragma unroll
+    for (int i = 0; i < K - 1; ++i) store_vec<float, 8>(keep + (int64_t)i * C, last[i]);
+  }
+}
+
+template <typename T>
+int launch_conv(const T* in, int64_t in_stride, const float* taps, const float* bias, int32_t C, int32_t K, float* state, T* out,
+                int64_t out_stride, const msa_seq_batch& b, hipStream_t st) {
+  const int row_blocks = (b.max_rows + kConvRows - 1) / kConvRows;
+  if (K >= 2 && K <= 5 && vec_ok(8, {in, bias, state, out}, {in_stride, out_stride, C})) {
+    const dim3 grid((C / 8 + 255) / 256, row_blocks, b.n_seq);
+    if (K == 2) conv_silu_vec_kernel<T, 2><<<grid, 256, 0, st>>>(in, in_stride, taps, bias, C, state, out, out_stride, b);
+    else if (K == 3) conv_silu_vec_kernel<T, 3><<<grid, 256, 0, st>>>(in, in_stride, taps, bias, C, state, out, out_stride, b);
+    else if (K == 4) conv_silu_vec_kernel<T, 4><<<grid, 256, 0, st>>>(in, in_stride, taps, bias, C, state, out, out_stride, b);
+    else conv_silu_vec_kernel<T, 5><<<grid, 256, 0, st>>>(in, in_stride, taps, bias, C, state, out, out_stride, b);
+  } else {
+    conv_silu_kernel<T><<<dim3((C + 255) / 256, row_blocks, b.n_seq), 256, 0, st>>>(in, in_stride, taps, bias, C, K, state, out, out_stride, b);
+  }
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+
 // ------------------------------------------------------------------------------------------------ state-space recurrence
-// A workgroup owns (sequence, head, 64 state columns): lane = column p, wavefront w holds the state rows n = w + waves i in
-// registers.  kScanRows tokens are staged at a time: every wavefront adds its share of S^T C into LDS, one barrier, and all
-// threads finish the outputs.
-constexpr int kScanRows = 8;
+// A workgroup owns (sequence, head, 64 state columns): lane = column p, wavefront w holds state rows w NI .. + NI in
+// registers.  A few tokens are staged at a time (B and C in LDS as fp32, read back four to an instruction): every wavefront
+// adds its share of S^T C into LDS, one barrier, and all threads finish the outputs.
 
 struct SsdArgs {
   const void* xbc;
@@ -65,39 +131,46 @@ struct SsdArgs {
 
 template <typename T, int NI, int WAVES>
 __global__ __launch_bounds__(WAVES * 64) void ssd_scan_kernel(SsdArgs a, msa_seq_batch b) {
-  __shared__ float part[WAVES][kScanRows][64];
+  constexpr int kRows = WAVES > 4 ? 2 : 8, kN = NI * WAVES;        // tokens per stage, state rows padded
+  __shared__ float part[WAVES][kRows][64];
+  __shared__ __align__(16) float bc[kRows][2][kN];
+  __shared__ float dts[kRows], decays[kRows];
   const int s = blockIdx.z, head = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int p = blockIdx.x * 64 + lane;
   const bool live = p < a.P;
   const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo;
   const int grp = head / (a.H / a.G), inner = a.H * a.P;
-  float* st = a.state + (((int64_t)b.slot[s] * a.H + head) * a.N) * a.P + p;
+  float* st = a.state + (((int64_t)b.slot[s] * a.H + head) * a.N + wave * NI) * a.P + p;
   float S[NI];
 #pragma unroll
-  for (int i = 0; i < NI; ++i) {
-    const int n = wave + WAVES * i;
-    S[i] = live && n < a.N ? st[(int64_t)n * a.P] : 0.f;
-  }
+  for (int i = 0; i < NI; ++i) S[i] = live && wave * NI + i < a.N ? st[(int64_t)i * a.P] : 0.f;
   const float rate = -expf(a.A_log[head]), bias = a.dt_bias[head], Dh = a.D[head];
   const T* xbc = static_cast<const T*>(a.xbc) + (int64_t)lo * a.xbc_stride;
   const T* dtp = static_cast<const T*>(a.dt_raw) + (int64_t)lo * a.dt_stride + head;
-  for (int t0 = 0; t0 < n_tok; t0 += kScanRows) {
-    const int rows = min(kScanRows, n_tok - t0);
+  for (int t0 = 0; t0 < n_tok; t0 += kRows) {
+    const int rows = min(kRows, n_tok - t0);
+    for (int i = threadIdx.x; i < rows * 2 * kN; i += WAVES * 64) {
+      const int r = i / (2 * kN), which = i / kN & 1, n = i % kN;
+      bc[r][which][n] = n < a.N ? to_f32<T>(xbc[(int64_t)(t0 + r) * a.xbc_stride + inner + (which * a.G + grp) * a.N + n]) : 0.f;
+    }
+    if (threadIdx.x < rows) {
+      const float dt = softplus_f(to_f32<T>(dtp[(int64_t)(t0 + threadIdx.x) * a.dt_stride]) + bias);
+      dts[threadIdx.x] = dt;
+      decays[threadIdx.x] = expf(rate * dt);
+    }
+    __syncthreads();
     for (int r = 0; r < rows; ++r) {
-      const T* row = xbc + (int64_t)(t0 + r) * a.xbc_stride;
-      const float dt = softplus_f(to_f32<T>(dtp[(int64_t)(t0 + r) * a.dt_stride]) + bias);
-      const float decay = expf(rate * dt);
-      const float x = live ? dt * to_f32<T>(row[head * a.P + p]) : 0.f;
-      const T* Bt = row + inner + grp * a.N;
-      const T* Ct = Bt + a.G * a.N;
+      const float decay = decays[r];
+      const float x = live ? dts[r] * to_f32<T>(xbc[(int64_t)(t0 + r) * a.xbc_stride + head * a.P + p]) : 0.f;
       float y = 0.f;
 #pragma unroll
-      for (int i = 0; i < NI; ++i) {
-        const int n = wave + WAVES * i;
-        if (n < a.N) {
-          S[i] = decay * S[i] + to_f32<T>(Bt[n]) * x;
-          y += S[i] * to_f32<T>(Ct[n]);
-        }
+      for (int i = 0; i < NI; i += 4) {
+        const float4 Bv = *reinterpret_cast<const float4*>(&bc[r][0][wave * NI + i]);
+        const float4 Cv = *reinterpret_cast<const float4*>(&bc[r][1][wave * NI + i]);
+        S[i] = decay * S[i] + Bv.x * x; y += S[i] * Cv.x;
+        S[i + 1] = decay * S[i + 1] + Bv.y * x; y += S[i + 1] * Cv.y;
+        S[i + 2] = decay * S[i + 2] + Bv.z * x; y += S[i + 2] * Cv.z;
+        S[i + 3] = decay * S[i + 3] + Bv.w * x; y += S[i + 3] * Cv.w;
       }
       part[wave][r][lane] = y;
     }
@@ -113,13 +186,10 @@ __global__ __launch_bounds__(WAVES * 64) void ssd_scan_kernel(SsdArgs a, msa_seq
         static_cast<T*>(a.v)[row * inner + head * a.P + p] = from_f32<T>(y);
       }
     }
-    __syncthreads();
   }
 #pragma unroll
-  for (int i = 0; i < NI; ++i) {
-    const int n = wave + WAVES * i;
-    if (live && n < a.N) st[(int64_t)n * a.P] = S[i];
-  }
+  for (int i = 0; i < NI; ++i)
+    if (live && wave * NI + i < a.N) st[(int64_t)i * a.P] = S[i];
 }
 
 // ------------------------------------------------------------------------------------------------ minimal gated recurrence
@@ -141,32 +211,57 @@ struct GruArgs {
   int32_t n, n_chunks;
 };
 
-template <typename T>
-__device__ __forceinline__ void gru_terms(const T* row, int c, float zb, float ub, float& keep, float& add) {
-  const float z = sigmoid_f(to_f32<T>(row[c]) + zb);
-  const float u = to_f32<T>(row[c + kGruGroup]) + ub;
+// The raw columns of a few rows, all loads issued before the first is needed (rows behind the portion repeat the last one).
+constexpr int kGruBatch = 8;
+template <typename T, int VEC, int COLS>
+struct GruRows {
+  float v[kGruBatch][COLS][VEC];
+  __device__ __forceinline__ void load(const T* row, int64_t stride, int left) {
+#pragma unroll
+    for (int r = 0; r < kGruBatch; ++r) {
+      const T* at = row + min(r, left - 1) * stride;
+#pragma unroll
+      for (int k = 0; k < COLS; ++k) load_vec<T, VEC>(at + k * kGruGroup, v[r][k]);
+    }
+  }
+};
+// keep = 1 - z and add = z * candidate.
+__device__ __forceinline__ void gru_terms(float z_raw, float u_raw, float zb, float ub, float& keep, float& add) {
+  const float z = sigmoid_f(z_raw + zb), u = u_raw + ub;
   keep = 1.0f - z;
   add = z * (u >= 0.f ? u + 0.5f : sigmoid_f(u));
 }
 
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void gru_chunk_kernel(GruArgs a, msa_seq_batch b) {
-  const int c = blockIdx.x * 256 + threadIdx.x, s = blockIdx.z;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * VEC, s = blockIdx.z;
   const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo, t0 = blockIdx.y * kGruRows;
   if (c >= a.n || t0 >= n_tok) return;
-  const int t1 = min(n_tok, t0 + kGruRows);
-  const float zb = a.z_bias[c], ub = a.u_bias[c];
-  const int at = gru_column(c);
-  float A = 1.f, S = 0.f;
-  const T* row = static_cast<const T*>(a.zug) + (int64_t)(lo + t0) * a.stride;
-#pragma unroll 4
-  for (int t = t0; t < t1; ++t, row += a.stride) {
-    float k, d;
-    gru_terms<T>(row, at, zb, ub, k, d);
-    A *= k;
-    S = k * S + d;
+  const int n = min(n_tok - t0, kGruRows);
+  float zb[VEC], ub[VEC], A[VEC], S[VEC];
+  load_vec<float, VEC>(a.z_bias + c, zb);
+  load_vec<float, VEC>(a.u_bias + c, ub);
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) A[e] = 1.f, S[e] = 0.f;
+  const T* row = static_cast<const T*>(a.zug) + (int64_t)(lo + t0) * a.stride + gru_column(c);
+  for (int t = 0; t < n; t += kGruBatch, row += kGruBatch * a.stride) {
+    GruRows<T, VEC, 2> in;
+    in.load(row, a.stride, n - t);
+#pragma unroll
+    for (int r = 0; r < kGruBatch; ++r) {
+      if (t + r >= n) break;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        float k, d;
+        gru_terms(in.v[r][0][e], in.v[r][1][e], zb[e], ub[e], k, d);
+        A[e] *= k;
+        S[e] = k * S[e] + d;
+      }
+    }
   }
-  a.chunk[((int64_t)s * a.n_chunks + blockIdx.y) * a.n + c] = make_float2(A, S);
+  float2* dst = a.chunk + ((int64_t)s * a.n_chunks + blockIdx.y) * a.n + c;
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) dst[e] = make_float2(A[e], S[e]);
 }
 
 __global__ __launch_bounds__(64) void gru_carry_kernel(GruArgs a, msa_seq_batch b) {
@@ -184,39 +279,53 @@ __global__ __launch_bounds__(64) void gru_carry_kernel(GruArgs a, msa_seq_batch 
   a.state[(int64_t)b.slot[s] * a.n + c] = S;
 }
 
-template <typename T, bool kCarried>
+template <typename T, int VEC, bool kCarried>
 __global__ __launch_bounds__(256) void gru_out_kernel(GruArgs a, msa_seq_batch b) {
-  const int c = blockIdx.x * 256 + threadIdx.x, s = blockIdx.z;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * VEC, s = blockIdx.z;
   const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo, t0 = blockIdx.y * kGruRows;
   if (c >= a.n || t0 >= n_tok) return;
-  const int t1 = min(n_tok, t0 + kGruRows);
-  const float zb = a.z_bias[c], ub = a.u_bias[c];
-  const int at = gru_column(c);
+  const int n = min(n_tok - t0, kGruRows);
+  float zb[VEC], ub[VEC], S[VEC];
+  load_vec<float, VEC>(a.z_bias + c, zb);
+  load_vec<float, VEC>(a.u_bias + c, ub);
   float* st = a.state + (int64_t)b.slot[s] * a.n + c;
-  float S = kCarried ? a.chunk[((int64_t)s * a.n_chunks + blockIdx.y) * a.n + c].x : *st;
-  const T* row = static_cast<const T*>(a.zug) + (int64_t)(lo + t0) * a.stride;
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) S[e] = kCarried ? a.chunk[((int64_t)s * a.n_chunks + blockIdx.y) * a.n + c + e].x : st[e];
+  const T* row = static_cast<const T*>(a.zug) + (int64_t)(lo + t0) * a.stride + gru_column(c);
   T* out = static_cast<T*>(a.out) + (int64_t)(lo + t0) * a.n + c;
-#pragma unroll 4
-  for (int t = t0; t < t1; ++t, row += a.stride, out += a.n) {
-    float k, d;
-    gru_terms<T>(row, at, zb, ub, k, d);
-    S = k * S + d;
-    *out = from_f32<T>(S * silu_f(to_f32<T>(row[at + 2 * kGruGroup])));
+  for (int t = 0; t < n; t += kGruBatch, row += kGruBatch * a.stride) {
+    GruRows<T, VEC, 3> in;
+    in.load(row, a.stride, n - t);
+#pragma unroll
+    for (int r = 0; r < kGruBatch; ++r) {
+      if (t + r >= n) break;
+      float y[VEC];
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        float k, d;
+        gru_terms(in.v[r][0][e], in.v[r][1][e], zb[e], ub[e], k, d);
+        S[e] = k * S[e] + d;
+        y[e] = S[e] * silu_f(in.v[r][2][e]);
+      }
+      store_vec<T, VEC>(out + (int64_t)(t + r) * a.n, y);
+    }
   }
-  if (!kCarried) *st = S;
+  if (!kCarried)
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) st[e] = S[e];
 }
 
-template <typename T>
+template <typename T, int VEC>
 int launch_gru(const GruArgs& a, const msa_seq_batch& b, hipStream_t st) {
-  const dim3 grid((a.n + 255) / 256, a.n_chunks, b.n_seq);
+  const dim3 grid((a.n / VEC + 255) / 256, a.n_chunks, b.n_seq);
   if (a.n_chunks > 1) {
-    gru_chunk_kernel<T><<<grid, 256, 0, st>>>(a, b);
+    gru_chunk_kernel<T, VEC><<<grid, 256, 0, st>>>(a, b);
     MSA_LAUNCH_CHECK();
     gru_carry_kernel<<<dim3((a.n + 63) / 64, b.n_seq), 64, 0, st>>>(a, b);
     MSA_LAUNCH_CHECK();
-    gru_out_kernel<T, true><<<grid, 256, 0, st>>>(a, b);
+    gru_out_kernel<T, VEC, true><<<grid, 256, 0, st>>>(a, b);
   } else {
-    gru_out_kernel<T, false><<<grid, 256, 0, st>>>(a, b);
+    gru_out_kernel<T, VEC, false><<<grid, 256, 0, st>>>(a, b);
   }
   MSA_LAUNCH_CHECK();
   return MSA_OK;
@@ -244,13 +353,9 @@ extern "C" int msa_seq_conv_silu(const void* in, int64_t in_stride, const float*
   MSA_REQUIRE(in && taps && bias && out && C > 0 && in_stride >= C && out_stride >= C, "msa_seq_conv_silu: bad arguments");
   MSA_REQUIRE(K >= 1 && K - 1 <= kConvRows && (K == 1 || state), "msa_seq_conv_silu: K=%d (1..%d taps)", K, kConvRows + 1);
   MSA_REQUIRE(batch->n_seq <= 65535 && (batch->max_rows + kConvRows - 1) / kConvRows <= 65535, "msa_seq_conv_silu: step too large");
-  const dim3 grid((C + 255) / 256, (batch->max_rows + kConvRows - 1) / kConvRows, batch->n_seq);
   if (dtype == MSA_BF16)
-    conv_silu_kernel<bf16_t><<<grid, 256, 0, as_stream(stream)>>>((const bf16_t*)in, in_stride, taps, bias, C, K, state, (bf16_t*)out, out_stride, *batch);
-  else
-    conv_silu_kernel<float><<<grid, 256, 0, as_stream(stream)>>>((const float*)in, in_stride, taps, bias, C, K, state, (float*)out, out_stride, *batch);
-  MSA_LAUNCH_CHECK();
-  return MSA_OK;
+    return launch_conv<bf16_t>((const bf16_t*)in, in_stride, taps, bias, C, K, state, (bf16_t*)out, out_stride, *batch, as_stream(stream));
+  return launch_conv<float>((const float*)in, in_stride, taps, bias, C, K, state, (float*)out, out_stride, *batch, as_stream(stream));
 }
 
 extern "C" int msa_seq_ssd_scan(const void* xbc, int64_t xbc_stride, const void* z, int64_t z_stride, const void* dt_raw,
@@ -285,5 +390,8 @@ extern "C" int msa_seq_min_gru(const void* zug, int64_t zug_stride, const float*
   const int chunks = (batch->max_rows + kGruRows - 1) / kGruRows;
   MSA_REQUIRE(chunks <= 65535 && batch->n_seq <= 65535, "msa_seq_min_gru: step too large");
   const GruArgs a{zug, z_bias, u_bias, state, out, static_cast<float2*>(workspace), zug_stride, n, chunks};
-  return dtype == MSA_BF16 ? launch_gru<bf16_t>(a, *batch, as_stream(stream)) : launch_gru<float>(a, *batch, as_stream(stream));
+  hipStream_t st = as_stream(stream);
+  const bool vec = vec_ok(2, {zug, z_bias, u_bias, out}, {zug_stride, n});
+  if (dtype == MSA_BF16) return vec ? launch_gru<bf16_t, 2>(a, *batch, st) : launch_gru<bf16_t, 1>(a, *batch, st);
+  return vec ? launch_gru<float, 2>(a, *batch, st) : launch_gru<float, 1>(a, *batch, st);
 }

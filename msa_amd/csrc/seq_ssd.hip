@@ -85,17 +85,29 @@ __device__ __forceinline__ void chunk_decays(const ChunkArgs& a, int row0, int r
   }
 }
 
-// `n` columns of the chunk's rows into an LDS tile of `width` columns (zeros behind n and behind the sequence).
-template <int Q>
-__device__ __forceinline__ void stage_rows(const bf16_t* src, int64_t stride, int rows, int n, int width, bf16_t* dst, int dst_stride) {
-  const int units = width / 8;
-  for (int i = threadIdx.x; i < Q * units; i += blockDim.x) {
-    const int r = i / units, u = i % units * 8;
-    uint4 w = make_uint4(0, 0, 0, 0);
-    if (r < rows && u < n) w = *reinterpret_cast<const uint4*>(src + (int64_t)r * stride + u);
-    *reinterpret_cast<uint4*>(dst + r * dst_stride + u) = w;
+// `n` columns of the chunk's rows on their way into an LDS tile of WIDTH columns (zeros behind n and behind the sequence): all
+// loads of a tile are issued before anything waits for one, and several tiles' loads before the first is stored.
+template <int Q, int WIDTH, int THREADS>
+struct RowTile {
+  static constexpr int kUnits = WIDTH / 8, kPieces = Q * kUnits / THREADS;
+  static_assert(Q * kUnits % THREADS == 0, "whole pieces per thread");
+  uint4 w[kPieces];
+  __device__ __forceinline__ void load(const bf16_t* src, int64_t stride, int rows, int n) {
+#pragma unroll
+    for (int k = 0; k < kPieces; ++k) {
+      const int i = threadIdx.x + k * THREADS, r = i / kUnits, u = i % kUnits * 8;
+      w[k] = make_uint4(0, 0, 0, 0);
+      if (r < rows && u < n) w[k] = *reinterpret_cast<const uint4*>(src + (int64_t)r * stride + u);
+    }
   }
-}
+  __device__ __forceinline__ void store(bf16_t* dst, int dst_stride) const {
+#pragma unroll
+    for (int k = 0; k < kPieces; ++k) {
+      const int i = threadIdx.x + k * THREADS;
+      *reinterpret_cast<uint4*>(dst + i / kUnits * dst_stride + i % kUnits * 8) = w[k];
+    }
+  }
+};
 
 template <int Q, int NP>
 __global__ __launch_bounds__(4 * Q) void ssd_local_kernel(ChunkArgs a, msa_seq_batch b) {
@@ -111,11 +123,15 @@ __global__ __launch_bounds__(4 * Q) void ssd_local_kernel(ChunkArgs a, msa_seq_b
   const int rows = min(Q, n_tok - t0), row0 = lo + t0;
   const int grp = head / (a.H / a.G), inner = a.H * a.P;
   const bf16_t* src = a.xbc + (int64_t)row0 * a.xbc_stride;
-  stage_rows<Q>(src + inner + grp * a.N, a.xbc_stride, rows, a.N, NP, Bs, kBS);
-  stage_rows<Q>(src + head * a.P + p0, a.xbc_stride, rows, a.P - p0, kPB, xs, kXS);
+  RowTile<Q, NP, 4 * Q> tb;
+  RowTile<Q, kPB, 4 * Q> tx;
+  tb.load(src + inner + grp * a.N, a.xbc_stride, rows, a.N);
+  tx.load(src + head * a.P + p0, a.xbc_stride, rows, a.P - p0);
   chunk_decays<Q>(a, row0, rows, head, ws, acs);
+  tb.store(Bs, kBS);
+  tx.store(xs, kXS);
   const float a_end = acs[Q - 1];
-  if (threadIdx.x < Q) ws[threadIdx.x] *= exp2f(a_end - acs[threadIdx.x]);
+  if (threadIdx.x < Q) ws[threadIdx.x] *= __builtin_amdgcn_exp2f(a_end - acs[threadIdx.x]);
   __syncthreads();
   const int64_t chunk = ((int64_t)s * a.n_chunks + blockIdx.y) * a.H + head;
   if (threadIdx.x == 0 && p0 == 0) a.chunk_decay[chunk] = a_end;
@@ -171,7 +187,7 @@ __global__ __launch_bounds__(256) void ssd_carry_kernel(ChunkArgs a, msa_seq_bat
   for (int c = 0; c < chunks; ++c) {
     float4* at = reinterpret_cast<float4*>(a.chunk_state + (first + (int64_t)c * a.H) * per + i);
     const float4 loc = *at;
-    const float d = exp2f(a.chunk_decay[first + (int64_t)c * a.H]);
+    const float d = __builtin_amdgcn_exp2f(a.chunk_decay[first + (int64_t)c * a.H]);
     *at = make_float4(pack_split(S.x), pack_split(S.y), pack_split(S.z), pack_split(S.w));
     S = make_float4(d * S.x + loc.x, d * S.y + loc.y, d * S.z + loc.z, d * S.w + loc.w);
   }
@@ -195,21 +211,34 @@ __global__ __launch_bounds__(4 * Q) void ssd_output_kernel(ChunkArgs a, msa_seq_
   const int rows = min(Q, n_tok - t0), row0 = lo + t0;
   const int grp = head / (a.H / a.G), inner = a.H * a.P;
   const bf16_t* src = a.xbc + (int64_t)row0 * a.xbc_stride;
-  stage_rows<Q>(src + inner + grp * a.N, a.xbc_stride, rows, a.N, NP, Bs, kBS);
-  stage_rows<Q>(src + inner + (a.G + grp) * a.N, a.xbc_stride, rows, a.N, NP, Cs, kBS);
-  stage_rows<Q>(src + head * a.P + p0, a.xbc_stride, rows, a.P - p0, kPB, xs, kXS);
+  RowTile<Q, NP, 4 * Q> tileB, tileC;
+  RowTile<Q, kPB, 4 * Q> tileX;
+  tileB.load(src + inner + grp * a.N, a.xbc_stride, rows, a.N);
+  tileC.load(src + inner + (a.G + grp) * a.N, a.xbc_stride, rows, a.N);
+  tileX.load(src + head * a.P + p0, a.xbc_stride, rows, a.P - p0);
   const int64_t chunk = ((int64_t)s * a.n_chunks + blockIdx.y) * a.H + head;
+  constexpr int kSPieces = NP * (kPB / 4) / (4 * Q);
+  uint4 sw[kSPieces];
   {
     const uint32_t* packed = reinterpret_cast<const uint32_t*>(a.chunk_state + chunk * a.N * a.P) + p0;
-    for (int i = threadIdx.x; i < NP * (kPB / 4); i += blockDim.x) {
-      const int n = i / (kPB / 4), p = i % (kPB / 4) * 4;
-      uint4 w = make_uint4(0, 0, 0, 0);
-      if (n < a.N && p0 + p < a.P) w = *reinterpret_cast<const uint4*>(packed + (int64_t)n * a.P + p);
-      *reinterpret_cast<uint2*>(Sh + n * kXS + p) = make_uint2((w.x & 0xffffu) | (w.y << 16), (w.z & 0xffffu) | (w.w << 16));
-      *reinterpret_cast<uint2*>(Sl + n * kXS + p) = make_uint2((w.x >> 16) | (w.y & 0xffff0000u), (w.z >> 16) | (w.w & 0xffff0000u));
+#pragma unroll
+    for (int k = 0; k < kSPieces; ++k) {
+      const int i = threadIdx.x + k * 4 * Q, n = i / (kPB / 4), p = i % (kPB / 4) * 4;
+      sw[k] = make_uint4(0, 0, 0, 0);
+      if (n < a.N && p0 + p < a.P) sw[k] = *reinterpret_cast<const uint4*>(packed + (int64_t)n * a.P + p);
     }
   }
   chunk_decays<Q>(a, row0, rows, head, dts, acs);
+  tileB.store(Bs, kBS);
+  tileC.store(Cs, kBS);
+  tileX.store(xs, kXS);
+#pragma unroll
+  for (int k = 0; k < kSPieces; ++k) {
+    const int i = threadIdx.x + k * 4 * Q, n = i / (kPB / 4), p = i % (kPB / 4) * 4;
+    const uint4 w = sw[k];
+    *reinterpret_cast<uint2*>(Sh + n * kXS + p) = make_uint2((w.x & 0xffffu) | (w.y << 16), (w.z & 0xffffu) | (w.w << 16));
+    *reinterpret_cast<uint2*>(Sl + n * kXS + p) = make_uint2((w.x >> 16) | (w.y & 0xffff0000u), (w.z >> 16) | (w.w & 0xffff0000u));
+  }
   __syncthreads();
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, half = lane >> 5, l16 = lane & 15, l32 = lane & 31;
   const int tb = wave >> 1, pb = wave % 2 * 32;
@@ -228,7 +257,7 @@ __global__ __launch_bounds__(4 * Q) void ssd_output_kernel(ChunkArgs a, msa_seq_
     acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(read_tr8(Sh + at, 4 * kXS), cf[kk], acc, 0, 0, 0);
     acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(read_tr8(Sl + at, 4 * kXS), cf[kk], acc, 0, 0, 0);
   }
-  const float in = exp2f(a_t);
+  const float in = __builtin_amdgcn_exp2f(a_t);
 #pragma unroll
   for (int e = 0; e < 16; ++e) acc[e] *= in;
   for (int sb = 0; sb <= tb; ++sb) {
@@ -249,7 +278,7 @@ __global__ __launch_bounds__(4 * Q) void ssd_output_kernel(ChunkArgs a, msa_seq_
         const float4 as = *reinterpret_cast<const float4*>(acs + s0), ds = *reinterpret_cast<const float4*>(dts + s0);
         const float av[4] = {as.x, as.y, as.z, as.w}, dv[4] = {ds.x, ds.y, ds.z, ds.w};
 #pragma unroll
-        for (int x = 0; x < 4; ++x) m[4 * q + x] = s0 + x <= t ? g[8 * j + 4 * q + x] * (exp2f(a_t - av[x]) * dv[x]) : 0.f;
+        for (int x = 0; x < 4; ++x) m[4 * q + x] = s0 + x <= t ? g[8 * j + 4 * q + x] * (__builtin_amdgcn_exp2f(a_t - av[x]) * dv[x]) : 0.f;
       }
       bf16x8_t hi, low;
       split8(m, hi, low);
