@@ -110,30 +110,33 @@ struct DecArgs {
   int32_t H, rank, n_split;
 };
 
-// HT tiles of 16 heads, RP: the rank padded to 64, 128, 256 or 512 (zeros in LDS).  Wavefront w scores keys 16 w .. + 16 of a
-// tile and owns the latent columns of tiles w, w + 4, ... of the product with the probabilities.
+// HT (1 or 2) tiles of 16 heads, RP: the rank padded to 64, 128, 256 or 512 (zeros in LDS).  Eight wavefronts: wavefront w
+// scores keys 16 (w % 4) .. + 16 of a tile for head tile w / 4, whose queries it holds in registers, and owns the latent columns
+// of 16-column tiles w, w + 8, ... of the product with the probabilities.
+constexpr int kDecWaves = 8, kDecThreads = kDecWaves * 64;
 template <int HT, int RP>
-__global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_batch b) {
-  constexpr int kHeads = 16 * HT, kPStride = kDecKeys + 8, kPer = 256 / kHeads;   // threads per head in the softmax
+__global__ __launch_bounds__(kDecThreads) void latent_decode_kernel(DecArgs a, msa_seq_batch b) {
+  constexpr int kHeads = 16 * HT, kPStride = kDecKeys + 8, kPer = kDecThreads / kHeads;   // threads per head in the softmax
   constexpr int kSStride = kDecKeys + 4, stride = RP + 8;
-  constexpr int kCT = RP / 16 / 4, units = RP / 8;               // 16-byte pieces of a row, zero behind the rank
+  constexpr int kCT = (RP / 16 + kDecWaves - 1) / kDecWaves, units = RP / 8;     // 16-byte pieces of a row, zero behind the rank
   extern __shared__ __align__(16) char lds[];
   bf16_t* cs = reinterpret_cast<bf16_t*>(lds);                   // [64][stride]
-  bf16_t* qs = cs + kDecKeys * stride;                           // [kHeads][stride]
-  bf16_t* ps = qs + kHeads * stride;                             // [kHeads][kPStride]
+  bf16_t* ps = cs + kDecKeys * stride;                           // [kHeads][kPStride]
   float* ss = reinterpret_cast<float*>(ps + kHeads * kPStride);  // [kHeads][kSStride]
   float* al = ss + kHeads * kSStride;                            // [kHeads]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
   const int split = blockIdx.x, h0 = blockIdx.y * kHeads, row = blockIdx.z;
+  const int kt = wave & 3, ht = wave >> 2;                       // score tile of this wavefront (ht < HT)
   const int s = b.row_seq[row];
   const int n_keys = (int)(b.pos[s] + (row - b.cu[s]) + 1);
   const int tiles = (n_keys + kDecKeys - 1) / kDecKeys, per = (tiles + a.n_split - 1) / a.n_split;
   const int first = split * per * kDecKeys, last = min(n_keys, first + per * kDecKeys);
   const bf16_t* c = a.cache + (int64_t)b.slot[s] * a.Lcap * a.rank;
 
-  // a thread's pieces: column u of rows r0, r0 + 256 / units, ...
+  // a thread's pieces: column u of rows r0, r0 + kStep, ...
   const int u = tid % units * 8, r0 = tid / units;
-  constexpr int kStep = 256 / units, kPieces = kDecKeys / kStep, kQPieces = (kHeads + kStep - 1) / kStep;
+  constexpr int kStep = kDecThreads / units, kPieces = (kDecKeys + kStep - 1) / kStep;
+  static_assert(kPieces * kStep == kDecKeys, "whole pieces per thread");
   uint4 next[kPieces];
   auto fetch = [&](int k0) {
     const bf16_t* at = c + (int64_t)(k0 + r0) * a.rank + u;
@@ -148,17 +151,15 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_b
     for (int i = 0; i < kPieces; ++i) *reinterpret_cast<uint4*>(cs + (r0 + kStep * i) * stride + u) = next[i];
   };
   if (first < last) fetch(first);
+  bf16x8_t qf[RP / 32];
   {
-    uint4 qw[kQPieces];
+    const int h = h0 + ht * 16 + l16;
+    const bf16_t* at = a.q + ((int64_t)row * a.H + h) * a.rank + 8 * g;
 #pragma unroll
-    for (int i = 0; i < kQPieces; ++i) {
-      const int h = h0 + r0 + kStep * i;
-      qw[i] = make_uint4(0, 0, 0, 0);
-      if (h < a.H && u < a.rank) qw[i] = *reinterpret_cast<const uint4*>(a.q + ((int64_t)row * a.H + h) * a.rank + u);
+    for (int kk = 0; kk < RP / 32; ++kk) {
+      const bool in = ht < HT && h < a.H && 32 * kk + 8 * g < a.rank;
+      qf[kk] = __builtin_bit_cast(bf16x8_t, in ? *reinterpret_cast<const uint4*>(at + 32 * kk) : make_uint4(0, 0, 0, 0));
     }
-#pragma unroll
-    for (int i = 0; i < kQPieces; ++i)
-      if (kHeads >= kStep || r0 < kHeads) *reinterpret_cast<uint4*>(qs + (r0 + kStep * i) * stride + u) = qw[i];
   }
   floatx4_t o[HT][kCT];
 #pragma unroll
@@ -171,22 +172,15 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_b
     stash();
     __syncthreads();
     if (k0 + kDecKeys < last) fetch(k0 + kDecKeys);
-    floatx4_t sc[HT];
+    if (ht < HT) {
+      floatx4_t sc = floatx4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int h = 0; h < HT; ++h) sc[h] = floatx4_t{0.f, 0.f, 0.f, 0.f};
+      for (int kk = 0; kk < RP / 32; ++kk)
+        sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            qf[kk], *reinterpret_cast<const bf16x8_t*>(cs + (kt * 16 + l16) * stride + 32 * kk + 8 * g), sc, 0, 0, 0);
 #pragma unroll
-    for (int kk = 0; kk < RP; kk += 32) {
-      const bf16x8_t kb = *reinterpret_cast<const bf16x8_t*>(cs + (wave * 16 + l16) * stride + kk + 8 * g);
-#pragma unroll
-      for (int h = 0; h < HT; ++h) {
-        const bf16x8_t qa = *reinterpret_cast<const bf16x8_t*>(qs + (h * 16 + l16) * stride + kk + 8 * g);
-        sc[h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qa, kb, sc[h], 0, 0, 0);
-      }
+      for (int e = 0; e < 4; ++e) ss[(ht * 16 + 4 * g + e) * kSStride + kt * 16 + l16] = sc[e] * a.scale_log2e;
     }
-#pragma unroll
-    for (int h = 0; h < HT; ++h)
-#pragma unroll
-      for (int e = 0; e < 4; ++e) ss[(h * 16 + 4 * g + e) * kSStride + wave * 16 + l16] = sc[h][e] * a.scale_log2e;
     __syncthreads();
     {
       constexpr int kEach = kDecKeys / kPer;                     // keys per thread
@@ -232,20 +226,21 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(DecArgs a, msa_seq_b
       for (int h = 0; h < HT; ++h) pa[h] = *reinterpret_cast<const bf16x8_t*>(ps + (h * 16 + l16) * kPStride + kk + 8 * g);
 #pragma unroll
       for (int t = 0; t < kCT; ++t) {
-        const bf16_t* at = cs + (kk + 8 * g + (l16 >> 2)) * stride + (wave + 4 * t) * 16 + (l16 & 3) * 4;
+        if (wave + kDecWaves * t >= RP / 16) break;
+        const bf16_t* at = cs + (kk + 8 * g + (l16 >> 2)) * stride + (wave + kDecWaves * t) * 16 + (l16 & 3) * 4;
         const bf16x8_t vb = join8(lds_read_tr16(at), lds_read_tr16(at + 4 * stride));
 #pragma unroll
         for (int h = 0; h < HT; ++h) o[h][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[h], vb, o[h][t], 0, 0, 0);
       }
     }
   }
-  // o[h][t][e] belongs to head 16 h + 4 g + e, latent column 16 (wave + 4 t) + l16
+  // o[h][t][e] belongs to head 16 h + 4 g + e, latent column 16 (wave + 8 t) + l16
   const int64_t at = ((int64_t)row * a.n_split + split) * a.H;
 #pragma unroll
   for (int h = 0; h < HT; ++h)
 #pragma unroll
     for (int t = 0; t < kCT; ++t) {
-      const int col = (wave + 4 * t) * 16 + l16;
+      const int col = (wave + kDecWaves * t) * 16 + l16;
       if (col >= a.rank) continue;
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
@@ -484,11 +479,11 @@ int launch_flash(const FlashArgs& a, const msa_seq_batch& b, hipStream_t st) {
 template <int HT, int RP>
 int launch_decode(const DecArgs& a, const msa_seq_batch& b, hipStream_t st) {
   constexpr int stride = RP + 8, heads = 16 * HT;
-  constexpr int lds = (kDecKeys + heads) * stride * 2 + heads * (kDecKeys + 8) * 2 + heads * (kDecKeys + 4) * 4 + heads * 4;
+  constexpr int lds = kDecKeys * stride * 2 + heads * (kDecKeys + 8) * 2 + heads * (kDecKeys + 4) * 4 + heads * 4;
   static_assert(lds <= 160 * 1024, "tiles must fit LDS");
   static std::atomic<int> raised{0};
   MSA_HIP(raise_dynamic_lds_limit(raised, reinterpret_cast<const void*>(latent_decode_kernel<HT, RP>), lds));
-  latent_decode_kernel<HT, RP><<<dim3(a.n_split, (a.H + heads - 1) / heads, b.rows), 256, lds, st>>>(a, b);
+  latent_decode_kernel<HT, RP><<<dim3(a.n_split, (a.H + heads - 1) / heads, b.rows), kDecThreads, lds, st>>>(a, b);
   MSA_LAUNCH_CHECK();
   return MSA_OK;
 }

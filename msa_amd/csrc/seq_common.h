@@ -31,9 +31,8 @@ __device__ __forceinline__ float tanh_f(float x) {
   const float small = x * (1.0f + s * (-0.33333333f + s * (0.13333333f + s * (-0.053968254f + s * 0.021869488f))));
   return fabsf(x) < 0.15f ? small : big;
 }
-__device__ __forceinline__ float gelu_tanh_f(float z) {
-  return 0.5f * z * (1.0f + tanh_f(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-}
+// z (1 + tanh(y)) / 2 = z / (1 + exp(-2 y)), y = sqrt(2 / pi) (z + 0.044715 z^3)
+__device__ __forceinline__ float gelu_tanh_f(float z) { return z * sigmoid_f(1.5957691216057308f * (z + 0.044715f * z * z * z)); }
 
 // VEC consecutive elements of a row (aligned to their size, at most 16 bytes), as fp32.
 template <typename T, int VEC>

@@ -5,6 +5,7 @@
 // and are added in wavefront order.  Everything behind the sums is element-wise in this model (dynamic tanh has no row
 // statistics), so a layer's chain of launches is one per weight matrix plus the state-space / attention step.
 #include <algorithm>
+#include <type_traits>
 
 #include "seq_common.h"
 
@@ -20,6 +21,51 @@ constexpr int kGruGroup = 16;
 // Units of 32 J elements of K (J 16-byte vectors per lane): shorter when three row groups share the registers.
 template <int R>
 constexpr int kVectors = R == 3 ? 2 : 4;
+
+// The element-wise end of product (m, n), `col` its column in the output.
+template <int EPI>
+__device__ __forceinline__ void finish(const msa_rows_args& a, int m, int n, int64_t col, float v) {
+  bf16_t* out16 = static_cast<bf16_t*>(a.out);
+  if constexpr (EPI == MSA_ROWS_PLAIN || EPI == MSA_ROWS_GRU) {
+    if (EPI == MSA_ROWS_PLAIN && n < a.gelu_n) v = gelu_tanh_f(v);
+    out16[m * a.out_stride + col] = f32_to_bf16(v);
+  } else if constexpr (EPI == MSA_ROWS_F32) {
+    if (a.cap > 0.f) v = a.cap * tanh_f(v / a.cap);
+    if (a.add) v += a.add[col];
+    static_cast<float*>(a.out)[m * a.out_stride + col] = v;
+  } else if constexpr (EPI == MSA_ROWS_MAMBA) {
+    const int c = n - a.conv_lo;
+    if (c >= 0 && c < a.conv_n) {
+      float* keep = a.conv_state + (int64_t)a.slot[m] * (a.conv_k - 1) * a.conv_n + c;
+      const float* tp = a.taps + (int64_t)c * a.conv_k;
+      float y = a.conv_bias[c];
+      for (int j = 0; j + 1 < a.conv_k; ++j) {
+        const float old = keep[(int64_t)j * a.conv_n];
+        y += tp[j] * old;
+        if (j > 0) keep[(int64_t)(j - 1) * a.conv_n] = old;
+      }
+      y += tp[a.conv_k - 1] * v;
+      if (a.conv_k > 1) keep[(int64_t)(a.conv_k - 2) * a.conv_n] = v;
+      v = silu_f(y);
+    }
+    out16[m * a.out_stride + col] = f32_to_bf16(v);
+  } else {
+    const int64_t at = (int64_t)m * a.N + n;
+    const float gate = bf16_to_f32(static_cast<const bf16_t*>(a.gate)[m * a.gate_stride + n]) + a.gate_bias[n];
+    const float x = a.x_in[at] + sigmoid_f(gate) * v;
+    a.x_out[at] = x;
+    if (a.norm.w) {
+      const float h = tanh_f(a.norm.alpha * x) * a.norm.w[n] + a.norm.b[n];
+      if (a.h) static_cast<bf16_t*>(a.h)[at] = f32_to_bf16(h);
+      if (a.shift) {
+        float* prev = a.prev + (int64_t)a.slot[m] * a.N + n;
+        const float before = *prev;
+        *prev = h;
+        static_cast<bf16_t*>(a.h_shift)[at] = f32_to_bf16(h + (before - h) * a.shift[n]);
+      }
+    }
+  }
+}
 
 template <int EPI, int R>
 __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_args a, int32_t rows_per_wg) {
@@ -88,8 +134,6 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_ar
   };
   auto row_of = [](int i) { return 4 * (i >> 6) + (i & 3); };
   auto col_of = [](int i) { return (i >> 2) & 15; };
-  bf16_t* out16 = static_cast<bf16_t*>(a.out);
-
   if constexpr (EPI == MSA_ROWS_GRU) {
     if (!second) {
       for (int i = tid; i < 256; i += blockDim.x) {
@@ -108,48 +152,114 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_ar
     const int r = o >> 8, i = o & 255;
     const int m = row_of(i), nr = 16 * r + col_of(i), n = n_base + nr;
     if (m >= a.M || nr >= rows_w) continue;
-    float v = total(r, i);
-    const int64_t col = (int64_t)grp * a.N + n;
-    if constexpr (EPI == MSA_ROWS_PLAIN || EPI == MSA_ROWS_GRU) {
-      if (EPI == MSA_ROWS_PLAIN && n < a.gelu_n) v = gelu_tanh_f(v);
-      out16[m * a.out_stride + col] = f32_to_bf16(v);
-    } else if constexpr (EPI == MSA_ROWS_F32) {
-      if (a.cap > 0.f) v = a.cap * tanh_f(v / a.cap);
-      if (a.add) v += a.add[col];
-      static_cast<float*>(a.out)[m * a.out_stride + col] = v;
-    } else if constexpr (EPI == MSA_ROWS_MAMBA) {
-      const int c = n - a.conv_lo;
-      if (c >= 0 && c < a.conv_n) {
-        float* keep = a.conv_state + (int64_t)a.slot[m] * (a.conv_k - 1) * a.conv_n + c;
-        const float* tp = a.taps + (int64_t)c * a.conv_k;
-        float y = a.conv_bias[c];
-        for (int j = 0; j + 1 < a.conv_k; ++j) {
-          const float old = keep[(int64_t)j * a.conv_n];
-          y += tp[j] * old;
-          if (j > 0) keep[(int64_t)(j - 1) * a.conv_n] = old;
-        }
-        y += tp[a.conv_k - 1] * v;
-        if (a.conv_k > 1) keep[(int64_t)(a.conv_k - 2) * a.conv_n] = v;
-        v = silu_f(y);
-      }
-      out16[m * a.out_stride + col] = f32_to_bf16(v);
-    } else {
-      const int64_t at = (int64_t)m * a.N + n;
-      const float gate = bf16_to_f32(static_cast<const bf16_t*>(a.gate)[m * a.gate_stride + n]) + a.gate_bias[n];
-      const float x = a.x_in[at] + sigmoid_f(gate) * v;
-      a.x_out[at] = x;
-      if (a.norm.w) {
-        const float h = tanh_f(a.norm.alpha * x) * a.norm.w[n] + a.norm.b[n];
-        if (a.h) static_cast<bf16_t*>(a.h)[at] = f32_to_bf16(h);
-        if (a.shift) {
-          float* prev = a.prev + (int64_t)a.slot[m] * a.N + n;
-          const float before = *prev;
-          *prev = h;
-          static_cast<bf16_t*>(a.h_shift)[at] = f32_to_bf16(h + (before - h) * a.shift[n]);
-        }
-      }
-    }
+    finish<EPI>(a, m, n, (int64_t)grp * a.N + n, total(r, i));
   }
+}
+
+// Streaming form for matrices with many rows per compute unit (input projections, up, the head): a workgroup stays for the
+// whole launch.  Wavefront w owns the K slice [32 F w, 32 F (w + 1)) for every item the workgroup visits and keeps its
+// activations of that slice in registers, so they are read once per workgroup.  An item is up to 16 weight rows (as many as
+// make every workgroup's share equal), its F vectors per lane requested kStages - 1 items ahead; partial sums meet in two LDS
+// buffers behind one barrier per item, four threads add up an output.  A workgroup's items are contiguous, so it changes from
+// the first operand's rows to the second's at most once.
+constexpr int kPartStride = 260;            // floats per wavefront's partial block: the four adders of an output hit distinct banks
+
+template <int EPI, int F>
+__global__ __launch_bounds__(kMaxWaves * 64) void rows_stream_kernel(msa_rows_args a, int32_t rows_per_item, int32_t items_a,
+                                                                     int32_t items, int32_t per_wg) {
+  constexpr int kStages = F <= 5 ? 3 : 2;
+  __shared__ __align__(16) float part[2][kMaxWaves][kPartStride];
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int n_l = lane & 15, g = lane >> 4;
+  const int row_bytes = a.K * 2, slice = wave * (F * 64);
+  constexpr int kFar = 0x7ff00000;
+  const int i0 = blockIdx.x * per_wg, i1 = min(items, i0 + per_wg);
+  int at[F];                                // this lane's byte offsets in a row, or past every extent
+#pragma unroll
+  for (int f = 0; f < F; ++f) at[f] = slice + f * 64 + g * 16 < row_bytes ? slice + f * 64 + g * 16 : kFar;
+  auto base_of = [&](int item) { return item < items_a ? item * rows_per_item : a.n_b + (item - items_a) * rows_per_item; };
+  auto rows_of = [&](int item) {
+    if (item >= i1) return 0;
+    return min(rows_per_item, (item < items_a ? min(a.n_b, a.N) : a.N) - base_of(item));
+  };
+  u32x4_t xf[F];
+  auto load_x = [&](bool second) {
+    const int64_t xs = second ? a.x_b_stride : a.x_stride;
+    const __amdgpu_buffer_rsrc_t rs_x = __builtin_amdgcn_make_buffer_rsrc(
+        const_cast<char*>(static_cast<const char*>(second ? a.x_b : a.x)), 0, (int)((a.M - 1) * xs * 2 + row_bytes), 0x00020000);
+#pragma unroll
+    for (int f = 0; f < F; ++f) xf[f] = __builtin_amdgcn_raw_buffer_load_b128(rs_x, at[f] == kFar ? kFar : n_l * (int)(xs * 2) + at[f], 0, 0);
+  };
+  u32x4_t fw[kStages][F];
+  auto load_w = [&](auto slot_tag, int item) {
+    constexpr int slot = decltype(slot_tag)::value;
+    // an empty extent (behind the last item) reads zeros and touches no memory
+    const int extent = __builtin_amdgcn_readfirstlane(max(0, rows_of(item)) * row_bytes);
+    const int base = __builtin_amdgcn_readfirstlane(item < i1 ? base_of(item) : 0);
+    const __amdgpu_buffer_rsrc_t rs_w = __builtin_amdgcn_make_buffer_rsrc(
+        const_cast<char*>(static_cast<const char*>(a.w)) + (int64_t)base * row_bytes, 0, extent, 0x00020000);
+#pragma unroll
+    for (int f = 0; f < F; ++f)
+      fw[slot][f] = __builtin_amdgcn_raw_buffer_load_b128(rs_w, at[f] == kFar ? kFar : n_l * row_bytes + at[f], 0, 0);
+  };
+  bool second = i0 >= items_a;
+  load_x(second);
+  load_w(std::integral_constant<int, 0>{}, i0);
+  if constexpr (kStages == 3) load_w(std::integral_constant<int, 1>{}, i0 + 1);
+  const int o = tid >> 2, quarter = tid & 3;
+  const int m = 4 * (o >> 6) + (o & 3), nr = (o >> 2) & 15;
+  auto step = [&](int item, auto slot_tag) {
+    constexpr int slot = decltype(slot_tag)::value;
+    load_w(std::integral_constant<int, (slot + kStages - 1) % kStages>{}, item + kStages - 1);
+    if (!second && item >= items_a && item < i1) {
+      second = true;
+      load_x(true);
+    }
+    floatx4_t acc = floatx4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int f = 0; f < F; ++f)
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, xf[f]), __builtin_bit_cast(bf16x8_t, fw[slot][f]), acc, 0, 0, 0);
+    float(*buf)[kPartStride] = part[item & 1];
+    *reinterpret_cast<floatx4_t*>(&buf[wave][lane * 4]) = acc;
+    __syncthreads();
+    float v = (buf[4 * quarter][o] + buf[4 * quarter + 1][o]) + (buf[4 * quarter + 2][o] + buf[4 * quarter + 3][o]);
+    v += __shfl_xor(v, 1);
+    v += __shfl_xor(v, 2);
+    if (quarter == 0 && m < a.M && nr < rows_of(item)) {
+      const int n = base_of(item) + nr;
+      finish<EPI>(a, m, n, n, v);
+    }
+  };
+  for (int item = i0; item < i1; item += kStages) {       // whole rounds: items behind the last read zeros and store nothing
+    step(item, std::integral_constant<int, 0>{});
+    step(item + 1, std::integral_constant<int, 1>{});
+    if constexpr (kStages == 3) step(item + 2, std::integral_constant<int, 2>{});
+  }
+}
+
+template <int EPI, int F>
+int launch_stream(const msa_rows_args& a, hipStream_t st) {
+  const int cus = device_compute_units();
+  const int n_a = std::min(a.n_b, a.N), n_b = a.N - n_a;
+  const int iters = (a.N + 16 * cus - 1) / (16 * cus);
+  int rpi = std::min(16, std::max(1, (a.N + iters * cus - 1) / (iters * cus)));
+  auto split = [&] { return (n_a + rpi - 1) / rpi + (n_b + rpi - 1) / rpi; };   // the second operand's rows start an item of their own
+  while (rpi < 16 && split() > iters * cus) ++rpi;
+  const int items_a = (n_a + rpi - 1) / rpi, items = split();
+  const int per_wg = (items + cus - 1) / cus;
+  rows_stream_kernel<EPI, F><<<(items + per_wg - 1) / per_wg, kMaxWaves * 64, 0, st>>>(a, rpi, items_a, items, per_wg);
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+template <int EPI>
+int launch_stream(const msa_rows_args& a, hipStream_t st) {
+  const int f = (a.K + 511) / 512;
+  if (f <= 2) return launch_stream<EPI, 2>(a, st);
+  if (f <= 3) return launch_stream<EPI, 3>(a, st);
+  if (f <= 4) return launch_stream<EPI, 4>(a, st);
+  if (f <= 5) return launch_stream<EPI, 5>(a, st);
+  return launch_stream<EPI, 8>(a, st);
 }
 
 template <int EPI, int R>
@@ -212,6 +322,12 @@ extern "C" int msa_rows_linear(const msa_rows_args* args, int32_t epilogue, void
   for (int cand = waves; cand >= std::max(1, waves / 2); --cand)
     if (units % cand == 0) { waves = cand; break; }
   hipStream_t st = as_stream(stream);
+  // Many rows per compute unit: the streaming form.
+  if (a.groups == 1 && a.K > 512 && a.K <= 4096 && a.N >= 2 * 16 * device_compute_units()) {
+    if (epilogue == MSA_ROWS_PLAIN) return launch_stream<MSA_ROWS_PLAIN>(a, st);
+    if (epilogue == MSA_ROWS_F32) return launch_stream<MSA_ROWS_F32>(a, st);
+    if (epilogue == MSA_ROWS_MAMBA) return launch_stream<MSA_ROWS_MAMBA>(a, st);
+  }
   switch (epilogue * 4 + R) {
     case MSA_ROWS_PLAIN * 4 + 1: return launch_rows<MSA_ROWS_PLAIN, 1>(a, waves, rows_per_wg, st);
     case MSA_ROWS_PLAIN * 4 + 2: return launch_rows<MSA_ROWS_PLAIN, 2>(a, waves, rows_per_wg, st);

@@ -270,11 +270,17 @@ __global__ __launch_bounds__(64) void gru_carry_kernel(GruArgs a, msa_seq_batch 
   const int n_tok = b.cu[s + 1] - b.cu[s], chunks = (n_tok + kGruRows - 1) / kGruRows;
   float S = a.state[(int64_t)b.slot[s] * a.n + c];
   float2* ch = a.chunk + (int64_t)s * a.n_chunks * a.n + c;
-#pragma unroll 8
-  for (int i = 0; i < chunks; ++i) {
-    const float2 t = ch[(int64_t)i * a.n];
-    ch[(int64_t)i * a.n].x = S;
-    S = t.x * S + t.y;
+  constexpr int kBatch = 16;
+  for (int i = 0; i < chunks; i += kBatch) {
+    float2 t[kBatch];
+#pragma unroll
+    for (int k = 0; k < kBatch; ++k) t[k] = ch[(int64_t)min(i + k, chunks - 1) * a.n];
+#pragma unroll
+    for (int k = 0; k < kBatch; ++k) {
+      if (i + k >= chunks) break;
+      ch[(int64_t)(i + k) * a.n].x = S;
+      S = t[k].x * S + t[k].y;
+    }
   }
   a.state[(int64_t)b.slot[s] * a.n + c] = S;
 }

@@ -183,13 +183,25 @@ __global__ __launch_bounds__(256) void ssd_carry_kernel(ChunkArgs a, msa_seq_bat
   float4* keep = reinterpret_cast<float4*>(a.state + ((int64_t)b.slot[s] * a.H + head) * per + i);
   float4 S = *keep;
   const int64_t first = (int64_t)s * a.n_chunks * a.H + head;
-#pragma unroll 4
-  for (int c = 0; c < chunks; ++c) {
-    float4* at = reinterpret_cast<float4*>(a.chunk_state + (first + (int64_t)c * a.H) * per + i);
-    const float4 loc = *at;
-    const float d = __builtin_amdgcn_exp2f(a.chunk_decay[first + (int64_t)c * a.H]);
-    *at = make_float4(pack_split(S.x), pack_split(S.y), pack_split(S.z), pack_split(S.w));
-    S = make_float4(d * S.x + loc.x, d * S.y + loc.y, d * S.z + loc.z, d * S.w + loc.w);
+  constexpr int kBatch = 8;
+  for (int c = 0; c < chunks; c += kBatch) {
+    float4 loc[kBatch];
+    float d[kBatch];
+    float4* at[kBatch];
+#pragma unroll
+    for (int k = 0; k < kBatch; ++k) {
+      const int64_t chunk = first + (int64_t)min(c + k, chunks - 1) * a.H;
+      at[k] = reinterpret_cast<float4*>(a.chunk_state + chunk * per + i);
+      loc[k] = *at[k];
+      d[k] = a.chunk_decay[chunk];
+    }
+#pragma unroll
+    for (int k = 0; k < kBatch; ++k) {
+      if (c + k >= chunks) break;
+      *at[k] = make_float4(pack_split(S.x), pack_split(S.y), pack_split(S.z), pack_split(S.w));
+      const float f = __builtin_amdgcn_exp2f(d[k]);
+      S = make_float4(f * S.x + loc[k].x, f * S.y + loc[k].y, f * S.z + loc[k].z, f * S.w + loc[k].w);
+    }
   }
   *keep = S;
 }

@@ -343,7 +343,8 @@ def test_flash_far_keys_at_every_edge():
 
 
 # ------------------------------------------------------------------------------------------------ decode products
-@pytest.mark.parametrize("M,N,K", [(1, 16, 8), (16, 37, 136), (3, 200, 72), (7, 2600, 264), (16, 6200, 128), (5, 48, 1000)])
+@pytest.mark.parametrize("M,N,K", [(1, 16, 8), (16, 37, 136), (3, 200, 72), (7, 2600, 264), (16, 6200, 128), (5, 48, 1000), (16, 8200, 520), (3, 9001, 1032),
+                                   (5, 8192, 2560), (2, 8300, 1800), (9, 20000, 4096), (1, 8192, 3000)])
 def test_rows_linear_plain_and_f32(M, N, K):
     r = Rand(M + K)
     (x, x_), (w, w_) = r(M, K, dtype=BF16), r(N, K, dtype=BF16, scale=K ** -0.5)
@@ -356,10 +357,10 @@ def test_rows_linear_plain_and_f32(M, N, K):
     close(seq_ops.rows_linear_f32(x, w, cap=0.8), 0.8 * torch.tanh(want / 0.8), F32)
 
 
-@pytest.mark.parametrize("N_a,N_b", [(32, 40), (64, 6200), (3200, 3000)])
-def test_rows_linear_two_operands(N_a, N_b):
+@pytest.mark.parametrize("N_a,N_b,K", [(32, 40, 80), (64, 6200, 80), (3200, 3000, 80), (8192, 200, 648), (32, 9000, 1160), (6400, 6000, 2568)])
+def test_rows_linear_two_operands(N_a, N_b, K):
     r = Rand(N_a)
-    (x, x_), (y, y_), (w, w_) = r(9, 80, dtype=BF16), r(9, 80, dtype=BF16), r(N_a + N_b, 80, dtype=BF16, scale=0.1)
+    (x, x_), (y, y_), (w, w_) = r(9, K, dtype=BF16), r(9, K, dtype=BF16), r(N_a + N_b, K, dtype=BF16, scale=K ** -0.5)
     got = seq_ops.rows_linear(x, w, x_b=y, n_b=N_a)
     close(got, torch.cat([x_ @ w_[:N_a].T, y_ @ w_[N_a:].T], 1), BF16, 4e-3)
 
@@ -389,11 +390,12 @@ def test_rows_residual(M, N, K):
     close(prev, prev_, F32)
 
 
+@pytest.mark.parametrize("W,rows", [(64, 32), (600, 8200)])
 @pytest.mark.parametrize("K", [1, 2, 5])
-def test_rows_conv_equals_the_block_form(K):
+def test_rows_conv_equals_the_block_form(K, W, rows):
     r = Rand(K)
-    W, lo, C = 64, 40, 56
-    (w, _), (taps, _), (b, _) = r(160, W, dtype=BF16, scale=0.2), r(C, K), r(C)
+    lo, C = 40, 56
+    (w, _), (taps, _), (b, _) = r(128 + rows, W, dtype=BF16, scale=1.6 * W ** -0.5), r(C, K), r(C)
     s1, s2 = torch.zeros(4, K - 1, C, device="cuda"), torch.zeros(4, K - 1, C, device="cuda")
     for step in range(6):
         (x, x_), (y, _) = r(3, W, dtype=BF16), r(3, W, dtype=BF16)
