@@ -22,50 +22,94 @@ constexpr int kGruGroup = 16;
 template <int R>
 constexpr int kVectors = R == 3 ? 2 : 4;
 
-// The element-wise end of product (m, n), `col` its column in the output.
+// The element-wise end of product (m, n), `col` its column in the output.  What it reads besides the product is fetched by
+// `load`, which the kernels call before they multiply, so that it arrives with the weights instead of behind the sums.
 template <int EPI>
-__device__ __forceinline__ void finish(const msa_rows_args& a, int m, int n, int64_t col, float v) {
-  bf16_t* out16 = static_cast<bf16_t*>(a.out);
-  if constexpr (EPI == MSA_ROWS_PLAIN || EPI == MSA_ROWS_GRU) {
-    if (EPI == MSA_ROWS_PLAIN && n < a.gelu_n) v = gelu_tanh_f(v);
-    out16[m * a.out_stride + col] = f32_to_bf16(v);
-  } else if constexpr (EPI == MSA_ROWS_F32) {
-    if (a.cap > 0.f) v = a.cap * tanh_f(v / a.cap);
-    if (a.add) v += a.add[col];
-    static_cast<float*>(a.out)[m * a.out_stride + col] = v;
-  } else if constexpr (EPI == MSA_ROWS_MAMBA) {
-    const int c = n - a.conv_lo;
-    if (c >= 0 && c < a.conv_n) {
-      float* keep = a.conv_state + (int64_t)a.slot[m] * (a.conv_k - 1) * a.conv_n + c;
-      const float* tp = a.taps + (int64_t)c * a.conv_k;
-      float y = a.conv_bias[c];
-      for (int j = 0; j + 1 < a.conv_k; ++j) {
-        const float old = keep[(int64_t)j * a.conv_n];
-        y += tp[j] * old;
-        if (j > 0) keep[(int64_t)(j - 1) * a.conv_n] = old;
-      }
-      y += tp[a.conv_k - 1] * v;
-      if (a.conv_k > 1) keep[(int64_t)(a.conv_k - 2) * a.conv_n] = v;
-      v = silu_f(y);
-    }
-    out16[m * a.out_stride + col] = f32_to_bf16(v);
-  } else {
-    const int64_t at = (int64_t)m * a.N + n;
-    const float gate = bf16_to_f32(static_cast<const bf16_t*>(a.gate)[m * a.gate_stride + n]) + a.gate_bias[n];
-    const float x = a.x_in[at] + sigmoid_f(gate) * v;
-    a.x_out[at] = x;
-    if (a.norm.w) {
-      const float h = tanh_f(a.norm.alpha * x) * a.norm.w[n] + a.norm.b[n];
-      if (a.h) static_cast<bf16_t*>(a.h)[at] = f32_to_bf16(h);
-      if (a.shift) {
-        float* prev = a.prev + (int64_t)a.slot[m] * a.N + n;
-        const float before = *prev;
-        *prev = h;
-        static_cast<bf16_t*>(a.h_shift)[at] = f32_to_bf16(h + (before - h) * a.shift[n]);
-      }
+struct Finish {
+  __device__ __forceinline__ void load(const msa_rows_args& a, int m, int n) {}
+  __device__ __forceinline__ void apply(const msa_rows_args& a, int m, int n, int64_t col, float v) const {
+    if constexpr (EPI == MSA_ROWS_F32) {
+      if (a.cap > 0.f) v = a.cap * tanh_f(v / a.cap);
+      if (a.add) v += a.add[col];
+      static_cast<float*>(a.out)[m * a.out_stride + col] = v;
+    } else {
+      if (EPI == MSA_ROWS_PLAIN && n < a.gelu_n) v = gelu_tanh_f(v);
+      static_cast<bf16_t*>(a.out)[m * a.out_stride + col] = f32_to_bf16(v);
     }
   }
-}
+};
+
+template <>
+struct Finish<MSA_ROWS_MAMBA> {
+  static constexpr int kTaps = 4;            // more taps than this are read when they are needed
+  float keep[kTaps - 1], tap[kTaps], bias;
+  __device__ __forceinline__ void load(const msa_rows_args& a, int m, int n) {
+    const int c = n - a.conv_lo;
+    if (c < 0 || c >= a.conv_n) return;
+    const float* kp = a.conv_state + (int64_t)a.slot[m] * (a.conv_k - 1) * a.conv_n + c;
+    const float* tp = a.taps + (int64_t)c * a.conv_k;
+    bias = a.conv_bias[c];
+#pragma unroll
+    for (int j = 0; j < kTaps; ++j) {
+      if (j + 1 < a.conv_k && j < kTaps - 1) keep[j] = kp[(int64_t)j * a.conv_n];
+      if (j < a.conv_k) tap[j] = tp[j];
+    }
+  }
+  __device__ __forceinline__ void apply(const msa_rows_args& a, int m, int n, int64_t col, float v) const {
+    const int c = n - a.conv_lo;
+    if (c >= 0 && c < a.conv_n) {
+      float* kp = a.conv_state + (int64_t)a.slot[m] * (a.conv_k - 1) * a.conv_n + c;
+      float y = bias;
+      if (a.conv_k <= kTaps) {
+#pragma unroll
+        for (int j = 0; j < kTaps; ++j) {
+          if (j + 1 < a.conv_k && j < kTaps - 1) {
+            y += tap[j] * keep[j];
+            if (j > 0) kp[(int64_t)(j - 1) * a.conv_n] = keep[j];
+          }
+          if (j + 1 == a.conv_k) y += tap[j] * v;
+        }
+      } else {
+        const float* tp = a.taps + (int64_t)c * a.conv_k;
+        for (int j = 0; j + 1 < a.conv_k; ++j) {
+          const float old = kp[(int64_t)j * a.conv_n];
+          y += tp[j] * old;
+          if (j > 0) kp[(int64_t)(j - 1) * a.conv_n] = old;
+        }
+        y += tp[a.conv_k - 1] * v;
+      }
+      if (a.conv_k > 1) kp[(int64_t)(a.conv_k - 2) * a.conv_n] = v;
+      v = silu_f(y);
+    }
+    static_cast<bf16_t*>(a.out)[m * a.out_stride + col] = f32_to_bf16(v);
+  }
+};
+
+template <>
+struct Finish<MSA_ROWS_RESIDUAL> {
+  float x, gate, w, b, mix, before;
+  __device__ __forceinline__ void load(const msa_rows_args& a, int m, int n) {
+    x = a.x_in[(int64_t)m * a.N + n];
+    gate = bf16_to_f32(static_cast<const bf16_t*>(a.gate)[m * a.gate_stride + n]) + a.gate_bias[n];
+    if (!a.norm.w) return;
+    w = a.norm.w[n];
+    b = a.norm.b[n];
+    if (!a.shift) return;
+    mix = a.shift[n];
+    before = a.prev[(int64_t)a.slot[m] * a.N + n];
+  }
+  __device__ __forceinline__ void apply(const msa_rows_args& a, int m, int n, int64_t, float v) const {
+    const int64_t at = (int64_t)m * a.N + n;
+    const float y = x + sigmoid_f(gate) * v;
+    a.x_out[at] = y;
+    if (!a.norm.w) return;
+    const float h = tanh_f(a.norm.alpha * y) * w + b;
+    if (a.h) static_cast<bf16_t*>(a.h)[at] = f32_to_bf16(h);
+    if (!a.shift) return;
+    a.prev[(int64_t)a.slot[m] * a.N + n] = h;
+    static_cast<bf16_t*>(a.h_shift)[at] = f32_to_bf16(h + (before - h) * mix);
+  }
+};
 
 template <int EPI, int R>
 __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_args a, int32_t rows_per_wg) {
@@ -88,6 +132,15 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_ar
   constexpr int kFar = 0x7ff00000;          // past every extent, whatever is added: reads zeros
   const int units = (a.K + kUnit - 1) / kUnit;
   const int u0 = units * wave / waves, u1 = units * (wave + 1) / waves;
+
+  // output i of a row group: lane i / 4, element i % 4 of its accumulator
+  auto row_of = [](int i) { return 4 * (i >> 6) + (i & 3); };
+  auto col_of = [](int i) { return (i >> 2) & 15; };
+  Finish<EPI> fin;                          // of this thread's first output
+  {
+    const int m = row_of(tid & 255), nr = 16 * (tid >> 8) + col_of(tid & 255);
+    if (tid < R * 256 && m < a.M && nr < rows_w) fin.load(a, m, n_base + nr);
+  }
 
   floatx4_t acc[R];
 #pragma unroll
@@ -126,22 +179,20 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_ar
   for (int r = 0; r < R; ++r) *reinterpret_cast<floatx4_t*>(&part[((wave * R + r) * 64 + lane) * 4]) = acc[r];
   __syncthreads();
 
-  // output i of a row group: lane i / 4, element i % 4 of its accumulator
   auto total = [&](int r, int i) {
     float v = 0.f;
     for (int w = 0; w < waves; ++w) v += part[(w * R + r) * 256 + i];
     return v;
   };
-  auto row_of = [](int i) { return 4 * (i >> 6) + (i & 3); };
-  auto col_of = [](int i) { return (i >> 2) & 15; };
   if constexpr (EPI == MSA_ROWS_GRU) {
     if (!second) {
       for (int i = tid; i < 256; i += blockDim.x) {
         const int m = row_of(i), c = n_base / (3 * kGruGroup) * kGruGroup + col_of(i);
         if (m >= a.M || c >= a.gru_n) continue;
-        const float z = sigmoid_f(total(0, i) + a.z_bias[c]), uu = total(1, i) + a.u_bias[c], gt = total(2, i);
         float* st = a.gru_state + (int64_t)a.slot[m] * a.gru_n + c;
-        const float S = (1.0f - z) * *st + z * (uu >= 0.f ? uu + 0.5f : sigmoid_f(uu));
+        const float before = *st, zb = a.z_bias[c], ub = a.u_bias[c];
+        const float z = sigmoid_f(total(0, i) + zb), uu = total(1, i) + ub, gt = total(2, i);
+        const float S = (1.0f - z) * before + z * (uu >= 0.f ? uu + 0.5f : sigmoid_f(uu));
         *st = S;
         static_cast<bf16_t*>(a.out2)[(int64_t)m * a.gru_n + c] = f32_to_bf16(S * silu_f(gt));
       }
@@ -152,7 +203,8 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_ar
     const int r = o >> 8, i = o & 255;
     const int m = row_of(i), nr = 16 * r + col_of(i), n = n_base + nr;
     if (m >= a.M || nr >= rows_w) continue;
-    finish<EPI>(a, m, n, (int64_t)grp * a.N + n, total(r, i));
+    if (o != tid) fin.load(a, m, n);
+    fin.apply(a, m, n, (int64_t)grp * a.N + n, total(r, i));
   }
 }
 
@@ -216,6 +268,10 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_stream_kernel(msa_rows_ar
       second = true;
       load_x(true);
     }
+    const bool mine = quarter == 0 && m < a.M && nr < rows_of(item);
+    const int n = base_of(item) + nr;
+    Finish<EPI> fin;
+    if (mine) fin.load(a, m, n);
     floatx4_t acc = floatx4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int f = 0; f < F; ++f)
@@ -226,10 +282,7 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_stream_kernel(msa_rows_ar
     float v = (buf[4 * quarter][o] + buf[4 * quarter + 1][o]) + (buf[4 * quarter + 2][o] + buf[4 * quarter + 3][o]);
     v += __shfl_xor(v, 1);
     v += __shfl_xor(v, 2);
-    if (quarter == 0 && m < a.M && nr < rows_of(item)) {
-      const int n = base_of(item) + nr;
-      finish<EPI>(a, m, n, n, v);
-    }
+    if (mine) fin.apply(a, m, n, n, v);
   };
   for (int item = i0; item < i1; item += kStages) {       // whole rounds: items behind the last read zeros and store nothing
     step(item, std::integral_constant<int, 0>{});
@@ -258,8 +311,8 @@ int launch_stream(const msa_rows_args& a, hipStream_t st) {
   if (f <= 2) return launch_stream<EPI, 2>(a, st);
   if (f <= 3) return launch_stream<EPI, 3>(a, st);
   if (f <= 4) return launch_stream<EPI, 4>(a, st);
-  if (f <= 5) return launch_stream<EPI, 5>(a, st);
-  return launch_stream<EPI, 8>(a, st);
+  if constexpr (EPI == MSA_ROWS_MAMBA) return launch_stream<EPI, 5>(a, st);    // (its operands would not fit beside eight vectors)
+  else return f <= 5 ? launch_stream<EPI, 5>(a, st) : launch_stream<EPI, 8>(a, st);
 }
 
 template <int EPI, int R>
@@ -326,7 +379,7 @@ extern "C" int msa_rows_linear(const msa_rows_args* args, int32_t epilogue, void
   if (a.groups == 1 && a.K > 512 && a.K <= 4096 && a.N >= 2 * 16 * device_compute_units()) {
     if (epilogue == MSA_ROWS_PLAIN) return launch_stream<MSA_ROWS_PLAIN>(a, st);
     if (epilogue == MSA_ROWS_F32) return launch_stream<MSA_ROWS_F32>(a, st);
-    if (epilogue == MSA_ROWS_MAMBA) return launch_stream<MSA_ROWS_MAMBA>(a, st);
+    if (epilogue == MSA_ROWS_MAMBA && a.K <= 2560) return launch_stream<MSA_ROWS_MAMBA>(a, st);
   }
   switch (epilogue * 4 + R) {
     case MSA_ROWS_PLAIN * 4 + 1: return launch_rows<MSA_ROWS_PLAIN, 1>(a, waves, rows_per_wg, st);

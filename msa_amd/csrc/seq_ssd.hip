@@ -6,6 +6,8 @@
 //   (1) ssd_local_kernel   every chunk's S_loc
 //   (2) ssd_carry_kernel   the chunk-to-chunk recurrence, element by element; leaves each chunk's S_in in its place
 //   (3) ssd_output_kernel  the outputs
+// A workgroup takes one chunk and several heads of one group, whose B, C and B . C^T are the same: those are read / formed once
+// and stay in registers; a head's x and S_in are fetched while the head before is multiplied.
 // Operands that carry decays or states are fp32 values: they enter the bf16 products as a high and a low part (two products
 // with about 16 bits of mantissa), so only x, B and C, which are bf16 to begin with, set the precision.
 //
@@ -57,31 +59,34 @@ struct ChunkArgs {
   float* chunk_state;      // [n_seq, n_chunks, H, N, P]: S_loc (fp32), then S_in as packed (high, low) bf16 pairs
   float* chunk_decay;      // [n_seq, n_chunks, H]: a_end in powers of two
   int64_t xbc_stride, z_stride, dt_stride;
-  int32_t H, P, N, G, n_chunks;
+  int32_t H, P, N, G, n_chunks, heads_per_wg;
 };
 
-// dt and the running log-decay (base 2) of the chunk's tokens into LDS; tokens behind the sequence have dt = 0.
+constexpr int kMaxHeads = 8;             // heads of a group per workgroup
+
+// dt and the running log-decay (base 2) of the chunk's tokens for `heads` heads from `head0` on, [heads][Q] each: a wavefront per
+// head.  Tokens behind the sequence have dt = 0.  The caller synchronises.
 template <int Q>
-__device__ __forceinline__ void chunk_decays(const ChunkArgs& a, int row0, int rows, int head, float* dts, float* acs) {
-  const int tid = threadIdx.x;
-  float dt = 0.f, ac = 0.f;
-  if (tid < Q) {
-    if (tid < rows) dt = softplus_f(bf16_to_f32(a.dt_raw[(int64_t)(row0 + tid) * a.dt_stride + head]) + a.dt_bias[head]);
-    ac = -expf(a.A_log[head]) * dt * kLog2e;
+__device__ __forceinline__ void chunk_decays(const ChunkArgs& a, int row0, int rows, int head0, int heads, float* dts, float* acs) {
+  const int lane = threadIdx.x & 63;
+  for (int hh = threadIdx.x >> 6; hh < heads; hh += blockDim.x >> 6) {
+    const int head = head0 + hh;
+    const float rate = -expf(a.A_log[head]) * kLog2e, bias = a.dt_bias[head];
+    float before = 0.f;
 #pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const float up = __shfl_up(ac, o);
-      if ((tid & 63) >= o) ac += up;
+    for (int t = lane; t < Q; t += 64) {
+      const float dt = t < rows ? softplus_f(bf16_to_f32(a.dt_raw[(int64_t)(row0 + t) * a.dt_stride + head]) + bias) : 0.f;
+      float ac = rate * dt;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const float up = __shfl_up(ac, o);
+        if (lane >= o) ac += up;
+      }
+      ac += before;
+      before = __shfl(ac, 63);
+      dts[hh * Q + t] = dt;
+      acs[hh * Q + t] = ac;
     }
-    dts[tid] = dt;
-    acs[tid] = ac;
-  }
-  __syncthreads();
-  if (Q == 128) {
-    const float first = acs[63];
-    __syncthreads();
-    if (tid >= 64 && tid < 128) acs[tid] = ac + first;
-    __syncthreads();
   }
 }
 
@@ -109,61 +114,100 @@ struct RowTile {
   }
 };
 
+// What a workgroup of kernels (1) and (3) works on.
+struct Unit {
+  int head0, heads, grp, p0, lo, t0, rows, row0;
+  int64_t chunk0;          // chunk index of head0
+};
+template <int Q>
+__device__ __forceinline__ bool unit_of(const ChunkArgs& a, const msa_seq_batch& b, Unit& u) {
+  const int per_group = a.H / a.G, sets = (per_group + a.heads_per_wg - 1) / a.heads_per_wg;
+  const int set = blockIdx.x % sets, rest = blockIdx.x / sets, s = blockIdx.z;
+  u.grp = rest % a.G;
+  u.p0 = rest / a.G * kPB;
+  u.head0 = u.grp * per_group + set * a.heads_per_wg;
+  u.heads = min(a.heads_per_wg, per_group - set * a.heads_per_wg);
+  u.lo = b.cu[s];
+  u.t0 = blockIdx.y * Q;
+  const int n_tok = b.cu[s + 1] - u.lo;
+  u.rows = min(Q, n_tok - u.t0);
+  u.row0 = u.lo + u.t0;
+  u.chunk0 = ((int64_t)s * a.n_chunks + blockIdx.y) * a.H + u.head0;
+  return u.t0 < n_tok;
+}
+
 template <int Q, int NP>
 __global__ __launch_bounds__(4 * Q) void ssd_local_kernel(ChunkArgs a, msa_seq_batch b) {
-  constexpr int kBS = NP + 8, kWaves = Q / 16;
+  constexpr int kBS = NP + 8, kWaves = Q / 16, kTiles = (NP / 32 * 2 + kWaves - 1) / kWaves;
+  constexpr int kBX = Q * kBS > 2 * Q * kXS ? Q * kBS : 2 * Q * kXS;
   extern __shared__ __align__(16) bf16_t sm[];
-  bf16_t* Bs = sm;                                  // [Q][kBS]
-  bf16_t* xs = Bs + Q * kBS;                        // [Q][kXS]
-  float* ws = reinterpret_cast<float*>(xs + Q * kXS);
-  float* acs = ws + Q;
-  const int head = blockIdx.x % a.H, p0 = blockIdx.x / a.H * kPB, s = blockIdx.z;
-  const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo, t0 = blockIdx.y * Q;
-  if (t0 >= n_tok) return;
-  const int rows = min(Q, n_tok - t0), row0 = lo + t0;
-  const int grp = head / (a.H / a.G), inner = a.H * a.P;
-  const bf16_t* src = a.xbc + (int64_t)row0 * a.xbc_stride;
+  bf16_t* Bs = sm;                                  // [Q][kBS], until its fragments are in registers; then
+  bf16_t* xh = sm;                                  // [Q][kXS] high and
+  bf16_t* xl = xh + Q * kXS;                        // [Q][kXS] low parts of the weighted x
+  float* ws = reinterpret_cast<float*>(sm + kBX);   // [heads][Q]
+  float* acs = ws + kMaxHeads * Q;
+  Unit u;
+  if (!unit_of<Q>(a, b, u)) return;
+  const int inner = a.H * a.P;
+  const bf16_t* src = a.xbc + (int64_t)u.row0 * a.xbc_stride;
   RowTile<Q, NP, 4 * Q> tb;
   RowTile<Q, kPB, 4 * Q> tx;
-  tb.load(src + inner + grp * a.N, a.xbc_stride, rows, a.N);
-  tx.load(src + head * a.P + p0, a.xbc_stride, rows, a.P - p0);
-  chunk_decays<Q>(a, row0, rows, head, ws, acs);
+  tb.load(src + inner + u.grp * a.N, a.xbc_stride, u.rows, a.N);
+  tx.load(src + u.head0 * a.P + u.p0, a.xbc_stride, u.rows, a.P - u.p0);
+  chunk_decays<Q>(a, u.row0, u.rows, u.head0, u.heads, ws, acs);
   tb.store(Bs, kBS);
-  tx.store(xs, kXS);
-  const float a_end = acs[Q - 1];
-  if (threadIdx.x < Q) ws[threadIdx.x] *= __builtin_amdgcn_exp2f(a_end - acs[threadIdx.x]);
   __syncthreads();
-  const int64_t chunk = ((int64_t)s * a.n_chunks + blockIdx.y) * a.H + head;
-  if (threadIdx.x == 0 && p0 == 0) a.chunk_decay[chunk] = a_end;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, half = lane >> 5, l16 = lane & 15;
-  float* out = a.chunk_state + chunk * a.N * a.P;
-  for (int tile = wave; tile < NP / 32 * 2; tile += kWaves) {
-    const int n0 = tile / 2 * 32, pb = tile % 2 * 32;
-    if (n0 >= a.N || p0 + pb >= a.P) continue;
-    floatx16_t acc;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), half = lane >> 5, l16 = lane & 15;
+  const int r = 8 * half + (l16 >> 2), c = (lane & 16) + (l16 & 3) * 4;
+  bf16x8_t bf[kTiles][Q / 16];                      // B^T operands of this wavefront's tiles, for every head
 #pragma unroll
-    for (int e = 0; e < 16; ++e) acc[e] = 0.f;
-    const int r = 8 * half + (l16 >> 2), c = (lane & 16) + (l16 & 3) * 4;
+  for (int i = 0; i < kTiles; ++i) {
+    const int n0 = (wave + kWaves * i) / 2 * 32;
+    if (n0 < NP)
 #pragma unroll
-    for (int kk = 0; kk < Q; kk += 16) {
-      const bf16x8_t bf = read_tr8(Bs + (kk + r) * kBS + n0 + c, 4 * kBS);
-      const bf16x8_t xf = read_tr8(xs + (kk + r) * kXS + pb + c, 4 * kXS);
-      const uint4 xw = __builtin_bit_cast(uint4, xf);
-      const float4 w0 = *reinterpret_cast<const float4*>(ws + kk + 8 * half), w1 = *reinterpret_cast<const float4*>(ws + kk + 8 * half + 4);
-      const float sx[8] = {bf16lo(xw.x) * w0.x, bf16hi(xw.x) * w0.y, bf16lo(xw.y) * w0.z, bf16hi(xw.y) * w0.w,
-                           bf16lo(xw.z) * w1.x, bf16hi(xw.z) * w1.y, bf16lo(xw.w) * w1.z, bf16hi(xw.w) * w1.w};
+      for (int kk = 0; kk < Q / 16; ++kk) bf[i][kk] = read_tr8(Bs + (kk * 16 + r) * kBS + n0 + c, 4 * kBS);
+  }
+  for (int i = threadIdx.x; i < u.heads * Q; i += 4 * Q) ws[i] *= __builtin_amdgcn_exp2f(acs[i / Q * Q + Q - 1] - acs[i]);
+  if (threadIdx.x < u.heads && u.p0 == 0) a.chunk_decay[u.chunk0 + threadIdx.x] = acs[threadIdx.x * Q + Q - 1];
+  for (int hh = 0; hh < u.heads; ++hh) {
+    __syncthreads();                                // the last reads of B or of the head before, and the weights
+    // x times its token's weight, split
+#pragma unroll
+    for (int k = 0; k < tx.kPieces; ++k) {
+      const int i = threadIdx.x + k * 4 * Q, t = i / tx.kUnits, at = t * kXS + i % tx.kUnits * 8;
+      const float w = ws[hh * Q + t];
+      const uint4 xw = tx.w[k];
+      const float v[8] = {bf16lo(xw.x) * w, bf16hi(xw.x) * w, bf16lo(xw.y) * w, bf16hi(xw.y) * w,
+                          bf16lo(xw.z) * w, bf16hi(xw.z) * w, bf16lo(xw.w) * w, bf16hi(xw.w) * w};
       bf16x8_t hi, low;
-      split8(sx, hi, low);
-      acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf, hi, acc, 0, 0, 0);
-      acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf, low, acc, 0, 0, 0);
+      split8(v, hi, low);
+      *reinterpret_cast<bf16x8_t*>(xh + at) = hi;
+      *reinterpret_cast<bf16x8_t*>(xl + at) = low;
     }
-    const int p = p0 + pb + (lane & 31);
-    if (p < a.P)
+    __syncthreads();
+    if (hh + 1 < u.heads) tx.load(src + (u.head0 + hh + 1) * a.P + u.p0, a.xbc_stride, u.rows, a.P - u.p0);
+    float* out = a.chunk_state + (u.chunk0 + hh) * a.N * a.P;
 #pragma unroll
-      for (int e = 0; e < 16; ++e) {
-        const int n = n0 + 8 * (e >> 2) + 4 * half + (e & 3);
-        if (n < a.N) out[(int64_t)n * a.P + p] = acc[e];
+    for (int i = 0; i < kTiles; ++i) {
+      const int tile = wave + kWaves * i, n0 = tile / 2 * 32, pb = tile % 2 * 32;
+      if (n0 >= a.N || u.p0 + pb >= a.P) continue;
+      floatx16_t acc;
+#pragma unroll
+      for (int e = 0; e < 16; ++e) acc[e] = 0.f;
+#pragma unroll
+      for (int kk = 0; kk < Q / 16; ++kk) {
+        const int at = (kk * 16 + r) * kXS + pb + c;
+        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[i][kk], read_tr8(xh + at, 4 * kXS), acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[i][kk], read_tr8(xl + at, 4 * kXS), acc, 0, 0, 0);
       }
+      const int p = u.p0 + pb + (lane & 31);
+      if (p < a.P)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) {
+          const int n = n0 + 8 * (e >> 2) + 4 * half + (e & 3);
+          if (n < a.N) out[(int64_t)n * a.P + p] = acc[e];
+        }
+    }
   }
 }
 
@@ -208,125 +252,185 @@ __global__ __launch_bounds__(256) void ssd_carry_kernel(ChunkArgs a, msa_seq_bat
 
 template <int Q, int NP>
 __global__ __launch_bounds__(4 * Q) void ssd_output_kernel(ChunkArgs a, msa_seq_batch b) {
-  constexpr int kBS = NP + 8;
+  constexpr int kBS = NP + 8, kBlocks = Q / 32;
+  constexpr int kBSt = Q * kBS > 2 * NP * kXS ? Q * kBS : 2 * NP * kXS;
+  constexpr int kBefore = kBlocks * (kBlocks - 1) / 2 * 32;         // (block, earlier token) pairs
   extern __shared__ __align__(16) bf16_t sm[];
-  bf16_t* Bs = sm;                                  // [Q][kBS]
-  bf16_t* Cs = Bs + Q * kBS;                        // [Q][kBS]
-  bf16_t* xs = Cs + Q * kBS;                        // [Q][kXS]
-  bf16_t* Sh = xs + Q * kXS;                        // [NP][kXS] high parts of S_in
-  bf16_t* Sl = Sh + NP * kXS;                       // [NP][kXS] low parts
-  float* dts = reinterpret_cast<float*>(Sl + NP * kXS);
-  float* acs = dts + Q;
-  const int head = blockIdx.x % a.H, p0 = blockIdx.x / a.H * kPB, s = blockIdx.z;
-  const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo, t0 = blockIdx.y * Q;
-  if (t0 >= n_tok) return;
-  const int rows = min(Q, n_tok - t0), row0 = lo + t0;
-  const int grp = head / (a.H / a.G), inner = a.H * a.P;
-  const bf16_t* src = a.xbc + (int64_t)row0 * a.xbc_stride;
-  RowTile<Q, NP, 4 * Q> tileB, tileC;
+  bf16_t* Bs = sm;                                  // [Q][kBS], until B . C^T is in registers; then
+  bf16_t* Sh = sm;                                  // [NP][kXS] high and
+  bf16_t* Sl = Sh + NP * kXS;                       // [NP][kXS] low parts of S_in
+  bf16_t* xs = sm + kBSt;                           // [Q][kXS]
+  float* dts = reinterpret_cast<float*>(xs + Q * kXS);
+  float* acs = dts + kMaxHeads * Q;
+  float* wbs = acs + kMaxHeads * Q;                 // [heads][kBefore] weights of earlier blocks' tokens at a block's start
+  Unit u;
+  if (!unit_of<Q>(a, b, u)) return;
+  const int inner = a.H * a.P;
+  const bf16_t* src = a.xbc + (int64_t)u.row0 * a.xbc_stride;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), half = lane >> 5, l16 = lane & 15, l32 = lane & 31;
+  // a wavefront's token block and half of the columns; the two wavefronts of a SIMD get a long and a short block
+  const int tb = Q == 128 ? (wave < 4 ? wave >> 1 : 3 - ((wave - 4) >> 1)) : wave >> 1, pb = wave % 2 * 32;
+  const int t = tb * 32 + l32;
+  const int64_t row = u.row0 + t;
+
+  RowTile<Q, NP, 4 * Q> tileB;
   RowTile<Q, kPB, 4 * Q> tileX;
-  tileB.load(src + inner + grp * a.N, a.xbc_stride, rows, a.N);
-  tileC.load(src + inner + (a.G + grp) * a.N, a.xbc_stride, rows, a.N);
-  tileX.load(src + head * a.P + p0, a.xbc_stride, rows, a.P - p0);
-  const int64_t chunk = ((int64_t)s * a.n_chunks + blockIdx.y) * a.H + head;
   constexpr int kSPieces = NP * (kPB / 4) / (4 * Q);
   uint4 sw[kSPieces];
-  {
-    const uint32_t* packed = reinterpret_cast<const uint32_t*>(a.chunk_state + chunk * a.N * a.P) + p0;
+  auto fetch = [&](int hh) {
+    tileX.load(src + (u.head0 + hh) * a.P + u.p0, a.xbc_stride, u.rows, a.P - u.p0);
+    const uint32_t* packed = reinterpret_cast<const uint32_t*>(a.chunk_state + (u.chunk0 + hh) * a.N * a.P) + u.p0;
 #pragma unroll
     for (int k = 0; k < kSPieces; ++k) {
       const int i = threadIdx.x + k * 4 * Q, n = i / (kPB / 4), p = i % (kPB / 4) * 4;
       sw[k] = make_uint4(0, 0, 0, 0);
-      if (n < a.N && p0 + p < a.P) sw[k] = *reinterpret_cast<const uint4*>(packed + (int64_t)n * a.P + p);
+      if (n < a.N && u.p0 + p < a.P) sw[k] = *reinterpret_cast<const uint4*>(packed + (int64_t)n * a.P + p);
     }
-  }
-  chunk_decays<Q>(a, row0, rows, head, dts, acs);
-  tileB.store(Bs, kBS);
-  tileC.store(Cs, kBS);
-  tileX.store(xs, kXS);
-#pragma unroll
-  for (int k = 0; k < kSPieces; ++k) {
-    const int i = threadIdx.x + k * 4 * Q, n = i / (kPB / 4), p = i % (kPB / 4) * 4;
-    const uint4 w = sw[k];
-    *reinterpret_cast<uint2*>(Sh + n * kXS + p) = make_uint2((w.x & 0xffffu) | (w.y << 16), (w.z & 0xffffu) | (w.w << 16));
-    *reinterpret_cast<uint2*>(Sl + n * kXS + p) = make_uint2((w.x >> 16) | (w.y & 0xffff0000u), (w.z >> 16) | (w.w & 0xffff0000u));
-  }
-  __syncthreads();
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, half = lane >> 5, l16 = lane & 15, l32 = lane & 31;
-  const int tb = wave >> 1, pb = wave % 2 * 32;
-  if (p0 + pb >= a.P || tb * 32 >= rows) return;
-  const int t = tb * 32 + l32;
-  const float a_t = acs[t];
-  const int r = l16 >> 2, c = (lane & 16) + (l16 & 3) * 4;
-  floatx16_t acc;
-#pragma unroll
-  for (int e = 0; e < 16; ++e) acc[e] = 0.f;
+  };
+  tileB.load(src + inner + u.grp * a.N, a.xbc_stride, u.rows, a.N);
   bf16x8_t cf[NP / 16];
 #pragma unroll
   for (int kk = 0; kk < NP / 16; ++kk) {
-    cf[kk] = *reinterpret_cast<const bf16x8_t*>(Cs + t * kBS + kk * 16 + 8 * half);
-    const int at = (kk * 16 + 8 * half + r) * kXS + pb + c;
-    acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(read_tr8(Sh + at, 4 * kXS), cf[kk], acc, 0, 0, 0);
-    acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(read_tr8(Sl + at, 4 * kXS), cf[kk], acc, 0, 0, 0);
+    const int n = kk * 16 + 8 * half;
+    const bool in = t < u.rows && n < a.N;
+    cf[kk] = __builtin_bit_cast(bf16x8_t, in ? *reinterpret_cast<const uint4*>(src + (int64_t)t * a.xbc_stride + inner + (a.G + u.grp) * a.N + n)
+                                             : make_uint4(0, 0, 0, 0));
   }
-  const float in = __builtin_amdgcn_exp2f(a_t);
+  fetch(0);
+  chunk_decays<Q>(a, u.row0, u.rows, u.head0, u.heads, dts, acs);
+  tileB.store(Bs, kBS);
+  __syncthreads();
+  for (int i = threadIdx.x; i < u.heads * kBefore; i += 4 * Q) {
+    const int hh = i / kBefore, j = i % kBefore;
+    const int blk = j < 32 ? 1 : j < 96 ? 2 : 3, s = j - 16 * blk * (blk - 1);
+    wbs[i] = dts[hh * Q + s] * __builtin_amdgcn_exp2f(acs[hh * Q + blk * 32 - 1] - acs[hh * Q + s]);
+  }
+  floatx16_t g[kBlocks];                            // (B . C^T)[s, t] of block sb, the same for every head
 #pragma unroll
-  for (int e = 0; e < 16; ++e) acc[e] *= in;
-  for (int sb = 0; sb <= tb; ++sb) {
-    floatx16_t g;
+  for (int sb = 0; sb < kBlocks; ++sb)
+    if (sb <= tb) {
 #pragma unroll
-    for (int e = 0; e < 16; ++e) g[e] = 0.f;
+      for (int e = 0; e < 16; ++e) g[sb][e] = 0.f;
+#pragma unroll
+      for (int kk = 0; kk < NP / 16; ++kk) {
+        const bf16x8_t bf = *reinterpret_cast<const bf16x8_t*>(Bs + (sb * 32 + l32) * kBS + kk * 16 + 8 * half);
+        g[sb] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf, cf[kk], g[sb], 0, 0, 0);
+      }
+    }
+  const bool work = u.p0 + pb < a.P && tb * 32 < u.rows;
+  const int r = l16 >> 2, c = (lane & 16) + (l16 & 3) * 4;
+  for (int hh = 0; hh < u.heads; ++hh) {
+    const int head = u.head0 + hh;
+    __syncthreads();                                // the last reads of B or of the head before, and the weights
+    tileX.store(xs, kXS);
+#pragma unroll
+    for (int k = 0; k < kSPieces; ++k) {
+      const int i = threadIdx.x + k * 4 * Q, n = i / (kPB / 4), p = i % (kPB / 4) * 4;
+      const uint4 w = sw[k];
+      *reinterpret_cast<uint2*>(Sh + n * kXS + p) = make_uint2((w.x & 0xffffu) | (w.y << 16), (w.z & 0xffffu) | (w.w << 16));
+      *reinterpret_cast<uint2*>(Sl + n * kXS + p) = make_uint2((w.x >> 16) | (w.y & 0xffff0000u), (w.z >> 16) | (w.w & 0xffff0000u));
+    }
+    __syncthreads();
+    if (hh + 1 < u.heads) fetch(hh + 1);
+    if (!work) continue;
+    const bf16_t* zp = a.z + row * a.z_stride + head * a.P + u.p0 + pb + 4 * half;
+    uint2 zw[4];
+#pragma unroll
+    for (int q = 0; q < 4; ++q)
+      zw[q] = t < u.rows && u.p0 + pb + 8 * q + 4 * half < a.P ? *reinterpret_cast<const uint2*>(zp + 8 * q) : make_uint2(0, 0);
+    const float* ac = acs + hh * Q;
+    const float a_t = ac[t], a_ref = tb > 0 ? ac[tb * 32 - 1] : 0.f;
+    floatx16_t acc;
+#pragma unroll
+    for (int e = 0; e < 16; ++e) acc[e] = 0.f;
 #pragma unroll
     for (int kk = 0; kk < NP / 16; ++kk) {
-      const bf16x8_t bf = *reinterpret_cast<const bf16x8_t*>(Bs + (sb * 32 + l32) * kBS + kk * 16 + 8 * half);
-      g = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf, cf[kk], g, 0, 0, 0);
+      const int at = (kk * 16 + 8 * half + r) * kXS + pb + c;
+      acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(read_tr8(Sh + at, 4 * kXS), cf[kk], acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(read_tr8(Sl + at, 4 * kXS), cf[kk], acc, 0, 0, 0);
     }
+    const float in = __builtin_amdgcn_exp2f(a_ref);
 #pragma unroll
-    for (int j = 0; j < 2; ++j) {
-      float m[8];
+    for (int e = 0; e < 16; ++e) acc[e] *= in;
+    auto add_block = [&](int sb, const float (&m)[16]) {
 #pragma unroll
-      for (int q = 0; q < 2; ++q) {
-        const int s0 = sb * 32 + 16 * j + 8 * q + 4 * half;
-        const float4 as = *reinterpret_cast<const float4*>(acs + s0), ds = *reinterpret_cast<const float4*>(dts + s0);
-        const float av[4] = {as.x, as.y, as.z, as.w}, dv[4] = {ds.x, ds.y, ds.z, ds.w};
-#pragma unroll
-        for (int x = 0; x < 4; ++x) m[4 * q + x] = s0 + x <= t ? g[8 * j + 4 * q + x] * (__builtin_amdgcn_exp2f(a_t - av[x]) * dv[x]) : 0.f;
+      for (int j = 0; j < 2; ++j) {
+        const float part[8] = {m[8 * j], m[8 * j + 1], m[8 * j + 2], m[8 * j + 3], m[8 * j + 4], m[8 * j + 5], m[8 * j + 6], m[8 * j + 7]};
+        bf16x8_t hi, low;
+        split8(part, hi, low);
+        const bf16x8_t xf = read_tr8(xs + (sb * 32 + 16 * j + 4 * half + r) * kXS + pb + c, 8 * kXS);
+        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(xf, hi, acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(xf, low, acc, 0, 0, 0);
       }
-      bf16x8_t hi, low;
-      split8(m, hi, low);
-      const bf16x8_t xf = read_tr8(xs + (sb * 32 + 16 * j + 4 * half + r) * kXS + pb + c, 8 * kXS);
-      acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(xf, hi, acc, 0, 0, 0);
-      acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(xf, low, acc, 0, 0, 0);
+    };
+    // earlier blocks, relative to this block's start; then on to token t
+    const float* wb = wbs + hh * kBefore + 16 * tb * (tb - 1);
+#pragma unroll
+    for (int sb = 0; sb < kBlocks - 1; ++sb)
+      if (sb < tb) {
+        float m[16];
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          const float4 w = *reinterpret_cast<const float4*>(wb + sb * 32 + 8 * q + 4 * half);
+          m[4 * q] = g[sb][4 * q] * w.x;
+          m[4 * q + 1] = g[sb][4 * q + 1] * w.y;
+          m[4 * q + 2] = g[sb][4 * q + 2] * w.z;
+          m[4 * q + 3] = g[sb][4 * q + 3] * w.w;
+        }
+        add_block(sb, m);
+      }
+    const float on = __builtin_amdgcn_exp2f(a_t - a_ref);
+#pragma unroll
+    for (int e = 0; e < 16; ++e) acc[e] *= on;
+#pragma unroll
+    for (int sb = 0; sb < kBlocks; ++sb)
+      if (sb == tb) {
+        float m[16];
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          const int s0 = sb * 32 + 8 * q + 4 * half;
+          const float4 as = *reinterpret_cast<const float4*>(ac + s0), ds = *reinterpret_cast<const float4*>(dts + hh * Q + s0);
+          const float av[4] = {as.x, as.y, as.z, as.w}, dv[4] = {ds.x, ds.y, ds.z, ds.w};
+#pragma unroll
+          for (int x = 0; x < 4; ++x)
+            m[4 * q + x] = s0 + x <= t ? g[sb][4 * q + x] * (__builtin_amdgcn_exp2f(a_t - av[x]) * dv[x]) : 0.f;
+        }
+        add_block(sb, m);
+      }
+    // acc[e] is y of token t, column pb + 8 (e / 4) + 4 half + e % 4
+    const float Dh = a.D[head];
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int p = pb + 8 * q + 4 * half;
+      if (t >= u.rows || u.p0 + p >= a.P) continue;
+      float xv[4], y[4];
+      load_vec<bf16_t, 4>(xs + t * kXS + p, xv);
+      const float zv[4] = {bf16lo(zw[q].x), bf16hi(zw[q].x), bf16lo(zw[q].y), bf16hi(zw[q].y)};
+#pragma unroll
+      for (int x = 0; x < 4; ++x) y[x] = (acc[4 * q + x] + Dh * xv[x]) * silu_f(zv[x]);
+      store_vec<bf16_t, 4>(a.v + row * inner + head * a.P + u.p0 + p, y);
     }
-  }
-  // acc[e] is y of token t, column pb + 8 (e / 4) + 4 half + e % 4
-  if (t >= rows) return;
-  const float Dh = a.D[head];
-  const int64_t row = row0 + t;
-#pragma unroll
-  for (int q = 0; q < 4; ++q) {
-    const int p = pb + 8 * q + 4 * half;
-    if (p0 + p >= a.P) continue;
-    float xv[4], zv[4], y[4];
-    load_vec<bf16_t, 4>(xs + t * kXS + p, xv);
-    load_vec<bf16_t, 4>(a.z + row * a.z_stride + head * a.P + p0 + p, zv);
-#pragma unroll
-    for (int x = 0; x < 4; ++x) y[x] = (acc[4 * q + x] + Dh * xv[x]) * silu_f(zv[x]);
-    store_vec<bf16_t, 4>(a.v + row * inner + head * a.P + p0 + p, y);
   }
 }
 
 int chunk_tokens(int32_t N) { return N <= 128 ? 128 : 64; }
 
 template <int Q, int NP>
-int launch_chunked(const ChunkArgs& a, const msa_seq_batch& b, hipStream_t st) {
-  constexpr int lds1 = Q * (NP + 8 + kXS) * 2 + 2 * Q * 4;
-  constexpr int lds3 = (2 * Q * (NP + 8) + (Q + 2 * NP) * kXS) * 2 + 2 * Q * 4;
-  static_assert(lds3 <= 160 * 1024, "tiles of a chunk must fit LDS");
+int launch_chunked(ChunkArgs a, const msa_seq_batch& b, hipStream_t st) {
+  constexpr int tile = Q * (NP + 8), x = Q * kXS, state = 2 * NP * kXS;
+  constexpr int lds1 = (tile > 2 * x ? tile : 2 * x) * 2 + 2 * kMaxHeads * Q * 4;
+  constexpr int lds3 = ((tile > state ? tile : state) + x) * 2 + kMaxHeads * (2 * Q + (Q / 32) * (Q / 32 - 1) * 16) * 4;
+  static_assert(lds1 <= 160 * 1024 && lds3 <= 160 * 1024, "tiles of a chunk must fit LDS");
+  // as many heads per workgroup as leave the launch two workgroups per compute unit
+  const int per_group = a.H / a.G, blocks = (a.P + kPB - 1) / kPB;
+  auto wgs = [&](int h) { return (int64_t)a.n_chunks * b.n_seq * a.G * blocks * ((per_group + h - 1) / h); };
+  a.heads_per_wg = std::min(kMaxHeads, per_group);
+  while (a.heads_per_wg > 1 && wgs(a.heads_per_wg) < 2 * device_compute_units()) --a.heads_per_wg;
+  a.heads_per_wg = (per_group + (per_group + a.heads_per_wg - 1) / a.heads_per_wg - 1) / ((per_group + a.heads_per_wg - 1) / a.heads_per_wg);
   static std::atomic<int> raised1{0}, raised3{0};
   MSA_HIP(raise_dynamic_lds_limit(raised1, reinterpret_cast<const void*>(ssd_local_kernel<Q, NP>), lds1));
   MSA_HIP(raise_dynamic_lds_limit(raised3, reinterpret_cast<const void*>(ssd_output_kernel<Q, NP>), lds3));
-  const dim3 grid((unsigned)(a.H * ((a.P + kPB - 1) / kPB)), a.n_chunks, b.n_seq);
+  const dim3 grid((unsigned)(a.G * blocks * ((per_group + a.heads_per_wg - 1) / a.heads_per_wg)), a.n_chunks, b.n_seq);
   ssd_local_kernel<Q, NP><<<grid, 4 * Q, lds1, st>>>(a, b);
   MSA_LAUNCH_CHECK();
   ssd_carry_kernel<<<dim3((a.N * a.P / 4 + 255) / 256, a.H, b.n_seq), 256, 0, st>>>(a, b, Q);
@@ -364,7 +468,7 @@ extern "C" int msa_seq_ssd_chunked(const void* xbc, int64_t xbc_stride, const vo
   }
   float* states = static_cast<float*>(workspace);
   const ChunkArgs a{(const bf16_t*)xbc, (const bf16_t*)z, (const bf16_t*)dt_raw, dt_bias, A_log, D, state, (bf16_t*)v, states,
-                    states + (int64_t)batch->n_seq * chunks * H * N * P, xbc_stride, z_stride, dt_stride, H, P, N, G, chunks};
+                    states + (int64_t)batch->n_seq * chunks * H * N * P, xbc_stride, z_stride, dt_stride, H, P, N, G, chunks, 1};
   hipStream_t st = as_stream(stream);
   if (N <= 32) return launch_chunked<128, 32>(a, *batch, st);
   if (N <= 64) return launch_chunked<128, 64>(a, *batch, st);
