@@ -15,6 +15,7 @@ namespace {
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8_t;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4_t;
 typedef __attribute__((__vector_size__(16 * sizeof(float)))) float floatx16_t;
+typedef unsigned int u32x4_t __attribute__((ext_vector_type(4)));
 typedef short shortx4_t __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) shortx4_t lds_shortx4_t;
 
@@ -103,7 +104,7 @@ constexpr int kDecMaxRank = 512;
 struct DecArgs {
   const bf16_t* q;
   const bf16_t* cache;
-  float* part_acc;     // [rows, n_split, H, rank]
+  bf16_t* part_acc;    // [rows, n_split, H, rank]
   float* part_ml;      // [rows, n_split, H, 2]
   int64_t Lcap;
   float scale_log2e;
@@ -135,22 +136,22 @@ __global__ __launch_bounds__(kDecThreads) void latent_decode_kernel(DecArgs a, m
 
   // a thread's pieces: column u of rows r0, r0 + kStep, ...
   const int u = tid % units * 8, r0 = tid / units;
-  constexpr int kStep = kDecThreads / units, kPieces = (kDecKeys + kStep - 1) / kStep;
+  constexpr int kStep = kDecThreads / units, kPieces = (kDecKeys + kStep - 1) / kStep, kQPieces = (kHeads + kStep - 1) / kStep;
   static_assert(kPieces * kStep == kDecKeys, "whole pieces per thread");
-  uint4 next[kPieces];
-  auto fetch = [&](int k0) {
-    const bf16_t* at = c + (int64_t)(k0 + r0) * a.rank + u;
+  // Two register sets: a tile is requested two tiles ahead of its use, through a buffer resource whose extent is the tile's
+  // valid rows (what lies outside reads as zero), so that no load is conditional and the waits can be counted.
+  struct Tile { u32x4_t w[kPieces]; } set0, set1;
+  const int row_bytes = a.rank * 2;
+  const int voff = u < a.rank ? r0 * row_bytes + u * 2 : 0x40000000;
+  auto fetch = [&](Tile& next, int k0) {
+    const int extent = __builtin_amdgcn_readfirstlane(max(0, min(kDecKeys, last - k0)) * row_bytes);
+    const int at = __builtin_amdgcn_readfirstlane(k0 < last ? k0 : 0);
+    const __amdgpu_buffer_rsrc_t rs = __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t*>(c + (int64_t)at * a.rank), 0, extent, 0x00020000);
 #pragma unroll
-    for (int i = 0; i < kPieces; ++i) {
-      next[i] = make_uint4(0, 0, 0, 0);
-      if (k0 + r0 + kStep * i < last && u < a.rank) next[i] = *reinterpret_cast<const uint4*>(at + (int64_t)(kStep * i) * a.rank);
-    }
+    for (int i = 0; i < kPieces; ++i) next.w[i] = __builtin_amdgcn_raw_buffer_load_b128(rs, voff + kStep * i * row_bytes, 0, 0);
   };
-  auto stash = [&]() {
-#pragma unroll
-    for (int i = 0; i < kPieces; ++i) *reinterpret_cast<uint4*>(cs + (r0 + kStep * i) * stride + u) = next[i];
-  };
-  if (first < last) fetch(first);
+  fetch(set0, first);
+  fetch(set1, first + kDecKeys);
   bf16x8_t qf[RP / 32];
   {
     const int h = h0 + ht * 16 + l16;
@@ -167,19 +168,29 @@ __global__ __launch_bounds__(kDecThreads) void latent_decode_kernel(DecArgs a, m
 #pragma unroll
     for (int t = 0; t < kCT; ++t) o[h][t] = floatx4_t{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;        // of head tid / kPer, the same in its kPer threads
-  for (int k0 = first; k0 < last; k0 += kDecKeys) {
+  auto tile_step = [&](Tile& mine, int k0) {
     __syncthreads();
-    stash();
+#pragma unroll
+    for (int i = 0; i < kPieces; ++i) *reinterpret_cast<u32x4_t*>(cs + (r0 + kStep * i) * stride + u) = mine.w[i];
     __syncthreads();
-    if (k0 + kDecKeys < last) fetch(k0 + kDecKeys);
+    fetch(mine, k0 + 2 * kDecKeys);
     if (ht < HT) {
-      floatx4_t sc = floatx4_t{0.f, 0.f, 0.f, 0.f};
+      // two chains of products, keys read from LDS a few products ahead
+      floatx4_t sc[2] = {floatx4_t{0.f, 0.f, 0.f, 0.f}, floatx4_t{0.f, 0.f, 0.f, 0.f}};
+      constexpr int kAhead = RP / 32 < 6 ? RP / 32 : 6;
+      const bf16_t* kr = cs + (kt * 16 + l16) * stride + 8 * g;
+      bf16x8_t kb[kAhead];
 #pragma unroll
-      for (int kk = 0; kk < RP / 32; ++kk)
-        sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-            qf[kk], *reinterpret_cast<const bf16x8_t*>(cs + (kt * 16 + l16) * stride + 32 * kk + 8 * g), sc, 0, 0, 0);
+      for (int kk = 0; kk < kAhead; ++kk) kb[kk] = *reinterpret_cast<const bf16x8_t*>(kr + 32 * kk);
+      __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) ss[(ht * 16 + 4 * g + e) * kSStride + kt * 16 + l16] = sc[e] * a.scale_log2e;
+      for (int kk = 0; kk < RP / 32; ++kk) {
+        sc[kk & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[kk], kb[kk % kAhead], sc[kk & 1], 0, 0, 0);
+        if (kk + kAhead < RP / 32) kb[kk % kAhead] = *reinterpret_cast<const bf16x8_t*>(kr + 32 * (kk + kAhead));
+        __builtin_amdgcn_sched_barrier(0);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss[(ht * 16 + 4 * g + e) * kSStride + kt * 16 + l16] = (sc[0][e] + sc[1][e]) * a.scale_log2e;
     }
     __syncthreads();
     {
@@ -211,6 +222,7 @@ __global__ __launch_bounds__(kDecThreads) void latent_decode_kernel(DecArgs a, m
 #pragma unroll
     for (int h = 0; h < HT; ++h) {
       const float4 f = *reinterpret_cast<const float4*>(al + h * 16 + 4 * g);
+      if (!__any(f.x * f.y * f.z * f.w != 1.0f)) continue;       // no maximum moved
 #pragma unroll
       for (int t = 0; t < kCT; ++t) {
         o[h][t][0] *= f.x;
@@ -233,34 +245,47 @@ __global__ __launch_bounds__(kDecThreads) void latent_decode_kernel(DecArgs a, m
         for (int h = 0; h < HT; ++h) o[h][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[h], vb, o[h][t], 0, 0, 0);
       }
     }
+  };
+  for (int k0 = first; k0 < last; k0 += 2 * kDecKeys) {
+    tile_step(set0, k0);
+    if (k0 + kDecKeys < last) tile_step(set1, k0 + kDecKeys);
   }
-  // o[h][t][e] belongs to head 16 h + 4 g + e, latent column 16 (wave + 8 t) + l16
+  // o[h][t][e] belongs to head 16 h + 4 g + e, latent column 16 (wave + 8 t) + l16.  The sums leave in bf16 (as the context that
+  // is made of them will), through LDS so that a row's pieces are stored 16 bytes at a time.
   const int64_t at = ((int64_t)row * a.n_split + split) * a.H;
+  __syncthreads();
+  static_assert(kHeads <= kDecKeys, "the key tile's LDS holds the sums");
 #pragma unroll
   for (int h = 0; h < HT; ++h)
 #pragma unroll
     for (int t = 0; t < kCT; ++t) {
       const int col = (wave + kDecWaves * t) * 16 + l16;
-      if (col >= a.rank) continue;
+      if (col >= RP) continue;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int head = h0 + h * 16 + 4 * g + e;
-        if (head < a.H) a.part_acc[(at + head) * a.rank + col] = o[h][t][e];
-      }
+      for (int e = 0; e < 4; ++e) cs[(h * 16 + 4 * g + e) * stride + col] = f32_to_bf16(o[h][t][e]);
     }
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < kQPieces; ++i) {
+    const int h = r0 + kStep * i;
+    if (h < kHeads && h0 + h < a.H && u < a.rank)
+      *reinterpret_cast<uint4*>(a.part_acc + (at + h0 + h) * a.rank + u) = *reinterpret_cast<const uint4*>(cs + h * stride + u);
+  }
   if (tid % kPer == 0 && h0 + tid / kPer < a.H) {
     a.part_ml[(at + h0 + tid / kPer) * 2] = m;
     a.part_ml[(at + h0 + tid / kPer) * 2 + 1] = l;
   }
 }
 
-// A workgroup per (row, head): folds the key ranges and the sink.  The ranges' weights first, then one pass over their sums.
+// A workgroup per (row, head): folds the key ranges and the sink.  The ranges' weights first, then their sums: four wavefronts
+// take a quarter of the ranges each, eight columns a lane.
 constexpr int kMaxSplits = 128;
-__global__ __launch_bounds__(128) void latent_combine_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
+__global__ __launch_bounds__(256) void latent_combine_kernel(const bf16_t* __restrict__ part_acc, const float* __restrict__ part_ml,
                                                              const float* __restrict__ sink, int32_t H, int32_t rank, int32_t n_split,
                                                              bf16_t* __restrict__ ctx) {
-  __shared__ float ws[kMaxSplits], red[4];
-  const int row = blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
+  __shared__ float ws[kMaxSplits], red[8];
+  __shared__ float sums[4][64 * 8];
+  const int row = blockIdx.x, head = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int64_t first = (int64_t)row * n_split * H + head;
   const float sk = sink[head] * kLog2e;
   float mi = -INFINITY, li = 0.f;
@@ -272,29 +297,37 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(const float* __rest
   float m = fmaxf(mi, sk);
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) m = fmaxf(m, __shfl_xor(m, o));
-  if ((tid & 63) == 0) red[tid >> 6] = m;
+  if (lane == 0) red[wave] = m;
   __syncthreads();
-  m = fmaxf(red[0], red[1]);
+  m = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
   const float w = __builtin_amdgcn_exp2f(mi - m);                // 0 for a range without keys
   float l = w * li;
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) l += __shfl_xor(l, o);
-  if ((tid & 63) == 0) red[2 + (tid >> 6)] = l;
-  ws[tid] = w;
+  if (lane == 0) red[4 + wave] = l;
+  if (tid < kMaxSplits) ws[tid] = w;
   __syncthreads();
-  const float inv = 1.0f / (red[2] + red[3] + __builtin_amdgcn_exp2f(sk - m));
-  for (int c = tid * 4; c < rank; c += 512) {
-    float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-    const float* src = part_acc + first * rank + c;
-#pragma unroll 8
-    for (int i = 0; i < n_split; ++i) {
-      const float4 p = *reinterpret_cast<const float4*>(src + (int64_t)i * H * rank);
+  const float inv = 1.0f / (red[4] + red[5] + red[6] + red[7] + __builtin_amdgcn_exp2f(sk - m));
+  float v[8] = {};
+  const int c = lane * 8;                                        // rank <= 512
+  if (c < rank) {
+    const bf16_t* src = part_acc + first * rank + c;
+#pragma unroll 4
+    for (int i = wave; i < n_split; i += 4) {
+      float p[8];
+      load_vec<bf16_t, 8>(src + (int64_t)i * H * rank, p);
       const float f = ws[i];
-      v.x += f * p.x; v.y += f * p.y; v.z += f * p.z; v.w += f * p.w;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] += f * p[e];
     }
-    *reinterpret_cast<uint2*>(ctx + ((int64_t)row * H + head) * rank + c) =
-        make_uint2(pack_bf16x2(v.x * inv, v.y * inv), pack_bf16x2(v.z * inv, v.w * inv));
   }
+#pragma unroll
+  for (int e = 0; e < 8; ++e) sums[wave][e * 64 + lane] = v[e];
+  __syncthreads();
+  if (wave != 0 || c >= rank) return;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] = (sums[0][e * 64 + lane] + sums[1][e * 64 + lane] + sums[2][e * 64 + lane] + sums[3][e * 64 + lane]) * inv;
+  store_vec<bf16_t, 8>(ctx + ((int64_t)row * H + head) * rank + c, v);
 }
 
 int latent_splits(int32_t rows, int32_t H, int64_t max_keys) {
@@ -350,29 +383,40 @@ __global__ __launch_bounds__(256, (DP + EP <= 256) ? 2 : 1) void flash_sink_kern
       qf[i] = __builtin_bit_cast(bf16x8_t, w);
     }
   }
-  uint4 kn[kKP], vn[kVP];
+  // tile loads through buffer resources whose extent is the tile's valid rows: rows and dims outside read as zero
+  u32x4_t kn[kKP], vn[kVP];
+  int kv_off[kKP], vv_off[kVP];
+#pragma unroll
+  for (int i = 0; i < kKP; ++i) {
+    const int idx = tid + 256 * i, key = idx / (DP / 8), d = idx % (DP / 8) * 8;
+    kv_off[i] = d < a.D ? (int)(key * a.k_stride + d) * 2 : 0x7ffffff0;
+  }
+#pragma unroll
+  for (int i = 0; i < kVP; ++i) {
+    const int idx = tid + 256 * i, key = idx / (EP / 8), d = idx % (EP / 8) * 8;
+    vv_off[i] = d < a.E ? (int)(key * a.v_stride + d) * 2 : 0x7ffffff0;
+  }
   auto fetch = [&](int k0) {
+    const int rows = min(kFlashKeys, kmax - k0);
+    const __amdgpu_buffer_rsrc_t rk = __builtin_amdgcn_make_buffer_rsrc(
+        const_cast<bf16_t*>(kg + (int64_t)k0 * a.k_stride), 0, (int)((rows - 1) * a.k_stride + a.D) * 2, 0x00020000);
+    const __amdgpu_buffer_rsrc_t rv = __builtin_amdgcn_make_buffer_rsrc(
+        const_cast<bf16_t*>(vg + (int64_t)k0 * a.v_stride), 0, (int)((rows - 1) * a.v_stride + a.E) * 2, 0x00020000);
 #pragma unroll
-    for (int i = 0; i < kKP; ++i) {
-      const int idx = tid + 256 * i, key = idx / (DP / 8), d = idx % (DP / 8) * 8;
-      kn[i] = k0 + key < kmax && d < a.D ? *reinterpret_cast<const uint4*>(kg + (int64_t)(k0 + key) * a.k_stride + d) : make_uint4(0, 0, 0, 0);
-    }
+    for (int i = 0; i < kKP; ++i) kn[i] = __builtin_amdgcn_raw_buffer_load_b128(rk, kv_off[i], 0, 0);
 #pragma unroll
-    for (int i = 0; i < kVP; ++i) {
-      const int idx = tid + 256 * i, key = idx / (EP / 8), d = idx % (EP / 8) * 8;
-      vn[i] = k0 + key < kmax && d < a.E ? *reinterpret_cast<const uint4*>(vg + (int64_t)(k0 + key) * a.v_stride + d) : make_uint4(0, 0, 0, 0);
-    }
+    for (int i = 0; i < kVP; ++i) vn[i] = __builtin_amdgcn_raw_buffer_load_b128(rv, vv_off[i], 0, 0);
   };
   auto stash = [&](int stage) {
 #pragma unroll
     for (int i = 0; i < kKP; ++i) {
       const int idx = tid + 256 * i;
-      *reinterpret_cast<uint4*>(kt + (stage * kFlashKeys + idx / (DP / 8)) * kKS + idx % (DP / 8) * 8) = kn[i];
+      *reinterpret_cast<u32x4_t*>(kt + (stage * kFlashKeys + idx / (DP / 8)) * kKS + idx % (DP / 8) * 8) = kn[i];
     }
 #pragma unroll
     for (int i = 0; i < kVP; ++i) {
       const int idx = tid + 256 * i;
-      *reinterpret_cast<uint4*>(vt + (stage * kFlashKeys + idx / (EP / 8)) * kVS + idx % (EP / 8) * 8) = vn[i];
+      *reinterpret_cast<u32x4_t*>(vt + (stage * kFlashKeys + idx / (EP / 8)) * kVS + idx % (EP / 8) * 8) = vn[i];
     }
   };
   floatx16_t o[EP / 32];
@@ -517,7 +561,7 @@ extern "C" int msa_seq_latent_attn(const void* q, const void* cache, int64_t Lca
 
 extern "C" size_t msa_seq_latent_decode_workspace_bytes(int32_t rows, int32_t H, int32_t rank, int64_t max_keys) {
   if (rows <= 0 || H <= 0 || rank <= 0 || max_keys <= 0) return 0;
-  return (size_t)rows * latent_splits(rows, H, max_keys) * H * (rank + 2) * sizeof(float);
+  return (size_t)rows * latent_splits(rows, H, max_keys) * H * (2 * sizeof(float) + (size_t)rank * sizeof(bf16_t));
 }
 
 extern "C" int msa_seq_latent_decode(const void* q, const void* cache, int64_t Lcap, const float* sink, float scale, int32_t dtype,
@@ -530,19 +574,19 @@ extern "C" int msa_seq_latent_decode(const void* q, const void* cache, int64_t L
               H, rank, kDecMaxRank);
   MSA_REQUIRE(batch->rows <= 65535 && max_keys > 0 && max_keys <= Lcap && Lcap < ((int64_t)1 << 31), "msa_seq_latent_decode: %d rows, %lld keys",
               batch->rows, (long long)max_keys);
-  MSA_REQUIRE((((uintptr_t)q | (uintptr_t)cache) & 15) == 0, "msa_seq_latent_decode: q and cache must be 16-byte aligned");
+  MSA_REQUIRE((((uintptr_t)q | (uintptr_t)cache | (uintptr_t)ctx | (uintptr_t)workspace) & 15) == 0, "msa_seq_latent_decode: q, cache, ctx and workspace must be 16-byte aligned");
   const int splits = latent_splits(batch->rows, H, max_keys);
   if (workspace_bytes < msa_seq_latent_decode_workspace_bytes(batch->rows, H, rank, max_keys)) {
     msa_set_error("msa_seq_latent_decode: workspace of %zu bytes is too small", workspace_bytes);
     return MSA_ESIZE;
   }
-  float* acc = static_cast<float*>(workspace);
-  float* ml = acc + (int64_t)batch->rows * splits * H * rank;
+  bf16_t* acc = static_cast<bf16_t*>(workspace);                 // (rank is a multiple of 8: the pairs behind stay aligned)
+  float* ml = reinterpret_cast<float*>(acc + (int64_t)batch->rows * splits * H * rank);
   const DecArgs a{(const bf16_t*)q, (const bf16_t*)cache, acc, ml, Lcap, scale * kLog2e, H, rank, splits};
   hipStream_t st = as_stream(stream);
   const int rc = H <= 16 ? launch_decode<1>(a, *batch, st) : launch_decode<2>(a, *batch, st);
   if (rc != MSA_OK) return rc;
-  latent_combine_kernel<<<dim3(batch->rows, H), 128, 0, st>>>(acc, ml, sink, H, rank, splits, (bf16_t*)ctx);
+  latent_combine_kernel<<<dim3(batch->rows, H), 256, 0, st>>>(acc, ml, sink, H, rank, splits, (bf16_t*)ctx);
   MSA_LAUNCH_CHECK();
   return MSA_OK;
 }
@@ -555,7 +599,7 @@ extern "C" int msa_seq_flash(const void* q, int64_t q_stride, const void* k, int
   MSA_REQUIRE(q && k && v && kv_off && sink && out && scale > 0.f, "msa_seq_flash: null pointer or scale <= 0");
   MSA_REQUIRE(H > 0 && D > 0 && E > 0 && D % 8 == 0 && E % 8 == 0 && D <= 256 && E <= 256, "msa_seq_flash: D=%d E=%d (multiples of 8 up to 256)", D, E);
   MSA_REQUIRE(q_stride >= (int64_t)H * D && k_stride >= (int64_t)H * D && v_stride >= (int64_t)H * E && q_stride % 8 == 0 &&
-                  k_stride % 8 == 0 && v_stride % 8 == 0 && (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)out) & 15) == 0,
+                  k_stride % 8 == 0 && v_stride % 8 == 0 && k_stride <= (1 << 22) && v_stride <= (1 << 22) && (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)out) & 15) == 0,
               "msa_seq_flash: strides or alignment");
   MSA_REQUIRE(batch->n_seq <= 65535 && (batch->max_rows + kFlashRows - 1) / kFlashRows <= 65535, "msa_seq_flash: step too large");
   const FlashArgs a{(const bf16_t*)q, (const bf16_t*)k, (const bf16_t*)v, kv_off, sink, (bf16_t*)out, q_stride, k_stride, v_stride,

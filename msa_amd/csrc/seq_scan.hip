@@ -196,7 +196,7 @@ __global__ __launch_bounds__(WAVES * 64) void ssd_scan_kernel(SsdArgs a, msa_seq
 // S_t = a_t S_(t-1) + b_t per channel.  Long portions run in chunks of kGruRows tokens: (1) every chunk's (product of a,
 // last b-part), (2) the chunk-to-chunk recurrence, which leaves each chunk's incoming state, (3) the chunks again from
 // their incoming states.  A portion of one chunk is phase (3) alone.
-constexpr int kGruRows = 64;
+constexpr int kGruRows = 32;
 constexpr int kGruGroup = 16;       // channels per group of the [16 z | 16 u | 16 g] row layout
 __device__ __forceinline__ int gru_column(int c) { return (c / kGruGroup) * 3 * kGruGroup + c % kGruGroup; }
 
