@@ -211,25 +211,44 @@ struct GruArgs {
   int32_t n, n_chunks;
 };
 
-// The raw columns of a few rows, all loads issued before the first is needed (rows behind the portion repeat the last one).
+// The raw columns of a few rows of a portion, through a buffer resource whose extent is the portion's rows: nothing is
+// conditional, so the compiler can count the loads in flight, and a batch is requested while the one before is worked on.
 constexpr int kGruBatch = 8;
 template <typename T, int VEC, int COLS>
 struct GruRows {
-  float v[kGruBatch][COLS][VEC];
-  __device__ __forceinline__ void load(const T* row, int64_t stride, int left) {
+  static constexpr int kBytes = VEC * sizeof(T);
+  uint32_t v[kGruBatch][COLS][kBytes <= 4 ? 1 : kBytes / 4];
+  __device__ __forceinline__ void load(__amdgpu_buffer_rsrc_t rs, int at, int stride) {
 #pragma unroll
-    for (int r = 0; r < kGruBatch; ++r) {
-      const T* at = row + min(r, left - 1) * stride;
+    for (int r = 0; r < kGruBatch; ++r)
 #pragma unroll
-      for (int k = 0; k < COLS; ++k) load_vec<T, VEC>(at + k * kGruGroup, v[r][k]);
-    }
+      for (int k = 0; k < COLS; ++k) {
+        const int off = at + r * stride + k * kGruGroup * (int)sizeof(T);
+        if constexpr (kBytes == 2) v[r][k][0] = __builtin_amdgcn_raw_buffer_load_b16(rs, off, 0, 0);
+        else if constexpr (kBytes == 4) v[r][k][0] = __builtin_amdgcn_raw_buffer_load_b32(rs, off, 0, 0);
+        else {
+          const auto w = __builtin_amdgcn_raw_buffer_load_b64(rs, off, 0, 0);
+          v[r][k][0] = w[0];
+          v[r][k][1] = w[1];
+        }
+      }
+  }
+  __device__ __forceinline__ float get(int r, int k, int e) const {
+    if constexpr (sizeof(T) == 4) return __uint_as_float(v[r][k][e]);
+    else return e == 0 ? bf16lo(v[r][k][0]) : bf16hi(v[r][k][0]);
   }
 };
-// keep = 1 - z and add = z * candidate.
+// keep = 1 - z and add = z * candidate, from the raw columns and the biases times -log2(e).  With ez = exp(-z_raw - z_bias) and
+// eu = exp(-u) one reciprocal r = 1 / ((1 + ez) (1 + eu)) gives both: z = r (1 + eu), and z sigmoid(u) = r.  (The kernel is bound by
+// instructions, the transcendental ones above all; exponents stop at 60, where a sigmoid is 1e-18.)
 __device__ __forceinline__ void gru_terms(float z_raw, float u_raw, float zb, float ub, float& keep, float& add) {
-  const float z = sigmoid_f(z_raw + zb), u = u_raw + ub;
-  keep = 1.0f - z;
-  add = z * (u >= 0.f ? u + 0.5f : sigmoid_f(u));
+  constexpr float kNegLog2e = -1.4426950408889634f, kHalfLog2e = 0.7213475204444817f, kLn2 = -0.6931471805599453f;
+  const float un = fmaf(u_raw, kNegLog2e, ub);                       // -u log2(e)
+  const float ez = __builtin_amdgcn_exp2f(fminf(fmaf(z_raw, kNegLog2e, zb), 60.f));
+  const float q = 1.0f + __builtin_amdgcn_exp2f(fminf(un, 60.f));
+  const float r = __builtin_amdgcn_rcpf((1.0f + ez) * q), z = r * q;
+  keep = ez * z;
+  add = un <= 0.f ? z * ((un - kHalfLog2e) * kLn2) : r;              // u + 1/2 = (un - log2(e) / 2) * -ln 2
 }
 
 template <typename T, int VEC>
@@ -242,22 +261,31 @@ __global__ __launch_bounds__(256) void gru_chunk_kernel(GruArgs a, msa_seq_batch
   load_vec<float, VEC>(a.z_bias + c, zb);
   load_vec<float, VEC>(a.u_bias + c, ub);
 #pragma unroll
-  for (int e = 0; e < VEC; ++e) A[e] = 1.f, S[e] = 0.f;
-  const T* row = static_cast<const T*>(a.zug) + (int64_t)(lo + t0) * a.stride + gru_column(c);
-  for (int t = 0; t < n; t += kGruBatch, row += kGruBatch * a.stride) {
-    GruRows<T, VEC, 2> in;
-    in.load(row, a.stride, n - t);
+  for (int e = 0; e < VEC; ++e) zb[e] *= -1.4426950408889634f, ub[e] *= -1.4426950408889634f;
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) A[e]  = 1.f, S[e] = 0.f;
+  const int row_bytes = (int)a.stride * (int)sizeof(T);
+  const __amdgpu_buffer_rsrc_t rs = __builtin_amdgcn_make_buffer_rsrc(
+      const_cast<T*>(static_cast<const T*>(a.zug) + (int64_t)(lo + t0) * a.stride), 0, n * row_bytes, 0x00020000);
+  int at = gru_column(c) * (int)sizeof(T);
+  GruRows<T, VEC, 2> cur, next;
+  cur.load(rs, at, row_bytes);
+  for (int t = 0; t < n; t += kGruBatch) {
+    at += kGruBatch * row_bytes;
+    next.load(rs, at, row_bytes);
+    const int live = n - t;
 #pragma unroll
     for (int r = 0; r < kGruBatch; ++r) {
-      if (t + r >= n) break;
+      if (r >= live) break;
 #pragma unroll
       for (int e = 0; e < VEC; ++e) {
         float k, d;
-        gru_terms(in.v[r][0][e], in.v[r][1][e], zb[e], ub[e], k, d);
+        gru_terms(cur.get(r, 0, e), cur.get(r, 1, e), zb[e], ub[e], k, d);
         A[e] *= k;
         S[e] = k * S[e] + d;
       }
     }
+    cur = next;
   }
   float2* dst = a.chunk + ((int64_t)s * a.n_chunks + blockIdx.y) * a.n + c;
 #pragma unroll
@@ -294,27 +322,47 @@ __global__ __launch_bounds__(256) void gru_out_kernel(GruArgs a, msa_seq_batch b
   float zb[VEC], ub[VEC], S[VEC];
   load_vec<float, VEC>(a.z_bias + c, zb);
   load_vec<float, VEC>(a.u_bias + c, ub);
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) zb[e] *= -1.4426950408889634f, ub[e] *= -1.4426950408889634f;
   float* st = a.state + (int64_t)b.slot[s] * a.n + c;
 #pragma unroll
   for (int e = 0; e < VEC; ++e) S[e] = kCarried ? a.chunk[((int64_t)s * a.n_chunks + blockIdx.y) * a.n + c + e].x : st[e];
-  const T* row = static_cast<const T*>(a.zug) + (int64_t)(lo + t0) * a.stride + gru_column(c);
-  T* out = static_cast<T*>(a.out) + (int64_t)(lo + t0) * a.n + c;
-  for (int t = 0; t < n; t += kGruBatch, row += kGruBatch * a.stride) {
-    GruRows<T, VEC, 3> in;
-    in.load(row, a.stride, n - t);
+  const int row_bytes = (int)a.stride * (int)sizeof(T), out_bytes = a.n * (int)sizeof(T);
+  const __amdgpu_buffer_rsrc_t rs = __builtin_amdgcn_make_buffer_rsrc(
+      const_cast<T*>(static_cast<const T*>(a.zug) + (int64_t)(lo + t0) * a.stride), 0, n * row_bytes, 0x00020000);
+  const __amdgpu_buffer_rsrc_t ro = __builtin_amdgcn_make_buffer_rsrc(static_cast<T*>(a.out) + (int64_t)(lo + t0) * a.n, 0, n * out_bytes, 0x00020000);
+  int at = gru_column(c) * (int)sizeof(T), to = c * (int)sizeof(T);
+  GruRows<T, VEC, 3> cur, next;
+  cur.load(rs, at, row_bytes);
+  for (int t = 0; t < n; t += kGruBatch, to += kGruBatch * out_bytes) {
+    at += kGruBatch * row_bytes;
+    next.load(rs, at, row_bytes);
+    const int live = n - t;
+    float ys[kGruBatch][VEC];
 #pragma unroll
     for (int r = 0; r < kGruBatch; ++r) {
-      if (t + r >= n) break;
-      float y[VEC];
+      if (r >= live) break;
 #pragma unroll
       for (int e = 0; e < VEC; ++e) {
         float k, d;
-        gru_terms(in.v[r][0][e], in.v[r][1][e], zb[e], ub[e], k, d);
+        gru_terms(cur.get(r, 0, e), cur.get(r, 1, e), zb[e], ub[e], k, d);
         S[e] = k * S[e] + d;
-        y[e] = S[e] * silu_f(in.v[r][2][e]);
+        ys[r][e] = S[e] * silu_f(cur.get(r, 2, e));
       }
-      store_vec<T, VEC>(out + (int64_t)(t + r) * a.n, y);
     }
+#pragma unroll
+    for (int r = 0; r < kGruBatch; ++r) {
+      const float(&y)[VEC] = ys[r];
+      const int off = to + r * out_bytes;                   // rows behind the portion are not written
+      if constexpr (VEC == 1 && sizeof(T) == 2) __builtin_amdgcn_raw_buffer_store_b16(f32_to_bf16(y[0]), ro, off, 0, 0);
+      else if constexpr (VEC == 1) __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(y[0]), ro, off, 0, 0);
+      else if constexpr (sizeof(T) == 2) __builtin_amdgcn_raw_buffer_store_b32(pack_bf16x2(y[0], y[1]), ro, off, 0, 0);
+      else {
+        typedef unsigned int u32x2_t __attribute__((ext_vector_type(2)));
+        __builtin_amdgcn_raw_buffer_store_b64(u32x2_t{__float_as_uint(y[0]), __float_as_uint(y[1])}, ro, off, 0, 0);
+      }
+    }
+    cur = next;
   }
   if (!kCarried)
 #pragma unroll
@@ -387,7 +435,7 @@ extern "C" int msa_seq_min_gru(const void* zug, int64_t zug_stride, const float*
                                void* stream) {
   MSA_CHECK_BATCH(batch, "msa_seq_min_gru");
   MSA_CHECK_DTYPE(dtype, "msa_seq_min_gru");
-  MSA_REQUIRE(zug && z_bias && u_bias && state && out && n > 0 && zug_stride >= 48LL * ((n + 15) / 16), "msa_seq_min_gru: bad arguments");
+  MSA_REQUIRE(zug && z_bias && u_bias && state && out && n > 0 && zug_stride >= 48LL * ((n + 15) / 16) && zug_stride < (1 << 22), "msa_seq_min_gru: bad arguments");
   const size_t need = msa_seq_min_gru_workspace_bytes(batch->rows, batch->n_seq, batch->max_rows, n);
   if (need > workspace_bytes || (need && !workspace)) {
     msa_set_error("msa_seq_min_gru: workspace of %zu bytes, need %zu", workspace_bytes, need);

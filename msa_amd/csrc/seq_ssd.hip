@@ -3,11 +3,12 @@
 // a_t = sum of the chunk's log-decays up to t, inside a chunk
 //   y_t = exp(a_t) S_in^T C_t + sum_{s <= t} exp(a_t - a_s) dt_s (B_s . C_t) x_s,   S_out = exp(a_end) S_in + S_loc,
 //   S_loc = sum_s exp(a_end - a_s) dt_s B_s x_s^T.
-//   (1) ssd_local_kernel   every chunk's S_loc
-//   (2) ssd_carry_kernel   the chunk-to-chunk recurrence, element by element; leaves each chunk's S_in in its place
-//   (3) ssd_output_kernel  the outputs
-// A workgroup takes one chunk and several heads of one group, whose B, C and B . C^T are the same: those are read / formed once
-// and stay in registers; a head's x and S_in are fetched while the head before is multiplied.
+//   (1) ssd_decay_kernel   dt and a_t of every token and head
+//   (2) ssd_state_kernel   the states: a workgroup owns 32 columns of a head's state and walks over the chunks with it in its
+//                          accumulators, leaving every chunk's S_in behind for
+//   (3) ssd_output_kernel  the outputs: a workgroup takes one chunk and several heads of one group, whose B, C and B . C^T are
+//                          the same (read / formed once, kept in registers); a head's x and S_in are fetched while the head
+//                          before is multiplied.
 // Operands that carry decays or states are fp32 values: they enter the bf16 products as a high and a low part (two products
 // with about 16 bits of mantissa), so only x, B and C, which are bf16 to begin with, set the precision.
 //
@@ -22,6 +23,8 @@ namespace {
 
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8_t;
 typedef __attribute__((__vector_size__(16 * sizeof(float)))) float floatx16_t;
+typedef unsigned int u32x4_t __attribute__((ext_vector_type(4)));
+typedef unsigned int u32x2_t __attribute__((ext_vector_type(2)));
 typedef short shortx4_t __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) shortx4_t lds_shortx4_t;
 
@@ -56,38 +59,46 @@ struct ChunkArgs {
   const float* D;
   float* state;
   bf16_t* v;
-  float* chunk_state;      // [n_seq, n_chunks, H, N, P]: S_loc (fp32), then S_in as packed (high, low) bf16 pairs
-  float* chunk_decay;      // [n_seq, n_chunks, H]: a_end in powers of two
+  uint32_t* chunk_state;   // [n_seq, n_chunks, H, N, P]: S_in as packed (high, low) bf16 pairs
+  float* dts;              // [n_seq, n_chunks, H, Q]: dt, and
+  float* acs;              // the running log-decay of the chunk (in powers of two)
   int64_t xbc_stride, z_stride, dt_stride;
   int32_t H, P, N, G, n_chunks, heads_per_wg;
 };
 
 constexpr int kMaxHeads = 8;             // heads of a group per workgroup
 
-// dt and the running log-decay (base 2) of the chunk's tokens for `heads` heads from `head0` on, [heads][Q] each: a wavefront per
-// head.  Tokens behind the sequence have dt = 0.  The caller synchronises.
+// A wavefront per (chunk, head).  Tokens behind the sequence have dt = 0.
 template <int Q>
-__device__ __forceinline__ void chunk_decays(const ChunkArgs& a, int row0, int rows, int head0, int heads, float* dts, float* acs) {
-  const int lane = threadIdx.x & 63;
-  for (int hh = threadIdx.x >> 6; hh < heads; hh += blockDim.x >> 6) {
-    const int head = head0 + hh;
-    const float rate = -expf(a.A_log[head]) * kLog2e, bias = a.dt_bias[head];
-    float before = 0.f;
+__global__ __launch_bounds__(256) void ssd_decay_kernel(ChunkArgs a, msa_seq_batch b) {
+  const int lane = threadIdx.x & 63, head = blockIdx.x * 4 + (threadIdx.x >> 6), s = blockIdx.z;
+  const int lo = b.cu[s], t0 = blockIdx.y * Q, rows = min(Q, b.cu[s + 1] - lo - t0);
+  if (head >= a.H || rows <= 0) return;
+  const float rate = -expf(a.A_log[head]) * kLog2e, bias = a.dt_bias[head];
+  const int64_t at = (((int64_t)s * a.n_chunks + blockIdx.y) * a.H + head) * Q;
+  float before = 0.f;
 #pragma unroll
-    for (int t = lane; t < Q; t += 64) {
-      const float dt = t < rows ? softplus_f(bf16_to_f32(a.dt_raw[(int64_t)(row0 + t) * a.dt_stride + head]) + bias) : 0.f;
-      float ac = rate * dt;
+  for (int t = lane; t < Q; t += 64) {
+    const float dt = t < rows ? softplus_f(bf16_to_f32(a.dt_raw[(int64_t)(lo + t0 + t) * a.dt_stride + head]) + bias) : 0.f;
+    float ac = rate * dt;
 #pragma unroll
-      for (int o = 1; o < 64; o <<= 1) {
-        const float up = __shfl_up(ac, o);
-        if (lane >= o) ac += up;
-      }
-      ac += before;
-      before = __shfl(ac, 63);
-      dts[hh * Q + t] = dt;
-      acs[hh * Q + t] = ac;
+    for (int o = 1; o < 64; o <<= 1) {
+      const float up = __shfl_up(ac, o);
+      if (lane >= o) ac += up;
     }
+    ac += before;
+    before = __shfl(ac, 63);
+    a.dts[at + t] = dt;
+    a.acs[at + t] = ac;
   }
+}
+
+// All global accesses inside the loops below go through buffer resources whose extent is the valid rows: what lies outside
+// reads as zero and is not written, nothing is conditional, and the compiler can count the loads and stores in flight (behind a
+// conditional one it would wait for every store of the step before).
+constexpr int kOutside = 0x40000000;
+__device__ __forceinline__ __amdgpu_buffer_rsrc_t rows_rsrc(const bf16_t* p, int rows, int64_t stride, int n) {
+  return __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t*>(p), 0, __builtin_amdgcn_readfirstlane((int)((rows - 1) * stride + n) * 2), 0x00020000);
 }
 
 // `n` columns of the chunk's rows on their way into an LDS tile of WIDTH columns (zeros behind n and behind the sequence): all
@@ -96,25 +107,157 @@ template <int Q, int WIDTH, int THREADS>
 struct RowTile {
   static constexpr int kUnits = WIDTH / 8, kPieces = Q * kUnits / THREADS;
   static_assert(Q * kUnits % THREADS == 0, "whole pieces per thread");
-  uint4 w[kPieces];
-  __device__ __forceinline__ void load(const bf16_t* src, int64_t stride, int rows, int n) {
+  u32x4_t w[kPieces];
+  // A thread's byte offsets in a chunk's rows, the same for every chunk and head.
+  struct Offsets {
+    int at[kPieces];
+    __device__ __forceinline__ Offsets(int stride, int n) {
 #pragma unroll
-    for (int k = 0; k < kPieces; ++k) {
-      const int i = threadIdx.x + k * THREADS, r = i / kUnits, u = i % kUnits * 8;
-      w[k] = make_uint4(0, 0, 0, 0);
-      if (r < rows && u < n) w[k] = *reinterpret_cast<const uint4*>(src + (int64_t)r * stride + u);
+      for (int k = 0; k < kPieces; ++k) {
+        const int i = threadIdx.x + k * THREADS, u = i % kUnits * 8, in = (i / kUnits * stride + u) * 2;
+        at[k] = u < n ? in : kOutside;
+      }
     }
+  };
+  __device__ __forceinline__ void load(const Offsets& off, const bf16_t* src, int stride, int rows, int n) {
+    const __amdgpu_buffer_rsrc_t rs = rows_rsrc(src, rows, stride, n);
+#pragma unroll
+    for (int k = 0; k < kPieces; ++k) w[k] = __builtin_amdgcn_raw_buffer_load_b128(rs, off.at[k], 0, 0);
   }
   __device__ __forceinline__ void store(bf16_t* dst, int dst_stride) const {
 #pragma unroll
     for (int k = 0; k < kPieces; ++k) {
       const int i = threadIdx.x + k * THREADS;
-      *reinterpret_cast<uint4*>(dst + i / kUnits * dst_stride + i % kUnits * 8) = w[k];
+      *reinterpret_cast<u32x4_t*>(dst + i / kUnits * dst_stride + i % kUnits * 8) = w[k];
     }
   }
 };
 
-// What a workgroup of kernels (1) and (3) works on.
+__device__ __forceinline__ uint32_t pack_split(float v) {
+  const uint32_t hi = f32_to_bf16(v);
+  return hi | ((uint32_t)f32_to_bf16(v - bf16_to_f32((bf16_t)hi)) << 16);
+}
+
+// A workgroup per (sequence, head, 32 state columns); wavefront w owns the state rows of 32-row tiles w, w + 4, ...
+constexpr int kStateCols = 32, kSX = kStateCols + 8;
+template <int Q, int NP>
+__global__ __launch_bounds__(256) void ssd_state_kernel(ChunkArgs a, msa_seq_batch b) {
+  constexpr int kBS = NP + 8, kTiles = (NP / 32 + 3) / 4;
+  extern __shared__ __align__(16) bf16_t sm[];
+  bf16_t* Bs = sm;                                  // [Q][kBS]
+  bf16_t* xh = Bs + Q * kBS;                        // [Q][kSX] high and
+  bf16_t* xl = xh + Q * kSX;                        // [Q][kSX] low parts of the weighted x
+  const int head = blockIdx.x % a.H, p0 = blockIdx.x / a.H * kStateCols, s = blockIdx.z;
+  const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo, chunks = (n_tok + Q - 1) / Q;
+  const int grp = head / (a.H / a.G), inner = a.H * a.P;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), half = lane >> 5, l16 = lane & 15;
+  const int p = p0 + (lane & 31);
+  const bf16_t* src = a.xbc + (int64_t)lo * a.xbc_stride;
+  const int64_t first = (int64_t)s * a.n_chunks * a.H + head;
+
+  const int stride = (int)a.xbc_stride;
+  const typename RowTile<Q, NP, 256>::Offsets off_b(stride, a.N);
+  const typename RowTile<Q, kStateCols, 256>::Offsets off_x(stride, a.P - p0);
+  // two sets of a chunk's operands on their way: a chunk is requested two chunks ahead of its use
+  struct Operands {
+    RowTile<Q, NP, 256> tb;
+    RowTile<Q, kStateCols, 256> tx;
+    float w_dt[RowTile<Q, kStateCols, 256>::kPieces], w_ac[RowTile<Q, kStateCols, 256>::kPieces], a_end;
+  } set0, set1;
+  auto fetch = [&](Operands& o, int c) {
+    __builtin_amdgcn_sched_barrier(0);              // (the waits count on the sets being loaded one behind the other)
+    c = min(c, chunks - 1);                         // the last chunk again instead of one that is not there
+    const int rows = min(Q, n_tok - c * Q);
+    const bf16_t* at = src + (int64_t)c * Q * a.xbc_stride;
+    const int64_t d = (first + (int64_t)c * a.H) * Q;
+    o.tb.load(off_b, at + inner + grp * a.N, stride, rows, a.N);
+    o.tx.load(off_x, at + head * a.P + p0, stride, rows, a.P - p0);
+#pragma unroll
+    for (int k = 0; k < o.tx.kPieces; ++k) {
+      const int t = (threadIdx.x + k * 256) / o.tx.kUnits;
+      o.w_dt[k] = a.dts[d + t];
+      o.w_ac[k] = a.acs[d + t];
+    }
+    o.a_end = a.acs[d + Q - 1];
+    __builtin_amdgcn_sched_barrier(0);
+  };
+  float* keep = a.state + (((int64_t)b.slot[s] * a.H + head) * a.N) * a.P + p;
+  floatx16_t S[kTiles];                             // rows n0 + 8 (e / 4) + 4 half + e % 4 of column p
+#pragma unroll
+  for (int i = 0; i < kTiles; ++i)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) {
+      const int n = (wave + 4 * i) * 32 + 8 * (e >> 2) + 4 * half + (e & 3);
+      S[i][e] = n < a.N && p < a.P ? keep[(int64_t)n * a.P] : 0.f;
+    }
+  const int r = 8 * half + (l16 >> 2), c0 = (lane & 16) + (l16 & 3) * 4;
+  auto step = [&](Operands& o, int c) {
+    __syncthreads();
+    o.tb.store(Bs, kBS);
+#pragma unroll
+    for (int k = 0; k < o.tx.kPieces; ++k) {        // x times its token's weight, split
+      const int i = threadIdx.x + k * 256, at = i / o.tx.kUnits * kSX + i % o.tx.kUnits * 8;
+      const float w = o.w_dt[k] * __builtin_amdgcn_exp2f(o.a_end - o.w_ac[k]);
+      const u32x4_t xw = o.tx.w[k];
+      const float v[8] = {bf16lo(xw.x) * w, bf16hi(xw.x) * w, bf16lo(xw.y) * w, bf16hi(xw.y) * w,
+                          bf16lo(xw.z) * w, bf16hi(xw.z) * w, bf16lo(xw.w) * w, bf16hi(xw.w) * w};
+      bf16x8_t hi, low;
+      split8(v, hi, low);
+      *reinterpret_cast<bf16x8_t*>(xh + at) = hi;
+      *reinterpret_cast<bf16x8_t*>(xl + at) = low;
+    }
+    const float decay = __builtin_amdgcn_exp2f(o.a_end);
+    __syncthreads();
+    fetch(o, c + 2);
+    const __amdgpu_buffer_rsrc_t out = __builtin_amdgcn_make_buffer_rsrc(a.chunk_state + (first + (int64_t)c * a.H) * a.N * a.P, 0,
+                                                                          a.N * a.P * 4, 0x00020000);
+#pragma unroll
+    for (int i = 0; i < kTiles; ++i) {
+      const int n0 = (wave + 4 * i) * 32;
+      if (NP < 128 && n0 >= NP) continue;           // (the wavefront has no rows)
+      // every operand of the tile's products first, so that their LDS reads overlap; high and low parts in chains of their own
+      bf16x8_t bf[Q / 16], hi[Q / 16], low[Q / 16];
+#pragma unroll
+      for (int kk = 0; kk < Q / 16; ++kk) {
+        const int at = (kk * 16 + r) * kSX + c0;
+        bf[kk] = read_tr8(Bs + (kk * 16 + r) * kBS + n0 + c0, 4 * kBS);
+        hi[kk] = read_tr8(xh + at, 4 * kSX);
+        low[kk] = read_tr8(xl + at, 4 * kSX);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+      const int in_out = ((n0 + 4 * half) * a.P + p) * 4, at_out = p < a.P ? in_out : kOutside;
+      floatx16_t rest;
+#pragma unroll
+      for (int e = 0; e < 16; ++e) {
+        __builtin_amdgcn_raw_buffer_store_b32(pack_split(S[i][e]), out, at_out + (8 * (e >> 2) + (e & 3)) * a.P * 4, 0, 0);
+        S[i][e] *= decay;
+        rest[e] = 0.f;
+      }
+#pragma unroll
+      for (int kk = 0; kk < Q / 16; ++kk) {
+        S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[kk], hi[kk], S[i], 0, 0, 0);
+        rest = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[kk], low[kk], rest, 0, 0, 0);
+      }
+#pragma unroll
+      for (int e = 0; e < 16; ++e) S[i][e] += rest[e];
+    }
+  };
+  fetch(set0, 0);
+  fetch(set1, 1);
+  for (int c = 0; c < chunks; c += 2) {
+    step(set0, c);
+    if (c + 1 < chunks) step(set1, c + 1);
+  }
+#pragma unroll
+  for (int i = 0; i < kTiles; ++i)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) {
+      const int n = (wave + 4 * i) * 32 + 8 * (e >> 2) + 4 * half + (e & 3);
+      if (n < a.N && p < a.P) keep[(int64_t)n * a.P] = S[i][e];
+    }
+}
+
+// What a workgroup of the output kernel works on.
 struct Unit {
   int head0, heads, grp, p0, lo, t0, rows, row0;
   int64_t chunk0;          // chunk index of head0
@@ -134,120 +277,6 @@ __device__ __forceinline__ bool unit_of(const ChunkArgs& a, const msa_seq_batch&
   u.row0 = u.lo + u.t0;
   u.chunk0 = ((int64_t)s * a.n_chunks + blockIdx.y) * a.H + u.head0;
   return u.t0 < n_tok;
-}
-
-template <int Q, int NP>
-__global__ __launch_bounds__(4 * Q) void ssd_local_kernel(ChunkArgs a, msa_seq_batch b) {
-  constexpr int kBS = NP + 8, kWaves = Q / 16, kTiles = (NP / 32 * 2 + kWaves - 1) / kWaves;
-  constexpr int kBX = Q * kBS > 2 * Q * kXS ? Q * kBS : 2 * Q * kXS;
-  extern __shared__ __align__(16) bf16_t sm[];
-  bf16_t* Bs = sm;                                  // [Q][kBS], until its fragments are in registers; then
-  bf16_t* xh = sm;                                  // [Q][kXS] high and
-  bf16_t* xl = xh + Q * kXS;                        // [Q][kXS] low parts of the weighted x
-  float* ws = reinterpret_cast<float*>(sm + kBX);   // [heads][Q]
-  float* acs = ws + kMaxHeads * Q;
-  Unit u;
-  if (!unit_of<Q>(a, b, u)) return;
-  const int inner = a.H * a.P;
-  const bf16_t* src = a.xbc + (int64_t)u.row0 * a.xbc_stride;
-  RowTile<Q, NP, 4 * Q> tb;
-  RowTile<Q, kPB, 4 * Q> tx;
-  tb.load(src + inner + u.grp * a.N, a.xbc_stride, u.rows, a.N);
-  tx.load(src + u.head0 * a.P + u.p0, a.xbc_stride, u.rows, a.P - u.p0);
-  chunk_decays<Q>(a, u.row0, u.rows, u.head0, u.heads, ws, acs);
-  tb.store(Bs, kBS);
-  __syncthreads();
-  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), half = lane >> 5, l16 = lane & 15;
-  const int r = 8 * half + (l16 >> 2), c = (lane & 16) + (l16 & 3) * 4;
-  bf16x8_t bf[kTiles][Q / 16];                      // B^T operands of this wavefront's tiles, for every head
-#pragma unroll
-  for (int i = 0; i < kTiles; ++i) {
-    const int n0 = (wave + kWaves * i) / 2 * 32;
-    if (n0 < NP)
-#pragma unroll
-      for (int kk = 0; kk < Q / 16; ++kk) bf[i][kk] = read_tr8(Bs + (kk * 16 + r) * kBS + n0 + c, 4 * kBS);
-  }
-  for (int i = threadIdx.x; i < u.heads * Q; i += 4 * Q) ws[i] *= __builtin_amdgcn_exp2f(acs[i / Q * Q + Q - 1] - acs[i]);
-  if (threadIdx.x < u.heads && u.p0 == 0) a.chunk_decay[u.chunk0 + threadIdx.x] = acs[threadIdx.x * Q + Q - 1];
-  for (int hh = 0; hh < u.heads; ++hh) {
-    __syncthreads();                                // the last reads of B or of the head before, and the weights
-    // x times its token's weight, split
-#pragma unroll
-    for (int k = 0; k < tx.kPieces; ++k) {
-      const int i = threadIdx.x + k * 4 * Q, t = i / tx.kUnits, at = t * kXS + i % tx.kUnits * 8;
-      const float w = ws[hh * Q + t];
-      const uint4 xw = tx.w[k];
-      const float v[8] = {bf16lo(xw.x) * w, bf16hi(xw.x) * w, bf16lo(xw.y) * w, bf16hi(xw.y) * w,
-                          bf16lo(xw.z) * w, bf16hi(xw.z) * w, bf16lo(xw.w) * w, bf16hi(xw.w) * w};
-      bf16x8_t hi, low;
-      split8(v, hi, low);
-      *reinterpret_cast<bf16x8_t*>(xh + at) = hi;
-      *reinterpret_cast<bf16x8_t*>(xl + at) = low;
-    }
-    __syncthreads();
-    if (hh + 1 < u.heads) tx.load(src + (u.head0 + hh + 1) * a.P + u.p0, a.xbc_stride, u.rows, a.P - u.p0);
-    float* out = a.chunk_state + (u.chunk0 + hh) * a.N * a.P;
-#pragma unroll
-    for (int i = 0; i < kTiles; ++i) {
-      const int tile = wave + kWaves * i, n0 = tile / 2 * 32, pb = tile % 2 * 32;
-      if (n0 >= a.N || u.p0 + pb >= a.P) continue;
-      floatx16_t acc;
-#pragma unroll
-      for (int e = 0; e < 16; ++e) acc[e] = 0.f;
-#pragma unroll
-      for (int kk = 0; kk < Q / 16; ++kk) {
-        const int at = (kk * 16 + r) * kXS + pb + c;
-        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[i][kk], read_tr8(xh + at, 4 * kXS), acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[i][kk], read_tr8(xl + at, 4 * kXS), acc, 0, 0, 0);
-      }
-      const int p = u.p0 + pb + (lane & 31);
-      if (p < a.P)
-#pragma unroll
-        for (int e = 0; e < 16; ++e) {
-          const int n = n0 + 8 * (e >> 2) + 4 * half + (e & 3);
-          if (n < a.N) out[(int64_t)n * a.P + p] = acc[e];
-        }
-    }
-  }
-}
-
-__device__ __forceinline__ float pack_split(float v) {
-  const uint32_t hi = f32_to_bf16(v);
-  const uint32_t low = f32_to_bf16(v - bf16_to_f32((bf16_t)hi));
-  return __uint_as_float(hi | (low << 16));
-}
-
-// Four state elements per thread (N P is a multiple of 8).
-__global__ __launch_bounds__(256) void ssd_carry_kernel(ChunkArgs a, msa_seq_batch b, int32_t Q) {
-  const int64_t per = (int64_t)a.N * a.P;
-  const int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * 4;
-  const int head = blockIdx.y, s = blockIdx.z;
-  if (i >= per) return;
-  const int n_tok = b.cu[s + 1] - b.cu[s], chunks = (n_tok + Q - 1) / Q;
-  float4* keep = reinterpret_cast<float4*>(a.state + ((int64_t)b.slot[s] * a.H + head) * per + i);
-  float4 S = *keep;
-  const int64_t first = (int64_t)s * a.n_chunks * a.H + head;
-  constexpr int kBatch = 8;
-  for (int c = 0; c < chunks; c += kBatch) {
-    float4 loc[kBatch];
-    float d[kBatch];
-    float4* at[kBatch];
-#pragma unroll
-    for (int k = 0; k < kBatch; ++k) {
-      const int64_t chunk = first + (int64_t)min(c + k, chunks - 1) * a.H;
-      at[k] = reinterpret_cast<float4*>(a.chunk_state + chunk * per + i);
-      loc[k] = *at[k];
-      d[k] = a.chunk_decay[chunk];
-    }
-#pragma unroll
-    for (int k = 0; k < kBatch; ++k) {
-      if (c + k >= chunks) break;
-      *at[k] = make_float4(pack_split(S.x), pack_split(S.y), pack_split(S.z), pack_split(S.w));
-      const float f = __builtin_amdgcn_exp2f(d[k]);
-      S = make_float4(f * S.x + loc[k].x, f * S.y + loc[k].y, f * S.z + loc[k].z, f * S.w + loc[k].w);
-    }
-  }
-  *keep = S;
 }
 
 template <int Q, int NP>
@@ -271,23 +300,26 @@ __global__ __launch_bounds__(4 * Q) void ssd_output_kernel(ChunkArgs a, msa_seq_
   // a wavefront's token block and half of the columns; the two wavefronts of a SIMD get a long and a short block
   const int tb = Q == 128 ? (wave < 4 ? wave >> 1 : 3 - ((wave - 4) >> 1)) : wave >> 1, pb = wave % 2 * 32;
   const int t = tb * 32 + l32;
-  const int64_t row = u.row0 + t;
 
+  const int stride = (int)a.xbc_stride;
   RowTile<Q, NP, 4 * Q> tileB;
   RowTile<Q, kPB, 4 * Q> tileX;
+  const typename RowTile<Q, kPB, 4 * Q>::Offsets off_x(stride, a.P - u.p0);
   constexpr int kSPieces = NP * (kPB / 4) / (4 * Q);
-  uint4 sw[kSPieces];
-  auto fetch = [&](int hh) {
-    tileX.load(src + (u.head0 + hh) * a.P + u.p0, a.xbc_stride, u.rows, a.P - u.p0);
-    const uint32_t* packed = reinterpret_cast<const uint32_t*>(a.chunk_state + (u.chunk0 + hh) * a.N * a.P) + u.p0;
+  u32x4_t sw[kSPieces];
+  int s_at[kSPieces];
 #pragma unroll
-    for (int k = 0; k < kSPieces; ++k) {
-      const int i = threadIdx.x + k * 4 * Q, n = i / (kPB / 4), p = i % (kPB / 4) * 4;
-      sw[k] = make_uint4(0, 0, 0, 0);
-      if (n < a.N && u.p0 + p < a.P) sw[k] = *reinterpret_cast<const uint4*>(packed + (int64_t)n * a.P + p);
-    }
+  for (int k = 0; k < kSPieces; ++k) {
+    const int i = threadIdx.x + k * 4 * Q, p = u.p0 + i % (kPB / 4) * 4, in = (i / (kPB / 4) * a.P + p) * 4;
+    s_at[k] = p < a.P ? in : kOutside;
+  }
+  auto fetch = [&](int hh) {
+    tileX.load(off_x, src + (u.head0 + hh) * a.P + u.p0, stride, u.rows, a.P - u.p0);
+    const __amdgpu_buffer_rsrc_t rs = __builtin_amdgcn_make_buffer_rsrc(a.chunk_state + (u.chunk0 + hh) * a.N * a.P, 0, a.N * a.P * 4, 0x00020000);
+#pragma unroll
+    for (int k = 0; k < kSPieces; ++k) sw[k] = __builtin_amdgcn_raw_buffer_load_b128(rs, s_at[k], 0, 0);
   };
-  tileB.load(src + inner + u.grp * a.N, a.xbc_stride, u.rows, a.N);
+  tileB.load(typename RowTile<Q, NP, 4 * Q>::Offsets(stride, a.N), src + inner + u.grp * a.N, stride, u.rows, a.N);
   bf16x8_t cf[NP / 16];
 #pragma unroll
   for (int kk = 0; kk < NP / 16; ++kk) {
@@ -297,7 +329,10 @@ __global__ __launch_bounds__(4 * Q) void ssd_output_kernel(ChunkArgs a, msa_seq_
                                              : make_uint4(0, 0, 0, 0));
   }
   fetch(0);
-  chunk_decays<Q>(a, u.row0, u.rows, u.head0, u.heads, dts, acs);
+  for (int i = threadIdx.x; i < u.heads * Q; i += 4 * Q) {
+    dts[i] = a.dts[u.chunk0 * Q + i];
+    acs[i] = a.acs[u.chunk0 * Q + i];
+  }
   tileB.store(Bs, kBS);
   __syncthreads();
   for (int i = threadIdx.x; i < u.heads * kBefore; i += 4 * Q) {
@@ -317,8 +352,16 @@ __global__ __launch_bounds__(4 * Q) void ssd_output_kernel(ChunkArgs a, msa_seq_
         g[sb] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf, cf[kk], g[sb], 0, 0, 0);
       }
     }
-  const bool work = u.p0 + pb < a.P && tb * 32 < u.rows;
+  const __amdgpu_buffer_rsrc_t rs_z = rows_rsrc(a.z + (int64_t)u.row0 * a.z_stride, u.rows, a.z_stride, inner);
+  const __amdgpu_buffer_rsrc_t rs_v = rows_rsrc(a.v + (int64_t)u.row0 * inner, u.rows, inner, inner);
   const int r = l16 >> 2, c = (lane & 16) + (l16 & 3) * 4;
+  int z_at[4], v_at[4];                             // of token t's four pieces, without the head
+#pragma unroll
+  for (int q = 0; q < 4; ++q) {
+    const int p = u.p0 + pb + 8 * q + 4 * half, zin = (t * (int)a.z_stride + p) * 2, vin = (t * inner + p) * 2;
+    z_at[q] = p < a.P ? zin : kOutside;
+    v_at[q] = p < a.P ? vin : kOutside;
+  }
   for (int hh = 0; hh < u.heads; ++hh) {
     const int head = u.head0 + hh;
     __syncthreads();                                // the last reads of B or of the head before, and the weights
@@ -326,18 +369,15 @@ __global__ __launch_bounds__(4 * Q) void ssd_output_kernel(ChunkArgs a, msa_seq_
 #pragma unroll
     for (int k = 0; k < kSPieces; ++k) {
       const int i = threadIdx.x + k * 4 * Q, n = i / (kPB / 4), p = i % (kPB / 4) * 4;
-      const uint4 w = sw[k];
+      const u32x4_t w = sw[k];
       *reinterpret_cast<uint2*>(Sh + n * kXS + p) = make_uint2((w.x & 0xffffu) | (w.y << 16), (w.z & 0xffffu) | (w.w << 16));
       *reinterpret_cast<uint2*>(Sl + n * kXS + p) = make_uint2((w.x >> 16) | (w.y & 0xffff0000u), (w.z >> 16) | (w.w & 0xffff0000u));
     }
     __syncthreads();
     if (hh + 1 < u.heads) fetch(hh + 1);
-    if (!work) continue;
-    const bf16_t* zp = a.z + row * a.z_stride + head * a.P + u.p0 + pb + 4 * half;
-    uint2 zw[4];
+    u32x2_t zw[4];
 #pragma unroll
-    for (int q = 0; q < 4; ++q)
-      zw[q] = t < u.rows && u.p0 + pb + 8 * q + 4 * half < a.P ? *reinterpret_cast<const uint2*>(zp + 8 * q) : make_uint2(0, 0);
+    for (int q = 0; q < 4; ++q) zw[q] = __builtin_amdgcn_raw_buffer_load_b64(rs_z, z_at[q], head * a.P * 2, 0);
     const float* ac = acs + hh * Q;
     const float a_t = ac[t], a_ref = tb > 0 ? ac[tb * 32 - 1] : 0.f;
     floatx16_t acc;
@@ -401,14 +441,12 @@ __global__ __launch_bounds__(4 * Q) void ssd_output_kernel(ChunkArgs a, msa_seq_
     const float Dh = a.D[head];
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
-      const int p = pb + 8 * q + 4 * half;
-      if (t >= u.rows || u.p0 + p >= a.P) continue;
       float xv[4], y[4];
-      load_vec<bf16_t, 4>(xs + t * kXS + p, xv);
+      load_vec<bf16_t, 4>(xs + t * kXS + pb + 8 * q + 4 * half, xv);
       const float zv[4] = {bf16lo(zw[q].x), bf16hi(zw[q].x), bf16lo(zw[q].y), bf16hi(zw[q].y)};
 #pragma unroll
       for (int x = 0; x < 4; ++x) y[x] = (acc[4 * q + x] + Dh * xv[x]) * silu_f(zv[x]);
-      store_vec<bf16_t, 4>(a.v + row * inner + head * a.P + u.p0 + p, y);
+      __builtin_amdgcn_raw_buffer_store_b64(u32x2_t{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])}, rs_v, v_at[q], head * a.P * 2, 0);
     }
   }
 }
@@ -418,24 +456,23 @@ int chunk_tokens(int32_t N) { return N <= 128 ? 128 : 64; }
 template <int Q, int NP>
 int launch_chunked(ChunkArgs a, const msa_seq_batch& b, hipStream_t st) {
   constexpr int tile = Q * (NP + 8), x = Q * kXS, state = 2 * NP * kXS;
-  constexpr int lds1 = (tile > 2 * x ? tile : 2 * x) * 2 + 2 * kMaxHeads * Q * 4;
+  constexpr int lds2 = (tile + 2 * Q * kSX) * 2;
   constexpr int lds3 = ((tile > state ? tile : state) + x) * 2 + kMaxHeads * (2 * Q + (Q / 32) * (Q / 32 - 1) * 16) * 4;
-  static_assert(lds1 <= 160 * 1024 && lds3 <= 160 * 1024, "tiles of a chunk must fit LDS");
-  // as many heads per workgroup as leave the launch two workgroups per compute unit
+  static_assert(lds2 <= 160 * 1024 && lds3 <= 160 * 1024, "tiles of a chunk must fit LDS");
+  // as many heads per workgroup as leave the output launch two workgroups per compute unit
   const int per_group = a.H / a.G, blocks = (a.P + kPB - 1) / kPB;
-  auto wgs = [&](int h) { return (int64_t)a.n_chunks * b.n_seq * a.G * blocks * ((per_group + h - 1) / h); };
-  a.heads_per_wg = std::min(kMaxHeads, per_group);
-  while (a.heads_per_wg > 1 && wgs(a.heads_per_wg) < 2 * device_compute_units()) --a.heads_per_wg;
-  a.heads_per_wg = (per_group + (per_group + a.heads_per_wg - 1) / a.heads_per_wg - 1) / ((per_group + a.heads_per_wg - 1) / a.heads_per_wg);
-  static std::atomic<int> raised1{0}, raised3{0};
-  MSA_HIP(raise_dynamic_lds_limit(raised1, reinterpret_cast<const void*>(ssd_local_kernel<Q, NP>), lds1));
+  auto sets = [&](int h) { return (per_group + h - 1) / h; };
+  int heads = std::min(kMaxHeads, per_group);
+  while (heads > 1 && (int64_t)a.n_chunks * b.n_seq * a.G * blocks * sets(heads) < 2 * device_compute_units()) --heads;
+  a.heads_per_wg = (per_group + sets(heads) - 1) / sets(heads);
+  static std::atomic<int> raised2{0}, raised3{0};
+  MSA_HIP(raise_dynamic_lds_limit(raised2, reinterpret_cast<const void*>(ssd_state_kernel<Q, NP>), lds2));
   MSA_HIP(raise_dynamic_lds_limit(raised3, reinterpret_cast<const void*>(ssd_output_kernel<Q, NP>), lds3));
-  const dim3 grid((unsigned)(a.G * blocks * ((per_group + a.heads_per_wg - 1) / a.heads_per_wg)), a.n_chunks, b.n_seq);
-  ssd_local_kernel<Q, NP><<<grid, 4 * Q, lds1, st>>>(a, b);
+  ssd_decay_kernel<Q><<<dim3((a.H + 3) / 4, a.n_chunks, b.n_seq), 256, 0, st>>>(a, b);
   MSA_LAUNCH_CHECK();
-  ssd_carry_kernel<<<dim3((a.N * a.P / 4 + 255) / 256, a.H, b.n_seq), 256, 0, st>>>(a, b, Q);
+  ssd_state_kernel<Q, NP><<<dim3((unsigned)(a.H * ((a.P + kStateCols - 1) / kStateCols)), 1, b.n_seq), 256, lds2, st>>>(a, b);
   MSA_LAUNCH_CHECK();
-  ssd_output_kernel<Q, NP><<<grid, 4 * Q, lds3, st>>>(a, b);
+  ssd_output_kernel<Q, NP><<<dim3((unsigned)(a.G * blocks * sets(a.heads_per_wg)), a.n_chunks, b.n_seq), 4 * Q, lds3, st>>>(a, b);
   MSA_LAUNCH_CHECK();
   return MSA_OK;
 }
@@ -445,7 +482,7 @@ int launch_chunked(ChunkArgs a, const msa_seq_batch& b, hipStream_t st) {
 extern "C" size_t msa_seq_ssd_chunked_workspace_bytes(int32_t max_rows, int32_t n_seq, int32_t H, int32_t P, int32_t N) {
   if (max_rows <= 0 || n_seq <= 0 || H <= 0 || P <= 0 || N <= 0) return 0;
   const int Q = chunk_tokens(N);
-  return (size_t)n_seq * ((max_rows + Q - 1) / Q) * H * ((size_t)N * P + 1) * sizeof(float);
+  return (size_t)n_seq * ((max_rows + Q - 1) / Q) * H * ((size_t)N * P + 2 * Q) * sizeof(float);
 }
 
 extern "C" int msa_seq_ssd_chunked(const void* xbc, int64_t xbc_stride, const void* z, int64_t z_stride, const void* dt_raw,
@@ -457,7 +494,8 @@ extern "C" int msa_seq_ssd_chunked(const void* xbc, int64_t xbc_stride, const vo
   MSA_REQUIRE(xbc && z && dt_raw && dt_bias && A_log && D && state && v && workspace, "msa_seq_ssd_chunked: null pointer");
   MSA_REQUIRE(H > 0 && P > 0 && G > 0 && H % G == 0 && H <= 65535 && P % 8 == 0 && N > 0 && N % 8 == 0 && N <= 256,
               "msa_seq_ssd_chunked: H=%d P=%d N=%d (multiples of 8, N up to 256) G=%d", H, P, N, G);
-  MSA_REQUIRE(xbc_stride >= (int64_t)H * P + 2LL * G * N && z_stride >= (int64_t)H * P && dt_stride >= H && xbc_stride % 8 == 0 &&
+  MSA_REQUIRE(xbc_stride >= (int64_t)H * P + 2LL * G * N && z_stride >= (int64_t)H * P && dt_stride >= H && xbc_stride % 8 == 0 && xbc_stride < (1 << 21) &&
+                  z_stride < (1 << 21) &&
                   z_stride % 4 == 0 && (((uintptr_t)xbc | (uintptr_t)workspace | (uintptr_t)state) & 15) == 0 &&
                   (((uintptr_t)z | (uintptr_t)v) & 7) == 0, "msa_seq_ssd_chunked: strides or alignment");
   const int Q = chunk_tokens(N), chunks = (batch->max_rows + Q - 1) / Q;
@@ -466,9 +504,10 @@ extern "C" int msa_seq_ssd_chunked(const void* xbc, int64_t xbc_stride, const vo
     msa_set_error("msa_seq_ssd_chunked: workspace of %zu bytes is too small", workspace_bytes);
     return MSA_ESIZE;
   }
-  float* states = static_cast<float*>(workspace);
-  const ChunkArgs a{(const bf16_t*)xbc, (const bf16_t*)z, (const bf16_t*)dt_raw, dt_bias, A_log, D, state, (bf16_t*)v, states,
-                    states + (int64_t)batch->n_seq * chunks * H * N * P, xbc_stride, z_stride, dt_stride, H, P, N, G, chunks, 1};
+  uint32_t* states = static_cast<uint32_t*>(workspace);
+  float* dts = reinterpret_cast<float*>(states + (int64_t)batch->n_seq * chunks * H * N * P);
+  const ChunkArgs a{(const bf16_t*)xbc, (const bf16_t*)z, (const bf16_t*)dt_raw, dt_bias, A_log, D, state, (bf16_t*)v, states, dts,
+                    dts + (int64_t)batch->n_seq * chunks * H * Q, xbc_stride, z_stride, dt_stride, H, P, N, G, chunks, 1};
   hipStream_t st = as_stream(stream);
   if (N <= 32) return launch_chunked<128, 32>(a, *batch, st);
   if (N <= 64) return launch_chunked<128, 64>(a, *batch, st);
