@@ -59,7 +59,7 @@ def time_us(fn, reps=20, warm=3):
     return best * 1e3 / reps
 
 
-def row(us, bytes_=0.0, flops=0.0):
+def row(us: float, bytes_: float = 0.0, flops: float = 0.0) -> dict:
     """A kernel's line: time and the fraction of whichever roofline binds it."""
     hbm, mfma = bytes_ / (HBM_GBS * 1e3), flops / (MFMA_TFLOPS * 1e6)
     bound, floor = ("hbm", hbm) if hbm >= mfma else ("mfma", mfma)
@@ -107,7 +107,7 @@ def kernels(size: str, dev) -> dict:
     st = torch.zeros(1, SH, N, P, device=dev)
     Q = 128 if N <= 128 else 64
     ssd_fl = SH * T * (2.0 * Q / 2 * (N + 2 * P) + 2.0 * N * P * 4)      # (two products per decay- or state-carrying operand)
-    p["state-space scan (3 launches)"] = row(time_us(lambda: seq_ops.ssd(xbc_in, zz, dtr, dtb, al, D, SH, P, N, G, st, pb, chunked=True)),
+    p["state-space scan (4 launches)"] = row(time_us(lambda: seq_ops.ssd(xbc_in, zz, dtr, dtb, al, D, SH, P, N, G, st, pb, chunked=True)),
                                              T * (C + 2 * inner + SH) * 2, ssd_fl)
     v, nw = bf(T, inner), f32(inner)
     p["grouped rms norm"] = row(time_us(lambda: seq_ops.group_rmsnorm(v, nw, 8, 1e-5)), T * inner * 4)
@@ -175,6 +175,10 @@ def kernels(size: str, dev) -> dict:
     qa = bf(B, H, rank)
     ring = Ring(lambda: bf(B, L, rank), B * L * rank * 2)
     d["latent attention + combine"] = row(time_us(lambda: seq_ops.latent_attn(qa, ring(), sink, 0.1, db, L), reps=24), B * L * rank * 2)
+    long = seq_ops.StepBatch([1] * B, list(range(B)), [4 * L - 1] * B, dev)
+    far = Ring(lambda: bf(B, 4 * L, rank), B * 4 * L * rank * 2)
+    d[f"latent attention + combine at {4 * L} tokens"] = row(time_us(lambda: seq_ops.latent_attn(qa, far(), sink, 0.1, long, 4 * L), reps=12),
+                                                             B * 4 * L * rank * 2)
     vB = bf(B, inner)
     d["grouped rms norm"] = row(time_us(lambda: seq_ops.group_rmsnorm(vB, nw, 8, 1e-5)), B * inner * 4)
     d["latent norm + append"] = row(time_us(lambda: seq_ops.latent_append(dkv[:B], lw, 1e-5, ring(), db)), B * rank * 4)

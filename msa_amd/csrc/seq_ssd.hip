@@ -4,11 +4,13 @@
 //   y_t = exp(a_t) S_in^T C_t + sum_{s <= t} exp(a_t - a_s) dt_s (B_s . C_t) x_s,   S_out = exp(a_end) S_in + S_loc,
 //   S_loc = sum_s exp(a_end - a_s) dt_s B_s x_s^T.
 //   (1) ssd_decay_kernel   dt and a_t of every token and head
-//   (2) ssd_state_kernel   the states: a workgroup owns 32 columns of a head's state and walks over the chunks with it in its
-//                          accumulators, leaving every chunk's S_in behind for
-//   (3) ssd_output_kernel  the outputs: a workgroup takes one chunk and several heads of one group, whose B, C and B . C^T are
-//                          the same (read / formed once, kept in registers); a head's x and S_in are fetched while the head
-//                          before is multiplied.
+//   (2) ssd_local_kernel   every chunk's S_loc
+//   (3) ssd_carry_kernel   the chunk-to-chunk recurrence, element by element; leaves each chunk's S_in in its place
+//   (4) ssd_output_kernel  the outputs
+// A workgroup of (2) and (4) takes one chunk and several heads of one group, whose B, C and B . C^T are the same: those are read /
+// formed once and stay in registers; a head's x and S_in are fetched while the head before is multiplied.  (Walking over the chunks
+// with the state in accumulators instead of (2) and (3) moves fewer bytes but is a chain of latencies: faster only with several
+// hundred heads in the step, 1.7 times slower with 32.)
 // Operands that carry decays or states are fp32 values: they enter the bf16 products as a high and a low part (two products
 // with about 16 bits of mantissa), so only x, B and C, which are bf16 to begin with, set the precision.
 //
@@ -59,7 +61,7 @@ struct ChunkArgs {
   const float* D;
   float* state;
   bf16_t* v;
-  uint32_t* chunk_state;   // [n_seq, n_chunks, H, N, P]: S_in as packed (high, low) bf16 pairs
+  uint32_t* chunk_state;   // [n_seq, n_chunks, H, N, P]: S_loc (fp32), then S_in as packed (high, low) bf16 pairs
   float* dts;              // [n_seq, n_chunks, H, Q]: dt, and
   float* acs;              // the running log-decay of the chunk (in powers of two)
   int64_t xbc_stride, z_stride, dt_stride;
@@ -138,126 +140,7 @@ __device__ __forceinline__ uint32_t pack_split(float v) {
   return hi | ((uint32_t)f32_to_bf16(v - bf16_to_f32((bf16_t)hi)) << 16);
 }
 
-// A workgroup per (sequence, head, 32 state columns); wavefront w owns the state rows of 32-row tiles w, w + 4, ...
-constexpr int kStateCols = 32, kSX = kStateCols + 8;
-template <int Q, int NP>
-__global__ __launch_bounds__(256) void ssd_state_kernel(ChunkArgs a, msa_seq_batch b) {
-  constexpr int kBS = NP + 8, kTiles = (NP / 32 + 3) / 4;
-  extern __shared__ __align__(16) bf16_t sm[];
-  bf16_t* Bs = sm;                                  // [Q][kBS]
-  bf16_t* xh = Bs + Q * kBS;                        // [Q][kSX] high and
-  bf16_t* xl = xh + Q * kSX;                        // [Q][kSX] low parts of the weighted x
-  const int head = blockIdx.x % a.H, p0 = blockIdx.x / a.H * kStateCols, s = blockIdx.z;
-  const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo, chunks = (n_tok + Q - 1) / Q;
-  const int grp = head / (a.H / a.G), inner = a.H * a.P;
-  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), half = lane >> 5, l16 = lane & 15;
-  const int p = p0 + (lane & 31);
-  const bf16_t* src = a.xbc + (int64_t)lo * a.xbc_stride;
-  const int64_t first = (int64_t)s * a.n_chunks * a.H + head;
-
-  const int stride = (int)a.xbc_stride;
-  const typename RowTile<Q, NP, 256>::Offsets off_b(stride, a.N);
-  const typename RowTile<Q, kStateCols, 256>::Offsets off_x(stride, a.P - p0);
-  // two sets of a chunk's operands on their way: a chunk is requested two chunks ahead of its use
-  struct Operands {
-    RowTile<Q, NP, 256> tb;
-    RowTile<Q, kStateCols, 256> tx;
-    float w_dt[RowTile<Q, kStateCols, 256>::kPieces], w_ac[RowTile<Q, kStateCols, 256>::kPieces], a_end;
-  } set0, set1;
-  auto fetch = [&](Operands& o, int c) {
-    __builtin_amdgcn_sched_barrier(0);              // (the waits count on the sets being loaded one behind the other)
-    c = min(c, chunks - 1);                         // the last chunk again instead of one that is not there
-    const int rows = min(Q, n_tok - c * Q);
-    const bf16_t* at = src + (int64_t)c * Q * a.xbc_stride;
-    const int64_t d = (first + (int64_t)c * a.H) * Q;
-    o.tb.load(off_b, at + inner + grp * a.N, stride, rows, a.N);
-    o.tx.load(off_x, at + head * a.P + p0, stride, rows, a.P - p0);
-#pragma unroll
-    for (int k = 0; k < o.tx.kPieces; ++k) {
-      const int t = (threadIdx.x + k * 256) / o.tx.kUnits;
-      o.w_dt[k] = a.dts[d + t];
-      o.w_ac[k] = a.acs[d + t];
-    }
-    o.a_end = a.acs[d + Q - 1];
-    __builtin_amdgcn_sched_barrier(0);
-  };
-  float* keep = a.state + (((int64_t)b.slot[s] * a.H + head) * a.N) * a.P + p;
-  floatx16_t S[kTiles];                             // rows n0 + 8 (e / 4) + 4 half + e % 4 of column p
-#pragma unroll
-  for (int i = 0; i < kTiles; ++i)
-#pragma unroll
-    for (int e = 0; e < 16; ++e) {
-      const int n = (wave + 4 * i) * 32 + 8 * (e >> 2) + 4 * half + (e & 3);
-      S[i][e] = n < a.N && p < a.P ? keep[(int64_t)n * a.P] : 0.f;
-    }
-  const int r = 8 * half + (l16 >> 2), c0 = (lane & 16) + (l16 & 3) * 4;
-  auto step = [&](Operands& o, int c) {
-    __syncthreads();
-    o.tb.store(Bs, kBS);
-#pragma unroll
-    for (int k = 0; k < o.tx.kPieces; ++k) {        // x times its token's weight, split
-      const int i = threadIdx.x + k * 256, at = i / o.tx.kUnits * kSX + i % o.tx.kUnits * 8;
-      const float w = o.w_dt[k] * __builtin_amdgcn_exp2f(o.a_end - o.w_ac[k]);
-      const u32x4_t xw = o.tx.w[k];
-      const float v[8] = {bf16lo(xw.x) * w, bf16hi(xw.x) * w, bf16lo(xw.y) * w, bf16hi(xw.y) * w,
-                          bf16lo(xw.z) * w, bf16hi(xw.z) * w, bf16lo(xw.w) * w, bf16hi(xw.w) * w};
-      bf16x8_t hi, low;
-      split8(v, hi, low);
-      *reinterpret_cast<bf16x8_t*>(xh + at) = hi;
-      *reinterpret_cast<bf16x8_t*>(xl + at) = low;
-    }
-    const float decay = __builtin_amdgcn_exp2f(o.a_end);
-    __syncthreads();
-    fetch(o, c + 2);
-    const __amdgpu_buffer_rsrc_t out = __builtin_amdgcn_make_buffer_rsrc(a.chunk_state + (first + (int64_t)c * a.H) * a.N * a.P, 0,
-                                                                          a.N * a.P * 4, 0x00020000);
-#pragma unroll
-    for (int i = 0; i < kTiles; ++i) {
-      const int n0 = (wave + 4 * i) * 32;
-      if (NP < 128 && n0 >= NP) continue;           // (the wavefront has no rows)
-      // every operand of the tile's products first, so that their LDS reads overlap; high and low parts in chains of their own
-      bf16x8_t bf[Q / 16], hi[Q / 16], low[Q / 16];
-#pragma unroll
-      for (int kk = 0; kk < Q / 16; ++kk) {
-        const int at = (kk * 16 + r) * kSX + c0;
-        bf[kk] = read_tr8(Bs + (kk * 16 + r) * kBS + n0 + c0, 4 * kBS);
-        hi[kk] = read_tr8(xh + at, 4 * kSX);
-        low[kk] = read_tr8(xl + at, 4 * kSX);
-      }
-      __builtin_amdgcn_sched_barrier(0);
-      const int in_out = ((n0 + 4 * half) * a.P + p) * 4, at_out = p < a.P ? in_out : kOutside;
-      floatx16_t rest;
-#pragma unroll
-      for (int e = 0; e < 16; ++e) {
-        __builtin_amdgcn_raw_buffer_store_b32(pack_split(S[i][e]), out, at_out + (8 * (e >> 2) + (e & 3)) * a.P * 4, 0, 0);
-        S[i][e] *= decay;
-        rest[e] = 0.f;
-      }
-#pragma unroll
-      for (int kk = 0; kk < Q / 16; ++kk) {
-        S[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[kk], hi[kk], S[i], 0, 0, 0);
-        rest = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[kk], low[kk], rest, 0, 0, 0);
-      }
-#pragma unroll
-      for (int e = 0; e < 16; ++e) S[i][e] += rest[e];
-    }
-  };
-  fetch(set0, 0);
-  fetch(set1, 1);
-  for (int c = 0; c < chunks; c += 2) {
-    step(set0, c);
-    if (c + 1 < chunks) step(set1, c + 1);
-  }
-#pragma unroll
-  for (int i = 0; i < kTiles; ++i)
-#pragma unroll
-    for (int e = 0; e < 16; ++e) {
-      const int n = (wave + 4 * i) * 32 + 8 * (e >> 2) + 4 * half + (e & 3);
-      if (n < a.N && p < a.P) keep[(int64_t)n * a.P] = S[i][e];
-    }
-}
-
-// What a workgroup of the output kernel works on.
+// What a workgroup of kernels (2) and (4) works on.
 struct Unit {
   int head0, heads, grp, p0, lo, t0, rows, row0;
   int64_t chunk0;          // chunk index of head0
@@ -277,6 +160,113 @@ __device__ __forceinline__ bool unit_of(const ChunkArgs& a, const msa_seq_batch&
   u.row0 = u.lo + u.t0;
   u.chunk0 = ((int64_t)s * a.n_chunks + blockIdx.y) * a.H + u.head0;
   return u.t0 < n_tok;
+}
+
+template <int Q, int NP>
+__global__ __launch_bounds__(4 * Q) void ssd_local_kernel(ChunkArgs a, msa_seq_batch b) {
+  constexpr int kBS = NP + 8, kWaves = Q / 16, kTiles = (NP / 32 * 2 + kWaves - 1) / kWaves;
+  constexpr int kBX = Q * kBS > 2 * Q * kXS ? Q * kBS : 2 * Q * kXS;
+  extern __shared__ __align__(16) bf16_t sm[];
+  bf16_t* Bs = sm;                                  // [Q][kBS], until its fragments are in registers; then
+  bf16_t* xh = sm;                                  // [Q][kXS] high and
+  bf16_t* xl = xh + Q * kXS;                        // [Q][kXS] low parts of the weighted x
+  float* ws = reinterpret_cast<float*>(sm + kBX);   // [heads][Q]
+  Unit u;
+  if (!unit_of<Q>(a, b, u)) return;
+  const int inner = a.H * a.P, stride = (int)a.xbc_stride;
+  const bf16_t* src = a.xbc + (int64_t)u.row0 * a.xbc_stride;
+  RowTile<Q, NP, 4 * Q> tb;
+  RowTile<Q, kPB, 4 * Q> tx;
+  const typename RowTile<Q, kPB, 4 * Q>::Offsets off_x(stride, a.P - u.p0);
+  tb.load(typename RowTile<Q, NP, 4 * Q>::Offsets(stride, a.N), src + inner + u.grp * a.N, stride, u.rows, a.N);
+  tx.load(off_x, src + u.head0 * a.P + u.p0, stride, u.rows, a.P - u.p0);
+  for (int i = threadIdx.x; i < u.heads * Q; i += 4 * Q) {      // weights of the tokens at the chunk's end
+    const float* ac = a.acs + u.chunk0 * Q;
+    ws[i] = a.dts[u.chunk0 * Q + i] * __builtin_amdgcn_exp2f(ac[i / Q * Q + Q - 1] - ac[i]);
+  }
+  tb.store(Bs, kBS);
+  __syncthreads();
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), half = lane >> 5, l16 = lane & 15;
+  const int r = 8 * half + (l16 >> 2), c = (lane & 16) + (l16 & 3) * 4;
+  bf16x8_t bf[kTiles][Q / 16];                      // B^T operands of this wavefront's tiles, for every head
+  int out_at[kTiles];
+#pragma unroll
+  for (int i = 0; i < kTiles; ++i) {
+    const int tile = wave + kWaves * i, n0 = tile / 2 * 32, p = u.p0 + tile % 2 * 32 + (lane & 31), in = ((n0 + 4 * half) * a.P + p) * 4;
+    out_at[i] = p < a.P ? in : kOutside;
+    if (n0 < NP)
+#pragma unroll
+      for (int kk = 0; kk < Q / 16; ++kk) bf[i][kk] = read_tr8(Bs + (kk * 16 + r) * kBS + n0 + c, 4 * kBS);
+  }
+  for (int hh = 0; hh < u.heads; ++hh) {
+    __syncthreads();                                // the last reads of B or of the head before
+#pragma unroll
+    for (int k = 0; k < tx.kPieces; ++k) {          // x times its token's weight, split
+      const int i = threadIdx.x + k * 4 * Q, t = i / tx.kUnits, at = t * kXS + i % tx.kUnits * 8;
+      const float w = ws[hh * Q + t];
+      const u32x4_t xw = tx.w[k];
+      const float v[8] = {bf16lo(xw.x) * w, bf16hi(xw.x) * w, bf16lo(xw.y) * w, bf16hi(xw.y) * w,
+                          bf16lo(xw.z) * w, bf16hi(xw.z) * w, bf16lo(xw.w) * w, bf16hi(xw.w) * w};
+      bf16x8_t hi, low;
+      split8(v, hi, low);
+      *reinterpret_cast<bf16x8_t*>(xh + at) = hi;
+      *reinterpret_cast<bf16x8_t*>(xl + at) = low;
+    }
+    __syncthreads();
+    tx.load(off_x, src + min(u.head0 + hh + 1, a.H - 1) * a.P + u.p0, stride, u.rows, a.P - u.p0);
+    const __amdgpu_buffer_rsrc_t out = __builtin_amdgcn_make_buffer_rsrc(a.chunk_state + (u.chunk0 + hh) * a.N * a.P, 0, a.N * a.P * 4, 0x00020000);
+#pragma unroll
+    for (int i = 0; i < kTiles; ++i) {
+      const int tile = wave + kWaves * i, pb = tile % 2 * 32;
+      if (NP / 32 * 2 < kWaves && tile / 2 * 32 >= NP) continue;      // (the wavefront has no tile)
+      floatx16_t acc;
+#pragma unroll
+      for (int e = 0; e < 16; ++e) acc[e] = 0.f;
+#pragma unroll
+      for (int kk = 0; kk < Q / 16; ++kk) {
+        const int at = (kk * 16 + r) * kXS + pb + c;
+        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[i][kk], read_tr8(xh + at, 4 * kXS), acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(bf[i][kk], read_tr8(xl + at, 4 * kXS), acc, 0, 0, 0);
+      }
+#pragma unroll
+      for (int e = 0; e < 16; ++e)                  // row 8 (e / 4) + 4 half + e % 4 of the tile; rows behind N are not written
+        __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(acc[e]), out, out_at[i] + (8 * (e >> 2) + (e & 3)) * a.P * 4, 0, 0);
+    }
+  }
+}
+
+// Four state elements per thread (N P is a multiple of 8), a batch of chunks requested at a time.
+template <int Q>
+__global__ __launch_bounds__(256) void ssd_carry_kernel(ChunkArgs a, msa_seq_batch b) {
+  const int64_t per = (int64_t)a.N * a.P;
+  const int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * 4;
+  const int head = blockIdx.y, s = blockIdx.z;
+  if (i >= per) return;
+  const int n_tok = b.cu[s + 1] - b.cu[s], chunks = (n_tok + Q - 1) / Q;
+  float4* keep = reinterpret_cast<float4*>(a.state + ((int64_t)b.slot[s] * a.H + head) * per + i);
+  float4 S = *keep;
+  const int64_t first = (int64_t)s * a.n_chunks * a.H + head;
+  constexpr int kBatch = 8;
+  for (int c = 0; c < chunks; c += kBatch) {
+    float4 loc[kBatch];
+    float d[kBatch];
+    float4* at[kBatch];
+#pragma unroll
+    for (int k = 0; k < kBatch; ++k) {
+      const int64_t chunk = first + (int64_t)min(c + k, chunks - 1) * a.H;
+      at[k] = reinterpret_cast<float4*>(a.chunk_state + chunk * per + i);
+      loc[k] = *at[k];
+      d[k] = a.acs[chunk * Q + Q - 1];
+    }
+#pragma unroll
+    for (int k = 0; k < kBatch; ++k) {
+      if (c + k >= chunks) break;
+      *reinterpret_cast<uint4*>(at[k]) = make_uint4(pack_split(S.x), pack_split(S.y), pack_split(S.z), pack_split(S.w));
+      const float f = __builtin_amdgcn_exp2f(d[k]);
+      S = make_float4(f * S.x + loc[k].x, f * S.y + loc[k].y, f * S.z + loc[k].z, f * S.w + loc[k].w);
+    }
+  }
+  *keep = S;
 }
 
 template <int Q, int NP>
@@ -456,23 +446,26 @@ int chunk_tokens(int32_t N) { return N <= 128 ? 128 : 64; }
 template <int Q, int NP>
 int launch_chunked(ChunkArgs a, const msa_seq_batch& b, hipStream_t st) {
   constexpr int tile = Q * (NP + 8), x = Q * kXS, state = 2 * NP * kXS;
-  constexpr int lds2 = (tile + 2 * Q * kSX) * 2;
+  constexpr int lds2 = (tile > 2 * x ? tile : 2 * x) * 2 + kMaxHeads * Q * 4;
   constexpr int lds3 = ((tile > state ? tile : state) + x) * 2 + kMaxHeads * (2 * Q + (Q / 32) * (Q / 32 - 1) * 16) * 4;
   static_assert(lds2 <= 160 * 1024 && lds3 <= 160 * 1024, "tiles of a chunk must fit LDS");
-  // as many heads per workgroup as leave the output launch two workgroups per compute unit
+  // as many heads per workgroup as leave a launch two workgroups per compute unit
   const int per_group = a.H / a.G, blocks = (a.P + kPB - 1) / kPB;
   auto sets = [&](int h) { return (per_group + h - 1) / h; };
   int heads = std::min(kMaxHeads, per_group);
   while (heads > 1 && (int64_t)a.n_chunks * b.n_seq * a.G * blocks * sets(heads) < 2 * device_compute_units()) --heads;
   a.heads_per_wg = (per_group + sets(heads) - 1) / sets(heads);
   static std::atomic<int> raised2{0}, raised3{0};
-  MSA_HIP(raise_dynamic_lds_limit(raised2, reinterpret_cast<const void*>(ssd_state_kernel<Q, NP>), lds2));
+  MSA_HIP(raise_dynamic_lds_limit(raised2, reinterpret_cast<const void*>(ssd_local_kernel<Q, NP>), lds2));
   MSA_HIP(raise_dynamic_lds_limit(raised3, reinterpret_cast<const void*>(ssd_output_kernel<Q, NP>), lds3));
   ssd_decay_kernel<Q><<<dim3((a.H + 3) / 4, a.n_chunks, b.n_seq), 256, 0, st>>>(a, b);
   MSA_LAUNCH_CHECK();
-  ssd_state_kernel<Q, NP><<<dim3((unsigned)(a.H * ((a.P + kStateCols - 1) / kStateCols)), 1, b.n_seq), 256, lds2, st>>>(a, b);
+  const dim3 grid((unsigned)(a.G * blocks * sets(a.heads_per_wg)), a.n_chunks, b.n_seq);
+  ssd_local_kernel<Q, NP><<<grid, 4 * Q, lds2, st>>>(a, b);
   MSA_LAUNCH_CHECK();
-  ssd_output_kernel<Q, NP><<<dim3((unsigned)(a.G * blocks * sets(a.heads_per_wg)), a.n_chunks, b.n_seq), 4 * Q, lds3, st>>>(a, b);
+  ssd_carry_kernel<Q><<<dim3((a.N * a.P / 4 + 255) / 256, a.H, b.n_seq), 256, 0, st>>>(a, b);
+  MSA_LAUNCH_CHECK();
+  ssd_output_kernel<Q, NP><<<grid, 4 * Q, lds3, st>>>(a, b);
   MSA_LAUNCH_CHECK();
   return MSA_OK;
 }
