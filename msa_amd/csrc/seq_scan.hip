@@ -298,7 +298,7 @@ __global__ __launch_bounds__(64) void gru_carry_kernel(GruArgs a, msa_seq_batch 
   const int n_tok = b.cu[s + 1] - b.cu[s], chunks = (n_tok + kGruRows - 1) / kGruRows;
   float S = a.state[(int64_t)b.slot[s] * a.n + c];
   float2* ch = a.chunk + (int64_t)s * a.n_chunks * a.n + c;
-  constexpr int kBatch = 16;
+  constexpr int kBatch = 32;
   for (int i = 0; i < chunks; i += kBatch) {
     float2 t[kBatch];
 #pragma unroll
