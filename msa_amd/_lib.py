@@ -98,10 +98,30 @@ class RowsArgs(C.Structure):
                 ("taps", _vp), ("conv_bias", _vp), ("conv_state", _vp), ("conv_lo", _i32), ("conv_n", _i32), ("conv_k", _i32),
                 ("reserved2", _i32),
                 ("z_bias", _vp), ("u_bias", _vp), ("gru_state", _vp), ("out2", _vp), ("gru_n", _i32), ("reserved3", _i32),
-                ("slot", _vp)]
+                ("slot", _vp), ("glu_limit", _f32), ("glu_alpha", _f32), ("glu_shift", _f32), ("reserved4", _i32)]
 
 
-ROWS_PLAIN, ROWS_F32, ROWS_RESIDUAL, ROWS_MAMBA, ROWS_GRU = range(5)
+class QKRopeArgs(C.Structure):
+    """``msa_qk_rope_args``."""
+    _fields_ = [("q", _vp), ("k", _vp), ("v", _vp), ("q_stride", _i64), ("k_stride", _i64), ("v_stride", _i64), ("q_norm", _vp),
+                ("k_norm", _vp), ("freqs", _vp), ("q_out", _vp), ("k_cache", _vp), ("v_cache", _vp), ("Lcap", _i64), ("H", _i32),
+                ("G", _i32), ("D", _i32), ("E", _i32), ("n_pairs", _i32), ("eps", _f32)]
+
+
+class KVAttnArgs(C.Structure):
+    """``msa_kv_attn_args``."""
+    _fields_ = [("q", _vp), ("k_cache", _vp), ("v_cache", _vp), ("gate", _vp), ("out", _vp), ("Lcap", _i64), ("gate_stride", _i64),
+                ("max_keys", _i64), ("H", _i32), ("G", _i32), ("D", _i32), ("E", _i32), ("chunk", _i32), ("scale", _f32)]
+
+
+class DeltaArgs(C.Structure):
+    """``msa_delta_args``."""
+    _fields_ = [("qkv", _vp), ("a", _vp), ("b", _vp), ("gate", _vp), ("qkv_stride", _i64), ("a_stride", _i64), ("b_stride", _i64),
+                ("gate_stride", _i64), ("A_log", _vp), ("dt_bias", _vp), ("norm", _vp), ("state", _vp), ("out", _vp), ("H", _i32),
+                ("G", _i32), ("D", _i32), ("E", _i32), ("eps", _f32), ("reserved", _i32)]
+
+
+ROWS_PLAIN, ROWS_F32, ROWS_RESIDUAL, ROWS_MAMBA, ROWS_GRU, ROWS_GLU = range(6)
 _batch = C.POINTER(SeqBatch)
 
 # include/msa_seq.h
@@ -124,7 +144,18 @@ SEQ_SIGNATURES = {
     "msa_seq_latent_attn": (C.c_int, [_vp, _vp, _i64, _vp, _f32, _i32, _i32, _i32, _vp, _batch, _vp]),
     "msa_seq_latent_decode_workspace_bytes": (_sz, [_i32, _i32, _i32, _i64]),
     "msa_seq_latent_decode": (C.c_int, [_vp, _vp, _i64, _vp, _f32, _i32, _i32, _i32, _i64, _vp, _batch, _vp, _sz, _vp]),
-    "msa_seq_flash": (C.c_int, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _f32, _i32, _i32, _i32, _i32, _vp, _batch, _vp]),
+    "msa_seq_flash": (C.c_int, [_vp, _i64, _vp, _i64, _vp, _i64, _vp, _vp, _f32, _i32, _i32, _i32, _i32, _i32, _i32, _vp, _i64, _vp,
+                                _batch, _vp]),
+    "msa_seq_qk_rope_append": (C.c_int, [C.POINTER(QKRopeArgs), _i32, _batch, _vp]),
+    "msa_seq_kv_attn": (C.c_int, [C.POINTER(KVAttnArgs), _i32, _batch, _vp]),
+    "msa_seq_kv_decode_workspace_bytes": (_sz, [C.POINTER(KVAttnArgs), _i32]),
+    "msa_seq_kv_decode": (C.c_int, [C.POINTER(KVAttnArgs), _batch, _vp, _sz, _vp]),
+    "msa_seq_delta_scan": (C.c_int, [C.POINTER(DeltaArgs), _i32, _batch, _vp]),
+    "msa_seq_delta_chunked_workspace_bytes": (_sz, [C.POINTER(DeltaArgs), _i32, _i32]),
+    "msa_seq_delta_chunked": (C.c_int, [C.POINTER(DeltaArgs), _batch, _vp, _sz, _vp]),
+    "msa_seq_head_norm_gate": (C.c_int, [_vp, _vp, _i64, _vp, _f32, _i32, _i32, _i32, _i32, _vp]),
+    "msa_seq_rms_residual": (C.c_int, [_vp, _vp, _i64, _vp, _f32, _vp, _vp, _vp, _i32, _i32, _i32, _vp]),
+    "msa_seq_clamped_glu": (C.c_int, [_vp, _i64, _i32, _i32, _i32, _f32, _f32, _f32, _vp, _vp]),
     "msa_rows_linear": (C.c_int, [C.POINTER(RowsArgs), _i32, _vp]),
 }
 # entry points of include/msa_amd.h that libmsa_seq.so holds too (the error text is per library)

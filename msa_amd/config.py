@@ -2,8 +2,9 @@
 and the msa_config block of the checkpoint's config.json, src/utils/resave_model.py:33-50)."""
 from __future__ import annotations
 
-from dataclasses import dataclass, field
-from typing import Dict, List, Union
+import math
+from dataclasses import MISSING, dataclass, field
+from typing import Dict, List, Optional, Union
 
 QWEN3_TEMPLATE = {"prompt": "<|im_start|>user\n{prompt}<|im_end|>\n",
                   "response": "<|im_start|>assistant\n<think>\n{think_content}\n</think>\n\n{output}<|im_end|>"}
@@ -101,13 +102,16 @@ class MSAConfig:
 # ------------------------------------------------------------------------------ recurrent / latent-attention decoders
 def _fields(cls, d: dict, where: str):
     """Builds dataclass ``cls`` from ``d``; unknown or missing keys are an error that names the place."""
-    names = [f for f in cls.__dataclass_fields__]
-    unknown = sorted(set(d) - set(names))
+    fields = cls.__dataclass_fields__
+    unknown = sorted(set(d) - set(fields))
     if unknown:
         raise ValueError(f"{where}: unknown keys {unknown}")
+    missing = [n for n, f in fields.items() if n not in d and f.default is MISSING and f.default_factory is MISSING]
+    if missing:
+        raise ValueError(f"{where}: missing keys {missing}")
     try:
         return cls(**d)
-    except TypeError as e:
+    except ValueError as e:
         raise ValueError(f"{where}: {e}") from None
 
 
@@ -150,6 +154,97 @@ class LatentAttentionConfig:
 
 
 @dataclass
+class ChannelDeltaConfig:
+    """Delta rule with a decay per key channel: ``heads`` of ``vdim`` value dimensions over ``kv_heads`` queries and keys of
+    ``dim``, ``conv`` taps in front."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError(f"{self.heads} heads over {self.kv_heads} keys")
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+
+@dataclass
+class RotaryScalingConfig:
+    """Wavelengths above ``original / low`` are stretched by ``factor``, those below ``original / high`` kept, others blended."""
+    factor: float
+    low: float
+    high: float
+    original: float
+
+
+@dataclass
+class RotaryConfig:
+    """Rotary positions on the first ``dims`` dimensions of a head, dimension i paired with i + dims / 2."""
+    base: float
+    dims: int
+    scaling: Optional[RotaryScalingConfig] = None
+
+    def __post_init__(self):
+        if isinstance(self.scaling, dict):
+            self.scaling = _fields(RotaryScalingConfig, self.scaling, "scaling")
+        if self.dims < 0 or self.dims % 2:
+            raise ValueError(f"{self.dims} rotated dimensions")
+
+    def frequencies(self) -> List[float]:
+        """Radians per position of every pair."""
+        c, out = self.scaling, []
+        for i in range(self.dims // 2):
+            f = float(self.base) ** (-2 * i / self.dims)
+            if c is not None:
+                turns = c.original * f / (2 * math.pi)          # full turns over the original context
+                if turns < c.low:
+                    f /= c.factor
+                elif turns <= c.high:
+                    s = (turns - c.low) / (c.high - c.low) if c.high > c.low else 1.0
+                    f = (1 - s) * f / c.factor + s * f
+            out.append(f)
+        return out
+
+
+@dataclass
+class ChunkMaskConfig:
+    """A position sees the positions up to itself in its own stretch of ``size``, counted from the sequence's start."""
+    size: int
+
+    def __post_init__(self):
+        if self.size < 1:
+            raise ValueError(f"chunks of {self.size}")
+
+
+@dataclass
+class AttentionConfig:
+    """Grouped-query attention with query / key norms, rotary positions, a chunk mask (none: causal) and a sigmoid gate per
+    head; with ``kv_from`` the keys and values are those of an earlier layer."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot: Optional[RotaryConfig] = None
+    mask: Optional[ChunkMaskConfig] = None
+    kv_from: Optional[int] = None
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError(f"{self.heads} heads over {self.kv_heads} keys")
+        if isinstance(self.rot, dict):
+            self.rot = _fields(RotaryConfig, self.rot, "rot")
+        if isinstance(self.mask, dict):
+            self.mask = _fields(ChunkMaskConfig, self.mask, "mask")
+        if self.rot is not None and self.rot.dims > self.dim:
+            raise ValueError(f"{self.rot.dims} rotated of {self.dim} dimensions")
+
+
+@dataclass
 class DenseMLPConfig:
     ff: int
     kind: str = "dense"
@@ -159,14 +254,43 @@ class DenseMLPConfig:
             raise NotImplementedError(f"unsupported feed-forward {self.kind!r}")
 
 
-MIXER_CONFIGS = {"mamba2": Mamba2Config, "mingru": MinGRUConfig, "latent_attention": LatentAttentionConfig}
+@dataclass
+class ClampedGLUConfig(DenseMLPConfig):
+    """``g sigmoid(1.702 g) (u + 1)`` with the gate capped at ``limit`` and the up projection clamped to ``+-limit``."""
+    limit: float = field(kw_only=True)
+
+
+MIXER_CONFIGS = {"mamba2": Mamba2Config, "mingru": MinGRUConfig, "latent_attention": LatentAttentionConfig,
+                 "channel_delta": ChannelDeltaConfig, "attention": AttentionConfig}
+MixerConfig = Union[Mamba2Config, MinGRUConfig, LatentAttentionConfig, ChannelDeltaConfig, AttentionConfig]
 
 
 @dataclass
 class HybridLayerConfig:
     type: str
-    mixer: Union[Mamba2Config, MinGRUConfig, LatentAttentionConfig]
+    mixer: MixerConfig
     mlp: Union[DenseMLPConfig, None]
+
+
+def _layers(entries: List[dict], mlp_config=DenseMLPConfig) -> List[HybridLayerConfig]:
+    """The layer list of a ``config.json``."""
+    layers = []
+    for i, e in enumerate(entries):
+        where = f"layers[{i}]"
+        if e["type"] not in MIXER_CONFIGS:
+            raise NotImplementedError(f"{where}: unsupported mixer {e['type']!r}")
+        mlp = e.get("mlp")
+        layers.append(HybridLayerConfig(e["type"], _fields(MIXER_CONFIGS[e["type"]], e["mixer"], where + ".mixer"),
+                                        None if mlp is None else _fields(mlp_config, mlp, where + ".mlp")))
+    for i, layer in enumerate(layers):
+        m, j = layer.mixer, getattr(layer.mixer, "kv_from", None)
+        if j is None:
+            continue
+        if not 0 <= j < i or layers[j].type != layer.type or layers[j].mixer.kv_from is not None:
+            raise ValueError(f"layers[{i}]: no keys of its own in layer {j}")
+        if any(getattr(m, n) != getattr(layers[j].mixer, n) for n in ("kv_heads", "dim", "vdim")):
+            raise ValueError(f"layers[{i}]: heads differ from those of layer {j}")
+    return layers
 
 
 @dataclass
@@ -190,14 +314,7 @@ class HybridConfig:
 
     @classmethod
     def from_dict(cls, d: dict) -> "HybridConfig":
-        layers = []
-        for i, e in enumerate(d["layers"]):
-            where = f"layers[{i}]"
-            if e["type"] not in MIXER_CONFIGS:
-                raise NotImplementedError(f"{where}: unsupported mixer {e['type']!r}")
-            mlp = e.get("mlp")
-            layers.append(HybridLayerConfig(e["type"], _fields(MIXER_CONFIGS[e["type"]], e["mixer"], where + ".mixer"),
-                                            None if mlp is None else _fields(DenseMLPConfig, mlp, where + ".mlp")))
+        layers = _layers(d["layers"])
         loop = d.get("loop")
         loop = None if loop is None else _fields(LoopConfig, loop, "loop")
         if loop is not None and not (0 <= loop.start < loop.stop <= len(layers) and loop.times >= 1):
@@ -212,3 +329,21 @@ class HybridConfig:
             return [(i, None) for i in range(n)]
         return ([(i, None) for i in range(lp.start)] + [(i, t) for t in range(lp.times) for i in range(lp.start, lp.stop)]
                 + [(i, None) for i in range(lp.stop, n)])
+
+
+@dataclass
+class PostNormConfig:
+    """A decoder whose layers each name their mixer and feed-forward, with RMS norms on the sublayers' outputs only (the Sugizen
+    architecture)."""
+    vocab: int
+    width: int
+    layers: List[HybridLayerConfig]
+    norm_eps: float
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "PostNormConfig":
+        return cls(d["vocab"], d["width"], _layers(d["layers"], ClampedGLUConfig), d["norm"]["eps"])
+
+    @property
+    def runs(self) -> List[tuple]:
+        return [(i, None) for i in range(len(self.layers))]

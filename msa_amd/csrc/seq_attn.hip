@@ -1,34 +1,18 @@
-// Attention over latents with a learned sink in the softmax denominator.
+// Attention over latents with a learned sink in the softmax denominator, and the prefill kernel of all attention layers.
 //
 // Decoding works on the latents themselves: a head's query is multiplied by its key matrix beforehand, so all heads of a
 // token share one pass over the cached rows (scores and values come from the same bytes).  Prefill works on keys and
 // values expanded per head, which costs a fraction of the multiplications per (query, key) pair.
 //   latent_attn_kernel    any rank and type: a workgroup per (row, head), fp32 arithmetic throughout
 //   latent_decode_kernel  bf16: a workgroup per (row, range of keys, up to 32 heads), 16x16x32 MFMA, then a combine step
-//   flash_sink_kernel     bf16 prefill: 32 query columns per wavefront, transposed score tile, 32x32x16 MFMA
+//   flash_sink_kernel     bf16 prefill: 32 query columns per wavefront, transposed score tile, 32x32x16 MFMA; query heads may share
+//                         keys, positions may see their own chunk only, sinks and a gate per head are optional
 #include <algorithm>
 
-#include "seq_common.h"
+#include "seq_mfma.h"
 
 namespace {
 
-typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8_t;
-typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4_t;
-typedef __attribute__((__vector_size__(16 * sizeof(float)))) float floatx16_t;
-typedef unsigned int u32x4_t __attribute__((ext_vector_type(4)));
-typedef short shortx4_t __attribute__((ext_vector_type(4)));
-typedef __attribute__((address_space(3))) shortx4_t lds_shortx4_t;
-
-constexpr float kLog2e = 1.4426950408889634f;
-
-// Transposing LDS read of 16-bit elements: within each group of 16 lanes, lanes 4 r .. 4 r + 3 name the four 8-byte
-// pieces of row r (r = 0..3, 16 elements) and lane j receives element j of rows 0..3.
-__device__ __forceinline__ shortx4_t lds_read_tr16(const bf16_t* p) {
-  return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_shortx4_t*)(p));
-}
-__device__ __forceinline__ bf16x8_t join8(shortx4_t lo, shortx4_t hi) {
-  return __builtin_bit_cast(bf16x8_t, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
-}
 __device__ __forceinline__ float half_wave_max(float x) {
   const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
   return fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
@@ -342,12 +326,15 @@ struct FlashArgs {
   const bf16_t* k;
   const bf16_t* v;
   const int64_t* kv_off;
-  const float* sink;
+  const float* sink;         // or null
+  const bf16_t* gate;        // [rows, H] or null: outputs times sigmoid(gate)
   bf16_t* out;
-  int64_t q_stride, k_stride, v_stride;
+  int64_t q_stride, k_stride, v_stride, gate_stride;
   float scale_log2e;
-  int32_t H, D, E;
+  int32_t H, D, E, group;    // `group` query heads share a key head
+  int32_t chunk;             // positions see keys from their last multiple of this on (0: all)
 };
+constexpr float kNoScore = -1e30f;       // below every score, and finite
 constexpr int kFlashKeys = 64, kFlashRows = 128;
 
 // DP / EP: D and E padded to a multiple of 32 (zeros in LDS).  Two stages of K and V tiles in LDS; the next tile is
@@ -369,9 +356,14 @@ __global__ __launch_bounds__(256, (DP + EP <= 256) ? 2 : 1) void flash_sink_kern
   const int base = (int)b.pos[s];
   const int limit = ok ? base + tok + 1 : 0;
   const int kmax = base + min(n_tok, (blk + 1) * kFlashRows);
-  const int wave_min = base + blk * kFlashRows + wave * 32 + 1;      // the wavefront's first column sees this many keys
-  const bf16_t* kg = a.k + a.kv_off[s] * a.k_stride + (int64_t)head * a.D;
-  const bf16_t* vg = a.v + a.kv_off[s] * a.v_stride + (int64_t)head * a.E;
+  auto floor_of = [&](int pos) { return a.chunk ? pos / a.chunk * a.chunk : 0; };   // first key that position sees
+  const int kmin = floor_of(base + blk * kFlashRows), lowest = floor_of(base + tok);
+  // the wavefront's first column sees keys wave_lo .. wave_min - 1, its last one keys wave_hi_lo .. wave_max - 1
+  const int wave_first = __builtin_amdgcn_readfirstlane(blk * kFlashRows + wave * 32), wave_last = min(n_tok, wave_first + 32) - 1;
+  const int wave_min = base + wave_first + 1, wave_max = wave_first < n_tok ? base + wave_last + 1 : 0;
+  const int wave_lo = floor_of(base + wave_first), wave_hi_lo = floor_of(base + max(wave_last, 0));
+  const bf16_t* kg = a.k + a.kv_off[s] * a.k_stride + (int64_t)(head / a.group) * a.D;
+  const bf16_t* vg = a.v + a.kv_off[s] * a.v_stride + (int64_t)(head / a.group) * a.E;
 
   bf16x8_t qf[DP / 16];
   {
@@ -424,14 +416,13 @@ __global__ __launch_bounds__(256, (DP + EP <= 256) ? 2 : 1) void flash_sink_kern
   for (int d = 0; d < EP / 32; ++d)
 #pragma unroll
     for (int e = 0; e < 16; ++e) o[d][e] = 0.f;
-  float m = a.sink[head] * kLog2e, l = half == 0 ? 1.f : 0.f;       // the sink: first member of every column's softmax
-  fetch(0);
+  // a sink is the first member of every column's softmax
+  float m = a.sink ? a.sink[head] * kLog2e : kNoScore, l = a.sink && half == 0 ? 1.f : 0.f;
+  fetch(kmin);
   stash(0);
   __syncthreads();
   int stage = 0;
-  for (int k0 = 0; k0 < kmax; k0 += kFlashKeys, stage ^= 1) {
-    const bool more = k0 + kFlashKeys < kmax;
-    if (more) fetch(k0 + kFlashKeys);
+  auto multiply = [&](int k0) {
     const bf16_t* kb = kt + stage * kFlashKeys * kKS;
     const bf16_t* vb = vt + stage * kFlashKeys * kVS;
     floatx16_t sc[2];
@@ -447,13 +438,13 @@ __global__ __launch_bounds__(256, (DP + EP <= 256) ? 2 : 1) void flash_sink_kern
         sc[rb] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[i], sc[rb], 0, 0, 0);
       }
     float mx = -INFINITY;
-    if (k0 + kFlashKeys > wave_min) {
+    if (k0 + kFlashKeys > wave_min || k0 < wave_hi_lo) {
 #pragma unroll
       for (int rb = 0; rb < 2; ++rb)
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
           const int key = k0 + 32 * rb + 8 * (e >> 2) + 4 * half + (e & 3);
-          sc[rb][e] = key < limit ? sc[rb][e] : -INFINITY;
+          sc[rb][e] = key < limit && key >= lowest ? sc[rb][e] : -INFINITY;
         }
     }
 #pragma unroll
@@ -492,12 +483,18 @@ __global__ __launch_bounds__(256, (DP + EP <= 256) ? 2 : 1) void flash_sink_kern
           o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, pb, o[d], 0, 0, 0);
         }
       }
+  };
+  for (int k0 = kmin; k0 < kmax; k0 += kFlashKeys, stage ^= 1) {
+    const bool more = k0 + kFlashKeys < kmax;
+    if (more) fetch(k0 + kFlashKeys);
+    if (k0 < wave_max && k0 + kFlashKeys > wave_lo) multiply(k0);      // (the wavefront's columns see some of the tile)
     if (more) stash(stage ^ 1);
     __syncthreads();
   }
   l = half_wave_sum(l);
   if (!ok) return;
-  const float inv = 1.0f / l;
+  float inv = 1.0f / l;
+  if (a.gate) inv *= sigmoid_f(bf16_to_f32(a.gate[(int64_t)(lo + tok) * a.gate_stride + head]));
   bf16_t* dst = a.out + ((int64_t)(lo + tok) * a.H + head) * a.E;
 #pragma unroll
   for (int d = 0; d < EP / 32; ++d)
@@ -592,18 +589,19 @@ extern "C" int msa_seq_latent_decode(const void* q, const void* cache, int64_t L
 }
 
 extern "C" int msa_seq_flash(const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v, int64_t v_stride,
-                             const int64_t* kv_off, const float* sink, float scale, int32_t dtype, int32_t H, int32_t D, int32_t E,
-                             void* out, const msa_seq_batch* batch, void* stream) {
+                             const int64_t* kv_off, const float* sink, float scale, int32_t dtype, int32_t H, int32_t G, int32_t D, int32_t E,
+                             int32_t chunk, const void* gate, int64_t gate_stride, void* out, const msa_seq_batch* batch, void* stream) {
   MSA_CHECK_BATCH(batch, "msa_seq_flash");
   MSA_REQUIRE(dtype == MSA_BF16, "msa_seq_flash: bf16 only");
-  MSA_REQUIRE(q && k && v && kv_off && sink && out && scale > 0.f, "msa_seq_flash: null pointer or scale <= 0");
-  MSA_REQUIRE(H > 0 && D > 0 && E > 0 && D % 8 == 0 && E % 8 == 0 && D <= 256 && E <= 256, "msa_seq_flash: D=%d E=%d (multiples of 8 up to 256)", D, E);
-  MSA_REQUIRE(q_stride >= (int64_t)H * D && k_stride >= (int64_t)H * D && v_stride >= (int64_t)H * E && q_stride % 8 == 0 &&
+  MSA_REQUIRE(q && k && v && kv_off && out && scale > 0.f && chunk >= 0, "msa_seq_flash: null pointer, scale <= 0 or chunk < 0");
+  MSA_REQUIRE(H > 0 && G > 0 && H % G == 0 && (!gate || gate_stride >= H), "msa_seq_flash: %d heads over %d, or the gate's stride", H, G);
+  MSA_REQUIRE(D > 0 && E > 0 && D % 8 == 0 && E % 8 == 0 && D <= 256 && E <= 256, "msa_seq_flash: D=%d E=%d (multiples of 8 up to 256)", D, E);
+  MSA_REQUIRE(q_stride >= (int64_t)H * D && k_stride >= (int64_t)G * D && v_stride >= (int64_t)G * E && q_stride % 8 == 0 &&
                   k_stride % 8 == 0 && v_stride % 8 == 0 && k_stride <= (1 << 22) && v_stride <= (1 << 22) && (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)out) & 15) == 0,
               "msa_seq_flash: strides or alignment");
   MSA_REQUIRE(batch->n_seq <= 65535 && (batch->max_rows + kFlashRows - 1) / kFlashRows <= 65535, "msa_seq_flash: step too large");
-  const FlashArgs a{(const bf16_t*)q, (const bf16_t*)k, (const bf16_t*)v, kv_off, sink, (bf16_t*)out, q_stride, k_stride, v_stride,
-                    scale * kLog2e, H, D, E};
+  const FlashArgs a{(const bf16_t*)q, (const bf16_t*)k, (const bf16_t*)v, kv_off, sink, (const bf16_t*)gate, (bf16_t*)out, q_stride, k_stride,
+                    v_stride, gate_stride, scale * kLog2e, H, D, E, H / G, chunk};
   hipStream_t st = as_stream(stream);
   if (D <= 64 && E <= 64) return launch_flash<64, 64>(a, *batch, st);
   if (D <= 128 && E <= 64) return launch_flash<128, 64>(a, *batch, st);

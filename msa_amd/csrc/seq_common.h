@@ -34,6 +34,12 @@ __device__ __forceinline__ float tanh_f(float x) {
 // z (1 + tanh(y)) / 2 = z / (1 + exp(-2 y)), y = sqrt(2 / pi) (z + 0.044715 z^3)
 __device__ __forceinline__ float gelu_tanh_f(float z) { return z * sigmoid_f(1.5957691216057308f * (z + 0.044715f * z * z * z)); }
 
+// g sigmoid(alpha g) (u + shift) of a gate and an up projection, clamped from above and on both sides
+__device__ __forceinline__ float clamped_glu_f(float gate, float up, float limit, float alpha, float shift) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g * sigmoid_f(alpha * g) * (u + shift);
+}
+
 // VEC consecutive elements of a row (aligned to their size, at most 16 bytes), as fp32.
 template <typename T, int VEC>
 __device__ __forceinline__ void load_vec(const T* p, float (&v)[VEC]) {

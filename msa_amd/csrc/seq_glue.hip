@@ -1,5 +1,6 @@
 // Element-wise and row-wise steps of the recurrent / latent-attention decoder: gated residual + dynamic-tanh norm + token
-// shift in one pass, gelu, logit softcap, grouped RMS norm, latent norm + cache append.  All are bound by the bytes they
+// shift in one pass, residual + RMS norm, gelu, clamped gated units, logit softcap, grouped RMS norm, head norm + gate, latent
+// norm + cache append.  All are bound by the bytes they
 // move: the residual step reads the stream, one sublayer output and one gate and writes the stream and the next
 // sublayer's operands, with no intermediate tensor (dynamic tanh needs no row statistics, so a thread owns columns and
 // walks over tokens; the token before is the value it had in registers one step earlier).
@@ -219,6 +220,191 @@ __global__ __launch_bounds__(256) void latent_append_kernel(const T* __restrict_
   }
 }
 
+// A workgroup per row: x' = x + rms_norm(y) w, and the next sublayer's operand.  A row of up to 256 * kKeep vectors stays in
+// registers between its sums and the outputs; what lies behind is read again (by the thread that owns it).
+struct RmsResidual {
+  const float* x_in;
+  const void* y;
+  const float* w;
+  float* x_out;
+  const float* next_w;
+  void* h;
+  int64_t y_stride;
+  float eps;
+  int32_t W;
+};
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void rms_residual_kernel(RmsResidual a) {
+  constexpr int kKeep = 4;
+  __shared__ float red[2][4];
+  const int64_t row = blockIdx.x;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const float* xr = a.x_in + row * a.W;
+  const T* yr = a.y ? static_cast<const T*>(a.y) + row * a.y_stride : nullptr;
+  float* xo = a.y ? a.x_out + row * a.W : nullptr;
+  float x[kKeep][VEC], y[kKeep][VEC];
+  auto sum_of = [&](float v, int which) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+    if (lane == 0) red[which][wave] = v;
+    __syncthreads();
+    return red[which][0] + red[which][1] + red[which][2] + red[which][3];
+  };
+  float ssq = 0.f;
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k) {
+    const int i = (k * 256 + tid) * VEC;
+    if (i >= a.W) break;
+    load_vec<float, VEC>(xr + i, x[k]);
+    if (!a.y) continue;
+    load_vec<T, VEC>(yr + i, y[k]);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ssq += y[k][e] * y[k][e];
+  }
+  if (a.y) {
+    for (int i = (kKeep * 256 + tid) * VEC; i < a.W; i += 256 * VEC) {
+      float v[VEC];
+      load_vec<T, VEC>(yr + i, v);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ssq += v[e] * v[e];
+    }
+    ssq = sum_of(ssq, 0);
+  }
+  const float inv = a.y ? 1.0f / sqrtf(ssq / (float)a.W + a.eps) : 0.f;
+  const bool norm = a.next_w != nullptr;
+  float next_ssq = 0.f;
+  auto combine = [&](int i, float (&xv)[VEC], const float (&yv)[VEC]) {
+    float w[VEC];
+    load_vec<float, VEC>(a.w + i, w);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) xv[e] += yv[e] * inv * w[e];
+    store_vec<float, VEC>(xo + i, xv);
+  };
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k) {
+    const int i = (k * 256 + tid) * VEC;
+    if (i >= a.W) break;
+    if (a.y) combine(i, x[k], y[k]);
+    if (norm)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) next_ssq += x[k][e] * x[k][e];
+    else if (a.h) store_vec<T, VEC>(static_cast<T*>(a.h) + row * a.W + i, x[k]);
+  }
+  for (int i = (kKeep * 256 + tid) * VEC; i < a.W; i += 256 * VEC) {
+    float xv[VEC], yv[VEC];
+    load_vec<float, VEC>(xr + i, xv);
+    if (a.y) {
+      load_vec<T, VEC>(yr + i, yv);
+      combine(i, xv, yv);
+    }
+    if (norm)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) next_ssq += xv[e] * xv[e];
+    else if (a.h) store_vec<T, VEC>(static_cast<T*>(a.h) + row * a.W + i, xv);
+  }
+  if (!norm) return;
+  const float next_inv = 1.0f / sqrtf(sum_of(next_ssq, 1) / (float)a.W + a.eps);
+  auto finish = [&](int i, float (&v)[VEC]) {
+    float w[VEC];
+    load_vec<float, VEC>(a.next_w + i, w);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] *= next_inv * w[e];
+    store_vec<T, VEC>(static_cast<T*>(a.h) + row * a.W + i, v);
+  };
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k) {
+    const int i = (k * 256 + tid) * VEC;
+    if (i < a.W) finish(i, x[k]);
+  }
+  for (int i = (kKeep * 256 + tid) * VEC; i < a.W; i += 256 * VEC) {
+    float v[VEC];
+    load_vec<float, VEC>((xo ? xo : xr) + i, v);
+    finish(i, v);
+  }
+}
+
+// VEC pairs per thread and turn.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void clamped_glu_kernel(const T* __restrict__ in, int64_t stride, int64_t rows, int32_t n, float limit,
+                                                          float alpha, float shift, T* __restrict__ out) {
+  const int64_t per_row = n / VEC, total = rows * per_row;
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (int64_t)gridDim.x * 256) {
+    const int64_t row = i / per_row, c = i % per_row * VEC;
+    const T* p = in + row * stride + 2 * c;
+    float y[VEC];
+    if constexpr (VEC == 4) {
+      float v[8];
+      load_vec<T, 8>(p, v);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[e] = clamped_glu_f(v[2 * e], v[2 * e + 1], limit, alpha, shift);
+    } else {
+      y[0] = clamped_glu_f(to_f32<T>(p[0]), to_f32<T>(p[1]), limit, alpha, shift);
+    }
+    store_vec<T, VEC>(out + row * n + c, y);
+  }
+}
+
+// LANES lanes per (row, head), a head's columns VEC at a time.
+template <typename T, int VEC, int LANES>
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(T* o, const T* __restrict__ gate, int64_t gate_stride, const float* __restrict__ w,
+                                                             float eps, int64_t items, int32_t H, int32_t E) {
+  constexpr int kKeep = VEC == 8 ? 2 : 4;
+  const int64_t item = ((int64_t)blockIdx.x * 256 + threadIdx.x) / LANES;
+  const int lane = threadIdx.x % LANES;
+  const bool live = item < items;
+  T* at = o + item * E;
+  const T* gt = gate + item / H * gate_stride + item % H * E;
+  float keep[kKeep][VEC], ssq = 0.f;
+  if (live) {
+#pragma unroll
+    for (int k = 0; k < kKeep; ++k) {
+      const int i = (k * LANES + lane) * VEC;
+      if (i < E) {
+        load_vec<T, VEC>(at + i, keep[k]);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) ssq += keep[k][e] * keep[k][e];
+      }
+    }
+    for (int i = (kKeep * LANES + lane) * VEC; i < E; i += LANES * VEC) {
+      float x[VEC];
+      load_vec<T, VEC>(at + i, x);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ssq += x[e] * x[e];
+    }
+  }
+#pragma unroll
+  for (int d = LANES / 2; d > 0; d >>= 1) ssq += __shfl_xor(ssq, d);
+  if (!live) return;
+  const float inv = 1.0f / sqrtf(ssq / (float)E + eps);
+  auto finish = [&](int i, float (&x)[VEC]) {
+    float g[VEC], n[VEC];
+    load_vec<T, VEC>(gt + i, g);
+    load_vec<float, VEC>(w + i, n);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) x[e] *= inv * n[e] * sigmoid_f(g[e]);
+    store_vec<T, VEC>(at + i, x);
+  };
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k) {
+    const int i = (k * LANES + lane) * VEC;
+    if (i < E) finish(i, keep[k]);
+  }
+  for (int i = (kKeep * LANES + lane) * VEC; i < E; i += LANES * VEC) {
+    float x[VEC];
+    load_vec<T, VEC>(at + i, x);
+    finish(i, x);
+  }
+}
+
+template <typename T, int VEC>
+void launch_head_norm(T* o, const T* gate, int64_t gate_stride, const float* w, float eps, int64_t items, int32_t H, int32_t E, hipStream_t st) {
+  const int units = (E + VEC - 1) / VEC;
+  auto grid = [&](int lanes) { return (unsigned)((items * lanes + 255) / 256); };
+  if (units <= 8) head_norm_gate_kernel<T, VEC, 8><<<grid(8), 256, 0, st>>>(o, gate, gate_stride, w, eps, items, H, E);
+  else if (units <= 16) head_norm_gate_kernel<T, VEC, 16><<<grid(16), 256, 0, st>>>(o, gate, gate_stride, w, eps, items, H, E);
+  else head_norm_gate_kernel<T, VEC, 64><<<grid(64), 256, 0, st>>>(o, gate, gate_stride, w, eps, items, H, E);
+}
+
 int grid_for(int64_t items) { return (int)std::min<int64_t>(std::max<int64_t>(1, (items + 255) / 256), 8192); }
 
 }  // namespace
@@ -324,6 +510,62 @@ extern "C" int msa_seq_latent_append(const void* in, int64_t in_stride, const fl
   } else {
     if (vec) latent_append_kernel<float, 8><<<grid, 256, 0, st>>>((const float*)in, in_stride, w, eps, rank, (float*)cache, Lcap, *batch);
     else latent_append_kernel<float, 1><<<grid, 256, 0, st>>>((const float*)in, in_stride, w, eps, rank, (float*)cache, Lcap, *batch);
+  }
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+
+extern "C" int msa_seq_rms_residual(const float* x_in, const void* y, int64_t y_stride, const float* w, float eps, float* x_out,
+                                    const float* next_w, void* h, int32_t dtype, int32_t rows, int32_t W, void* stream) {
+  MSA_REQUIRE(x_in && rows > 0 && W > 0 && (y || h), "msa_seq_rms_residual: null stream, rows=%d or W=%d", rows, W);
+  MSA_REQUIRE(!y || (w && x_out && y_stride >= W), "msa_seq_rms_residual: a sublayer output needs its norm, a stride of at least W and x_out");
+  MSA_REQUIRE(!next_w || h, "msa_seq_rms_residual: norm without an output");
+  MSA_CHECK_DTYPE(dtype, "msa_seq_rms_residual");
+  const RmsResidual a{x_in, y, w, x_out, next_w, h, y_stride, eps, W};
+  const bool vec = vec_ok(4, {x_in, y, w, x_out, next_w, h}, {W, y_stride});
+  hipStream_t st = as_stream(stream);
+  if (dtype == MSA_BF16) {
+    if (vec) rms_residual_kernel<bf16_t, 4><<<rows, 256, 0, st>>>(a);
+    else rms_residual_kernel<bf16_t, 1><<<rows, 256, 0, st>>>(a);
+  } else {
+    if (vec) rms_residual_kernel<float, 4><<<rows, 256, 0, st>>>(a);
+    else rms_residual_kernel<float, 1><<<rows, 256, 0, st>>>(a);
+  }
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+
+extern "C" int msa_seq_clamped_glu(const void* in, int64_t in_stride, int32_t dtype, int32_t rows, int32_t n, float limit, float alpha,
+                                   float shift, void* out, void* stream) {
+  MSA_REQUIRE(in && out && rows > 0 && n > 0 && in_stride >= 2LL * n && limit >= 0.f, "msa_seq_clamped_glu: bad arguments");
+  MSA_CHECK_DTYPE(dtype, "msa_seq_clamped_glu");
+  const bool vec = vec_ok(8, {in, out}, {in_stride}) && n % 4 == 0;
+  const int grid = grid_for((int64_t)rows * n / (vec ? 4 : 1));
+  hipStream_t st = as_stream(stream);
+  if (dtype == MSA_BF16) {
+    if (vec) clamped_glu_kernel<bf16_t, 4><<<grid, 256, 0, st>>>((const bf16_t*)in, in_stride, rows, n, limit, alpha, shift, (bf16_t*)out);
+    else clamped_glu_kernel<bf16_t, 1><<<grid, 256, 0, st>>>((const bf16_t*)in, in_stride, rows, n, limit, alpha, shift, (bf16_t*)out);
+  } else {
+    if (vec) clamped_glu_kernel<float, 4><<<grid, 256, 0, st>>>((const float*)in, in_stride, rows, n, limit, alpha, shift, (float*)out);
+    else clamped_glu_kernel<float, 1><<<grid, 256, 0, st>>>((const float*)in, in_stride, rows, n, limit, alpha, shift, (float*)out);
+  }
+  MSA_LAUNCH_CHECK();
+  return MSA_OK;
+}
+
+extern "C" int msa_seq_head_norm_gate(void* o, const void* gate, int64_t gate_stride, const float* norm, float eps, int32_t dtype, int32_t rows,
+                                      int32_t H, int32_t E, void* stream) {
+  MSA_REQUIRE(o && gate && norm && rows > 0 && H > 0 && E > 0 && gate_stride >= (int64_t)H * E, "msa_seq_head_norm_gate: bad arguments");
+  MSA_CHECK_DTYPE(dtype, "msa_seq_head_norm_gate");
+  const bool vec = vec_ok(8, {o, gate, norm}, {gate_stride, E});
+  const int64_t items = (int64_t)rows * H;
+  hipStream_t st = as_stream(stream);
+  if (dtype == MSA_BF16) {
+    if (vec) launch_head_norm<bf16_t, 8>((bf16_t*)o, (const bf16_t*)gate, gate_stride, norm, eps, items, H, E, st);
+    else launch_head_norm<bf16_t, 1>((bf16_t*)o, (const bf16_t*)gate, gate_stride, norm, eps, items, H, E, st);
+  } else {
+    if (vec) launch_head_norm<float, 8>((float*)o, (const float*)gate, gate_stride, norm, eps, items, H, E, st);
+    else launch_head_norm<float, 1>((float*)o, (const float*)gate, gate_stride, norm, eps, items, H, E, st);
   }
   MSA_LAUNCH_CHECK();
   return MSA_OK;

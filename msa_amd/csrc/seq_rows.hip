@@ -1,5 +1,5 @@
 // Weight-streaming linear for the rows of a decode step (M <= 16, bf16), with the recurrent decoder's element-wise work in
-// the epilogue: gelu, softcap, the gated residual with the next norm and token shift, the causal convolution, the minimal
+// the epilogue: gelu, clamped gated units, softcap, the gated residual with the next norm and token shift, the causal convolution, the minimal
 // gated recurrence.  Like the skinny linear of the attention model a workgroup owns a few 16-row groups of the weights and
 // splits K over its wavefronts (16x16x32 MFMA: the 16 activation rows are exactly one operand); partial sums meet in LDS
 // and are added in wavefront order.  Everything behind the sums is element-wise in this model (dynamic tanh has no row
@@ -7,13 +7,9 @@
 #include <algorithm>
 #include <type_traits>
 
-#include "seq_common.h"
+#include "seq_mfma.h"
 
 namespace {
-
-typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8_t;
-typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4_t;
-typedef unsigned int u32x4_t __attribute__((ext_vector_type(4)));
 
 constexpr int kMaxWaves = 16;
 constexpr int kGruGroup = 16;
@@ -48,7 +44,7 @@ struct Finish<MSA_ROWS_MAMBA> {
     if (c < 0 || c >= a.conv_n) return;
     const float* kp = a.conv_state + (int64_t)a.slot[m] * (a.conv_k - 1) * a.conv_n + c;
     const float* tp = a.taps + (int64_t)c * a.conv_k;
-    bias = a.conv_bias[c];
+    bias = a.conv_bias ? a.conv_bias[c] : 0.f;
 #pragma unroll
     for (int j = 0; j < kTaps; ++j) {
       if (j + 1 < a.conv_k && j < kTaps - 1) keep[j] = kp[(int64_t)j * a.conv_n];
@@ -108,6 +104,16 @@ struct Finish<MSA_ROWS_RESIDUAL> {
     if (!a.shift) return;
     a.prev[(int64_t)a.slot[m] * a.N + n] = h;
     static_cast<bf16_t*>(a.h_shift)[at] = f32_to_bf16(h + (before - h) * mix);
+  }
+};
+
+// A (gate, up) pair of neighbouring columns, in the lane of the even one.
+template <>
+struct Finish<MSA_ROWS_GLU> {
+  __device__ __forceinline__ void load(const msa_rows_args& a, int m, int n) {}
+  __device__ __forceinline__ void apply(const msa_rows_args& a, int m, int n, float gate, float up) const {
+    if (n & 1) return;
+    static_cast<bf16_t*>(a.out)[m * a.out_stride + (n >> 1)] = f32_to_bf16(clamped_glu_f(gate, up, a.glu_limit, a.glu_alpha, a.glu_shift));
   }
 };
 
@@ -203,8 +209,13 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_linear_kernel(msa_rows_ar
     const int r = o >> 8, i = o & 255;
     const int m = row_of(i), nr = 16 * r + col_of(i), n = n_base + nr;
     if (m >= a.M || nr >= rows_w) continue;
-    if (o != tid) fin.load(a, m, n);
-    fin.apply(a, m, n, (int64_t)grp * a.N + n, total(r, i));
+    if constexpr (EPI == MSA_ROWS_GLU) {    // (rows come in pairs: the neighbouring column is in this wavefront, four lanes on)
+      const float v = total(r, i), up = __shfl_xor(v, 4);
+      fin.apply(a, m, n, v, up);
+    } else {
+      if (o != tid) fin.load(a, m, n);
+      fin.apply(a, m, n, (int64_t)grp * a.N + n, total(r, i));
+    }
   }
 }
 
@@ -282,7 +293,12 @@ __global__ __launch_bounds__(kMaxWaves * 64) void rows_stream_kernel(msa_rows_ar
     float v = (buf[4 * quarter][o] + buf[4 * quarter + 1][o]) + (buf[4 * quarter + 2][o] + buf[4 * quarter + 3][o]);
     v += __shfl_xor(v, 1);
     v += __shfl_xor(v, 2);
-    if (mine) fin.apply(a, m, n, n, v);
+    if constexpr (EPI == MSA_ROWS_GLU) {
+      const float up = __shfl_xor(v, 16);
+      if (mine) fin.apply(a, m, n, v, up);
+    } else if (mine) {
+      fin.apply(a, m, n, n, v);
+    }
   };
   for (int item = i0; item < i1; item += kStages) {       // whole rounds: items behind the last read zeros and store nothing
     step(item, std::integral_constant<int, 0>{});
@@ -297,6 +313,7 @@ int launch_stream(const msa_rows_args& a, hipStream_t st) {
   const int n_a = std::min(a.n_b, a.N), n_b = a.N - n_a;
   const int iters = (a.N + 16 * cus - 1) / (16 * cus);
   int rpi = std::min(16, std::max(1, (a.N + iters * cus - 1) / (iters * cus)));
+  if (EPI == MSA_ROWS_GLU) rpi = (rpi + 1) & ~1;                      // pairs stay together
   auto split = [&] { return (n_a + rpi - 1) / rpi + (n_b + rpi - 1) / rpi; };   // the second operand's rows start an item of their own
   while (rpi < 16 && split() > iters * cus) ++rpi;
   const int items_a = (n_a + rpi - 1) / rpi, items = split();
@@ -347,8 +364,11 @@ extern "C" int msa_rows_linear(const msa_rows_args* args, int32_t epilogue, void
       MSA_REQUIRE(!a.shift || (a.norm.w && a.prev && a.h_shift && a.slot), "msa_rows_linear: shift arguments");
       break;
     case MSA_ROWS_MAMBA:
-      MSA_REQUIRE(a.out && a.out_stride >= a.N && a.groups == 1 && a.taps && a.conv_bias && a.slot && a.conv_k >= 1 && a.conv_lo >= 0 &&
+      MSA_REQUIRE(a.out && a.out_stride >= a.N && a.groups == 1 && a.taps && a.slot && a.conv_k >= 1 && a.conv_lo >= 0 &&
                       a.conv_n > 0 && a.conv_lo + a.conv_n <= a.n_b && (a.conv_k == 1 || a.conv_state), "msa_rows_linear: convolution arguments");
+      break;
+    case MSA_ROWS_GLU:
+      MSA_REQUIRE(a.out && a.N % 2 == 0 && a.out_stride >= a.N / 2 && a.groups == 1 && !two, "msa_rows_linear: gated unit arguments");
       break;
     case MSA_ROWS_GRU:
       MSA_REQUIRE(a.out2 && a.z_bias && a.u_bias && a.gru_state && a.slot && a.groups == 1 && a.gru_n > 0 &&
@@ -367,6 +387,7 @@ extern "C" int msa_rows_linear(const msa_rows_args* args, int32_t epilogue, void
   MSA_REQUIRE(!two || a.n_b % rows_per_wg == 0, "msa_rows_linear: n_b=%d must be a multiple of %d", a.n_b, rows_per_wg);
   if (R == 1 && !two && a.groups == 1 && (a.N + 15) / 16 < device_compute_units())
     rows_per_wg = std::min(16, std::max(8, (a.N + device_compute_units() - 1) / device_compute_units()));
+  if (epilogue == MSA_ROWS_GLU) rows_per_wg = (rows_per_wg + 1) & ~1;
   const int64_t wgs = (int64_t)((a.N + rows_per_wg - 1) / rows_per_wg) * a.groups;
   const int kUnit = 32 * (R == 3 ? kVectors<3> : kVectors<1>);
   const int units = (a.K + kUnit - 1) / kUnit;
@@ -379,6 +400,7 @@ extern "C" int msa_rows_linear(const msa_rows_args* args, int32_t epilogue, void
   if (a.groups == 1 && a.K > 512 && a.K <= 4096 && a.N >= 2 * 16 * device_compute_units()) {
     if (epilogue == MSA_ROWS_PLAIN) return launch_stream<MSA_ROWS_PLAIN>(a, st);
     if (epilogue == MSA_ROWS_F32) return launch_stream<MSA_ROWS_F32>(a, st);
+    if (epilogue == MSA_ROWS_GLU) return launch_stream<MSA_ROWS_GLU>(a, st);
     if (epilogue == MSA_ROWS_MAMBA && a.K <= 2560) return launch_stream<MSA_ROWS_MAMBA>(a, st);
   }
   switch (epilogue * 4 + R) {
@@ -390,6 +412,8 @@ extern "C" int msa_rows_linear(const msa_rows_args* args, int32_t epilogue, void
     case MSA_ROWS_RESIDUAL * 4 + 2: return launch_rows<MSA_ROWS_RESIDUAL, 2>(a, waves, rows_per_wg, st);
     case MSA_ROWS_MAMBA * 4 + 1: return launch_rows<MSA_ROWS_MAMBA, 1>(a, waves, rows_per_wg, st);
     case MSA_ROWS_MAMBA * 4 + 2: return launch_rows<MSA_ROWS_MAMBA, 2>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_GLU * 4 + 1: return launch_rows<MSA_ROWS_GLU, 1>(a, waves, rows_per_wg, st);
+    case MSA_ROWS_GLU * 4 + 2: return launch_rows<MSA_ROWS_GLU, 2>(a, waves, rows_per_wg, st);
     case MSA_ROWS_GRU * 4 + 3: return launch_rows<MSA_ROWS_GRU, 3>(a, waves, rows_per_wg, st);
   }
   msa_set_error("msa_rows_linear: no kernel for epilogue %d with %d row groups", epilogue, R);

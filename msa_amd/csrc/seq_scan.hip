@@ -26,7 +26,7 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(const T* __restrict__ in
   float* keep = state + (int64_t)b.slot[s] * (K - 1) * C + c;
   const T* src = in + (int64_t)lo * in_stride + c;
   const float* tp = taps + (int64_t)c * K;
-  const float bs = bias[c];
+  const float bs = bias ? bias[c] : 0.f;
   // Only the workgroup of the first rows reads the kept inputs, and only it replaces them; portions shorter than the
   // taps push them along.  (Rows t < K - 1 are in that workgroup as long as K - 1 <= kConvRows, which the host checks.)
   for (int t = t0; t < t1; ++t) {
@@ -57,12 +57,12 @@ __global__ __launch_bounds__(256) void conv_silu_vec_kernel(const T* __restrict_
   const int t1 = min(n, t0 + kConvRows);
   float* keep = state + (int64_t)b.slot[s] * (K - 1) * C + c;
   const T* src = in + (int64_t)lo * in_stride + c;
-  float tp[K][8], bs[8], win[K - 1][8];
+  float tp[K][8], bs[8] = {}, win[K - 1][8];
 #pragma unroll
   for (int e = 0; e < 8; ++e)
 #pragma unroll
     for (int j = 0; j < K; ++j) tp[j][e] = taps[(int64_t)(c + e) * K + j];
-  load_vec<float, 8>(bias + c, bs);
+  if (bias) load_vec<float, 8>(bias + c, bs);
   auto input = [&](int u, float (&x)[8]) {                   // input u of the sequence's new tokens, or a kept one (u < 0)
     if (u >= 0) load_vec<T, 8>(src + u * in_stride, x);
     else load_vec<float, 8>(keep + (int64_t)(K - 1 + u) * C, x);
@@ -404,7 +404,7 @@ extern "C" int msa_seq_conv_silu(const void* in, int64_t in_stride, const float*
                                  int32_t K, float* state, void* out, int64_t out_stride, const msa_seq_batch* batch, void* stream) {
   MSA_CHECK_BATCH(batch, "msa_seq_conv_silu");
   MSA_CHECK_DTYPE(dtype, "msa_seq_conv_silu");
-  MSA_REQUIRE(in && taps && bias && out && C > 0 && in_stride >= C && out_stride >= C, "msa_seq_conv_silu: bad arguments");
+  MSA_REQUIRE(in && taps && out && C > 0 && in_stride >= C && out_stride >= C, "msa_seq_conv_silu: bad arguments");
   MSA_REQUIRE(K >= 1 && K - 1 <= kConvRows && (K == 1 || state), "msa_seq_conv_silu: K=%d (1..%d taps)", K, kConvRows + 1);
   MSA_REQUIRE(batch->n_seq <= 65535 && (batch->max_rows + kConvRows - 1) / kConvRows <= 65535, "msa_seq_conv_silu: step too large");
   if (dtype == MSA_BF16)

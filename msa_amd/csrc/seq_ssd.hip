@@ -19,38 +19,12 @@
 // the transposing read.
 #include <algorithm>
 
-#include "seq_common.h"
+#include "seq_mfma.h"
 
 namespace {
 
-typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8_t;
-typedef __attribute__((__vector_size__(16 * sizeof(float)))) float floatx16_t;
-typedef unsigned int u32x4_t __attribute__((ext_vector_type(4)));
-typedef unsigned int u32x2_t __attribute__((ext_vector_type(2)));
-typedef short shortx4_t __attribute__((ext_vector_type(4)));
-typedef __attribute__((address_space(3))) shortx4_t lds_shortx4_t;
-
-constexpr float kLog2e = 1.4426950408889634f;
 constexpr int kPB = 64;                  // state columns (p) per workgroup
 constexpr int kXS = kPB + 8;             // LDS row stride of [.., p] tiles
-
-// Eight rows (two reads of four, `gap` rows apart in LDS elements) of a 16-bit tile, transposed: see flash_attn.hip.
-__device__ __forceinline__ bf16x8_t read_tr8(const bf16_t* p, int gap) {
-  const shortx4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_shortx4_t*)(p));
-  const shortx4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_shortx4_t*)(p + gap));
-  return __builtin_bit_cast(bf16x8_t, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
-}
-// fp32 values as bf16 operands: high part and what it leaves over.
-__device__ __forceinline__ void split8(const float (&v)[8], bf16x8_t& hi, bf16x8_t& lo) {
-  uint32_t h[4], l[4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    h[i] = pack_bf16x2(v[2 * i], v[2 * i + 1]);
-    l[i] = pack_bf16x2(v[2 * i] - bf16lo(h[i]), v[2 * i + 1] - bf16hi(h[i]));
-  }
-  hi = __builtin_bit_cast(bf16x8_t, make_uint4(h[0], h[1], h[2], h[3]));
-  lo = __builtin_bit_cast(bf16x8_t, make_uint4(l[0], l[1], l[2], l[3]));
-}
 
 struct ChunkArgs {
   const bf16_t* xbc;
@@ -98,7 +72,6 @@ __global__ __launch_bounds__(256) void ssd_decay_kernel(ChunkArgs a, msa_seq_bat
 // All global accesses inside the loops below go through buffer resources whose extent is the valid rows: what lies outside
 // reads as zero and is not written, nothing is conditional, and the compiler can count the loads and stores in flight (behind a
 // conditional one it would wait for every store of the step before).
-constexpr int kOutside = 0x40000000;
 __device__ __forceinline__ __amdgpu_buffer_rsrc_t rows_rsrc(const bf16_t* p, int rows, int64_t stride, int n) {
   return __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t*>(p), 0, __builtin_amdgcn_readfirstlane((int)((rows - 1) * stride + n) * 2), 0x00020000);
 }

@@ -7,13 +7,18 @@ from typing import Callable, Dict
 
 import torch
 
-from .config import HybridConfig, MSAConfig
+from .config import HybridConfig, MSAConfig, PostNormConfig
 from .weights import load_tensors
 
 
 def _build_hybrid(config: dict, tensors, dtype, device):
     from .hybrid import HybridForCausalLM
     return HybridForCausalLM.from_tensors(HybridConfig.from_dict(config), tensors, dtype, device)
+
+
+def _build_postnorm(config: dict, tensors, dtype, device):
+    from .postnorm import PostNormForCausalLM
+    return PostNormForCausalLM.from_tensors(PostNormConfig.from_dict(config), tensors, dtype, device)
 
 
 def _build_msa(config: dict, tensors, dtype, device):
@@ -28,7 +33,7 @@ def _build_msa(config: dict, tensors, dtype, device):
 
 
 # architecture -> builder(config dict, {name: tensor}, dtype, device)
-ARCHITECTURES: Dict[str, Callable] = {"Gevonex": _build_hybrid, "MSAForCausalLM": _build_msa}
+ARCHITECTURES: Dict[str, Callable] = {"Gevonex": _build_hybrid, "Sugizen": _build_postnorm, "MSAForCausalLM": _build_msa}
 
 
 def architecture(config: dict) -> str:

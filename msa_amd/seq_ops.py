@@ -72,6 +72,13 @@ class StepBatch:
         self.c = _lib.SeqBatch(ptr(self.cu), ptr(self.row_seq), ptr(self.slot), ptr(self.pos), n, self.rows, self.max_rows, 0)
         self.ref = C.byref(self.c)
         self.max_keys = max(p + c for p, c in zip(positions, counts))     # longest sequence at the end of the step
+        self._row_at = {}
+
+    def cache_rows(self, capacity: int) -> torch.Tensor:
+        """First row of every sequence in a cache of ``capacity`` rows a slot (int64, on the device)."""
+        if capacity not in self._row_at:
+            self._row_at[capacity] = self.slot.to(torch.int64) * capacity
+        return self._row_at[capacity]
 
 
 @dataclass
@@ -124,6 +131,42 @@ def residual_norm(x: torch.Tensor, batch: StepBatch, dtype: torch.dtype, y=None,
     return (x if y is None else x_out), h, hs
 
 
+def rms_residual(x: torch.Tensor, dtype: torch.dtype, y=None, w=None, eps: float = 0.0, next_w=None, out=None, want_h: bool = True):
+    """``(x', h)``: ``x' = x + rms_norm(y) * w`` (``x`` itself without ``y``; into ``out``, which may be ``x``), and ``h = x'``, or
+    ``rms_norm(x') * next_w``, in ``dtype``."""
+    _dense(x, out)
+    T, W = x.shape
+    if x.dtype != torch.float32 or (out is not None and (out.shape != x.shape or out.dtype != torch.float32)):
+        raise ValueError("the residual stream is fp32 [rows, W]")
+    if y is not None:
+        _f32(W, w)
+        if y.shape != x.shape or y.dtype != dtype:
+            raise ValueError("sublayer output must be [rows, W] of the activations' type")
+        out = torch.empty_like(x) if out is None else out
+    _f32(W, next_w)
+    h = torch.empty((T, W), dtype=dtype, device=x.device) if want_h or next_w is not None else None
+    _check(_lib.load_seq().msa_seq_rms_residual(ptr(x), ptr(y), _rows(y) if y is not None else 0, ptr(w), eps, ptr(out), ptr(next_w), ptr(h),
+                                                dtype_code(dtype), T, W, _stream()), "msa_seq_rms_residual")
+    return (x if y is None else out), h
+
+
+GLU_ALPHA, GLU_SHIFT = 1.702, 1.0
+
+
+def interleave_pairs(gate_w: torch.Tensor, up_w: torch.Tensor) -> torch.Tensor:
+    """Weight rows in (gate, up) pairs."""
+    return torch.stack([gate_w, up_w], dim=1).reshape(2 * gate_w.shape[0], gate_w.shape[1]).contiguous()
+
+
+def clamped_glu(gu: torch.Tensor, limit: float, alpha: float = GLU_ALPHA, shift: float = GLU_SHIFT) -> torch.Tensor:
+    """``g sigmoid(alpha g) (u + shift)`` of rows of (gate, up) pairs, the gate capped at ``limit``, up clamped to ``+-limit``."""
+    T, n = gu.shape[0], gu.shape[1] // 2
+    out = torch.empty((T, n), dtype=gu.dtype, device=gu.device)
+    _check(_lib.load_seq().msa_seq_clamped_glu(ptr(gu), _rows(gu), dtype_code(gu.dtype), T, n, limit, alpha, shift, ptr(out), _stream()),
+           "msa_seq_clamped_glu")
+    return out
+
+
 def gelu_(y: torch.Tensor) -> torch.Tensor:
     """tanh-form gelu in place on a ``[rows, n]`` column range."""
     _check(_lib.load_seq().msa_seq_gelu(ptr(y), _rows(y), dtype_code(y.dtype), y.shape[0], y.shape[1], _stream()), "msa_seq_gelu")
@@ -149,7 +192,7 @@ def join(x: torch.Tensor, x0: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
     return out
 
 
-def conv_silu(x: torch.Tensor, taps: torch.Tensor, bias: torch.Tensor, state: torch.Tensor, batch: StepBatch) -> torch.Tensor:
+def conv_silu(x: torch.Tensor, taps: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor, batch: StepBatch) -> torch.Tensor:
     """Causal per-channel convolution + silu of ``x [rows, C]``; ``state [slots, K - 1, C]`` is updated."""
     T, Cn = x.shape
     K = taps.shape[1]
@@ -194,6 +237,40 @@ def group_rmsnorm(v: torch.Tensor, w: torch.Tensor, parts: int, eps: float) -> t
     out = torch.empty_like(v)
     _check(_lib.load_seq().msa_seq_group_rmsnorm(ptr(v), dtype_code(v.dtype), T, n, parts, ptr(w), eps, ptr(out), _stream()),
            "msa_seq_group_rmsnorm")
+    return out
+
+
+DELTA_CHUNKED_ROWS = 64    # portions from this many tokens on are cut into chunks
+
+
+def delta_chunked_ok(dtype, D: int, E: int) -> bool:
+    return False
+
+
+def delta(qkv, a, b, gate, A_log, dt_bias, norm, eps: float, H: int, G: int, D: int, E: int, state, batch: StepBatch,
+          chunked: bool = False) -> torch.Tensor:
+    """Normed and gated read-outs ``[rows, H E]`` of the delta rule with a decay per key channel; ``qkv [rows, 2 G D + H E]``,
+    ``a [rows, H D]``, ``b [rows, H]``, ``gate [rows, H E]``; ``state [slots, H, D, E]`` fp32 is updated.  ``chunked`` takes the
+    matrix-core form (bf16)."""
+    T = batch.rows
+    _f32(H, A_log)
+    _f32(H * D, dt_bias)
+    _f32(E, norm)
+    _dense(state)
+    if state.dtype != torch.float32 or tuple(state.shape[1:]) != (H, D, E) or state.shape[0] <= max(batch.slots):
+        raise ValueError("state must be fp32 [slots, H, D, E]")
+    if qkv.shape != (T, 2 * G * D + H * E) or a.shape != (T, H * D) or b.shape != (T, H) or gate.shape != (T, H * E) or \
+            not (qkv.dtype == a.dtype == b.dtype == gate.dtype):
+        raise ValueError("qkv [rows, 2 G D + H E], a [rows, H D], b [rows, H] and gate [rows, H E] of one type")
+    out = torch.empty((T, H * E), dtype=qkv.dtype, device=qkv.device)
+    c = _lib.DeltaArgs(ptr(qkv), ptr(a), ptr(b), ptr(gate), _rows(qkv), _rows(a), _rows(b), _rows(gate), ptr(A_log), ptr(dt_bias), ptr(norm),
+                       ptr(state), ptr(out), H, G, D, E, eps, 0)
+    lib = _lib.load_seq()
+    if chunked:
+        ws = _workspace(qkv.device, lib.msa_seq_delta_chunked_workspace_bytes(C.byref(c), batch.max_rows, batch.n_seq))
+        _check(lib.msa_seq_delta_chunked(C.byref(c), batch.ref, ptr(ws), ws.numel(), _stream()), "msa_seq_delta_chunked")
+    else:
+        _check(lib.msa_seq_delta_scan(C.byref(c), dtype_code(qkv.dtype), batch.ref, _stream()), "msa_seq_delta_scan")
     return out
 
 
@@ -271,19 +348,80 @@ def flash_ok(dtype, D: int, E: int, scale: float) -> bool:
     return dtype == torch.bfloat16 and D % 8 == 0 and E % 8 == 0 and max(D, E) <= 256 and scale > 0
 
 
-def flash(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, kv_off: torch.Tensor, sink: torch.Tensor, scale: float, H: int,
-          batch: StepBatch) -> torch.Tensor:
-    """Causal attention of ``q [rows, H D]`` over expanded ``k [keys, H D]``, ``v [keys, H E]``; sequence ``s`` owns the rows
-    from ``kv_off[s]`` on."""
+def flash(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, kv_off: torch.Tensor, sink: Optional[torch.Tensor], scale: float, H: int,
+          batch: StepBatch, kv_heads: Optional[int] = None, chunk: int = 0, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Causal attention of ``q [rows, H D]`` over ``k [keys, G D]``, ``v [keys, G E]`` (``G = kv_heads``, H without); sequence ``s``
+    owns the rows from ``kv_off[s]`` on.  ``chunk``: a position sees its own stretch of that many positions only; ``gate [rows, H]``:
+    head outputs times its sigmoid."""
+    G = H if kv_heads is None else kv_heads
     _f32(H, sink)
-    D, E = q.shape[1] // H, v.shape[1] // H
-    if k.shape[1] != H * D or k.shape[0] != v.shape[0] or k.shape[0] < sum(p + c for p, c in zip(batch.positions, batch.counts)):
+    D, E = q.shape[1] // H, v.shape[1] // G
+    if k.shape[1] != G * D or k.shape[0] != v.shape[0] or k.shape[0] < sum(p + c for p, c in zip(batch.positions, batch.counts)):
         raise ValueError("k and v must hold every sequence's keys")
     if kv_off.dtype != torch.int64 or kv_off.numel() != batch.n_seq:
         raise ValueError("kv_off must be int64, one entry per sequence")
+    if gate is not None and (gate.shape != (batch.rows, H) or gate.dtype != q.dtype):
+        raise ValueError("gate must be [rows, H] of the activations' type")
     out = torch.empty((batch.rows, H * E), dtype=q.dtype, device=q.device)
     _check(_lib.load_seq().msa_seq_flash(ptr(q), _rows(q), ptr(k), _rows(k), ptr(v), _rows(v), ptr(kv_off), ptr(sink), scale,
-                                         dtype_code(q.dtype), H, D, E, ptr(out), batch.ref, _stream()), "msa_seq_flash")
+                                         dtype_code(q.dtype), H, G, D, E, chunk, ptr(gate), _rows(gate) if gate is not None else 0, ptr(out),
+                                         batch.ref, _stream()), "msa_seq_flash")
+    return out
+
+
+def _kv_caches(k_cache, v_cache, dtype, batch: StepBatch):
+    """``(capacity, G, D, E)`` of ``k_cache [slots, capacity, G, D]`` and ``v_cache [slots, capacity, G, E]``."""
+    _dense(k_cache, v_cache)
+    if k_cache.dim() != 4 or v_cache.dim() != 4 or k_cache.shape[:3] != v_cache.shape[:3] or not (k_cache.dtype == v_cache.dtype == dtype) \
+            or k_cache.shape[0] <= max(batch.slots):
+        raise ValueError("the caches must be [slots, capacity, G, D] and [slots, capacity, G, E] of the activations' type")
+    if batch.max_keys > k_cache.shape[1]:
+        raise ValueError(f"a cache of {k_cache.shape[1]} rows does not hold {batch.max_keys} tokens")
+    return k_cache.shape[1], k_cache.shape[2], k_cache.shape[3], v_cache.shape[3]
+
+
+def qk_rope_append(q, q_norm, freqs, eps: float, k_cache, v_cache, batch: StepBatch, k=None, v=None, k_norm=None) -> torch.Tensor:
+    """Normed and rotated queries ``[rows, H, D]`` of ``q [rows, H D]``; with ``k [rows, G D]`` and ``v [rows, G E]`` the normed and
+    rotated keys and the values go to the caches at their positions.  ``freqs`` (fp64): radians per position of each pair."""
+    Lcap, G, D, E = _kv_caches(k_cache, v_cache, q.dtype, batch)
+    H = q.shape[1] // D
+    _f32(D, q_norm)
+    if q.shape != (batch.rows, H * D) or freqs.dtype != torch.float64 or not freqs.is_cuda or 2 * freqs.numel() > D:
+        raise ValueError("q must be [rows, H D], freqs fp64 on the device")
+    if k is not None:
+        _f32(D, k_norm)
+        if k.shape != (batch.rows, G * D) or v.shape != (batch.rows, G * E) or not (k.dtype == v.dtype == q.dtype):
+            raise ValueError("k must be [rows, G D] and v [rows, G E] of the queries' type")
+    out = torch.empty((batch.rows, H, D), dtype=q.dtype, device=q.device)
+    c = _lib.QKRopeArgs(ptr(q), ptr(k), ptr(v), _rows(q), _rows(k) if k is not None else 0, _rows(v) if k is not None else 0, ptr(q_norm),
+                        ptr(k_norm), ptr(freqs), ptr(out), ptr(k_cache), ptr(v_cache), Lcap, H, G, D, E, freqs.numel(), eps)
+    _check(_lib.load_seq().msa_seq_qk_rope_append(C.byref(c), dtype_code(q.dtype), batch.ref, _stream()), "msa_seq_qk_rope_append")
+    return out
+
+
+def kv_attn(q: torch.Tensor, k_cache, v_cache, scale: float, batch: StepBatch, chunk: int = 0, gate: Optional[torch.Tensor] = None,
+            split: Optional[bool] = None) -> torch.Tensor:
+    """Causal attention ``[rows, H E]`` of prepared queries ``q [rows, H, D]`` over the caches, a few rows a sequence, with the chunk
+    mask and the gate of :func:`flash`.  bf16 of aligned sizes takes the split matrix-core kernel (``split`` chooses by hand)."""
+    _dense(q)
+    Lcap, G, D, E = _kv_caches(k_cache, v_cache, q.dtype, batch)
+    T, H = q.shape[:2]
+    if T != batch.rows or q.shape[2] != D or H % G:
+        raise ValueError("one query row [H, D] per row of the step")
+    if gate is not None and (gate.shape != (T, H) or gate.dtype != q.dtype):
+        raise ValueError("gate must be [rows, H] of the activations' type")
+    out = torch.empty((T, H * E), dtype=q.dtype, device=q.device)
+    c = _lib.KVAttnArgs(ptr(q), ptr(k_cache), ptr(v_cache), ptr(gate), ptr(out), Lcap, _rows(gate) if gate is not None else 0, batch.max_keys,
+                        H, G, D, E, chunk, scale)
+    lib = _lib.load_seq()
+    if split is None:
+        split = flash_ok(q.dtype, D, E, scale) and T <= 65535
+    if split:
+        need = lib.msa_seq_kv_decode_workspace_bytes(C.byref(c), T)
+        ws = _workspace(q.device, need) if need else None
+        _check(lib.msa_seq_kv_decode(C.byref(c), batch.ref, ptr(ws), ws.numel() if need else 0, _stream()), "msa_seq_kv_decode")
+    else:
+        _check(lib.msa_seq_kv_attn(C.byref(c), dtype_code(q.dtype), batch.ref, _stream()), "msa_seq_kv_attn")
     return out
 
 
@@ -329,6 +467,15 @@ def rows_linear_f32(x, w, cap: float = 0.0, add: Optional[torch.Tensor] = None) 
     return out
 
 
+def rows_glu(x, w, limit: float, alpha: float = GLU_ALPHA, shift: float = GLU_SHIFT) -> torch.Tensor:
+    """:func:`clamped_glu` of up to 16 rows' products with weights in the layout of :func:`interleave_pairs`."""
+    a = _rows_args(x, w)
+    out = torch.empty((x.shape[0], w.shape[0] // 2), dtype=torch.bfloat16, device=x.device)
+    a.out, a.out_stride, a.glu_limit, a.glu_alpha, a.glu_shift = ptr(out), out.shape[1], limit, alpha, shift
+    _run_rows(a, _lib.ROWS_GLU)
+    return out
+
+
 def rows_residual(x, w, stream: torch.Tensor, gate, gate_bias, slot, norm: Optional[DynTanhNorm] = None, shift=None, prev=None,
                   want_h: bool = True):
     """The output projection of a sublayer for up to 16 sequences' single rows, with :func:`residual_norm` behind it: the fp32
@@ -358,8 +505,8 @@ def rows_residual(x, w, stream: torch.Tensor, gate, gate_bias, slot, norm: Optio
     return h, hs
 
 
-def rows_conv(x, w, x_b, n_b: int, conv_lo: int, taps, bias, state, slot) -> torch.Tensor:
-    """Input projection of the state-space layer for up to 16 sequences' single rows: columns ``conv_lo ..`` leave through the
+def rows_conv(x, w, x_b, n_b: Optional[int], conv_lo: int, taps, bias, state, slot) -> torch.Tensor:
+    """Input projection of a layer with a convolution for up to 16 sequences' single rows: columns ``conv_lo ..`` leave through the
     causal convolution + silu, whose ``state [slots, K - 1, C]`` is updated."""
     a = _rows_args(x, w, 1, x_b, n_b)
     Cn, K = taps.shape
