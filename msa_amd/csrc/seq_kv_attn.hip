@@ -402,7 +402,7 @@ __global__ __launch_bounds__(256) void kv_combine_kernel(SplitArgs p, int64_t it
     for (int i = 0; i < p.n_split; ++i) {
       float x[4];
       load_vec<float, 4>(p.part_o + (first + (int64_t)i * a.H) * a.E + c, x);
-      const float wi = __shfl(w, i);
+      const float wi = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(w), i));    // (lanes without columns hold weights too)
 #pragma unroll
       for (int e = 0; e < 4; ++e) r[e] += wi * x[e];
     }

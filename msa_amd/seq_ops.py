@@ -244,7 +244,7 @@ DELTA_CHUNKED_ROWS = 64    # portions from this many tokens on are cut into chun
 
 
 def delta_chunked_ok(dtype, D: int, E: int) -> bool:
-    return False
+    return dtype == torch.bfloat16 and D % 8 == 0 and E % 8 == 0 and D <= 128
 
 
 def delta(qkv, a, b, gate, A_log, dt_bias, norm, eps: float, H: int, G: int, D: int, E: int, state, batch: StepBatch,

@@ -1,5 +1,5 @@
 """Plain restatement of the layer mechanisms of the Sugizen decoder (float64, one function per mechanism, token-by-token loops and
-explicit sums): the checker of ``msa_amd``'s channel-wise delta rule, rotary chunk attention, clamped gated feed-forward and
+explicit sums), which the tests compare ``msa_amd`` with: channel-wise delta rule, rotary chunk attention, clamped gated feed-forward and
 output-normed residuals.  It shares no code with the product path and reads a model as ``(config dict, {tensor name: tensor})``."""
 from __future__ import annotations
 
