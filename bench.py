@@ -425,10 +425,17 @@ def main():
     ap.add_argument("--hybrid", action="store_true",
                     help="run the hybrid decoder's benchmark (bench_hybrid.py) instead: prefill and decode throughput and every "
                          "kernel beside the attention model's")
+    ap.add_argument("--postnorm", action="store_true",
+                    help="run the output-normed decoder's benchmark (bench_postnorm.py) instead: prefill and decode throughput and "
+                         "every kernel beside the hybrid decoder's and the attention model's")
     args = ap.parse_args()
     if args.hybrid:
         import bench_hybrid
         bench_hybrid.main([])
+        return
+    if args.postnorm:
+        import bench_postnorm
+        bench_postnorm.main([])
         return
     if args.gpus != 1:
         sys.exit("bench.py: this build runs on exactly one GPU (no sharding, no collectives); use --gpus 1")

@@ -66,6 +66,18 @@ def row(us: float, bytes_: float = 0.0, flops: float = 0.0) -> dict:
     return {"us": round(us, 2), "bound": bound, "roofline_us": round(floor, 2), "frac": round(floor / us, 3)}
 
 
+class Ring:
+    """Successive operand sets, so that a set has left the caches when its turn comes again."""
+
+    def __init__(self, make, nbytes):
+        self.sets = [make() for _ in range(max(1, min(24, int(600e6 / max(nbytes, 1)))))]
+        self.i = 0
+
+    def __call__(self):
+        self.i = (self.i + 1) % len(self.sets)
+        return self.sets[self.i]
+
+
 def kernels(size: str, dev) -> dict:
     """Every kernel of the three layer kinds at prefill (one sequence of PREFILL tokens) and decode (16 sequences at CONTEXT
     tokens), and the attention model's like kernels at the same shapes.  Operands rotate through copies larger than the last-level
@@ -79,16 +91,6 @@ def kernels(size: str, dev) -> dict:
     T, B, L = PREFILL, 16, CONTEXT
     inner, C = SH * P, SH * P + 2 * G * N
     out = {"prefill": {}, "decode": {}, "prefill_like": {}, "decode_like": {}}
-
-    class Ring:
-        """Calls `fn` with successive operand sets, so that a set has left the caches when its turn comes again."""
-        def __init__(self, make, nbytes):
-            self.sets = [make() for _ in range(max(1, min(24, int(600e6 / max(nbytes, 1)))))]
-            self.i = 0
-
-        def __call__(self):
-            self.i = (self.i + 1) % len(self.sets)
-            return self.sets[self.i]
 
     # ---------------------------------------------------------------- prefill
     pb = seq_ops.StepBatch([T], [0], [0], dev)
@@ -214,9 +216,10 @@ def kernels(size: str, dev) -> dict:
     return out
 
 
-def model_throughput(size: str, dev) -> dict:
+def model_throughput(size: str, dev, others=None) -> dict:
     """Prefill of one prompt of PREFILL tokens and greedy decoding (HIP graph) of 1 and 16 sequences behind CONTEXT tokens, both
-    models at equal width, feed-forward, vocabulary and number of layers; timed in turn."""
+    models (and ``others``: name -> function of batch, prompt length, new tokens and generator that returns the timings) at equal
+    width, feed-forward, vocabulary and number of layers; timed in turn."""
     from msa_amd.cache import create_cache
     from msa_amd.config import MSAConfig
     from msa_amd.hybrid import HybridForCausalLM
@@ -233,13 +236,13 @@ def model_throughput(size: str, dev) -> dict:
         layer.self_attn.decode_reserve = STEPS + 8
     g = torch.Generator(device=dev).manual_seed(2)
 
-    def run_hybrid(B, S, new):
+    def run_hybrid(B, S, new, g):
         ids = torch.randint(0, z["vocab"], (B, S), generator=g, device=dev)
         t = {}
         hybrid.generate_greedy(ids, torch.ones_like(ids), new, timings=t, use_graph=True)
         return t
 
-    def run_msa(B, S, new):
+    def run_msa(B, S, new, g):
         ids = torch.randint(0, z["vocab"], (B, S), generator=g, device=dev)
         cache = create_cache()
         empty = torch.zeros((1, z["kv_heads"], 1, 128), dtype=torch.bfloat16, device=dev)
@@ -252,8 +255,8 @@ def model_throughput(size: str, dev) -> dict:
     for name, B, S, new in (("prefill", 1, PREFILL, 2), ("decode_1", 1, CONTEXT, STEPS), ("decode_16", 16, CONTEXT, STEPS)):
         best = {}
         for _ in range(3):
-            for who, fn in (("hybrid", run_hybrid), ("attention_model", run_msa)):
-                t = fn(B, S, new)
+            for who, fn in {"hybrid": run_hybrid, "attention_model": run_msa, **(others or {})}.items():
+                t = fn(B, S, new, g)
                 v = B * S / t["prefill_s"] if name == "prefill" else B * t["decode_steps"] / t["decode_s"]
                 best[who] = max(best.get(who, 0.0), v)
         res[name + "_tokens_per_s"] = {k: round(v, 1) for k, v in best.items()}
