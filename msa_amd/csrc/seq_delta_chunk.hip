@@ -7,7 +7,7 @@
 //   o_t = S_0^T (2^G_t q_t) + sum_{s <= t} A_ts u_s,   A_ts = sum_d q_td k_sd 2^(G_td - G_sd)
 //   S   = 2^G_end S_0 + sum_s (2^(G_end - G_s) k_s) u_s^T.
 //   (1) delta_prepare_kernel  a workgroup per (chunk, head): everything that does not need S_0
-//   (2) delta_state_kernel    a workgroup per (sequence, head, 32 value columns) walks over the chunks: U, o and S
+//   (2) delta_state_kernel    a workgroup per (sequence, head, 16 or 32 value columns) walks over the chunks: U, o and S
 //   (3) msa_seq_head_norm_gate
 // Chunks are prepared a segment at a time, which bounds the workspace.
 //
@@ -19,9 +19,9 @@
 // Operands that carry decays or states are fp32 values: what enters the state does so as a high and a low bf16 part (three
 // products, about 16 bits of mantissa).  The read-out's own operands (2^G q and A) are single bf16, like its result.
 //
-// The operands (2) reads lie in its own order, 16 bytes a lane.  A product's accumulator holds, in a lane of half h of the
-// wavefront, rows 8 x + 4 h + 0..3; taken as the next product's operand that names an order of its 16 summands,
-// {4 h + 0..3, 8 + 4 h + 0..3}, which the other operand follows: nothing is transposed on the way.
+// The operands (2) reads lie in its own order: fragments of 16 rows and 32 summands, 16 bytes a lane.  Two accumulator tiles of 16
+// rows hold, in a lane of quarter g of the wavefront, rows 4 g + 0..3 each; taken as the next product's operand that names an order
+// of its 32 summands, {4 g + 0..3, 16 + 4 g + 0..3}, which the other operand follows: nothing is transposed on the way.
 #include <algorithm>
 
 #include "seq_mfma.h"
@@ -38,18 +38,18 @@ constexpr float kMaxFall = 80.f;
 // Byte offsets of a (chunk, head)'s operands.  DP: D padded to a multiple of 32.
 template <int DP>
 struct Layout {
-  static constexpr int w = 0;                       // W: [row tile 2][DP / 16][high, low] fragments of 1 KB
-  static constexpr int q = w + DP * 256;            // 2^G q: [row tile 2][DP / 16]
-  static constexpr int k = q + DP * 128;            // 2^(G_end - G) k, transposed: [DP / 32][4][high, low]
-  static constexpr int a = k + DP * 256;            // A: row tile 0: two fragments, row tile 1: four
+  static constexpr int w = 0;                       // -W: [row tile 4][DP / 32][high, low] fragments of 1 KB
+  static constexpr int q = w + DP * 256;            // 2^G q: [row tile 4][DP / 32]
+  static constexpr int k = q + DP * 128;            // 2^(G_end - G) k, transposed: [DP / 16][2][high, low]
+  static constexpr int a = k + DP * 256;            // A: row tiles 0 and 1: one fragment each, 2 and 3: two
   static constexpr int gamma = a + 6 * 1024;        // 2^G_end: [DP] fp32
-  static constexpr int u = gamma + DP * 4;          // U': [E / 32][row tile 2] accumulators of 4 KB
+  static constexpr int u = gamma + DP * 4;          // U': [E / 16][row tile 4] accumulators of 1 KB
   static constexpr int64_t bytes(int E) { return u + (int64_t)(E + 31) / 32 * 8192; }
 };
 
 struct ChunkArgs {
   msa_delta_args d;
-  char* ws;                // [n_seq, seg, H] units of Layout::bytes
+  char* ws;                // [n_seq, H, seg] units of Layout::bytes
   int64_t unit;
   int32_t first, seg;      // first chunk and number of chunks of the segment
 };
@@ -58,12 +58,12 @@ __device__ __forceinline__ void wave_fence() {
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
   __builtin_amdgcn_wave_barrier();
 }
-// log2(1 + 2^y): its series where 1 + e would round e away.
+// log2(1 + 2^y): its series where 1 + e would round e away (above 24 it is y).
 __device__ __forceinline__ float softplus2_f(float y) {
-  const float e = __builtin_amdgcn_exp2f(y);
+  const float yc = fminf(y, 24.f), e = __builtin_amdgcn_exp2f(yc);
   const float small = e * (1.0f + e * (-0.5f + e * (0.33333333f - 0.25f * e))) * kLog2e;
   const float big = __builtin_amdgcn_logf(1.0f + e);
-  return y > 24.f ? y : e < 0.015625f ? small : big;
+  return (e < 0.015625f ? small : big) + (y - yc);
 }
 __device__ __forceinline__ float lane_value(float v, int lane) {
   return __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(v), lane));
@@ -111,7 +111,7 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
   const int head = blockIdx.x, s = blockIdx.z, kvh = head / (a.H / a.G);
   const int lo = b.cu[s], t0 = (c.first + blockIdx.y) * kC, rows = min(kC, b.cu[s + 1] - lo - t0);
   if (rows <= 0) return;
-  char* unit = c.ws + (((int64_t)s * c.seg + blockIdx.y) * a.H + head) * c.unit;
+  char* unit = c.ws + (((int64_t)s * a.H + head) * c.seg + blockIdx.y) * c.unit;
   const int brow = kB * wave, live = rows - brow;                // this wavefront's block and its tokens (may be none)
   const bf16_t* qkv = static_cast<const bf16_t*>(a.qkv) + (int64_t)(lo + t0) * a.qkv_stride;
   const bf16_t* kp = qkv + (int64_t)brow * a.qkv_stride + (int64_t)(a.G + kvh) * a.D;
@@ -122,13 +122,14 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
 
   // ---- a wavefront's block: unit vectors, decays from its start and to its end.  Lane = two channels.
   const int c0 = 2 * lane, row_bytes = (int)a.qkv_stride * 2;
-  const bool mine = lane < DP / 2, in = c0 < a.D;
+  const bool mine = DP == 128 || lane < DP / 2, in = c0 < a.D;
+  const int c_at = in ? c0 * 2 : kOutside;
   uint32_t kw[kB], qw[kB], aw[kB];
 #pragma unroll
   for (int t = 0; t < kB; ++t) {
-    kw[t] = __builtin_amdgcn_raw_buffer_load_b32(rs_k, in ? c0 * 2 + t * row_bytes : kOutside, 0, 0);
-    qw[t] = __builtin_amdgcn_raw_buffer_load_b32(rs_q, in ? c0 * 2 + t * row_bytes : kOutside, 0, 0);
-    aw[t] = __builtin_amdgcn_raw_buffer_load_b32(rs_a, in ? c0 * 2 + t * (int)a.a_stride * 2 : kOutside, 0, 0);
+    kw[t] = __builtin_amdgcn_raw_buffer_load_b32(rs_k, c_at + t * row_bytes, 0, 0);
+    qw[t] = __builtin_amdgcn_raw_buffer_load_b32(rs_q, c_at + t * row_bytes, 0, 0);
+    aw[t] = __builtin_amdgcn_raw_buffer_load_b32(rs_a, c_at + t * (int)a.a_stride * 2, 0, 0);
   }
   float kinv = 0.f, qinv = 0.f;                                  // of row lane / 4
 #pragma unroll
@@ -156,10 +157,9 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
     float x = 0.f, y = 0.f;
 #pragma unroll
     for (int t = 0; t < kB; ++t) {
-      if (t < live) {
-        x += rate * softplus2_f((bf16lo(aw[t]) + bias.x) * kLog2e);
-        y += rate * softplus2_f((bf16hi(aw[t]) + bias.y) * kLog2e);
-      }
+      const float on = t < live ? rate : 0.f;                    // no decay behind the sequence
+      x += on * softplus2_f((bf16lo(aw[t]) + bias.x) * kLog2e);
+      y += on * softplus2_f((bf16hi(aw[t]) + bias.y) * kLog2e);
       gx[t] = x;
       gy[t] = y;
     }
@@ -304,7 +304,7 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
       }
     }
   }
-  // ---- 2^G q of this block's rows: eight channels of a lane are four of either half's fragment slots
+  // ---- 2^G q of this block's rows: a lane's eight channels are half a slot of two quarters
 #pragma unroll
   for (int i = 0; i < kN; ++i) {
     const int d = 32 * i + 8 * g4;
@@ -316,22 +316,22 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
 #pragma unroll
       for (int e = 0; e < 8; ++e) x[e] *= w[e];
     }
-    char* dst = unit + Layout<DP>::q + ((wave >> 1) * (DP / 16) + 2 * i + (g4 >> 1)) * 1024 + ((wave & 1) * 16 + l15) * 16 + (g4 & 1) * 8;
+    char* dst = unit + Layout<DP>::q + (wave * kN + i) * 1024 + (l15 + 32 * (g4 & 1)) * 16 + (g4 >> 1) * 8;
     *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(x[0], x[1]), pack_bf16x2(x[2], x[3]));
-    *reinterpret_cast<uint2*>(dst + 512) = make_uint2(pack_bf16x2(x[4], x[5]), pack_bf16x2(x[6], x[7]));
+    *reinterpret_cast<uint2*>(dst + 256) = make_uint2(pack_bf16x2(x[4], x[5]), pack_bf16x2(x[6], x[7]));
   }
   // ---- 2^(G_end - G) k: more of it for the wavefronts with fewer score blocks
 #pragma unroll
   for (int f = 0; f < DP / 8; ++f) {
     const int share = f * 16 / (DP / 8), owner = share < 8 ? 0 : share < 13 ? 1 : 2;
     if (owner != wave) continue;
-    const int tile = f / 4, kk = f % 4, d = 32 * tile + (lane & 31), half = lane >> 5;
-    float post = 1.f;
-#pragma unroll
-    for (int j = kk + 1; j < 4; ++j) post *= e2[j * DP + d];
+    const int kk = f % 2, d = 16 * (f / 2) + l15;               // tokens of blocks 2 kk and 2 kk + 1
+    float post[2] = {1.f, 1.f};
+    if (kk == 0) post[1] = e2[2 * DP + d] * e2[3 * DP + d];
+    post[0] = post[1] * e2[(2 * kk + 1) * DP + d];
     float x[8];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) x[e] = ke[(kB * kk + 4 * half + (e & 3) + 8 * (e >> 2)) * kES + d] * post;
+    for (int e = 0; e < 8; ++e) x[e] = ke[(32 * kk + 4 * g4 + (e & 3) + 16 * (e >> 2)) * kES + d] * post[e >> 2];
     bf16x8_t hi, low;
     split8(x, hi, low);
     u32x4_t* dst = reinterpret_cast<u32x4_t*>(unit + Layout<DP>::k + f * 2048) + lane;
@@ -369,7 +369,12 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
     for (int r = 0; r < kB; ++r) {
       float v = r == l15 ? 1.f : 0.f;
 #pragma unroll
-      for (int k = 0; k < r; ++k) v -= lb[r * kLS + k] * x[k];
+      for (int k = 0; k < r; k += 4) {
+        const floatx4_t l = *reinterpret_cast<const floatx4_t*>(lb + r * kLS + k);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (k + e < r) v -= l[e] * x[k + e];
+      }
       x[r] = v;
     }
     wave_fence();
@@ -408,9 +413,9 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
 #pragma unroll
   for (int f = 0; f < 6; ++f) {                                  // A's fragments
     if ((f & 3) != wave) continue;
-    const int tile = f < 2 ? 0 : 1, kk = f < 2 ? f : f - 2;
-    const bf16_t* src = as + (32 * tile + (lane & 31)) * kTS + 16 * kk + 4 * (lane >> 5);
-    const uint2 x = *reinterpret_cast<const uint2*>(src), y = *reinterpret_cast<const uint2*>(src + 8);
+    const int tile = f < 2 ? f : f / 2 + 1, kk = f < 2 ? 0 : f & 1;
+    const bf16_t* src = as + (16 * tile + l15) * kTS + 32 * kk + 4 * g4;
+    const uint2 x = *reinterpret_cast<const uint2*>(src), y = *reinterpret_cast<const uint2*>(src + 16);
     reinterpret_cast<uint4*>(unit + Layout<DP>::a + f * 1024)[lane] = make_uint4(x.x, x.y, y.x, y.y);
   }
   __syncthreads();                                               // L and A are free
@@ -451,12 +456,13 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
         acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8_t*>(th + at), v, acc, 0, 0, 0);
         acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8_t*>(tl + at), v, acc, 0, 0, 0);
       }
-      floatx4_t* dst = reinterpret_cast<floatx4_t*>(unit + Layout<DP>::u + ((e0 + n0) / 32 * 2 + tile) * 4096) + lane;
+      // rows 8 x + 4 half + 0..3 of column l32: quarter 2 (x % 2) + half of row tile 2 tile + x / 2
+      floatx4_t* dst = reinterpret_cast<floatx4_t*>(unit + Layout<DP>::u + (((e0 + n0) / 16 + (l32 >> 4)) * 4 + 2 * tile) * 1024) + l15 + 16 * half;
 #pragma unroll
-      for (int x = 0; x < 4; ++x) dst[64 * x] = floatx4_t{acc[4 * x], acc[4 * x + 1], acc[4 * x + 2], acc[4 * x + 3]};
+      for (int x = 0; x < 4; ++x) dst[64 * (x >> 1) + 32 * (x & 1)] = floatx4_t{acc[4 * x], acc[4 * x + 1], acc[4 * x + 2], acc[4 * x + 3]};
     }
   }
-  // W^T = (2^G K)^T diag(beta) T^T, whose accumulators are W's fragments: (32 channels, token tile) per turn
+  // -W^T = -(2^G K)^T diag(beta) T^T, whose accumulators are -W's fragments: (32 channels, token tile) per turn
 #pragma unroll 1
   for (int task = wave; task < 2 * kN; task += 4) {
     const int d0 = task / 2 * 32, tile = task & 1;
@@ -482,162 +488,252 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
     }
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
-      const float x[8] = {acc[8 * i], acc[8 * i + 1], acc[8 * i + 2], acc[8 * i + 3], acc[8 * i + 4], acc[8 * i + 5], acc[8 * i + 6], acc[8 * i + 7]};
+      // channels 8 i + 4 half + 0..3 and 16 behind them: quarter 2 i + half
+      const float x[8] = {-acc[4 * i], -acc[4 * i + 1], -acc[4 * i + 2], -acc[4 * i + 3], -acc[4 * i + 8], -acc[4 * i + 9], -acc[4 * i + 10], -acc[4 * i + 11]};
       bf16x8_t hi, low;
       split8(x, hi, low);
-      u32x4_t* dst = reinterpret_cast<u32x4_t*>(unit + Layout<DP>::w + ((tile * (DP / 16) + d0 / 16 + i) * 2) * 1024) + lane;
+      u32x4_t* dst = reinterpret_cast<u32x4_t*>(unit + Layout<DP>::w + ((2 * tile + (l32 >> 4)) * kN + d0 / 32) * 2048) + l15 + 16 * (2 * i + half);
       dst[0] = as_u32(hi);
       dst[64] = as_u32(low);
     }
   }
 }
 
-// Wavefront w < 2 makes U of token tile w, w >= 2 the outputs of token tile w - 2, and w < DP / 32 owns 32 state rows, whose
-// fragments all of them read.  Two barriers a chunk; a chunk's operands are requested two chunks ahead.
-template <int DP>
-__global__ __launch_bounds__(256, 1) void delta_state_kernel(ChunkArgs c, msa_seq_batch b) {
-  constexpr int kN = DP / 16;
-  __shared__ u32x4_t sf[kN][2][64], uf[4][2][64];                // fragments of S and U, high and low
-  const msa_delta_args& a = c.d;
-  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), l32 = lane & 31, half = lane >> 5;
-  const int head = blockIdx.x, blk = blockIdx.y, s = blockIdx.z;
-  const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo - c.first * kC;
-  const int n = min(c.seg, (n_tok + kC - 1) / kC);
-  if (n_tok <= 0) return;
-  const int col = blk * 32 + l32;
-  const bool own = wave < DP / 32, makes_u = wave < 2;
-  const char* units = c.ws + ((int64_t)s * c.seg * a.H + head) * c.unit;
-  const int64_t step_bytes = (int64_t)a.H * c.unit;
-
-  floatx16_t S;
-  float* st = a.state + (((int64_t)b.slot[s] * a.H + head) * a.D + 32 * wave + 4 * half) * a.E + col;
-  const int d0 = 32 * wave + 4 * half;
-#pragma unroll
-  for (int e = 0; e < 16; ++e) {
-    const int r = 8 * (e >> 2) + (e & 3);
-    S[e] = own && col < a.E && d0 + r < a.D ? st[(int64_t)r * a.E] : 0.f;
-  }
+// A workgroup takes CT tiles of 16 value columns.  Wavefronts 0 and 1 make U of 32 tokens each, wavefronts 2 and 3 the outputs, and
+// wavefront w < DP / 32 owns 32 state rows, whose fragments all of them read.  Two barriers a chunk: S -> U, U -> S; the outputs'
+// part with U follows beside the next chunk's first half.  A chunk's operands are requested two chunks ahead.  The two kinds run
+// code of their own (with the same barriers), in which no load is conditional (what lies outside a buffer reads as zero), so that
+// the waits are counted.
+template <int DP, int CT>
+struct StateWalk {
+  static constexpr int kN = DP / 32;
+  struct Shared {
+    u32x4_t s[kN][CT][2][64];    // fragments of S, high and low
+    u32x4_t u[2][2][CT][2][64];  // of U, for even and odd chunks
+  };
+  template <bool kMakesU>
   struct Ops {
-    u32x4_t p[2 * kN];         // rows of W (high, low) or of 2^G q
-    u32x4_t k[8];              // rows of (2^(G_end - G) k)^T
-    u32x4_t x[4];              // U' or rows of A
-    floatx4_t gamma[4];
-  } x0, x1;
-  auto chunk_at = [&](int i) { return units + (int64_t)min(i, n - 1) * step_bytes; };
-  // (one address for either kind of wavefront, and no branch around loads both make)
-  const int p_at = makes_u ? Layout<DP>::w + wave * kN * 2048 : Layout<DP>::q + (wave - 2) * kN * 1024;
-  const int x_at = makes_u ? Layout<DP>::u + (blk * 2 + wave) * 4096 : Layout<DP>::a + (wave - 2) * 2048;
-  auto load_p = [&](Ops& o, int i) {
-    const u32x4_t* src = reinterpret_cast<const u32x4_t*>(chunk_at(i) + p_at) + lane;
-#pragma unroll
-    for (int f = 0; f < kN; ++f) o.p[f] = src[64 * f];
-    if (makes_u)
-#pragma unroll
-      for (int f = kN; f < 2 * kN; ++f) o.p[f] = src[64 * f];
+    u32x4_t p[2][kN][kMakesU ? 2 : 1];  // two row tiles of -W (high, low) or of 2^G q
+    u32x4_t k[2][2][2];                 // two row tiles of (2^(G_end - G) k)^T
+    u32x4_t a[kMakesU ? 1 : 4];         // two row tiles of A
+    floatx4_t u[kMakesU ? CT : 1][2];   // of U'
+    floatx4_t gamma[2];
   };
-  auto load_x = [&](Ops& o, int i) {                             // (of row tile 0's A two fragments are used, the others are tile 1's)
-    const u32x4_t* src = reinterpret_cast<const u32x4_t*>(chunk_at(i) + x_at) + lane;
+  struct Tiles { floatx4_t t[CT][2]; };
+
+  // accumulator tiles as a fragment per column tile
+  static __device__ __forceinline__ void share(const Tiles& v, u32x4_t (*to)[2][64], int lane) {
 #pragma unroll
-    for (int f = 0; f < 4; ++f) o.x[f] = src[64 * f];
-  };
-  auto load_k = [&](Ops& o, int i) {
-    if (!own) return;
-    const char* at = chunk_at(i);
-    const u32x4_t* src = reinterpret_cast<const u32x4_t*>(at + Layout<DP>::k + wave * 8192) + lane;
-#pragma unroll
-    for (int f = 0; f < 8; ++f) o.k[f] = src[64 * f];
-    const float* g = reinterpret_cast<const float*>(at + Layout<DP>::gamma) + d0;
-#pragma unroll
-    for (int x = 0; x < 4; ++x) o.gamma[x] = *reinterpret_cast<const floatx4_t*>(g + 8 * x);
-  };
-  load_p(x0, 0);
-  load_x(x0, 0);
-  load_k(x0, 0);
-  load_p(x1, 1);
-  load_x(x1, 1);
-  load_k(x1, 1);
-  auto share = [&](const floatx16_t& v, u32x4_t (*to)[2][64]) {  // an accumulator tile as two fragments
-#pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const float x[8] = {v[8 * i], v[8 * i + 1], v[8 * i + 2], v[8 * i + 3], v[8 * i + 4], v[8 * i + 5], v[8 * i + 6], v[8 * i + 7]};
+    for (int c = 0; c < CT; ++c) {
+      const float x[8] = {v.t[c][0][0], v.t[c][0][1], v.t[c][0][2], v.t[c][0][3], v.t[c][1][0], v.t[c][1][1], v.t[c][1][2], v.t[c][1][3]};
       bf16x8_t hi, low;
       split8(x, hi, low);
-      to[i][0][lane] = as_u32(hi);
-      to[i][1][lane] = as_u32(low);
+      to[c][0][lane] = as_u32(hi);
+      to[c][1][lane] = as_u32(low);
     }
-  };
-  if (own) share(S, sf + 2 * wave);
-  const int row_elems = a.H * a.E;
-  auto step = [&](Ops& o, int i) {
-    __syncthreads();
-    floatx16_t acc = zero16(), cross = zero16();
-    if (makes_u) {
-#pragma unroll
-      for (int kk = 0; kk < kN; ++kk) {
-        const bf16x8_t hi = as_bf16(sf[kk][0][lane]), low = as_bf16(sf[kk][1][lane]);
-        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.p[2 * kk]), hi, acc, 0, 0, 0);
-        cross = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.p[2 * kk]), low, cross, 0, 0, 0);
-        cross = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.p[2 * kk + 1]), hi, cross, 0, 0, 0);
-      }
-#pragma unroll
-      for (int e = 0; e < 16; ++e) acc[e] = __uint_as_float(o.x[e >> 2][e & 3]) - (acc[e] + cross[e]);
-      share(acc, uf + 2 * wave);
-      load_x(o, i + 2);
-    } else {
-#pragma unroll
-      for (int kk = 0; kk < kN; ++kk) {
-        const bf16x8_t hi = as_bf16(sf[kk][0][lane]), low = as_bf16(sf[kk][1][lane]);
-        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.p[kk]), hi, acc, 0, 0, 0);
-        cross = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.p[kk]), low, cross, 0, 0, 0);
-      }
-    }
-    load_p(o, i + 2);
-    __syncthreads();
-    if (own) {
-      floatx16_t add = zero16();
-#pragma unroll
-      for (int e = 0; e < 16; ++e) S[e] *= o.gamma[e >> 2][e & 3];
-#pragma unroll
-      for (int kk = 0; kk < 4; ++kk) {
-        const bf16x8_t hi = as_bf16(uf[kk][0][lane]), low = as_bf16(uf[kk][1][lane]);
-        S = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.k[2 * kk]), hi, S, 0, 0, 0);
-        add = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.k[2 * kk]), low, add, 0, 0, 0);
-        add = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.k[2 * kk + 1]), hi, add, 0, 0, 0);
-      }
-#pragma unroll
-      for (int e = 0; e < 16; ++e) S[e] += add[e];
-      share(S, sf + 2 * wave);
-      load_k(o, i + 2);
-    }
-    if (!makes_u) {
-#pragma unroll
-      for (int kk = 0; kk < 4; ++kk) {
-        if (kk >= 2 && wave == 2) continue;
-        const bf16x8_t hi = as_bf16(uf[kk][0][lane]), low = as_bf16(uf[kk][1][lane]);
-        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.x[kk]), hi, acc, 0, 0, 0);
-        cross = __builtin_amdgcn_mfma_f32_32x32x16_bf16(as_bf16(o.x[kk]), low, cross, 0, 0, 0);
-      }
-      load_x(o, i + 2);
-      // token 32 (wave - 2) + 8 x + 4 half + e, column col; tokens behind the sequence and columns behind the head are not written
-      const int rows = min(kC, n_tok - i * kC);
-      bf16_t* out = static_cast<bf16_t*>(a.out) + ((int64_t)(lo + (c.first + i) * kC) * a.H + head) * a.E;
-      const __amdgpu_buffer_rsrc_t rs = rows_rsrc(out, rows, row_elems, a.E);
-      const int at = col < a.E ? ((32 * (wave - 2) + 4 * half) * row_elems + col) * 2 : kOutside;
-#pragma unroll
-      for (int e = 0; e < 16; ++e)
-        __builtin_amdgcn_raw_buffer_store_b16(f32_to_bf16(acc[e] + cross[e]), rs, at + (8 * (e >> 2) + (e & 3)) * row_elems * 2, 0, 0);
-    }
-  };
-  for (int i = 0; i < n; i += 2) {
-    step(x0, i);
-    if (i + 1 < n) step(x1, i + 1);
   }
-  if (own && col < a.E)
+  static __device__ __forceinline__ floatx4_t mul(u32x4_t a, u32x4_t b, floatx4_t c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16(a), as_bf16(b), c, 0, 0, 0);
+  }
+  static __device__ __forceinline__ u32x4_t load(__amdgpu_buffer_rsrc_t rs, int at) { return __builtin_amdgcn_raw_buffer_load_b128(rs, at, 0, 0); }
+
+  template <bool kMakesU>
+  static __device__ __forceinline__ void run(const ChunkArgs& c, const msa_seq_batch& b, Shared& sh, int wave) {
+    const msa_delta_args& a = c.d;
+    const int lane = threadIdx.x & 63, l15 = lane & 15, g4 = lane >> 4, pair = wave & 1;
+    const int head = blockIdx.x, s = blockIdx.z, tile0 = blockIdx.y * CT;
+    const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo - c.first * kC;
+    const int n = min(c.seg, (n_tok + kC - 1) / kC);
+    const int col = tile0 * 16 + l15, d0 = 32 * wave + 4 * g4, row_elems = a.H * a.E;
+    const bool own = DP == 128 || wave < DP / 32;
+    const char* units = c.ws + ((int64_t)s * a.H + head) * c.seg * c.unit;
+
+    Tiles S;                                                     // rows d0 + 16 t + 0..3, column col + 16 i
+    float* st = a.state + (((int64_t)b.slot[s] * a.H + head) * a.D + d0) * a.E + col;
 #pragma unroll
-    for (int e = 0; e < 16; ++e) {
-      const int r = 8 * (e >> 2) + (e & 3);
-      if (d0 + r < a.D) st[(int64_t)r * a.E] = S[e];
+    for (int i = 0; i < CT; ++i)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int r = 16 * (e >> 2) + (e & 3);
+        S.t[i][e >> 2][e & 3] = own && col + 16 * i < a.E && d0 + r < a.D ? st[(int64_t)r * a.E + 16 * i] : 0.f;
+      }
+    const int p_at = (kMakesU ? Layout<DP>::w + pair * 2 * kN * 2048 : Layout<DP>::q + pair * 2 * kN * 1024) + lane * 16;
+    const int u_at = Layout<DP>::u + (tile0 * 4 + 2 * pair) * 1024 + lane * 16, a_at = Layout<DP>::a + pair * 2048 + lane * 16;
+    const int k_at = own ? Layout<DP>::k + wave * 8192 + lane * 16 : kOutside, g_at = own ? Layout<DP>::gamma + d0 * 4 : kOutside;
+    using O = Ops<kMakesU>;
+    auto chunk_rsrc = [&](int i) {
+      return __builtin_amdgcn_make_buffer_rsrc(const_cast<char*>(units + (int64_t)min(i, n - 1) * c.unit), 0, (int)c.unit, 0x00020000);
+    };
+    auto load_p = [&](O& o, int i) {
+      const __amdgpu_buffer_rsrc_t rs = chunk_rsrc(i);
+      constexpr int kParts = kMakesU ? 2 : 1;
+#pragma unroll
+      for (int f = 0; f < 2 * kN * kParts; ++f) o.p[f / (kN * kParts)][f / kParts % kN][f % kParts] = load(rs, p_at + 1024 * f);
+      __builtin_amdgcn_sched_barrier(0);
+    };
+    auto load_x = [&](O& o, int i) {
+      const __amdgpu_buffer_rsrc_t rs = chunk_rsrc(i);
+      if constexpr (kMakesU) {
+#pragma unroll
+        for (int f = 0; f < 2 * CT; ++f) o.u[f / 2][f % 2] = __builtin_bit_cast(floatx4_t, load(rs, u_at + 4096 * (f / 2) + 1024 * (f % 2)));
+      } else {                                                   // (of the first four two are tiles 0 and 1)
+#pragma unroll
+        for (int f = 0; f < 4; ++f) o.a[f] = load(rs, a_at + 1024 * f);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+    };
+    auto load_k = [&](O& o, int i) {
+      const __amdgpu_buffer_rsrc_t rs = chunk_rsrc(i);
+#pragma unroll
+      for (int f = 0; f < 8; ++f) o.k[f / 4][f / 2 % 2][f % 2] = load(rs, k_at + 1024 * f);
+#pragma unroll
+      for (int t = 0; t < 2; ++t) o.gamma[t] = __builtin_bit_cast(floatx4_t, load(rs, g_at + 64 * t));
+      __builtin_amdgcn_sched_barrier(0);
+    };
+    const floatx4_t none = {0.f, 0.f, 0.f, 0.f};
+    Tiles out;                                                   // 2^G q S of the chunk before
+#pragma unroll
+    for (int i = 0; i < CT; ++i) out.t[i][0] = out.t[i][1] = none;
+    // its stores: tokens 32 pair + 16 t + 4 g4 + 0..3 (what lies outside is not written)
+    auto store = [&](int i) {
+      const __amdgpu_buffer_rsrc_t rs = rows_rsrc(static_cast<bf16_t*>(a.out) + ((int64_t)(lo + (c.first + i) * kC) * a.H + head) * a.E,
+                                                  i < 0 ? 0 : min(kC, n_tok - i * kC), row_elems, a.E);
+#pragma unroll
+      for (int j = 0; j < CT; ++j) {
+        const int at = col + 16 * j < a.E ? ((32 * pair + 4 * g4) * row_elems + col + 16 * j) * 2 : kOutside;
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          __builtin_amdgcn_raw_buffer_store_b16(f32_to_bf16(out.t[j][e >> 2][e & 3]), rs, at + (16 * (e >> 2) + (e & 3)) * row_elems * 2, 0, 0);
+      }
+    };
+    // its part with U
+    auto finish = [&](O& o, int i) {
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk) {
+        if (kk > pair) continue;
+#pragma unroll
+        for (int h = 0; h < 2; ++h)
+#pragma unroll
+          for (int j = 0; j < CT; ++j)
+#pragma unroll
+            for (int t = 0; t < 2; ++t) out.t[j][t] = mul(pair ? o.a[2 * t + kk] : o.a[t], sh.u[i & 1][kk][j][h][lane], out.t[j][t]);
+      }
+      load_x(o, i + 2);
+      store(i);
+    };
+    auto step = [&](O& o, O& before, int i) {
+      __syncthreads();
+      u32x4_t f[kN][CT][2];
+#pragma unroll
+      for (int kk = 0; kk < kN; ++kk)
+#pragma unroll
+        for (int j = 0; j < CT; ++j)
+#pragma unroll
+          for (int h = 0; h < 2; ++h) f[kk][j][h] = sh.s[kk][j][h][lane];
+      __builtin_amdgcn_sched_barrier(0);
+      if constexpr (kMakesU) {
+        Tiles u;
+#pragma unroll
+        for (int j = 0; j < CT; ++j)
+#pragma unroll
+          for (int t = 0; t < 2; ++t) u.t[j][t] = o.u[j][t];
+#pragma unroll
+        for (int kk = 0; kk < kN; ++kk)
+#pragma unroll
+          for (int x = 0; x < 3; ++x)                            // high x high, high x low, low x high
+#pragma unroll
+            for (int j = 0; j < CT; ++j)
+#pragma unroll
+              for (int t = 0; t < 2; ++t) u.t[j][t] = mul(o.p[t][kk][x >> 1], f[kk][j][x & 1], u.t[j][t]);
+        share(u, sh.u[i & 1][pair], lane);
+        load_x(o, i + 2);
+      } else {
+        finish(before, i - 1);                                   // (in front of the first chunk: nothing is written)
+#pragma unroll
+        for (int j = 0; j < CT; ++j) out.t[j][0] = out.t[j][1] = none;
+#pragma unroll
+        for (int kk = 0; kk < kN; ++kk)
+#pragma unroll
+          for (int h = 0; h < 2; ++h)
+#pragma unroll
+            for (int j = 0; j < CT; ++j)
+#pragma unroll
+              for (int t = 0; t < 2; ++t) out.t[j][t] = mul(o.p[t][kk][0], f[kk][j][h], out.t[j][t]);
+      }
+      load_p(o, i + 2);
+      __syncthreads();
+      if (own) {
+        u32x4_t g[2][CT][2];
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk)
+#pragma unroll
+          for (int j = 0; j < CT; ++j)
+#pragma unroll
+            for (int h = 0; h < 2; ++h) g[kk][j][h] = sh.u[i & 1][kk][j][h][lane];
+#pragma unroll
+        for (int j = 0; j < CT; ++j)
+#pragma unroll
+          for (int t = 0; t < 2; ++t) S.t[j][t] *= o.gamma[t];
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk)
+#pragma unroll
+          for (int x = 0; x < 3; ++x)
+#pragma unroll
+            for (int j = 0; j < CT; ++j)
+#pragma unroll
+              for (int t = 0; t < 2; ++t) S.t[j][t] = mul(o.k[t][kk][x >> 1], g[kk][j][x & 1], S.t[j][t]);
+        share(S, sh.s[wave], lane);
+      }
+      load_k(o, i + 2);
+    };
+    O x0, x1;
+    // (in the order the loop makes them, stores included, so that the first pass counts like the others)
+    if constexpr (kMakesU) {
+      load_x(x0, 0);
+      load_p(x0, 0);
+      load_k(x0, 0);
+      load_x(x1, 1);
+      load_p(x1, 1);
+      load_k(x1, 1);
+    } else {
+      load_x(x1, 1);
+      store(-2);
+      load_p(x0, 0);
+      load_k(x0, 0);
+      load_x(x0, 0);
+      store(-1);
+      load_p(x1, 1);
+      load_k(x1, 1);
     }
+    if (own) share(S, sh.s[wave], lane);
+    for (int i = 0; i + 1 < n; i += 2) {
+      step(x0, x1, i);
+      step(x1, x0, i + 1);
+    }
+    if (n & 1) step(x0, x1, n - 1);
+    if constexpr (!kMakesU) {
+      if (n & 1) finish(x0, n - 1);
+      else finish(x1, n - 1);
+    }
+    if (!own) return;
+#pragma unroll
+    for (int i = 0; i < CT; ++i)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int r = 16 * (e >> 2) + (e & 3);
+        if (col + 16 * i < a.E && d0 + r < a.D) st[(int64_t)r * a.E + 16 * i] = S.t[i][e >> 2][e & 3];
+      }
+  }
+};
+
+template <int DP, int CT>
+__global__ __launch_bounds__(256, 1) void delta_state_kernel(ChunkArgs c, msa_seq_batch b) {
+  __shared__ typename StateWalk<DP, CT>::Shared sh;
+  if (b.cu[blockIdx.z + 1] - b.cu[blockIdx.z] <= c.first * kC) return;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  if (wave < 2) StateWalk<DP, CT>::template run<true>(c, b, sh, wave);
+  else StateWalk<DP, CT>::template run<false>(c, b, sh, wave);
 }
 
 constexpr int64_t kMaxWorkspace = (int64_t)1 << 29;
@@ -667,7 +763,10 @@ int launch_chunked(ChunkArgs c, const msa_seq_batch& b, hipStream_t st) {
   for (c.first = 0; c.first < chunks; c.first += c.seg) {
     delta_prepare_kernel<DP><<<dim3(c.d.H, std::min(c.seg, chunks - c.first), b.n_seq), 256, lds, st>>>(c, b);
     MSA_LAUNCH_CHECK();
-    delta_state_kernel<DP><<<dim3(c.d.H, (c.d.E + 31) / 32, b.n_seq), 256, 0, st>>>(c, b);
+    // narrow column tiles as long as they find compute units
+    const int tiles = (c.d.E + 15) / 16;
+    if ((int64_t)c.d.H * tiles * b.n_seq <= device_compute_units()) delta_state_kernel<DP, 1><<<dim3(c.d.H, tiles, b.n_seq), 256, 0, st>>>(c, b);
+    else delta_state_kernel<DP, 2><<<dim3(c.d.H, (tiles + 1) / 2, b.n_seq), 256, 0, st>>>(c, b);
     MSA_LAUNCH_CHECK();
   }
   return MSA_OK;

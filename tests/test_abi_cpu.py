@@ -80,8 +80,23 @@ def test_seq_validation_errors_without_gpu():
     assert lib.msa_rows_linear(C.byref(a), 0, None) == -1 and b"second operand" in lib.msa_last_error()
     assert lib.msa_seq_softcap(None, 0, 1, 0.0, None, None) == -1
     b = _lib.SeqBatch(4096, 4096, 4096, 4096, 1, 4, 4, 0)
-    assert lib.msa_seq_flash(4096, 96, 4096, 96, 4096, 96, 4096, 4096, 1.0, 0, 1, 300, 96, 4096, C.byref(b), None) == -1
-    assert b"D=300" in lib.msa_last_error()
+    flash = lambda H, G, D, chunk: lib.msa_seq_flash(4096, 96, 4096, 96, 4096, 96, 4096, 4096, 1.0, 0, H, G, D, 96, chunk, None, 0, 4096, C.byref(b), None)
+    assert flash(1, 1, 300, 0) == -1 and b"D=300" in lib.msa_last_error()
+    assert flash(3, 2, 96, 0) == -1 and b"3 heads over 2" in lib.msa_last_error()
+    assert flash(1, 1, 96, -1) == -1 and b"chunk" in lib.msa_last_error()
+    kv = _lib.KVAttnArgs(4096, 4096, 4096, None, 4096, 64, 0, 65, 4, 2, 64, 64, 0, 1.0)
+    assert lib.msa_seq_kv_decode(C.byref(kv), C.byref(b), None, 0, None) == -1 and b"65 keys" in lib.msa_last_error()
+    kv.max_keys, kv.D = 64, 60
+    assert lib.msa_seq_kv_decode(C.byref(kv), C.byref(b), None, 0, None) == -1 and b"D=60" in lib.msa_last_error()
+    rope = _lib.QKRopeArgs(4096, None, None, 128, 0, 0, 4096, None, 4096, 4096, None, None, 0, 2, 1, 64, 64, 33, 1e-5)
+    assert lib.msa_seq_qk_rope_append(C.byref(rope), 0, C.byref(b), None) == -1 and b"33 pairs" in lib.msa_last_error()
+    d = _lib.DeltaArgs(4096, 4096, 4096, 4096, 192, 64, 1, 64, 4096, 4096, 4096, 4096, 4096, 1, 1, 64, 64, 1e-5, 0)
+    assert lib.msa_seq_delta_chunked_workspace_bytes(C.byref(d), 640, 1) == 10 * lib.msa_seq_delta_chunked_workspace_bytes(C.byref(d), 64, 1) > 0
+    assert lib.msa_seq_delta_chunked(C.byref(d), C.byref(b), 4096, 16, None) == -3 and b"workspace" in lib.msa_last_error()
+    d.D = 520
+    assert lib.msa_seq_delta_scan(C.byref(d), 0, C.byref(b), None) == -1 and b"D=520" in lib.msa_last_error()
+    a.K, a.n_b, a.N, a.M = 64, 15, 15, 4
+    assert lib.msa_rows_linear(C.byref(a), 5, None) == -1 and b"gated unit" in lib.msa_last_error()
     assert lib.msa_seq_min_gru(4096, 96, 4096, 4096, 0, 32, 4096, 4096, C.byref(_lib.SeqBatch(4096, 4096, 4096, 4096, 1, 999, 999, 0)),
                                None, 0, None) == -3 and b"workspace" in lib.msa_last_error()
 
