@@ -52,7 +52,8 @@ def test_header_arity_matches_ctypes_table(header, table):
 def test_seq_structures_match_the_header(tmp_path):
     """Sizes and field offsets of the structures handed over by pointer, against the host compiler's."""
     import subprocess
-    structs = {"msa_seq_batch": _lib.SeqBatch, "msa_dyn_tanh": _lib.DynTanh, "msa_rows_args": _lib.RowsArgs}
+    structs = {"msa_seq_batch": _lib.SeqBatch, "msa_dyn_tanh": _lib.DynTanh, "msa_rows_args": _lib.RowsArgs,
+               "msa_qk_rope_args": _lib.QKRopeArgs, "msa_kv_attn_args": _lib.KVAttnArgs, "msa_delta_args": _lib.DeltaArgs}
     src = ['#include <stdio.h>', '#include "msa_seq.h"', "int main() {"]
     for c_name, py in structs.items():
         src.append(f'printf("{c_name} %zu\\n", sizeof({c_name}));')
