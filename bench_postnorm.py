@@ -140,6 +140,25 @@ def kernels(name: str, dev) -> dict:
     return {"prefill": p, "decode": d}
 
 
+def single_rows(name: str, dev) -> dict:
+    """The hybrid decoder's state update and attention for one sequence."""
+    from msa_amd import seq_ops
+    z = sizes(name)
+    SH, N, P, G, H, rank, L = z["ssm_heads"], z["state"], 64, 8, z["heads"], z["kv_rank"], CONTEXT
+    g = torch.Generator(device=dev).manual_seed(6)
+    bf = lambda *s: torch.randn(s, generator=g, device=dev).to(torch.bfloat16)
+    f32 = lambda *s: torch.randn(s, generator=g, device=dev)
+    one = seq_ops.StepBatch([1], [0], [L - 1], dev)
+    xbc, zz, dt = bf(1, SH * P + 2 * G * N), bf(1, SH * P), bf(1, SH)
+    bias, al, D, sink, qa = f32(SH) - 4.0, torch.rand(SH, device=dev), f32(SH), f32(H), bf(1, H, rank)
+    st = Ring(lambda: torch.zeros(1, SH, N, P, device=dev), 16 * SH * N * P * 4)
+    cache = Ring(lambda: bf(1, L, rank), 16 * L * rank * 2)
+    return {"state-space update, 1 sequence": row(time_us(lambda: seq_ops.ssd(xbc, zz, dt, bias, al, D, SH, P, N, G, st(), one), reps=24),
+                                                  2.0 * SH * N * P * 4),
+            "latent attention + combine, 1 sequence": row(time_us(lambda: seq_ops.latent_attn(qa, cache(), sink, 0.1, one, L), reps=24),
+                                                          L * rank * 2)}
+
+
 def model_throughput(name: str, dev) -> dict:
     """Prefill of one prompt of PREFILL tokens and greedy decoding (HIP graph) of 1 and 16 sequences behind CONTEXT tokens, the three
     models timed in turn."""
@@ -179,6 +198,7 @@ def main(argv=None) -> dict:
             print(f"[bench_postnorm] kernels {name} {time.time() - t0:.0f} s", file=sys.stderr, flush=True)
             if not args.no_like:
                 like = bench_hybrid.kernels(name, dev)
+                like["decode"].update(single_rows(name, dev))
                 out["kernels"][name]["like"] = {"hybrid": {k: like[k] for k in ("prefill", "decode")},
                                                 "attention_model": {"prefill": like["prefill_like"], "decode": like["decode_like"]}}
                 print(f"[bench_postnorm] like kernels {name} {time.time() - t0:.0f} s", file=sys.stderr, flush=True)

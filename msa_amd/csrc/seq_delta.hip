@@ -28,9 +28,6 @@ __global__ __launch_bounds__(RW * CW * 64) void delta_scan_kernel(msa_delta_args
   const bool live = col < a.E, whole = gridDim.x == 1;
   const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo, kvh = head / (a.H / a.G);
   float* st = a.state + (((int64_t)b.slot[s] * a.H + head) * a.D + rw * NI) * a.E + col;
-  float S[NI];
-#pragma unroll
-  for (int i = 0; i < NI; ++i) S[i] = live && rw * NI + i < a.D ? st[(int64_t)i * a.E] : 0.f;
   const float rate = -expf(a.A_log[head]), q_scale = 1.0f / sqrtf((float)a.D);
   const float* bias = a.dt_bias + (int64_t)head * a.D;
   const T* qkv = static_cast<const T*>(a.qkv) + (int64_t)lo * a.qkv_stride;
@@ -39,22 +36,53 @@ __global__ __launch_bounds__(RW * CW * 64) void delta_scan_kernel(msa_delta_args
   const T* vp = qkv + 2LL * a.G * a.D + (int64_t)head * a.E;
   const T* ap = static_cast<const T*>(a.a) + (int64_t)lo * a.a_stride + (int64_t)head * a.D;
   const T* bp = static_cast<const T*>(a.b) + (int64_t)lo * a.b_stride + head;
-  for (int t0 = 0; t0 < n_tok; t0 += kTok) {
+  const T* gp = static_cast<const T*>(a.gate) + (int64_t)lo * a.gate_stride + (int64_t)head * a.E;
+  constexpr int kEach = (kD + 63) / 64, kMine = (kTok + kWaves - 1) / kWaves;    // values of a lane, tokens of a wavefront in a stage
+  // What a stage reads is requested together, and the first one's in front of the state: loads arrive in the order they are made,
+  // and the vectors are ready by the time the state is there.
+  float k[kMine][kEach], q[kMine][kEach], x[kMine][kEach], bv[kMine], v[kTok], db[kEach];
+#pragma unroll
+  for (int j = 0; j < kEach; ++j) db[j] = lane + 64 * j < a.D ? bias[lane + 64 * j] : 0.f;
+  auto fetch = [&](int t0) {
     const int rows = min(kTok, n_tok - t0);
-    for (int r = wave; r < rows; r += kWaves) {          // a wavefront per token
-      const int64_t t = t0 + r;
-      constexpr int kEach = (kD + 63) / 64;
-      float k[kEach], q[kEach], kk = 0.f, qq = 0.f, dot = 0.f;
+#pragma unroll
+    for (int m = 0; m < kMine; ++m) {
+      const int r = wave + m * kWaves;
+      const int64_t t = t0 + min(r, rows - 1);
 #pragma unroll
       for (int j = 0; j < kEach; ++j) {
         const int i = lane + 64 * j;
         const bool in = i < a.D;
-        k[j] = in ? to_f32<T>(kp[t * a.qkv_stride + i]) : 0.f;
-        q[j] = in ? to_f32<T>(qp[t * a.qkv_stride + i]) : 0.f;
-        if (i < kD) gs[r][i] = in ? expf(rate * softplus_f(to_f32<T>(ap[t * a.a_stride + i]) + bias[i])) : 0.f;
-        kk += k[j] * k[j];
-        qq += q[j] * q[j];
-        dot += k[j] * q[j];
+        k[m][j] = in ? to_f32<T>(kp[t * a.qkv_stride + i]) : 0.f;
+        q[m][j] = in ? to_f32<T>(qp[t * a.qkv_stride + i]) : 0.f;
+        x[m][j] = in ? to_f32<T>(ap[t * a.a_stride + i]) : 0.f;
+      }
+      bv[m] = to_f32<T>(bp[t * a.b_stride]);
+    }
+#pragma unroll
+    for (int r = 0; r < kTok; ++r) v[r] = live && r < rows ? to_f32<T>(vp[(t0 + r) * a.qkv_stride + col]) : 0.f;
+  };
+  fetch(0);
+  const float out_w = live && whole ? a.norm[col] : 0.f;
+  const float gate0 = live && whole ? to_f32<T>(gp[col]) : 0.f;   // of the first token, all there is when decoding
+  float S[NI];
+#pragma unroll
+  for (int i = 0; i < NI; ++i) S[i] = live && rw * NI + i < a.D ? st[(int64_t)i * a.E] : 0.f;
+  for (int t0 = 0; t0 < n_tok; t0 += kTok) {
+    const int rows = min(kTok, n_tok - t0);
+    if (t0 > 0) fetch(t0);
+#pragma unroll
+    for (int m = 0; m < kMine; ++m) {                    // a wavefront per token
+      const int r = wave + m * kWaves;
+      if (r >= rows) break;
+      float kk = 0.f, qq = 0.f, dot = 0.f;
+#pragma unroll
+      for (int j = 0; j < kEach; ++j) {
+        const int i = lane + 64 * j;
+        if (i < kD) gs[r][i] = i < a.D ? expf(rate * softplus_f(x[m][j] + db[j])) : 0.f;
+        kk += k[m][j] * k[m][j];
+        qq += q[m][j] * q[m][j];
+        dot += k[m][j] * q[m][j];
       }
 #pragma unroll
       for (int o = 32; o > 0; o >>= 1) {
@@ -67,18 +95,15 @@ __global__ __launch_bounds__(RW * CW * 64) void delta_scan_kernel(msa_delta_args
       for (int j = 0; j < kEach; ++j) {
         const int i = lane + 64 * j;
         if (i < kD) {
-          ks[r][i] = k[j] * ki;
-          qs[r][i] = q[j] * qi;
+          ks[r][i] = k[m][j] * ki;
+          qs[r][i] = q[m][j] * qi;
         }
       }
       if (lane == 0) {
         kq[r] = dot * ki * qi;
-        beta[r] = sigmoid_f(to_f32<T>(bp[t * a.b_stride]));
+        beta[r] = sigmoid_f(bv[m]);
       }
     }
-    float v[kTok];
-#pragma unroll
-    for (int r = 0; r < kTok; ++r) v[r] = live && r < rows ? to_f32<T>(vp[(t0 + r) * a.qkv_stride + col]) : 0.f;
     __syncthreads();
 #pragma unroll
     for (int r = 0; r < kTok; ++r) {
@@ -117,25 +142,36 @@ __global__ __launch_bounds__(RW * CW * 64) void delta_scan_kernel(msa_delta_args
       }
     }
     __syncthreads();
-    for (int r = wave; r < rows; r += kWaves) {          // outputs, a wavefront per token
-      const int64_t row = lo + t0 + r;
-      T* dst = static_cast<T*>(a.out) + (row * a.H + head) * a.E + col0;
-      float inv = 1.f;
-      if (whole) {
-        float ssq = 0.f;
+    if (whole && n_tok == 1) {                           // decoding: every thread of the first row share finishes its column
+      float ssq = 0.f;
 #pragma unroll
-        for (int c = lane; c < kCols; c += 64) ssq += c < a.E ? os[r][c] * os[r][c] : 0.f;
+      for (int c = lane; c < kCols; c += 64) ssq += c < a.E ? os[0][c] * os[0][c] : 0.f;
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) ssq += __shfl_xor(ssq, o);
-        inv = 1.0f / sqrtf(ssq / (float)a.E + a.eps);
-      }
-      const T* gate = static_cast<const T*>(a.gate) + row * a.gate_stride + (int64_t)head * a.E;
+      for (int o = 32; o > 0; o >>= 1) ssq += __shfl_xor(ssq, o);
+      if (rw == 0 && live)
+        static_cast<T*>(a.out)[((int64_t)lo * a.H + head) * a.E + col] =
+            from_f32<T>(os[0][cl] * (1.0f / sqrtf(ssq / (float)a.E + a.eps)) * out_w * sigmoid_f(gate0));
+    } else {
+      for (int r = wave; r < rows; r += kWaves) {        // outputs, a wavefront per token
+        const int64_t row = lo + t0 + r;
+        T* dst = static_cast<T*>(a.out) + (row * a.H + head) * a.E + col0;
+        float inv = 1.f;
+        if (whole) {
+          float ssq = 0.f;
 #pragma unroll
-      for (int c = lane; c < kCols; c += 64) {
-        if (col0 + c >= a.E) break;
-        float y = os[r][c];
-        if (whole) y *= inv * a.norm[c] * sigmoid_f(to_f32<T>(gate[c]));
-        dst[c] = from_f32<T>(y);
+          for (int c = lane; c < kCols; c += 64) ssq += c < a.E ? os[r][c] * os[r][c] : 0.f;
+#pragma unroll
+          for (int o = 32; o > 0; o >>= 1) ssq += __shfl_xor(ssq, o);
+          inv = 1.0f / sqrtf(ssq / (float)a.E + a.eps);
+        }
+        const T* gate = gp + (int64_t)(t0 + r) * a.gate_stride;
+#pragma unroll
+        for (int c = lane; c < kCols; c += 64) {
+          if (col0 + c >= a.E) break;
+          float y = os[r][c];
+          if (whole) y *= inv * a.norm[c] * sigmoid_f(to_f32<T>(gate[c]));
+          dst[c] = from_f32<T>(y);
+        }
       }
     }
     // (the next stage's first barrier stands between these reads of `os` and its being written again)

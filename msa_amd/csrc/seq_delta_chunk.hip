@@ -14,7 +14,7 @@
 // Decays differ by channel, so L and A are products of operands that carry them: within blocks of 16 tokens everything is
 // relative to the block's start (rows, exponents <= 0) and its end (columns, exponents <= 0), and whole blocks' decays between
 // the two scale the columns.  Only inside a diagonal block the columns' exponents are positive; a block in which some channel
-// falls by more than 2^-80 is summed pair by pair instead.
+// falls by more than 2^-80 is taken apart once more, into four tokens a part (steep_block).
 //
 // Operands that carry decays or states are fp32 values: what enters the state does so as a high and a low bf16 part (three
 // products, about 16 bits of mantissa).  The read-out's own operands (2^G q and A) are single bf16, like its result.
@@ -78,6 +78,87 @@ __device__ __forceinline__ floatx16_t zero16() {
 #pragma unroll
   for (int e = 0; e < 16; ++e) z[e] = 0.f;
   return z;
+}
+
+// Sums over d of k_t k_s 2^(G_t - G_s) and q_t k_s 2^(G_t - G_s) of a 16-token block in which decays may be of any size, one
+// wavefront: parts of four tokens, factored at the row part's start where row and column lie in different ones (all exponents
+// <= 0), pair by pair within a part.  LDS rows of this block: g [16][DP + 4] log-decays, k and q [16][DP + 8].  Results: row
+// 4 (lane / 16) + e, column lane % 16.
+template <int DP>
+__device__ void steep_block(const float* g, const bf16_t* k, const bf16_t* q, floatx4_t& dk, floatx4_t& dq) {
+  constexpr int kKS = DP + 8, kES = DP + 4, kN = DP / 32;
+  const int lane = threadIdx.x & 63, l15 = lane & 15, g4 = lane >> 4;
+  // within parts: lane = (part, row, column)
+  float in_k = 0.f, in_q = 0.f;
+  {
+    const int t = 4 * g4 + (l15 >> 2), u = 4 * g4 + (l15 & 3);
+    for (int d = 0; d < DP; d += 4) {
+      float gt[4], gu[4], kt[4], ku[4], qt[4];
+      load_vec<float, 4>(g + t * kES + d, gt);
+      load_vec<float, 4>(g + u * kES + d, gu);
+      load_vec<bf16_t, 4>(k + t * kKS + d, kt);
+      load_vec<bf16_t, 4>(k + u * kKS + d, ku);
+      load_vec<bf16_t, 4>(q + t * kKS + d, qt);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float w = __builtin_amdgcn_exp2f(fminf(gt[e] - gu[e], 0.f)) * ku[e];
+        in_k += w * kt[e];
+        in_q += w * qt[e];
+      }
+    }
+  }
+  bf16x8_t kh[kN], kl[kN], qh[kN];                               // rows: decayed from their part's start
+#pragma unroll
+  for (int i = 0; i < kN; ++i) {
+    const int d = 32 * i + 8 * g4, start = 4 * (l15 >> 2) - 1;
+    float x[8], y[8], w[8], r[8] = {};
+    load_vec<float, 8>(g + l15 * kES + d, w);
+    if (start >= 0) load_vec<float, 8>(g + start * kES + d, r);
+    load_vec<bf16_t, 8>(k + l15 * kKS + d, x);
+    load_vec<bf16_t, 8>(q + l15 * kKS + d, y);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float f = __builtin_amdgcn_exp2f(w[e] - r[e]);
+      x[e] *= f;
+      y[e] *= f;
+    }
+    split8(x, kh[i], kl[i]);
+    bf16x8_t rest;
+    split8(y, qh[i], rest);
+  }
+#pragma unroll
+  for (int part = 1; part < 4; ++part) {
+    floatx4_t pk = {0.f, 0.f, 0.f, 0.f}, pq = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < kN; ++i) {
+      const int d = 32 * i + 8 * g4;
+      float x[8], w[8], r[8];
+      load_vec<float, 8>(g + l15 * kES + d, w);
+      load_vec<float, 8>(g + (4 * part - 1) * kES + d, r);
+      load_vec<bf16_t, 8>(k + l15 * kKS + d, x);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] *= __builtin_amdgcn_exp2f(fminf(r[e] - w[e], 0.f));
+      bf16x8_t hi, low;
+      split8(x, hi, low);
+      pk = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kh[i], hi, pk, 0, 0, 0);
+      pq = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh[i], hi, pq, 0, 0, 0);
+      pk = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kh[i], low, pk, 0, 0, 0);
+      pq = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh[i], low, pq, 0, 0, 0);
+      pk = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kl[i], hi, pk, 0, 0, 0);
+    }
+    if (g4 == part) {
+      dk = pk;
+      dq = pq;
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const float vk = __shfl(in_k, 16 * g4 + 4 * e + (l15 & 3)), vq = __shfl(in_q, 16 * g4 + 4 * e + (l15 & 3));
+    if ((l15 >> 2) == g4) {
+      dk[e] = vk;
+      dq[e] = vq;
+    }
+  }
 }
 
 template <int DP>
@@ -176,39 +257,19 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
   floatx4_t dk = {0.f, 0.f, 0.f, 0.f}, dq = {0.f, 0.f, 0.f, 0.f};    // a steep diagonal block's sums: row 4 g4 + e, column l15
   if (steep) {
 #pragma unroll
-    for (int t = 0; t < kB; ++t) {
-      const float ki = lane_value(kinv, 4 * t), x = bf16lo(kw[t]) * ki, y = bf16hi(kw[t]) * ki;
-      const uint32_t hi = pack_bf16x2(x, y);
+    for (int t = 0; t < kB; ++t) {                               // log-decays and the plain vectors, where products with them will be
       if (!mine) continue;
       *reinterpret_cast<float2*>(ke_b + t * kES + c0) = make_float2(gx[t], gy[t]);
-      *reinterpret_cast<uint32_t*>(kph_b + t * kKS + c0) = hi;
-      *reinterpret_cast<uint32_t*>(kpl_b + t * kKS + c0) = pack_bf16x2(x - bf16lo(hi), y - bf16hi(hi));
+      *reinterpret_cast<uint32_t*>(kph_b + t * kKS + c0) = kw[t];
+      *reinterpret_cast<uint32_t*>(kpl_b + t * kKS + c0) = qw[t];
     }
     wave_fence();
+    steep_block<DP>(ke_b, kph_b, kpl_b, dk, dq);
+    const float ks = __shfl(kinv, 4 * l15);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      const int t = 4 * g4 + e;
-      float sum = 0.f;
-      for (int d = 0; d < a.D; ++d) {
-        const float w = __builtin_amdgcn_exp2f(fminf(ke_b[t * kES + d] - ke_b[l15 * kES + d], 0.f));
-        sum += w * (bf16_to_f32(kph_b[t * kKS + d]) + bf16_to_f32(kpl_b[t * kKS + d])) * (bf16_to_f32(kph_b[l15 * kKS + d]) + bf16_to_f32(kpl_b[l15 * kKS + d]));
-      }
-      dk[e] = sum;
-    }
-    wave_fence();
-#pragma unroll
-    for (int t = 0; t < kB; ++t) {
-      const float qi = lane_value(qinv, 4 * t);
-      if (mine) *reinterpret_cast<uint32_t*>(kpl_b + t * kKS + c0) = pack_bf16x2(bf16lo(qw[t]) * qi, bf16hi(qw[t]) * qi);
-    }
-    wave_fence();
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int t = 4 * g4 + e;
-      float sum = 0.f;
-      for (int d = 0; d < a.D; ++d)
-        sum += __builtin_amdgcn_exp2f(fminf(ke_b[t * kES + d] - ke_b[l15 * kES + d], 0.f)) * bf16_to_f32(kpl_b[t * kKS + d]) * bf16_to_f32(kph_b[l15 * kKS + d]);
-      dq[e] = sum;
+      dk[e] *= ks * __shfl(kinv, 4 * (4 * g4 + e));
+      dq[e] *= ks * __shfl(qinv, 4 * (4 * g4 + e));
     }
     wave_fence();
   }

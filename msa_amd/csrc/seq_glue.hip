@@ -242,7 +242,7 @@ __global__ __launch_bounds__(256) void rms_residual_kernel(RmsResidual a) {
   const float* xr = a.x_in + row * a.W;
   const T* yr = a.y ? static_cast<const T*>(a.y) + row * a.y_stride : nullptr;
   float* xo = a.y ? a.x_out + row * a.W : nullptr;
-  float x[kKeep][VEC], y[kKeep][VEC];
+  float x[kKeep][VEC], y[kKeep][VEC], w[kKeep][VEC];             // (everything is requested before the first sum)
   auto sum_of = [&](float v, int which) {
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
@@ -258,10 +258,14 @@ __global__ __launch_bounds__(256) void rms_residual_kernel(RmsResidual a) {
     load_vec<float, VEC>(xr + i, x[k]);
     if (!a.y) continue;
     load_vec<T, VEC>(yr + i, y[k]);
-#pragma unroll
-    for (int e = 0; e < VEC; ++e) ssq += y[k][e] * y[k][e];
+    load_vec<float, VEC>(a.w + i, w[k]);
   }
   if (a.y) {
+#pragma unroll
+    for (int k = 0; k < kKeep; ++k)
+      if ((k * 256 + tid) * VEC < a.W)
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) ssq += y[k][e] * y[k][e];
     for (int i = (kKeep * 256 + tid) * VEC; i < a.W; i += 256 * VEC) {
       float v[VEC];
       load_vec<T, VEC>(yr + i, v);
@@ -273,29 +277,28 @@ __global__ __launch_bounds__(256) void rms_residual_kernel(RmsResidual a) {
   const float inv = a.y ? 1.0f / sqrtf(ssq / (float)a.W + a.eps) : 0.f;
   const bool norm = a.next_w != nullptr;
   float next_ssq = 0.f;
-  auto combine = [&](int i, float (&xv)[VEC], const float (&yv)[VEC]) {
-    float w[VEC];
-    load_vec<float, VEC>(a.w + i, w);
+  auto combine = [&](int i, float (&xv)[VEC], const float (&yv)[VEC], const float (&wv)[VEC]) {
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) xv[e] += yv[e] * inv * w[e];
+    for (int e = 0; e < VEC; ++e) xv[e] += yv[e] * inv * wv[e];
     store_vec<float, VEC>(xo + i, xv);
   };
 #pragma unroll
   for (int k = 0; k < kKeep; ++k) {
     const int i = (k * 256 + tid) * VEC;
     if (i >= a.W) break;
-    if (a.y) combine(i, x[k], y[k]);
+    if (a.y) combine(i, x[k], y[k], w[k]);
     if (norm)
 #pragma unroll
       for (int e = 0; e < VEC; ++e) next_ssq += x[k][e] * x[k][e];
     else if (a.h) store_vec<T, VEC>(static_cast<T*>(a.h) + row * a.W + i, x[k]);
   }
   for (int i = (kKeep * 256 + tid) * VEC; i < a.W; i += 256 * VEC) {
-    float xv[VEC], yv[VEC];
+    float xv[VEC], yv[VEC], wv[VEC];
     load_vec<float, VEC>(xr + i, xv);
     if (a.y) {
       load_vec<T, VEC>(yr + i, yv);
-      combine(i, xv, yv);
+      load_vec<float, VEC>(a.w + i, wv);
+      combine(i, xv, yv, wv);
     }
     if (norm)
 #pragma unroll

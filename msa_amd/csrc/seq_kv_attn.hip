@@ -20,39 +20,51 @@ __device__ __forceinline__ int64_t first_key(int64_t pos, int32_t chunk) { retur
 // ------------------------------------------------------------------------------------------------ preparation
 constexpr int kMaxPairs = 256;
 
-// cos and sin of position * freq for every pair.  The angle is reduced in fp64, so that its error does not grow with the position.
+// cos and sin of position * freq for every pair.  The angle is reduced to an eighth of a turn in fp64, so that its error does not
+// grow with the position; there the Taylor series are exact to fp32.
+__device__ __forceinline__ float2 cos_sin(double angle) {
+  const double t = angle * 0.63661977236758134308, n = rint(t);          // quarter turns
+  const float x = (float)((t - n) * 1.57079632679489661923), s = x * x;
+  const float sn = x * (1.f + s * (-1.6666667e-1f + s * (8.3333333e-3f + s * (-1.9841270e-4f + s * 2.7557319e-6f))));
+  const float cn = 1.f + s * (-0.5f + s * (4.1666667e-2f + s * (-1.3888889e-3f + s * (2.4801587e-5f - s * 2.7557319e-7f))));
+  const int quarter = (int)(n - 4.0 * floor(n * 0.25));
+  const float c = quarter & 1 ? sn : cn, v = quarter & 1 ? cn : sn;
+  return make_float2(quarter == 1 || quarter == 2 ? -c : c, quarter >= 2 ? -v : v);
+}
 __device__ __forceinline__ void rotation_table(float2* cs, const double* freqs, int32_t n_pairs, int64_t pos) {
-  for (int i = threadIdx.x; i < n_pairs; i += 256) {
-    const double a = (double)pos * freqs[i] * 0.3183098861837906715;        // half turns
-    const double r = a - 2.0 * rint(a * 0.5);
-    float s, c;
-    sincospif((float)r, &s, &c);
-    cs[i] = make_float2(c, s);
-  }
+  for (int i = threadIdx.x; i < n_pairs; i += 256) cs[i] = cos_sin((double)pos * freqs[i]);
   __syncthreads();
 }
 
 template <typename T, int LANES>
 __global__ __launch_bounds__(256) void qk_rope_append_vec_kernel(msa_qk_rope_args a, msa_seq_batch b) {
   __shared__ float2 cs[kMaxPairs];
+  constexpr int kHeads = 256 / LANES;
   const int row = blockIdx.x, s = b.row_seq[row];
   const int64_t pos = b.pos[s] + (row - b.cu[s]);
-  rotation_table(cs, a.freqs, a.n_pairs, pos);
   const int lane = threadIdx.x % LANES, d = lane * 8, half = a.n_pairs / 8;
   const int heads = a.H + (a.k ? a.G : 0);
   const int64_t cache_row = (int64_t)b.slot[s] * a.Lcap + pos;
-  for (int h0 = 0; h0 < heads; h0 += 256 / LANES) {
-    const int h = h0 + threadIdx.x / LANES;
-    const bool live = h < heads, query = h < a.H, in = live && d < a.D;
+  const int h_first = blockIdx.y * kHeads, h_step = gridDim.y * kHeads;
+  float x[8], w[8];
+  auto fetch = [&](int h0) {
+    // (lanes without a head or dimensions read some other's and count nothing)
+    const int h = min(h0 + (int)threadIdx.x / LANES, heads - 1), at = d < a.D ? d : 0;
+    const bool query = h < a.H;
     const T* src = query ? static_cast<const T*>(a.q) + row * a.q_stride + (int64_t)h * a.D
                          : static_cast<const T*>(a.k) + row * a.k_stride + (int64_t)(h - a.H) * a.D;
-    float x[8] = {}, w[8] = {}, ssq = 0.f;
-    if (in) {
-      load_vec<T, 8>(src + d, x);
-      load_vec<float, 8>((query ? a.q_norm : a.k_norm) + d, w);
-    }
+    load_vec<T, 8>(src + at, x);
+    load_vec<float, 8>((query ? a.q_norm : a.k_norm) + at, w);
+  };
+  fetch(h_first);                        // (on its way while the table is made)
+  rotation_table(cs, a.freqs, a.n_pairs, pos);
+  for (int h0 = h_first; h0 < heads; h0 += h_step) {
+    const int h = h0 + threadIdx.x / LANES;
+    const bool query = h < a.H, in = h < heads && d < a.D;
+    if (h0 != h_first) fetch(h0);
+    float ssq = 0.f;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) ssq += x[e] * x[e];
+    for (int e = 0; e < 8; ++e) ssq += in ? x[e] * x[e] : 0.f;
 #pragma unroll
     for (int o = LANES / 2; o > 0; o >>= 1) ssq += __shfl_xor(ssq, o);
     const float inv = 1.0f / sqrtf(ssq / (float)a.D + a.eps);
@@ -76,7 +88,7 @@ __global__ __launch_bounds__(256) void qk_rope_append_vec_kernel(msa_qk_rope_arg
     if (query || pos < a.Lcap) store_vec<T, 8>(dst + d, x);
   }
   if (a.k && pos < a.Lcap)
-    for (int i = threadIdx.x * 8; i < a.G * a.E; i += 256 * 8) {
+    for (int i = (blockIdx.y * 256 + threadIdx.x) * 8; i < a.G * a.E; i += gridDim.y * 256 * 8) {
       float v[8];
       load_vec<T, 8>(static_cast<const T*>(a.v) + row * a.v_stride + i, v);
       store_vec<T, 8>(static_cast<T*>(a.v_cache) + cache_row * a.G * a.E + i, v);
@@ -133,10 +145,15 @@ template <typename T>
 int launch_prepare(const msa_qk_rope_args& a, const msa_seq_batch& b, hipStream_t st) {
   const bool vec = vec_ok(8, {a.q, a.k, a.v, a.q_norm, a.k_norm, a.q_out, a.k_cache, a.v_cache},
                           {a.q_stride, a.k ? a.k_stride : 0, a.k ? a.v_stride : 0, a.D, a.E, a.n_pairs});
+  // few rows: a workgroup per set of heads
+  auto grid = [&](int lanes) {
+    const int heads = a.H + (a.k ? a.G : 0), per = 256 / lanes;
+    return dim3(b.rows, b.rows <= device_compute_units() ? (heads + per - 1) / per : 1);
+  };
   if (!vec) qk_rope_append_kernel<T><<<b.rows, 256, 0, st>>>(a, b);
-  else if (a.D <= 64) qk_rope_append_vec_kernel<T, 8><<<b.rows, 256, 0, st>>>(a, b);
-  else if (a.D <= 128) qk_rope_append_vec_kernel<T, 16><<<b.rows, 256, 0, st>>>(a, b);
-  else qk_rope_append_vec_kernel<T, 64><<<b.rows, 256, 0, st>>>(a, b);
+  else if (a.D <= 64) qk_rope_append_vec_kernel<T, 8><<<grid(8), 256, 0, st>>>(a, b);
+  else if (a.D <= 128) qk_rope_append_vec_kernel<T, 16><<<grid(16), 256, 0, st>>>(a, b);
+  else qk_rope_append_vec_kernel<T, 64><<<grid(64), 256, 0, st>>>(a, b);
   MSA_LAUNCH_CHECK();
   return MSA_OK;
 }
@@ -399,12 +416,17 @@ __global__ __launch_bounds__(256) void kv_combine_kernel(SplitArgs p, int64_t it
   if (a.gate) f *= sigmoid_f(bf16_to_f32(static_cast<const bf16_t*>(a.gate)[row * a.gate_stride + head]));
   for (int c = lane * 4; c < a.E; c += 256) {
     float r[4] = {};
-    for (int i = 0; i < p.n_split; ++i) {
-      float x[4];
-      load_vec<float, 4>(p.part_o + (first + (int64_t)i * a.H) * a.E + c, x);
-      const float wi = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(w), i));    // (lanes without columns hold weights too)
+    constexpr int kBatch = 8;                                    // ranges requested at a time
+    for (int i0 = 0; i0 < p.n_split; i0 += kBatch) {
+      float x[kBatch][4];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) r[e] += wi * x[e];
+      for (int i = 0; i < kBatch; ++i) load_vec<float, 4>(p.part_o + (first + (int64_t)min(i0 + i, p.n_split - 1) * a.H) * a.E + c, x[i]);
+#pragma unroll
+      for (int i = 0; i < kBatch; ++i) {                         // (lanes without columns hold weights too, 0 behind the last range)
+        const float wi = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(w), min(i0 + i, 63)));
+#pragma unroll
+        for (int e = 0; e < 4; ++e) r[e] += i0 + i < p.n_split ? wi * x[i][e] : 0.f;
+      }
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) r[e] *= f;
