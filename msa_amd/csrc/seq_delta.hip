@@ -197,6 +197,7 @@ int launch_scan(const msa_delta_args& a, const msa_seq_batch& b, hipStream_t st)
   if (a.D <= 16) launch_scan<T, 4, 4>(a, b, st);
   else if (a.D <= 32) launch_scan<T, 8, 4>(a, b, st);
   else if (a.D <= 64) launch_scan<T, 16, 4>(a, b, st);
+  else if (a.D <= 128 && (int64_t)a.H * b.n_seq <= device_compute_units() / 2) launch_scan<T, 16, 8>(a, b, st);    // (twice the wavefronts when compute units are free)
   else if (a.D <= 128) launch_scan<T, 32, 4>(a, b, st);
   else if (a.D <= 256) launch_scan<T, 32, 8>(a, b, st);
   else launch_scan<T, 64, 8>(a, b, st);

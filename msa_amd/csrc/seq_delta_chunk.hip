@@ -6,10 +6,11 @@
 //   U   = U' - W S_0,   U' = T diag(beta) V,   W = T diag(beta) (2^G K)
 //   o_t = S_0^T (2^G_t q_t) + sum_{s <= t} A_ts u_s,   A_ts = sum_d q_td k_sd 2^(G_td - G_sd)
 //   S   = 2^G_end S_0 + sum_s (2^(G_end - G_s) k_s) u_s^T.
-//   (1) delta_prepare_kernel  a workgroup per (chunk, head): everything that does not need S_0
-//   (2) delta_state_kernel    a workgroup per (sequence, head, 16 or 32 value columns) walks over the chunks: U, o and S
+//   (1) prepare_chunk  a workgroup per (chunk, head): everything that does not need S_0
+//   (2) StateWalk      a workgroup per (sequence, head, 16 or 32 value columns) walks over the chunks: U, o and S
 //   (3) msa_seq_head_norm_gate
-// Chunks are prepared a segment at a time, which bounds the workspace.
+// (1) is bound by memory and arithmetic, (2) by the latency of its chain, so they share launches: one launch prepares a segment of
+// chunks while it walks over the segment before.  Segments also bound the workspace (two of them).
 //
 // Decays differ by channel, so L and A are products of operands that carry them: within blocks of 16 tokens everything is
 // relative to the block's start (rows, exponents <= 0) and its end (columns, exponents <= 0), and whole blocks' decays between
@@ -168,10 +169,9 @@ constexpr int prepare_lds() {
 }
 
 template <int DP>
-__global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_seq_batch b) {
+__device__ __forceinline__ void prepare_chunk(const ChunkArgs& c, const msa_seq_batch& b, char* lds, int head, int chunk, int s) {
   constexpr int kKS = DP + 8, kES = DP + 4, kN = DP / 32;
   constexpr int kKE = kC * kES * 4, kTV = 2 * kC * kTS * 2 + kC * kVS * 2;
-  extern __shared__ __align__(16) char lds[];
   bf16_t* kph = reinterpret_cast<bf16_t*>(lds);                  // [64][kKS] 2^(G - block start) k, high
   bf16_t* kpl = kph + kC * kKS;                                  // and low parts
   char* shared = lds + 2 * kC * kKS * 2;
@@ -189,10 +189,10 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
 
   const msa_delta_args& a = c.d;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l15 = lane & 15, g4 = lane >> 4;
-  const int head = blockIdx.x, s = blockIdx.z, kvh = head / (a.H / a.G);
-  const int lo = b.cu[s], t0 = (c.first + blockIdx.y) * kC, rows = min(kC, b.cu[s + 1] - lo - t0);
+  const int kvh = head / (a.H / a.G);
+  const int lo = b.cu[s], t0 = (c.first + chunk) * kC, rows = min(kC, b.cu[s + 1] - lo - t0);
   if (rows <= 0) return;
-  char* unit = c.ws + (((int64_t)s * a.H + head) * c.seg + blockIdx.y) * c.unit;
+  char* unit = c.ws + (((int64_t)s * a.H + head) * c.seg + chunk) * c.unit;
   const int brow = kB * wave, live = rows - brow;                // this wavefront's block and its tokens (may be none)
   const bf16_t* qkv = static_cast<const bf16_t*>(a.qkv) + (int64_t)(lo + t0) * a.qkv_stride;
   const bf16_t* kp = qkv + (int64_t)brow * a.qkv_stride + (int64_t)(a.G + kvh) * a.D;
@@ -562,9 +562,9 @@ __global__ __launch_bounds__(256, 2) void delta_prepare_kernel(ChunkArgs c, msa_
 
 // A workgroup takes CT tiles of 16 value columns.  Wavefronts 0 and 1 make U of 32 tokens each, wavefronts 2 and 3 the outputs, and
 // wavefront w < DP / 32 owns 32 state rows, whose fragments all of them read.  Two barriers a chunk: S -> U, U -> S; the outputs'
-// part with U follows beside the next chunk's first half.  A chunk's operands are requested two chunks ahead.  The two kinds run
-// code of their own (with the same barriers), in which no load is conditional (what lies outside a buffer reads as zero), so that
-// the waits are counted.
+// part with U follows beside the next chunk's first half.  A chunk's operands are requested as soon as the registers of the chunk
+// before are free.  The two kinds run code of their own (with the same barriers), in which no load is conditional (what lies outside
+// a buffer reads as zero), so that the waits are counted.
 template <int DP, int CT>
 struct StateWalk {
   static constexpr int kN = DP / 32;
@@ -599,10 +599,9 @@ struct StateWalk {
   static __device__ __forceinline__ u32x4_t load(__amdgpu_buffer_rsrc_t rs, int at) { return __builtin_amdgcn_raw_buffer_load_b128(rs, at, 0, 0); }
 
   template <bool kMakesU>
-  static __device__ __forceinline__ void run(const ChunkArgs& c, const msa_seq_batch& b, Shared& sh, int wave) {
+  static __device__ __forceinline__ void run(const ChunkArgs& c, const msa_seq_batch& b, Shared& sh, int wave, int head, int tile0, int s) {
     const msa_delta_args& a = c.d;
     const int lane = threadIdx.x & 63, l15 = lane & 15, g4 = lane >> 4, pair = wave & 1;
-    const int head = blockIdx.x, s = blockIdx.z, tile0 = blockIdx.y * CT;
     const int lo = b.cu[s], n_tok = b.cu[s + 1] - lo - c.first * kC;
     const int n = min(c.seg, (n_tok + kC - 1) / kC);
     const int col = tile0 * 16 + l15, d0 = 32 * wave + 4 * g4, row_elems = a.H * a.E;
@@ -623,7 +622,7 @@ struct StateWalk {
     const int k_at = own ? Layout<DP>::k + wave * 8192 + lane * 16 : kOutside, g_at = own ? Layout<DP>::gamma + d0 * 4 : kOutside;
     using O = Ops<kMakesU>;
     auto chunk_rsrc = [&](int i) {
-      return __builtin_amdgcn_make_buffer_rsrc(const_cast<char*>(units + (int64_t)min(i, n - 1) * c.unit), 0, (int)c.unit, 0x00020000);
+      return __builtin_amdgcn_make_buffer_rsrc(const_cast<char*>(units + (int64_t)max(0, min(i, n - 1)) * c.unit), 0, (int)c.unit, 0x00020000);
     };
     auto load_p = [&](O& o, int i) {
       const __amdgpu_buffer_rsrc_t rs = chunk_rsrc(i);
@@ -679,10 +678,10 @@ struct StateWalk {
 #pragma unroll
             for (int t = 0; t < 2; ++t) out.t[j][t] = mul(pair ? o.a[2 * t + kk] : o.a[t], sh.u[i & 1][kk][j][h][lane], out.t[j][t]);
       }
-      load_x(o, i + 2);
+      load_x(o, i + 1);
       store(i);
     };
-    auto step = [&](O& o, O& before, int i) {
+    auto step = [&](O& o, int i) {
       __syncthreads();
       u32x4_t f[kN][CT][2];
 #pragma unroll
@@ -707,9 +706,9 @@ struct StateWalk {
 #pragma unroll
               for (int t = 0; t < 2; ++t) u.t[j][t] = mul(o.p[t][kk][x >> 1], f[kk][j][x & 1], u.t[j][t]);
         share(u, sh.u[i & 1][pair], lane);
-        load_x(o, i + 2);
+        load_x(o, i + 1);
       } else {
-        finish(before, i - 1);                                   // (in front of the first chunk: nothing is written)
+        finish(o, i - 1);                                   // (in front of the first chunk: nothing is written)
 #pragma unroll
         for (int j = 0; j < CT; ++j) out.t[j][0] = out.t[j][1] = none;
 #pragma unroll
@@ -721,7 +720,7 @@ struct StateWalk {
 #pragma unroll
               for (int t = 0; t < 2; ++t) out.t[j][t] = mul(o.p[t][kk][0], f[kk][j][h], out.t[j][t]);
       }
-      load_p(o, i + 2);
+      load_p(o, i + 1);
       __syncthreads();
       if (own) {
         u32x4_t g[2][CT][2];
@@ -746,37 +745,16 @@ struct StateWalk {
               for (int t = 0; t < 2; ++t) S.t[j][t] = mul(o.k[t][kk][x >> 1], g[kk][j][x & 1], S.t[j][t]);
         share(S, sh.s[wave], lane);
       }
-      load_k(o, i + 2);
+      load_k(o, i + 1);
     };
-    O x0, x1;
-    // (in the order the loop makes them, stores included, so that the first pass counts like the others)
-    if constexpr (kMakesU) {
-      load_x(x0, 0);
-      load_p(x0, 0);
-      load_k(x0, 0);
-      load_x(x1, 1);
-      load_p(x1, 1);
-      load_k(x1, 1);
-    } else {
-      load_x(x1, 1);
-      store(-2);
-      load_p(x0, 0);
-      load_k(x0, 0);
-      load_x(x0, 0);
-      store(-1);
-      load_p(x1, 1);
-      load_k(x1, 1);
-    }
+    O o;
+    load_x(o, 0);                // (in the order the loop makes them, stores included, so that the first pass counts like the others)
+    if constexpr (!kMakesU) store(-1);
+    load_p(o, 0);
+    load_k(o, 0);
     if (own) share(S, sh.s[wave], lane);
-    for (int i = 0; i + 1 < n; i += 2) {
-      step(x0, x1, i);
-      step(x1, x0, i + 1);
-    }
-    if (n & 1) step(x0, x1, n - 1);
-    if constexpr (!kMakesU) {
-      if (n & 1) finish(x0, n - 1);
-      else finish(x1, n - 1);
-    }
+    for (int i = 0; i < n; ++i) step(o, i);
+    if constexpr (!kMakesU) finish(o, n - 1);
     if (!own) return;
 #pragma unroll
     for (int i = 0; i < CT; ++i)
@@ -788,16 +766,28 @@ struct StateWalk {
   }
 };
 
+// Workgroups 0 .. n_walk - 1 walk over the chunks of `walk`, the others prepare those of `prep`.  Either part's workgroups of a head
+// follow one another at a distance of H, so that with a multiple of eight heads they share an L2.
 template <int DP, int CT>
-__global__ __launch_bounds__(256, 1) void delta_state_kernel(ChunkArgs c, msa_seq_batch b) {
-  __shared__ typename StateWalk<DP, CT>::Shared sh;
-  if (b.cu[blockIdx.z + 1] - b.cu[blockIdx.z] <= c.first * kC) return;
-  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  if (wave < 2) StateWalk<DP, CT>::template run<true>(c, b, sh, wave);
-  else StateWalk<DP, CT>::template run<false>(c, b, sh, wave);
+__global__ __launch_bounds__(256, 2) void delta_chunk_kernel(ChunkArgs walk, ChunkArgs prep, int32_t n_walk, int32_t n_prep, msa_seq_batch b) {
+  extern __shared__ __align__(16) char lds[];
+  static_assert(sizeof(typename StateWalk<DP, CT>::Shared) <= prepare_lds<DP>(), "either part's tiles");
+  const int H = walk.d.H;
+  if ((int)blockIdx.x < n_walk) {
+    const int head = blockIdx.x % H, rest = blockIdx.x / H, tiles = ((walk.d.E + 15) / 16 + CT - 1) / CT, s = rest / tiles;
+    if (b.cu[s + 1] - b.cu[s] <= walk.first * kC) return;
+    auto& sh = *reinterpret_cast<typename StateWalk<DP, CT>::Shared*>(lds);
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    if (wave < 2) StateWalk<DP, CT>::template run<true>(walk, b, sh, wave, head, rest % tiles * CT, s);
+    else StateWalk<DP, CT>::template run<false>(walk, b, sh, wave, head, rest % tiles * CT, s);
+  } else {
+    const int id = blockIdx.x - n_walk, head = id % H, rest = id / H;
+    prepare_chunk<DP>(prep, b, lds, head, rest % n_prep, rest / n_prep);
+  }
 }
 
-constexpr int64_t kMaxWorkspace = (int64_t)1 << 29;
+constexpr int64_t kMaxSegment = (int64_t)88 << 20;        // bytes: two segments stay in the memory-side cache
+constexpr int kSegments = 6, kLeastChunks = 22;           // segments of a long portion, chunks that are worth a launch
 
 int64_t unit_bytes(int32_t D, int32_t E) {
   switch ((D + 31) / 32) {
@@ -807,37 +797,48 @@ int64_t unit_bytes(int32_t D, int32_t E) {
     default: return Layout<128>::bytes(E);
   }
 }
-// Chunks prepared at a time: as many as the workspace holds, in segments of equal size.
+// Chunks of a segment: enough to be worth a launch, few enough to overlap, at most what the workspace holds.
 int segment(const msa_delta_args& a, int32_t max_rows, int32_t n_seq) {
   const int64_t chunks = (max_rows + kC - 1) / kC, per = unit_bytes(a.D, a.E) * a.H * n_seq;
-  const int64_t most = std::min<int64_t>(32768, std::max<int64_t>(1, kMaxWorkspace / per)), parts = (chunks + most - 1) / most;
+  const int64_t most = std::max<int64_t>(1, kMaxSegment / per), want = std::max<int64_t>(kLeastChunks, (chunks + kSegments - 1) / kSegments);
+  const int64_t parts = (chunks + std::min(most, want) - 1) / std::min(most, want);
   return (int)((chunks + parts - 1) / parts);
 }
 
-template <int DP>
-int launch_chunked(ChunkArgs c, const msa_seq_batch& b, hipStream_t st) {
+template <int DP, int CT>
+int launch_chunked(const ChunkArgs& c, const msa_seq_batch& b, hipStream_t st) {
   constexpr int lds = prepare_lds<DP>();
   static_assert(lds <= 80 * 1024, "two workgroups per compute unit");
   static std::atomic<int> raised{0};
-  MSA_HIP(raise_dynamic_lds_limit(raised, reinterpret_cast<const void*>(delta_prepare_kernel<DP>), lds));
-  const int chunks = (b.max_rows + kC - 1) / kC;
-  for (c.first = 0; c.first < chunks; c.first += c.seg) {
-    delta_prepare_kernel<DP><<<dim3(c.d.H, std::min(c.seg, chunks - c.first), b.n_seq), 256, lds, st>>>(c, b);
-    MSA_LAUNCH_CHECK();
-    // narrow column tiles as long as they find compute units
-    const int tiles = (c.d.E + 15) / 16;
-    if ((int64_t)c.d.H * tiles * b.n_seq <= device_compute_units()) delta_state_kernel<DP, 1><<<dim3(c.d.H, tiles, b.n_seq), 256, 0, st>>>(c, b);
-    else delta_state_kernel<DP, 2><<<dim3(c.d.H, (tiles + 1) / 2, b.n_seq), 256, 0, st>>>(c, b);
+  MSA_HIP(raise_dynamic_lds_limit(raised, reinterpret_cast<const void*>(delta_chunk_kernel<DP, CT>), lds));
+  const int chunks = (b.max_rows + kC - 1) / kC, parts = (chunks + c.seg - 1) / c.seg;
+  const int walks = c.d.H * (((c.d.E + 15) / 16 + CT - 1) / CT) * b.n_seq;
+  const int64_t half = c.unit * c.d.H * c.seg * b.n_seq;
+  for (int part = 0; part <= parts; ++part) {
+    ChunkArgs walk = c, prep = c;
+    walk.first = (part - 1) * c.seg;
+    walk.ws = c.ws + ((part + 1) & 1) * half;
+    prep.first = part * c.seg;
+    prep.ws = c.ws + (part & 1) * half;
+    const int n_walk = part > 0 ? walks : 0, n_prep = part < parts ? std::min(c.seg, chunks - prep.first) : 0;
+    delta_chunk_kernel<DP, CT><<<n_walk + c.d.H * n_prep * b.n_seq, 256, lds, st>>>(walk, prep, n_walk, n_prep, b);
     MSA_LAUNCH_CHECK();
   }
   return MSA_OK;
+}
+template <int DP>
+int launch_chunked(const ChunkArgs& c, const msa_seq_batch& b, hipStream_t st) {
+  // narrow column tiles as long as they find compute units
+  if ((int64_t)c.d.H * ((c.d.E + 15) / 16) * b.n_seq <= device_compute_units()) return launch_chunked<DP, 1>(c, b, st);
+  return launch_chunked<DP, 2>(c, b, st);
 }
 
 }  // namespace
 
 extern "C" size_t msa_seq_delta_chunked_workspace_bytes(const msa_delta_args* args, int32_t max_rows, int32_t n_seq) {
   if (!args || max_rows <= 0 || n_seq <= 0 || args->H <= 0 || args->D <= 0 || args->D > 128 || args->E <= 0) return 0;
-  return (size_t)unit_bytes(args->D, args->E) * args->H * n_seq * segment(*args, max_rows, n_seq);
+  const int chunks = (max_rows + kC - 1) / kC, seg = segment(*args, max_rows, n_seq);
+  return (size_t)unit_bytes(args->D, args->E) * args->H * n_seq * seg * (seg < chunks ? 2 : 1);
 }
 
 extern "C" int msa_seq_delta_chunked(const msa_delta_args* args, const msa_seq_batch* batch, void* workspace, size_t workspace_bytes, void* stream) {
@@ -856,6 +857,7 @@ extern "C" int msa_seq_delta_chunked(const msa_delta_args* args, const msa_seq_b
     return MSA_ESIZE;
   }
   const ChunkArgs c{a, static_cast<char*>(workspace), unit_bytes(a.D, a.E), 0, segment(a, batch->max_rows, batch->n_seq)};
+  MSA_REQUIRE((int64_t)a.H * batch->n_seq * std::max<int64_t>(2 * c.seg, (a.E + 15) / 8) < ((int64_t)1 << 30), "msa_seq_delta_chunked: step too large");
   hipStream_t st = as_stream(stream);
   const int tiles = (a.D + 31) / 32;
   const int rc = tiles == 1   ? launch_chunked<32>(c, *batch, st)

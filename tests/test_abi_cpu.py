@@ -92,7 +92,11 @@ def test_seq_validation_errors_without_gpu():
     rope = _lib.QKRopeArgs(4096, None, None, 128, 0, 0, 4096, None, 4096, 4096, None, None, 0, 2, 1, 64, 64, 33, 1e-5)
     assert lib.msa_seq_qk_rope_append(C.byref(rope), 0, C.byref(b), None) == -1 and b"33 pairs" in lib.msa_last_error()
     d = _lib.DeltaArgs(4096, 4096, 4096, 4096, 192, 64, 1, 64, 4096, 4096, 4096, 4096, 4096, 1, 1, 64, 64, 1e-5, 0)
-    assert lib.msa_seq_delta_chunked_workspace_bytes(C.byref(d), 640, 1) == 10 * lib.msa_seq_delta_chunked_workspace_bytes(C.byref(d), 64, 1) > 0
+    size = lambda rows: lib.msa_seq_delta_chunked_workspace_bytes(C.byref(d), rows, 1)
+    assert size(640) == 10 * size(64) > 0 and size(64 * 23) == 24 * size(64)          # (two segments of twelve chunks)
+    d.H = d.G = 64
+    assert size(1 << 20) <= 2 * (88 << 20)                                             # long portions take no more
+    d.H = d.G = 1
     assert lib.msa_seq_delta_chunked(C.byref(d), C.byref(b), 4096, 16, None) == -3 and b"workspace" in lib.msa_last_error()
     d.D = 520
     assert lib.msa_seq_delta_scan(C.byref(d), 0, C.byref(b), None) == -1 and b"D=520" in lib.msa_last_error()

@@ -230,7 +230,7 @@ def test_delta_reads_a_far_write():
 
 
 def test_delta_chunked_in_segments():
-    """More chunks than the workspace holds at a time: as the token-by-token form."""
+    """More chunks than are prepared at a time, in few and in many segments: as the token-by-token form."""
     H, G, D, E, T = 32, 4, 128, 128, 9300
     g = torch.Generator(device="cuda").manual_seed(2)
     bf = lambda *s: torch.randn(s, generator=g, device="cuda").to(BF16)
@@ -243,6 +243,13 @@ def test_delta_chunked_in_segments():
         states.append(state)
     close(outs[1], outs[0], BF16)
     close(states[1], states[0], F32, 2e-4)
+
+
+def test_delta_chunked_segments_of_a_ragged_batch():
+    """Sequences that end in different segments."""
+    c = DeltaCase(2, 1, 32, 24, [1700, 3, 1408, 1409, 900], BF16, seed=11)
+    c.step(c.lens, True)
+    c.finish(3e-4)
 
 
 # ------------------------------------------------------------------------------------------------ rotary attention
