@@ -1,5 +1,6 @@
 /*
- * msa_seq — C ABI of the gfx950 kernels behind the recurrent / latent-attention decoder layers (libmsa_seq.so).
+ * msa_seq — C ABI of the gfx950 kernels behind the decoders of mixed layers: recurrences, latent attention, grouped-query
+ * attention with chunk masks (libmsa_seq.so).
  *
  * Conventions are those of msa_amd.h (0 or a negative MSA_E* code, msa_last_error(), device pointers, everything
  * enqueued on `stream`, no allocation).  On top of them:

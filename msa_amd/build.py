@@ -1,5 +1,5 @@
 """Builds the C-ABI libraries from ``csrc/*.hip`` for gfx950 with hipcc: ``libmsa_amd.so`` (routing / sparse attention)
-and ``libmsa_seq.so`` (recurrent and latent-attention layers).
+and ``libmsa_seq.so`` (the layers of the decoders of mixed layers).
 
 ``python -m msa_amd.build`` compiles both in-tree; the libraries then travel with the source tree.
 """

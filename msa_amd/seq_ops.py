@@ -1,4 +1,4 @@
-"""Torch-tensor front end of ``include/msa_seq.h`` (recurrent and latent-attention layers).  As in :mod:`msa_amd.ops`
+"""Torch-tensor front end of ``include/msa_seq.h`` (the layers of the decoders of mixed layers).  As in :mod:`msa_amd.ops`
 PyTorch owns memory and names streams only; every function enqueues on the current stream and raises on any failure."""
 from __future__ import annotations
 

@@ -278,7 +278,7 @@ class Cache:
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("H,G,D,E,pairs", [(6, 2, 96, 96, 24), (4, 4, 40, 24, 20), (3, 1, 13, 11, 5), (5, 5, 16, 8, 0), (2, 1, 200, 136, 16), (9, 3, 64, 64, 32),
+@pytest.mark.parametrize("H,G,D,E,pairs", [(8, 2, 88, 104, 24), (4, 4, 40, 24, 20), (3, 1, 13, 11, 5), (5, 5, 16, 8, 0), (2, 1, 200, 136, 16), (9, 3, 64, 64, 32),
                                            (2, 2, 512, 16, 256), (1, 1, 1, 1, 0)])
 def test_norm_rotation_and_cache_rows(dtype, H, G, D, E, pairs):
     r = Rand(D)
@@ -319,7 +319,7 @@ def test_rotation_far_out():
     close(got, O.rotate(O.rms(q_.view(2, 1, 64), 1e-5) * w_, [pos, pos + 1], fr), F32)
 
 
-ATTN_SIZES = [(6, 2, 96, 96), (4, 4, 40, 24), (20, 1, 64, 128), (2, 1, 200, 136), (1, 1, 8, 8), (34, 2, 128, 128)]
+ATTN_SIZES = [(8, 2, 88, 104), (4, 4, 40, 24), (20, 1, 64, 128), (2, 1, 200, 136), (1, 1, 8, 8), (34, 2, 128, 128)]
 
 
 @pytest.mark.parametrize("chunk", [0, 1, 7, 64, 100])
@@ -355,7 +355,7 @@ def test_split_attention_long():
 
 
 @pytest.mark.parametrize("chunk", [0, 5, 32, 100, 128, 300])
-@pytest.mark.parametrize("H,G,D,E", [(6, 2, 96, 96), (4, 4, 40, 24), (8, 1, 64, 128), (2, 1, 200, 136), (3, 3, 8, 8)], ids=str)
+@pytest.mark.parametrize("H,G,D,E", [(8, 2, 88, 104), (4, 4, 40, 24), (8, 1, 64, 128), (2, 1, 200, 136), (3, 3, 8, 8)], ids=str)
 def test_prefill_attention(H, G, D, E, chunk):
     r = Rand(chunk + D)
     c = Cache(G, D, E, [0, 77, 0, 130], [150, 129, 1, 40], BF16, seed=H)
